@@ -6,7 +6,8 @@ gives them back when the whole batch is done
 (lite_llama/executor/mem_manager.py:134-263, lite_llama/generate_stream.py:136,188).
 Here the unit is a page of ``page_size`` tokens, pages are taken when a request's
 tokens need them and go back on the free list when the request ends or, for a
-group with a window, when every later query has moved past them. All of it is
+group whose queries read a window or a chunk of the positions, when every later query has moved
+past them. All of it is
 host-side bookkeeping: no device call, no synchronisation.
 
 Cache layers with the same needs form a group; a group has a page pool and, for
@@ -25,7 +26,7 @@ import numpy as np
 
 from ..parts.base import PagedSpec, StateSpec
 
-RELEASED = -1   # block-table entry of a page that was given back (left of the window)
+RELEASED = -1   # block-table entry of a page that was given back (left of the window or chunk)
 
 
 class OutOfPages(RuntimeError):
@@ -78,10 +79,8 @@ class PagedGroup:
     tables: Dict[Hashable, List[int]] = field(default_factory=dict)
 
     def first_needed_page(self, num_tokens: int) -> int:
-        """Index of the first page inside the window of a query at position >= num_tokens."""
-        if self.spec.window is None:
-            return 0
-        return max(0, num_tokens - self.spec.window + 1) // self.page_size
+        """Index of the first page that a query at position >= num_tokens reads (beside kept ones)."""
+        return self.spec.first_needed(num_tokens) // self.page_size
 
     def kept_pages(self) -> int:
         """Pages at the start of a sequence that are never given back: those of the first
@@ -211,12 +210,12 @@ class CacheManager:
 
     def release_behind_window(self, req) -> int:
         """Give back the pages of ``req`` that no later query can read (groups
-        with a window only). Their table entries become RELEASED. Returns the
+        with a window or chunks only). Their table entries become RELEASED. Returns the
         number of pages given back."""
         n = 0
         have = self.num_tokens[req]
         for g in self.paged:
-            if g.spec.window is None:
+            if not g.spec.gives_back:
                 continue
             table = g.tables[req]
             first = min(g.first_needed_page(have), len(table))

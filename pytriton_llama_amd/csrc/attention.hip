@@ -19,12 +19,14 @@
 // later query, at their true positions; their pages are never given back. A kernel walks the
 // keys 0 .. min(keep_first, window start) - 1 and then the window, as one list ("walk index":
 // index v below n_kept is key v, index v from n_kept on is key v + shift).
-// sink (or null): one float a query head; the softmax denominator of that head holds exp(sink)
-// once more, a term without key and value that is not scaled.
+// chunk > 0: a query sees the keys of its own chunk only, chunks of so many positions counted from
+// position 0; pages of chunks before it may be gone too.
+// sink, gate: one more term of a head's denominator, and a factor on its result (attention.h).
 //
 // ptl_attention_generic: vector-FMA kernel, float32 math, storage type T
 // (float32 or bfloat16), any page size, any D up to 640 (beyond 256 with more LDS than a
 // kernel gets unasked: the launcher asks for it).
+#include "attention.h"
 #include "common.h"
 #include "mfma.h"
 #include <math.h>
@@ -44,8 +46,7 @@ attn_generic_kernel(TO* __restrict__ out, long out_stride, const T* __restrict__
                     const int32_t* __restrict__ q_start, const int32_t* __restrict__ ctx_len,
                     const int32_t* __restrict__ block_table, int bt_stride,
                     const int32_t* __restrict__ work_seq, const int32_t* __restrict__ work_qoff,
-                    int Hq, int Hkv, int maps, int Dk, int Dv, int page_size, int window, int keep_first,
-                    const float* __restrict__ sink, float scale) {
+                    int Hq, int Hkv, int maps, int Dk, int Dv, int page_size, AttnExtras ex, float scale) {
   extern __shared__ float lds[];
   float* Qs = lds;                   // [BM][Dk]
   float* Ks = Qs + BM * Dk;          // [BN][Dk+1]
@@ -77,9 +78,10 @@ attn_generic_kernel(TO* __restrict__ out, long out_stride, const T* __restrict__
   const int qpos = cached + qoff + tm;
   const int first_q = cached + qoff;
   const int k_end = min(ctx, first_q + rows);
-  const int k_lo = window > 0 ? max(0, first_q - window + 1) : 0;
+  const int k_lo = first_seen(ex, first_q);
+  const int row_lo = first_seen(ex, qpos);
   // the walk: the kept first keys left of the window, then the keys from the window's start on
-  const int n_kept = min(max(keep_first, 0), k_lo);
+  const int n_kept = min(max(ex.keep_first, 0), k_lo);
   const int shift = k_lo - n_kept;
   const int n_walk = n_kept + (k_end - k_lo);
   const int nd = (Dv + 15) >> 4;
@@ -129,7 +131,7 @@ attn_generic_kernel(TO* __restrict__ out, long out_stride, const T* __restrict__
       float dot = 0.f;
       for (int d = 0; d < Dk; ++d) dot = fmaf(qr[d], kr[d], dot);
       const bool vis = row_valid && kw < n_walk && kp <= qpos &&
-                       (window <= 0 || kp > qpos - window || kp < keep_first);
+                       (kp >= row_lo || kp < ex.keep_first);
       s[j] = vis ? dot * scale : -INFINITY;
       tmax = fmaxf(tmax, s[j]);
     }
@@ -165,13 +167,13 @@ attn_generic_kernel(TO* __restrict__ out, long out_stride, const T* __restrict__
 
   if (row_valid) {
     float den = l_run, f = 1.f;
-    if (sink) {                            // one more term of the denominator: exp(sink)
-      const float sk = sink[head];
+    if (ex.sink) {                         // one more term of the denominator: exp(sink)
+      const float sk = ex.sink[head];
       const float mx = fmaxf(m_run, sk);
       f = expf(m_run - mx);
       den = l_run * f + expf(sk - mx);
     }
-    const float inv = den > 0.f ? f / den : 0.f;
+    const float inv = den > 0.f ? f / den * head_gate(ex, qs + qoff + tm, head) : 0.f;
     TO* o = out + (size_t)(qs + qoff + tm) * out_stride + head * Dv + tc;
 #pragma unroll
     for (int j = 0; j < NJ; ++j)
@@ -184,8 +186,8 @@ static int launch_generic(void* out, long out_stride, const void* q, long q_stri
                           const void* k_cache, const void* v_cache, const int32_t* q_start,
                           const int32_t* ctx_len, const int32_t* block_table, int bt_stride,
                           const int32_t* work_seq, const int32_t* work_qoff, int n_work,
-                          int Hq, int Hkv, int maps, int Dk, int Dv, int page_size, int window,
-                          int keep_first, const float* sink, float scale, hipStream_t stream) {
+                          int Hq, int Hkv, int maps, int Dk, int Dv, int page_size, const AttnExtras& ex,
+                          float scale, hipStream_t stream) {
   const size_t lds = (size_t)(BM * Dk + BN * (Dk + 1) + BN * Dv + BM * BN) * sizeof(float);
   if (lds > 64 * 1024) {
     // more dynamic LDS than a kernel may ask for without saying so beforehand (wide heads only)
@@ -202,8 +204,8 @@ static int launch_generic(void* out, long out_stride, const void* q, long q_stri
   dim3 grid(n_work, Hq);
   attn_generic_kernel<T, TO, BN, NJ><<<grid, 256, lds, stream>>>(
       (TO*)out, out_stride, (const T*)q, q_stride, (const T*)k_cache, (const T*)v_cache, q_start,
-      ctx_len, block_table, bt_stride, work_seq, work_qoff, Hq, Hkv, maps, Dk, Dv, page_size, window,
-      keep_first, sink, scale);
+      ctx_len, block_table, bt_stride, work_seq, work_qoff, Hq, Hkv, maps, Dk, Dv, page_size, ex,
+      scale);
   return ptl_launch_status();
 }
 
@@ -217,16 +219,18 @@ extern "C" int ptl_attention_generic_kv(void* out, long out_stride, int out_f32,
                                         const int32_t* block_table, int bt_stride,
                                         const int32_t* work_seq, const int32_t* work_qoff, int n_work,
                                         int Hq, int Hkv, int maps, int Dk, int Dv, int page_size,
-                                        int window, int keep_first, const float* sink, float scale,
-                                        int dtype, hipStream_t stream) {
+                                        int window, int keep_first, int chunk, const float* sink,
+                                        const float* gate, long gate_stride, float scale, int dtype,
+                                        hipStream_t stream) {
   if (n_work <= 0) return PTL_OK;
+  const AttnExtras ex{window, keep_first, chunk, sink, gate, gate_stride};
   if (Hq <= 0 || Hkv <= 0 || maps <= 0 || Hq % maps || (Hq / maps) % Hkv || Dk <= 0 || Dv <= 0 ||
-      Dk > 640 || Dv > 640 || page_size <= 0 || Hq > 65535)
+      Dk > 640 || Dv > 640 || page_size <= 0 || Hq > 65535 || !extras_ok(ex))
     return PTL_ERR_ARG;
 #define GO(T, TO, BN, NJ)                                                                         \
   launch_generic<T, TO, BN, NJ>(out, out_stride, q, q_stride, k_cache, v_cache, q_start, ctx_len, \
                                 block_table, bt_stride, work_seq, work_qoff, n_work, Hq, Hkv,    \
-                                maps, Dk, Dv, page_size, window, keep_first, sink, scale, stream)
+                                maps, Dk, Dv, page_size, ex, scale, stream)
 #define GO_SIZES(T, TO)                                                                           \
   {                                                                                               \
     /* wide heads (a latent cache of 512 + 64, say): 40 columns a thread, 16 keys a turn */       \
@@ -250,11 +254,12 @@ extern "C" int ptl_attention_generic(void* out, long out_stride, const void* q, 
                                      const int32_t* block_table, int bt_stride,
                                      const int32_t* work_seq, const int32_t* work_qoff, int n_work,
                                      int Hq, int Hkv, int D, int page_size, int window,
-                                     int keep_first, const float* sink, float scale,
-                                     int dtype, hipStream_t stream) {
+                                     int keep_first, int chunk, const float* sink, const float* gate,
+                                     long gate_stride, float scale, int dtype, hipStream_t stream) {
   return ptl_attention_generic_kv(out, out_stride, 0, q, q_stride, k_cache, v_cache, q_start, ctx_len,
                                   block_table, bt_stride, work_seq, work_qoff, n_work, Hq, Hkv, 1, D,
-                                  D, page_size, window, keep_first, sink, scale, dtype, stream);
+                                  D, page_size, window, keep_first, chunk, sink, gate, gate_stride, scale,
+                                  dtype, stream);
 }
 
 // ===========================================================================
@@ -315,8 +320,8 @@ attn_decode_kernel(TO* __restrict__ out, long out_stride, const T* __restrict__ 
                    const int32_t* __restrict__ q_start, const int32_t* __restrict__ ctx_len,
                    const int32_t* __restrict__ block_table, int bt_stride,
                    float* __restrict__ part_acc, float* __restrict__ part_ml,
-                   int Hq, int Hkv, int maps, int Dk, int Dv, int page_size, int window, int keep_first,
-                   const float* __restrict__ sink, float scale, int num_splits, int groups_per_kv) {
+                   int Hq, int Hkv, int maps, int Dk, int Dv, int page_size, AttnExtras ex, float scale,
+                   int num_splits, int groups_per_kv) {
   constexpr int KPW = 64 / LPK;           // keys a wave reads per turn
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int seq = blockIdx.x;
@@ -330,9 +335,9 @@ attn_decode_kernel(TO* __restrict__ out, long out_stride, const T* __restrict__ 
   const int nheads = min(GT, G - hg * GT);
   const int row = q_start[seq];
   const int ctx = ctx_len[seq];
-  const int k_lo = window > 0 ? max(0, ctx - window) : 0;
+  const int k_lo = first_seen(ex, ctx - 1);
   // the walk: the kept first keys left of the window, then the window (indices, not positions)
-  const int n_kept = min(max(keep_first, 0), k_lo);
+  const int n_kept = min(max(ex.keep_first, 0), k_lo);
   const int shift = k_lo - n_kept;
   const int span = ctx - shift;
   const int tile = 4 * KPW;
@@ -451,14 +456,15 @@ attn_decode_kernel(TO* __restrict__ out, long out_stride, const T* __restrict__ 
     }
     const int head = (head0 + h) * maps + map;
     if (num_splits == 1) {
-      if (sink) {                          // one more term of the denominator: exp(sink)
-        const float sk = sink[head];
+      if (ex.sink) {                       // one more term of the denominator: exp(sink)
+        const float sk = ex.sink[head];
         const float mx = fmaxf(mn, sk);
         const float f = expf(mn - mx);
         ll = ll * f + expf(sk - mx);
         a *= f;
       }
-      out[(size_t)row * out_stride + (size_t)head * Dv + d] = from_float<TO>(ll > 0.f ? a / ll : 0.f);
+      out[(size_t)row * out_stride + (size_t)head * Dv + d] =
+          from_float<TO>(ll > 0.f ? a / ll * head_gate(ex, row, head) : 0.f);
     } else {
       const size_t pi = ((size_t)seq * Hq + head) * num_splits + split;
       part_acc[pi * Dv + d] = a;
@@ -471,7 +477,7 @@ template <typename T>
 __global__ void __launch_bounds__(64)
 attn_decode_merge_kernel(T* __restrict__ out, long out_stride, const int32_t* __restrict__ q_start,
                          const float* __restrict__ part_acc, const float* __restrict__ part_ml,
-                         int Hq, int D, int num_splits, const float* __restrict__ sink) {
+                         int Hq, int D, int num_splits, AttnExtras ex) {
   // one wave per (sequence, head): lanes take the splits' (max, denominator) side by side,
   // then the head dimension, with the splits' weights in LDS. The partial results come from
   // other compute units' writes, a long way off: the first 16 splits of the lane's first
@@ -489,7 +495,7 @@ attn_decode_merge_kernel(T* __restrict__ out, long out_stride, const int32_t* __
   float mn = -INFINITY;
   for (int s = lane; s < num_splits; s += 64) mn = fmaxf(mn, part_ml[(base + s) * 2]);
   mn = wave_max(mn);
-  const float sk = sink ? sink[head] : -INFINITY;      // the denominator's term without a key
+  const float sk = ex.sink ? ex.sink[head] : -INFINITY;      // the denominator's term without a key
   mn = fmaxf(mn, sk);
   const float ms = mn == -INFINITY ? 0.f : mn;
   float ll = 0.f;
@@ -499,9 +505,9 @@ attn_decode_merge_kernel(T* __restrict__ out, long out_stride, const int32_t* __
     ll += part_ml[(base + s) * 2 + 1] * w;
   }
   ll = wave_sum(ll);
-  if (sink) ll += expf(sk - ms);
+  if (ex.sink) ll += expf(sk - ms);
   __syncthreads();
-  const float inv = ll > 0.f ? 1.0f / ll : 0.f;
+  const float inv = ll > 0.f ? head_gate(ex, row, head) / ll : 0.f;
   for (int d = lane; d < D; d += 64) {
     float a = 0.f;
     const float* pa = part_acc + base * D + d;
@@ -522,8 +528,8 @@ static int launch_decode(void* out, long out_stride, const void* q, long q_strid
                          const void* k_cache, const void* v_cache, const int32_t* q_start,
                          const int32_t* ctx_len, const int32_t* block_table, int bt_stride,
                          float* part_acc, float* part_ml, int n_seq, int Hq, int Hkv, int maps, int Dk,
-                         int Dv, int page_size, int window, int keep_first, const float* sink,
-                         float scale, int num_splits, hipStream_t stream) {
+                         int Dv, int page_size, const AttnExtras& ex, float scale, int num_splits,
+                         hipStream_t stream) {
   constexpr int GT = 4;
   const int G = (Hq / maps) / Hkv;
   const int groups = (G + GT - 1) / GT;
@@ -531,13 +537,13 @@ static int launch_decode(void* out, long out_stride, const void* q, long q_strid
   const size_t lds = (size_t)(4 * GT * Dv + 4 * GT * 2) * sizeof(float);
   attn_decode_kernel<T, TO, GT, LPK><<<grid, 256, lds, stream>>>(
       (TO*)out, out_stride, (const T*)q, q_stride, (const T*)k_cache, (const T*)v_cache, q_start,
-      ctx_len, block_table, bt_stride, part_acc, part_ml, Hq, Hkv, maps, Dk, Dv, page_size, window,
-      keep_first, sink, scale, num_splits, groups);
+      ctx_len, block_table, bt_stride, part_acc, part_ml, Hq, Hkv, maps, Dk, Dv, page_size, ex,
+      scale, num_splits, groups);
   if (hipGetLastError() != hipSuccess) return PTL_ERR_LAUNCH;
   if (num_splits > 1) {
     dim3 mgrid(n_seq, Hq);
     attn_decode_merge_kernel<TO><<<mgrid, 64, 0, stream>>>((TO*)out, out_stride, q_start, part_acc,
-                                                          part_ml, Hq, Dv, num_splits, sink);
+                                                          part_ml, Hq, Dv, num_splits, ex);
   }
   return ptl_launch_status();
 }
@@ -552,21 +558,22 @@ extern "C" int ptl_attention_decode_kv(void* out, long out_stride, int out_f32, 
                                        const int32_t* q_start, const int32_t* ctx_len,
                                        const int32_t* block_table, int bt_stride, float* part_acc,
                                        float* part_ml, int n_seq, int Hq, int Hkv, int maps, int Dk,
-                                       int Dv, int page_size, int window, int keep_first,
-                                       const float* sink, float scale, int num_splits,
-                                       int dtype, hipStream_t stream) {
+                                       int Dv, int page_size, int window, int keep_first, int chunk,
+                                       const float* sink, const float* gate, long gate_stride,
+                                       float scale, int num_splits, int dtype, hipStream_t stream) {
   if (n_seq <= 0) return PTL_OK;
+  const AttnExtras ex{window, keep_first, chunk, sink, gate, gate_stride};
   if (Hq <= 0 || Hkv <= 0 || maps <= 0 || Hq % maps || (Hq / maps) % Hkv || Dk <= 0 || Dk % 16 ||
       Dk > 256 || Dv <= 0 || Dv % 16 || Dv > 256 || page_size <= 0 || num_splits < 1 ||
-      num_splits > 1024 || (num_splits > 1 && (!part_acc || !part_ml)))
+      num_splits > 1024 || (num_splits > 1 && (!part_acc || !part_ml)) || !extras_ok(ex))
     return PTL_ERR_ARG;
   const int chunks = (Dk > Dv ? Dk : Dv) / 16;
   int lpk = 1;
   while (lpk < chunks) lpk <<= 1;
 #define GO(T, TO, L) launch_decode<T, TO, L>(out, out_stride, q, q_stride, k_cache, v_cache, q_start, \
                                              ctx_len, block_table, bt_stride, part_acc, part_ml,    \
-                                             n_seq, Hq, Hkv, maps, Dk, Dv, page_size, window,       \
-                                             keep_first, sink, scale, num_splits, stream)
+                                             n_seq, Hq, Hkv, maps, Dk, Dv, page_size, ex, scale,    \
+                                             num_splits, stream)
 #define BY_LPK(T, TO)                                                                              \
   switch (lpk) {                                                                                   \
     case 1: return GO(T, TO, 1);                                                                   \
@@ -591,11 +598,13 @@ extern "C" int ptl_attention_decode(void* out, long out_stride, const void* q, l
                                     const int32_t* q_start, const int32_t* ctx_len,
                                     const int32_t* block_table, int bt_stride, float* part_acc,
                                     float* part_ml, int n_seq, int Hq, int Hkv, int D, int page_size,
-                                    int window, int keep_first, const float* sink, float scale,
-                                    int num_splits, int dtype, hipStream_t stream) {
+                                    int window, int keep_first, int chunk, const float* sink,
+                                    const float* gate, long gate_stride, float scale, int num_splits,
+                                    int dtype, hipStream_t stream) {
   return ptl_attention_decode_kv(out, out_stride, 0, q, q_stride, k_cache, v_cache, q_start, ctx_len,
                                  block_table, bt_stride, part_acc, part_ml, n_seq, Hq, Hkv, 1, D, D,
-                                 page_size, window, keep_first, sink, scale, num_splits, dtype, stream);
+                                 page_size, window, keep_first, chunk, sink, gate, gate_stride, scale,
+                                 num_splits, dtype, stream);
 }
 
 // ===========================================================================
@@ -637,8 +646,8 @@ attn_decode_mfma_kernel(bf16_t* __restrict__ out, long out_stride, const bf16_t*
                         const bf16_t* __restrict__ v_cache, const int32_t* __restrict__ q_start,
                         const int32_t* __restrict__ ctx_len, const int32_t* __restrict__ block_table,
                         int bt_stride, float* __restrict__ part_acc, float* __restrict__ part_ml,
-                        int Hq, int Hkv, int page_size, int page_shift, int window, int keep_first,
-                        const float* __restrict__ sink, float scale_log2, int num_splits) {
+                        int Hq, int Hkv, int page_size, int page_shift, AttnExtras ex, float scale_log2,
+                        int num_splits) {
   constexpr int D = 32 * NDT;
   constexpr int NT = 2 * NDT;             // 16-wide tiles of the head dimension
   constexpr int TILE = 64 * UNR;          // keys per turn of the workgroup
@@ -652,10 +661,10 @@ attn_decode_mfma_kernel(bf16_t* __restrict__ out, long out_stride, const bf16_t*
   const int head0 = kvh * G;
   const int row = q_start[seq];
   const int ctx = ctx_len[seq];
-  const int k_lo = window > 0 ? max(0, ctx - window) : 0;
+  const int k_lo = first_seen(ex, ctx - 1);
   // the walk: the kept first keys left of the window, then the window; k_begin, k_end and the
   // keys of a turn are indices of the walk, key_at gives the position
-  const int n_kept = KEPT ? min(max(keep_first, 0), k_lo) : 0;
+  const int n_kept = KEPT ? min(max(ex.keep_first, 0), k_lo) : 0;
   const int shift = k_lo - n_kept;
   const int span = ctx - shift;
   const int per_split = ((span + num_splits - 1) / num_splits + TILE - 1) / TILE * TILE;
@@ -832,14 +841,15 @@ attn_decode_mfma_kernel(bf16_t* __restrict__ out, long out_stride, const bf16_t*
     }
     const int head = head0 + h;
     if (num_splits == 1) {
-      if (sink) {                          // one more term of the denominator: exp(sink)
-        const float sk = sink[head] * 1.4426950408889634f;
+      if (ex.sink) {                       // one more term of the denominator: exp(sink)
+        const float sk = ex.sink[head] * 1.4426950408889634f;
         const float mx = fmaxf(mn, sk);
         const float f = __builtin_amdgcn_exp2f(mn - mx);
         ll = ll * f + __builtin_amdgcn_exp2f(sk - mx);
         a *= f;
       }
-      out[(size_t)row * out_stride + (size_t)head * D + d] = float_to_bf16(ll > 0.f ? a / ll : 0.f);
+      out[(size_t)row * out_stride + (size_t)head * D + d] =
+          float_to_bf16(ll > 0.f ? a / ll * head_gate(ex, row, head) : 0.f);
     } else {
       const size_t pi = ((size_t)seq * Hq + head) * num_splits + split;
       part_acc[pi * D + d] = a;
@@ -854,8 +864,8 @@ static int launch_decode_mfma(void* out, long out_stride, const void* q, long q_
                               const void* k_cache, const void* v_cache, const int32_t* q_start,
                               const int32_t* ctx_len, const int32_t* block_table, int bt_stride,
                               float* part_acc, float* part_ml, int n_seq, int Hq, int Hkv,
-                              int page_size, int window, int keep_first, const float* sink,
-                              float scale, int num_splits, hipStream_t stream) {
+                              int page_size, const AttnExtras& ex, float scale, int num_splits,
+                              hipStream_t stream) {
   constexpr int D = 32 * NDT;
   dim3 grid(n_seq, Hkv, num_splits);
   int page_shift = 0;
@@ -863,21 +873,21 @@ static int launch_decode_mfma(void* out, long out_stride, const void* q, long q_
   const size_t lds_merge = (size_t)(4 * 16 * D + 4 * 16 * 2) * sizeof(float);
   const size_t lds_values = (size_t)4 * UNR * 16 * (D + 16) * sizeof(bf16_t);
   const size_t lds = lds_merge > lds_values ? lds_merge : lds_values;
-  if (window > 0 && keep_first > 0)
+  if (ex.window > 0 && ex.keep_first > 0)
     attn_decode_mfma_kernel<NDT, UNR, true><<<grid, 256, lds, stream>>>(
         (bf16_t*)out, out_stride, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache,
         (const bf16_t*)v_cache, q_start, ctx_len, block_table, bt_stride, part_acc, part_ml, Hq, Hkv,
-        page_size, page_shift, window, keep_first, sink, scale * 1.4426950408889634f, num_splits);
+        page_size, page_shift, ex, scale * 1.4426950408889634f, num_splits);
   else
     attn_decode_mfma_kernel<NDT, UNR, false><<<grid, 256, lds, stream>>>(
         (bf16_t*)out, out_stride, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache,
         (const bf16_t*)v_cache, q_start, ctx_len, block_table, bt_stride, part_acc, part_ml, Hq, Hkv,
-        page_size, page_shift, window, 0, sink, scale * 1.4426950408889634f, num_splits);
+        page_size, page_shift, ex, scale * 1.4426950408889634f, num_splits);
   if (hipGetLastError() != hipSuccess) return PTL_ERR_LAUNCH;
   if (num_splits > 1) {
     dim3 mgrid(n_seq, Hq);
     attn_decode_merge_kernel<bf16_t><<<mgrid, 64, 0, stream>>>((bf16_t*)out, out_stride, q_start,
-                                                              part_acc, part_ml, Hq, D, num_splits, sink);
+                                                              part_acc, part_ml, Hq, D, num_splits, ex);
   }
   return ptl_launch_status();
 }
@@ -888,19 +898,21 @@ extern "C" int ptl_attention_decode_mfma(void* out, long out_stride, const void*
                                          const int32_t* q_start, const int32_t* ctx_len,
                                          const int32_t* block_table, int bt_stride, float* part_acc,
                                          float* part_ml, int n_seq, int Hq, int Hkv, int D,
-                                         int page_size, int window, int keep_first, const float* sink,
+                                         int page_size, int window, int keep_first, int chunk,
+                                         const float* sink, const float* gate, long gate_stride,
                                          float scale, int num_splits, int unroll, hipStream_t stream) {
   if (n_seq <= 0) return PTL_OK;
+  const AttnExtras ex{window, keep_first, chunk, sink, gate, gate_stride};
   if (Hq <= 0 || Hkv <= 0 || Hq % Hkv || Hq / Hkv > 16 || D <= 0 || D % 32 || D > 128 ||
       page_size <= 0 || (page_size & (page_size - 1)) ||
       (long)Hkv * page_size * D * 2 >= (1L << 32) || q_stride % 8 || num_splits < 1 ||
-      num_splits > 1024 || (num_splits > 1 && (!part_acc || !part_ml)) || unroll < 0 || unroll > 2)
+      num_splits > 1024 || (num_splits > 1 && (!part_acc || !part_ml)) || unroll < 0 || unroll > 2 ||
+      !extras_ok(ex))
     return PTL_ERR_ARG;
   if (unroll == 0) unroll = 2;
 #define GO(N, U) launch_decode_mfma<N, U>(out, out_stride, q, q_stride, k_cache, v_cache, q_start,    \
                                           ctx_len, block_table, bt_stride, part_acc, part_ml, n_seq, \
-                                          Hq, Hkv, page_size, window, keep_first, sink, scale,       \
-                                          num_splits, stream)
+                                          Hq, Hkv, page_size, ex, scale, num_splits, stream)
   if (unroll == 1) {
     switch (D / 32) {
       case 1: return GO(1, 1);

@@ -2,6 +2,7 @@
 // The cache layout, the meaning of the arguments and the reference formulas are those of
 // attention.hip; this kernel has a source file of its own because it is compiled with one more
 // option (see max2 below).
+#include "attention.h"
 #include "common.h"
 #include "mfma.h"
 #include <math.h>
@@ -75,8 +76,7 @@ attn_prefill_mfma_kernel(TO* __restrict__ out, long out_stride, const bf16_t* __
                          const int32_t* __restrict__ ctx_len, const int32_t* __restrict__ block_table,
                          int bt_stride, const int32_t* __restrict__ work_seq,
                          const int32_t* __restrict__ work_qoff, int n_work, int Hq, int Hkv, int maps,
-                         int page_size, int page_shift, int window, int keep_first,
-                         const float* __restrict__ sink, float scale_log2) {
+                         int page_size, int page_shift, AttnExtras ex, float scale_log2) {
   constexpr int DK = 32 * NDK, DV = 32 * NDV;
   constexpr int PBM = 64 * RT;
   constexpr int CPRK = DK / 8, CPRV = DV / 8;      // 16-byte chunks per row
@@ -163,8 +163,8 @@ attn_prefill_mfma_kernel(TO* __restrict__ out, long out_stride, const bf16_t* __
   // list is the kept first keys left of the window (positions 0 .. n_kept - 1) and then the
   // positions from the window's start on, index 0 is its first entry, and key_at gives the
   // position of an index.
-  const int win_lo = window > 0 ? max(0, first_q - window + 1) : 0;
-  const int n_kept = KEPT ? min(max(keep_first, 0), win_lo) : 0;
+  const int win_lo = first_seen(ex, first_q);
+  const int n_kept = KEPT ? min(max(ex.keep_first, 0), win_lo) : 0;
   const int shift = KEPT ? win_lo - n_kept : 0;
   const int k_lo = KEPT ? 0 : win_lo;
   const int k_end = min(ctx, first_q + rows) - shift;
@@ -174,11 +174,17 @@ attn_prefill_mfma_kernel(TO* __restrict__ out, long out_stride, const bf16_t* __
   // What a row sees, in indices: its own key is index qw; with kept keys, an index from n_kept on
   // is a key of the window (position index + shift, which is no kept position when shift > 0),
   // an index below is a kept key (a position below keep_first), so key_at is not needed there:
-  //   seen = kw <= qw && kw < k_end && (kw > qw - window || kw < keep_lim)
-  int qw[RT];
+  //   seen = kw <= qw && kw < k_end && (kw >= lo || kw < keep_lim),  lo the row's first key
+  int qw[RT], lo[RT];
 #pragma unroll
-  for (int r = 0; r < RT; ++r) qw[r] = qpos[r] - shift;
-  const int keep_lim = shift == 0 ? keep_first : n_kept;
+  for (int r = 0; r < RT; ++r) {
+    qw[r] = qpos[r] - shift;
+    lo[r] = first_seen(ex, qpos[r]) - shift;
+  }
+  const int keep_lim = shift == 0 ? ex.keep_first : n_kept;
+  // the first keys of the wave's first and last row: left of the one nothing of a tile is seen (no
+  // kept keys), from the other on all rows see it
+  const int wave_lo_first = first_seen(ex, wave_min_q) - shift, wave_lo_last = first_seen(ex, wave_max_q) - shift;
 
   // This thread's chunks of a tile. A wave's load instruction fills 64 consecutive 16-byte
   // slots of LDS, lane l the l-th; slot s holds row s / CPR, chunk (s % CPR) ^ swz(row).
@@ -301,7 +307,7 @@ attn_prefill_mfma_kernel(TO* __restrict__ out, long out_stride, const bf16_t* __
           for (int i = 0; i < 4; ++i) {
             const int kw = k0 + 16 * kt + 4 * lg + i;
             const bool vis = kw <= qw[r] && kw < k_end &&
-                             (window <= 0 || kw > qw[r] - window || (KEPT && kw < keep_lim));
+                             (kw >= lo[r] || (KEPT && kw < keep_lim));
             st[r][kt][i] = vis ? st[r][kt][i] : -INFINITY;
           }
       }
@@ -366,9 +372,8 @@ attn_prefill_mfma_kernel(TO* __restrict__ out, long out_stride, const bf16_t* __
       load_pages(t + 2);
     }
     // a wave whose rows all lie before this tile has nothing to do in it
-    if (wave_has_rows && k0 <= wave_max_q - shift) {
-      // (without a window an index is a position)
-      const bool need_mask = (k0 + PF_BN - 1 > wave_min_q) || (k0 + PF_BN > k_end) || window > 0;
+    if (wave_has_rows && k0 <= wave_max_q - shift && (KEPT || k0 + PF_BN > wave_lo_first)) {
+      const bool need_mask = (k0 + PF_BN - 1 > wave_min_q - shift) || (k0 + PF_BN > k_end) || k0 < wave_lo_last;
       if (need_mask)
         tile(k0, Kb, Vb, std::true_type{});
       else
@@ -391,10 +396,10 @@ attn_prefill_mfma_kernel(TO* __restrict__ out, long out_stride, const bf16_t* __
   for (int r = 0; r < RT; ++r) {
     float l = o[r][2 * NDV][0];                // every row of that tile holds the column's sum
     // one more term of the denominator: exp(sink), in the units of what was summed
-    if (sink) l += __builtin_amdgcn_exp2f(sink[head] * 1.4426950408889634f - m_run[r] * scale_log2);
+    if (ex.sink) l += __builtin_amdgcn_exp2f(ex.sink[head] * 1.4426950408889634f - m_run[r] * scale_log2);
     if (row_ok[r]) {
-      const float inv = l > 0.f ? 1.0f / l : 0.f;
       const int my_row = 16 * (RT * wave + r) + ln;
+      const float inv = l > 0.f ? head_gate(ex, qs + qoff + my_row, head) / l : 0.f;
       TO* op = out + (size_t)(qs + qoff + my_row) * out_stride + (size_t)head * DV + 4 * lg;
 #pragma unroll
       for (int dt = 0; dt < 2 * NDV; ++dt) {
@@ -413,24 +418,22 @@ static int launch_prefill_mfma(void* out, long out_stride, const void* q, long q
                                const void* k_cache, const void* v_cache, const int32_t* q_start,
                                const int32_t* ctx_len, const int32_t* block_table, int bt_stride,
                                const int32_t* work_seq, const int32_t* work_qoff, int n_work,
-                               int n_groups, int Hq, int Hkv, int maps, int page_size, int window,
-                               int keep_first, const float* sink, float scale, hipStream_t stream) {
+                               int n_groups, int Hq, int Hkv, int maps, int page_size, const AttnExtras& ex,
+                               float scale, hipStream_t stream) {
   dim3 grid(Hq, n_groups < 65535 ? n_groups : 65535);
   int page_shift = -1;
   for (int sh = 0; sh < 31; ++sh)
     if ((1 << sh) == page_size) page_shift = sh;
-  if (window > 0 && keep_first > 0)
+  if (ex.window > 0 && ex.keep_first > 0)
     attn_prefill_mfma_kernel<NDK, NDV, RT, TO, true><<<grid, 256, 0, stream>>>(
         (TO*)out, out_stride, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache,
         (const bf16_t*)v_cache, q_start, ctx_len, block_table, bt_stride, work_seq, work_qoff,
-        n_work, Hq, Hkv, maps, page_size, page_shift, window, keep_first, sink,
-        scale * 1.4426950408889634f);
+        n_work, Hq, Hkv, maps, page_size, page_shift, ex, scale * 1.4426950408889634f);
   else
     attn_prefill_mfma_kernel<NDK, NDV, RT, TO, false><<<grid, 256, 0, stream>>>(
         (TO*)out, out_stride, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache,
         (const bf16_t*)v_cache, q_start, ctx_len, block_table, bt_stride, work_seq, work_qoff,
-        n_work, Hq, Hkv, maps, page_size, page_shift, window, 0, sink,
-        scale * 1.4426950408889634f);
+        n_work, Hq, Hkv, maps, page_size, page_shift, ex, scale * 1.4426950408889634f);
   return ptl_launch_status();
 }
 
@@ -441,12 +444,12 @@ static int prefill_same_size(int nd, void* out, long out_stride, const void* q, 
                              const void* k_cache, const void* v_cache, const int32_t* q_start,
                              const int32_t* ctx_len, const int32_t* block_table, int bt_stride,
                              const int32_t* work_seq, const int32_t* work_qoff, int n_work, int n_groups,
-                             int Hq, int Hkv, int page_size, int window, int keep_first, const float* sink,
-                             float scale, hipStream_t stream) {
+                             int Hq, int Hkv, int page_size, const AttnExtras& ex, float scale,
+                             hipStream_t stream) {
 #define GO(N) launch_prefill_mfma<N, N, RT, bf16_t>(out, out_stride, q, q_stride, k_cache, v_cache, q_start, \
                                                     ctx_len, block_table, bt_stride, work_seq, work_qoff,  \
-                                                    n_work, n_groups, Hq, Hkv, 1, page_size, window,     \
-                                                    keep_first, sink, scale, stream)
+                                                    n_work, n_groups, Hq, Hkv, 1, page_size, ex, scale,  \
+                                                    stream)
   switch (nd) {
     case 1: return GO(1);
     case 2: return GO(2);
@@ -467,21 +470,23 @@ extern "C" int ptl_attention_prefill_mfma(void* out, long out_stride, const void
                                           const int32_t* work_seq, const int32_t* work_qoff,
                                           int n_work, int n_groups, int block_rows, int Hq,
                                           int Hkv, int D,
-                                          int page_size, int window, int keep_first,
-                                          const float* sink, float scale, hipStream_t stream) {
+                                          int page_size, int window, int keep_first, int chunk,
+                                          const float* sink, const float* gate, long gate_stride,
+                                          float scale, hipStream_t stream) {
   if (n_work <= 0) return PTL_OK;
+  const AttnExtras ex{window, keep_first, chunk, sink, gate, gate_stride};
   if (Hq <= 0 || Hkv <= 0 || Hq % Hkv || D % 32 || D <= 0 || D > 128 || page_size <= 0 ||
       (page_size & (page_size - 1)) || (long)Hkv * page_size * D * 2 >= (1L << 32) ||
       Hq > 65535 || n_groups < 1 || n_groups > n_work || q_stride % 8 || out_stride % 4 ||
-      (block_rows != 64 && block_rows != 128))
+      (block_rows != 64 && block_rows != 128) || !extras_ok(ex))
     return PTL_ERR_ARG;
   if (block_rows == 64)
     return prefill_same_size<1>(D / 32, out, out_stride, q, q_stride, k_cache, v_cache, q_start, ctx_len,
                                 block_table, bt_stride, work_seq, work_qoff, n_work, n_groups, Hq, Hkv,
-                                page_size, window, keep_first, sink, scale, stream);
+                                page_size, ex, scale, stream);
   return prefill_same_size<2>(D / 32, out, out_stride, q, q_stride, k_cache, v_cache, q_start, ctx_len,
                               block_table, bt_stride, work_seq, work_qoff, n_work, n_groups, Hq, Hkv,
-                              page_size, window, keep_first, sink, scale, stream);
+                              page_size, ex, scale, stream);
 }
 
 // The general form: q [T, Hq, Dk] with Hq = heads * maps, k_cache [pages, Hkv * maps, page_size,
@@ -493,18 +498,20 @@ extern "C" int ptl_attention_prefill_mfma_kv(void* out, long out_stride, int out
                                              const int32_t* block_table, int bt_stride,
                                              const int32_t* work_seq, const int32_t* work_qoff,
                                              int n_work, int n_groups, int Hq, int Hkv, int maps, int Dk,
-                                             int Dv, int page_size, int window, int keep_first,
-                                             const float* sink, float scale, hipStream_t stream) {
+                                             int Dv, int page_size, int window, int keep_first, int chunk,
+                                             const float* sink, const float* gate, long gate_stride,
+                                             float scale, hipStream_t stream) {
   if (n_work <= 0) return PTL_OK;
+  const AttnExtras ex{window, keep_first, chunk, sink, gate, gate_stride};
   if (Hq <= 0 || Hkv <= 0 || maps <= 0 || Hq % maps || (Hq / maps) % Hkv || Dk % 32 || Dk <= 0 ||
       Dk > 128 || Dv % 32 || Dv <= 0 || Dv > 128 || page_size <= 0 || (page_size & (page_size - 1)) ||
       (long)Hkv * maps * page_size * Dk * 2 >= (1L << 32) || (long)Hkv * page_size * Dv * 2 >= (1L << 32) ||
-      Hq > 65535 || n_groups < 1 || n_groups > n_work || q_stride % 8 || out_stride % 4)
+      Hq > 65535 || n_groups < 1 || n_groups > n_work || q_stride % 8 || out_stride % 4 || !extras_ok(ex))
     return PTL_ERR_ARG;
 #define GO(NK, NV, TO)                                                                                  \
   launch_prefill_mfma<NK, NV, 1, TO>(out, out_stride, q, q_stride, k_cache, v_cache, q_start, ctx_len, \
                                      block_table, bt_stride, work_seq, work_qoff, n_work, n_groups, Hq, \
-                                     Hkv, maps, page_size, window, keep_first, sink, scale, stream)
+                                     Hkv, maps, page_size, ex, scale, stream)
 #define BY_V(NK, TO)                   \
   switch (Dv / 32) {                   \
     case 1: return GO(NK, 1, TO);      \

@@ -61,6 +61,17 @@ __device__ __forceinline__ float wave_max(float v) {
   return v;
 }
 
+// Activations of a gated feed-forward (act(gate) * up), float32. gelu_tanh is the tanh form of GELU;
+// (1 + tanh(u)) / 2 = sigmoid(2 u), so it is z * sigmoid(2 sqrt(2 / pi) (z + 0.044715 z^3)).
+#define GLU_SILU 0
+#define GLU_GELU_TANH 1
+__device__ __forceinline__ float gelu_tanh(float z) {
+  return z / (1.0f + expf(-1.5957691216057308f * (z + 0.044715f * z * z * z)));
+}
+__device__ __forceinline__ float glu_act(int act, float g) {
+  return act == GLU_GELU_TANH ? gelu_tanh(g) : g / (1.0f + expf(-g));
+}
+
 // block-wide sum for blockDim.x a multiple of 64, at most 1024; scratch holds 16 floats
 __device__ __forceinline__ float block_sum(float v, float* scratch) {
   v = wave_sum(v);

@@ -455,7 +455,8 @@ extern "C" int ptl_gemm_skinny_add_norm_bf16(void* y, const void* x, const void*
 // ===========================================================================
 // Decode-step products with their follow-up fused in, for at most 16 rows of x:
 //
-// ptl_gate_up_silu_bf16:  out[m, c] = silu(x . Wg[c]) * (x . Wu[c])   (W = [Wg; Wu], [2I, K])
+// ptl_gate_up_silu_bf16:  out[m, c] = act(x . Wg[c]) * (x . Wu[c])   (W = [Wg; Wu], [2I, K]; act SiLU or
+//     the tanh form of GELU)
 // ptl_qkv_rope_store_bf16: q, k, v = x . Wqkv^T; q and k rotated by the angles
 //     positions[m] * inv_freq[j] on the pairs (j, j + D/2); q written out, the
 //     rotated k and v written into the cache pages at slots[m].
@@ -493,7 +494,7 @@ template <int MODE, int U, int ROWS, int XR, bool BLOCKED>
 __global__ void __launch_bounds__(1024)
 gemm_pair_kernel(bf16_t* __restrict__ y, const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
                  int M, int N_out, int K, long ldx, long ldy, int k_per_wave, int pair_offset,
-                 int tiles_per_group, int group_rows, RopeStoreArgs rs, RowScaleArgs sc) {
+                 int tiles_per_group, int group_rows, RopeStoreArgs rs, RowScaleArgs sc, int act) {
   extern __shared__ float red[];                 // [waves][2][64][4]
   __shared__ float row_factor[16];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, ln = lane & 15, lg = lane >> 4;
@@ -612,7 +613,7 @@ gemm_pair_kernel(bf16_t* __restrict__ y, const bf16_t* __restrict__ x, const bf1
     for (int i = 0; i < 4; ++i) {
       // the gate and up products are rounded to bfloat16 as the unfused path stores them
       const float g = round_to<bf16_t>(acc1[i]), u = round_to<bf16_t>(acc2[i]);
-      o.e[i] = float_to_bf16(g / (1.0f + expf(-g)) * u);
+      o.e[i] = float_to_bf16(glu_act(act, g) * u);
     }
     const int c0 = r1 + 4 * lg;
     if ((N_out & 3) == 0 && (ldy & 3) == 0 && (reinterpret_cast<uintptr_t>(y) & 7) == 0) {
@@ -660,15 +661,15 @@ static int pair_waves(int blocks, int K) {
   return waves;
 }
 
-// out [M, I] = silu(x Wg^T) * (x Wu^T) for W = [Wg; Wu] of shape [2I, K]; M <= 16, I % 16 == 0
+// out [M, I] = act(x Wg^T) * (x Wu^T) for W = [Wg; Wu] of shape [2I, K]; M <= 16, I % 16 == 0
 // partials / n_partials / eps: the normalisation factor of x's rows that is still to be applied
 // (RowScaleArgs; K is the size of the normalised rows); partials == null: none.
 // w_blocked: as for ptl_gemm_skinny_bf16
 extern "C" int ptl_gate_up_silu_bf16(void* out, const void* x, const void* w, int w_blocked, int M, int I,
                                      int K, long ldx, const float* partials, int n_partials, float eps,
-                                     hipStream_t stream) {
+                                     int act, hipStream_t stream) {
   if (M <= 0 || I <= 0) return PTL_OK;
-  if (M > 16 || I % 16 || K <= 0 || K % 8 || ldx % 8 || ldx < K || (partials && n_partials <= 0) ||
+  if ((act != GLU_SILU && act != GLU_GELU_TANH) || M > 16 || I % 16 || K <= 0 || K % 8 || ldx % 8 || ldx < K || (partials && n_partials <= 0) ||
       (w_blocked && K % 32))
     return PTL_ERR_ARG;
   const RowScaleArgs sc = {partials, n_partials, 1.0f / (float)K, eps};
@@ -679,7 +680,7 @@ extern "C" int ptl_gate_up_silu_bf16(void* out, const void* x, const void* w, in
   RopeStoreArgs none = {};
 #define GO1(XR, BL)                                                                                   \
   gemm_pair_kernel<PAIR_SILU, 8, 16, XR, BL><<<blocks, waves * 64, lds, stream>>>(                    \
-      (bf16_t*)out, (const bf16_t*)x, (const bf16_t*)w, M, I, K, ldx, I, k_per_wave, I, blocks, 0, none, sc)
+      (bf16_t*)out, (const bf16_t*)x, (const bf16_t*)w, M, I, K, ldx, I, k_per_wave, I, blocks, 0, none, sc, act)
 #define GO(XR) if (w_blocked) GO1(XR, true); else GO1(XR, false)
   switch (gs_rows_of(M)) {
     case 4: GO(4); break;
@@ -715,7 +716,7 @@ extern "C" int ptl_qkv_rope_store_bf16(void* q_out, long ldq, const void* x, con
 #define GO1(ROWS, XR, BL)                                                                             \
   gemm_pair_kernel<PAIR_ROPE, 8, ROWS, XR, BL><<<blocks, waves * 64, lds, stream>>>(                  \
       (bf16_t*)q_out, (const bf16_t*)x, (const bf16_t*)w, M, Hq * D, K, ldx, ldq, k_per_wave, D / 2,  \
-      tiles, D, rs, sc)
+      tiles, D, rs, sc, 0)
 #define GO(ROWS, XR) if (w_blocked) GO1(ROWS, XR, true); else GO1(ROWS, XR, false)
 #define BY_ROWS(ROWS)                                                                                 \
   switch (gs_rows_of(M)) {                                                                            \

@@ -1,0 +1,681 @@
+// Linear recurrences: per head a matrix S [D, Dv] (keys x values) that decays and takes outer products,
+//
+//   S_t = diag(a_t) S_(t-1) + k_t v_t^T,     o_t = S_t^T q_t
+//
+// in two forms:
+//   MODE_SCALAR   one decay a head and token, a_t = exp(-exp(A_log) dt_t) with dt_t = softplus(raw +
+//                 bias); the value is dt_t v_t and skip v_t is added to the result: the state-space
+//                 duality of Mamba-2 (Dao, Gu: "Transformers are SSMs: Generalized Models and
+//                 Efficient Algorithms Through Structured State Space Duality") with S = state^T
+//   MODE_CHANNEL  a decay a key channel, a_t[d] in (0, 1]: gated linear attention (Yang, Wang, Shen,
+//                 Panda, Kim: "Gated Linear Attention Transformers with Hardware-Efficient Training")
+// Everything is float32. Query head h uses q/k head h / heads_per_qk. S lives in the request's state
+// slot as [H][Dv][DS] floats (a column of S after the other, DS = D rounded up to a multiple of 4).
+//
+// ptl_linear_decode: sequences of one token. A workgroup takes 16 columns of a head of a sequence, a
+//   column in 16 lanes (one row of a wave for the data-parallel lane moves); what is in front of the
+//   recurrence is done by the workgroup itself: the short causal convolution with SiLU (scalar form)
+//   or the low-rank decays (channel form). Bound by reading and writing S once.
+// ptl_linear_scan: portions. The rows of a sequence are walked in chunks of 32 tokens whose products
+//   run on the matrix cores in float32 (v_mfma_f32_16x16x4_f32):
+//     P[t, s] = sum_d q_t[d] k_s[d] a(s, t)[d]      s <= t, a(s, t) the decays of tokens s + 1 .. t
+//     O[t, :] = sum_s P[t, s] v_s + sum_d q_t[d] a(start, t)[d] S[d, :]
+//     S[d, :] = a(start, end)[d] S[d, :] + sum_s a(s, end)[d] k_s[d] v_s
+//   A workgroup of four waves takes 64 columns of a head; a wave keeps its 16 columns of S in the
+//   accumulators of the last product, which is also how the middle product wants them as an operand.
+//   Long sequences are cut into segments that are walked side by side: a local pass (what every
+//   segment makes of a zero state), a combine (the segments' start states) and the final pass.
+// ptl_lowrank_decay: a[t, c] = sigmoid(W2[c, :] . r_t + b[c])^(1 / tau) for all rows of a step.
+//
+// Decays between tokens are never formed as quotients or differences of large numbers: in the scalar
+// form the logarithms are summed in double, in the channel form products of decays are taken inside
+// blocks of 16 tokens, so decays that vanish do no harm.
+#include "common.h"
+#include <math.h>
+
+#define MODE_SCALAR 0
+#define MODE_CHANNEL 1
+#define QC 32                // tokens of a chunk
+#define XLD 68               // row stride of the values in LDS
+#define PLD 36               // row stride of P in LDS
+
+typedef float f32x4_t __attribute__((ext_vector_type(4)));
+
+__device__ __forceinline__ float row16_sum(float v) {
+  // the sum over the 16 lanes of a row, in every lane: rotations by 8, 4, 2 and 1 inside the row
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x128, 0xf, 0xf, false));
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x124, 0xf, 0xf, false));
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x122, 0xf, 0xf, false));
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x121, 0xf, 0xf, false));
+  return v;
+}
+__device__ __forceinline__ float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
+__device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
+// sigmoid(z)^p
+__device__ __forceinline__ float sigmoid_power(float z, float p) {
+  return expf((fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * p);
+}
+
+struct LinArgs {
+  float* out;                                     // [T, H, Dv]
+  const float* q; long ldq;                       // q[t * ldq + g * D + d]
+  const float* k; long ldk;
+  const float* v; long ldv;                       // v[t * ldv + h * Dv + c]
+  float qscale;
+  const float* dt; long ldt;                      // scalar: raw step sizes [t * ldt + h]
+  const float* A_log; const float* dt_bias; const float* skip;     // [H]
+  const float* decay; long lda;                   // channel: [t * lda + h * D + d]
+  float* state; long slot_stride;
+  float* work;                                    // per (sequence, segment): [H][Dv][DS], then the decays
+  const int32_t* q_start; const int32_t* state_slots;
+  int H, heads_per_qk, D, DS, Dv;
+  int P, seg_len;                                 // segments a sequence at most, tokens of one
+};
+
+// floats of one segment's work area: S, and its decays (one a head, or one a key channel)
+__host__ __device__ static inline size_t work_floats(const LinArgs& A, int mode) {
+  return (size_t)A.H * A.Dv * A.DS + (mode == MODE_SCALAR ? (size_t)(A.H + 3) / 4 * 4 : (size_t)A.H * A.DS);
+}
+
+// ---- chunks of 32 tokens on the matrix cores -----------------------------------------------------
+template <int NDT, int MODE, bool FINAL>
+constexpr size_t chunk_lds_floats() {
+  constexpr size_t rows = (size_t)QC * (16 * NDT + 4);
+  return rows * (1 + (FINAL ? 1 : 0) + (MODE == MODE_CHANNEL ? 1 : 0)) + (size_t)QC * XLD +
+         (FINAL ? (size_t)QC * PLD : 0) + (MODE == MODE_CHANNEL && FINAL ? (size_t)QC * 20 : 0) +
+         (MODE == MODE_CHANNEL ? 2 * 16 * NDT : 0) + 5 * QC;
+}
+
+template <int NDT, int MODE, bool FINAL>
+__global__ void __launch_bounds__(256) linear_chunk_kernel(LinArgs A, int vec) {
+  constexpr int DP = 16 * NDT;              // key channels, padded
+  constexpr int LD = DP + 4;                // row stride of q, k and the decays in LDS
+  constexpr int NQ = DP / 4;                // float4 of a row
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  float* Ks = lds;                                              // [QC][LD]
+  float* Qs = Ks + QC * LD;                                     // FINAL: [QC][LD]
+  float* As = Qs + (FINAL ? QC * LD : 0);                       // channel: [QC][LD]
+  float* Xs = As + (MODE == MODE_CHANNEL ? QC * LD : 0);        // [QC][XLD]
+  float* Ps = Xs + QC * XLD;                                    // FINAL: [QC][PLD]
+  float* Pd = Ps + (FINAL ? QC * PLD : 0);                      // channel, FINAL: [QC][20], second halves of the
+                                                                // sums over d of the two diagonal tiles
+  float* tot = Pd + (MODE == MODE_CHANNEL && FINAL ? QC * 20 : 0);   // channel: [2][DP]
+  double* cum = reinterpret_cast<double*>(tot + (MODE == MODE_CHANNEL ? 2 * DP : 0));     // scalar: [QC]
+  float* dts = reinterpret_cast<float*>(cum + QC);              // scalar: [QC] step sizes
+  float* es = dts + QC;                                         // scalar: [QC] decays from the chunk's start
+  float* ws = es + QC;                                          // scalar: [QC] dt x the decay to its end
+
+  const int tid = threadIdx.x, lane = tid & 63, ln = lane & 15, lg = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int h = blockIdx.y;
+  const int seq = blockIdx.z / A.P, seg = blockIdx.z % A.P;
+  const int row0 = A.q_start[seq];
+  const int qlen = A.q_start[seq + 1] - row0;
+  const int nseg = (qlen + A.seg_len - 1) / A.seg_len;
+  if (qlen <= 0 || seg >= nseg || (!FINAL && seg == nseg - 1)) return;
+  const int t_begin = seg * A.seg_len, t_end = min(qlen, t_begin + A.seg_len);
+  const int D = A.D, DS = A.DS, Dv = A.Dv, g = h / A.heads_per_qk;
+  const int c0 = blockIdx.x * 64;
+  const int c = c0 + 16 * wave + ln;                            // this lane's column
+  const bool wave_live = c0 + 16 * wave < Dv, live = c < Dv;
+  const size_t wsize = work_floats(A, MODE);
+  auto work_at = [&](int p) { return A.work + ((size_t)seq * A.P + p) * wsize; };
+  auto column = [&](float* base) { return base + ((size_t)h * Dv + c) * DS; };
+  float* slot = A.state + (size_t)A.state_slots[seq] * A.slot_stride;
+
+  f32x4_t S[NDT];                           // S[dt][i]: key channel 16 dt + 4 lg + i of column c
+#pragma unroll
+  for (int dt = 0; dt < NDT; ++dt) {
+    S[dt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    const int d = 16 * dt + 4 * lg;
+    if (FINAL && live && d < DS) S[dt] = *reinterpret_cast<const f32x4_t*>(column(A.P > 1 ? work_at(seg) : slot) + d);
+  }
+  double log_total = 0.0;                   // scalar, local pass: the segment's decay
+  float my_total = 1.f;                     // channel, local pass: of key channel tid
+  float neg_A = 0.f, dt_bias = 0.f, skip = 0.f;
+  if (MODE == MODE_SCALAR) {
+    neg_A = -expf(A.A_log[h]);
+    dt_bias = A.dt_bias[h];
+    skip = A.skip[h];
+  }
+
+  auto load_rows = [&](float* dst, const float* src, long ld, int col0, float f, int t0, int steps) {
+    for (int i = tid; i < QC * NQ; i += 256) {
+      const int r = i / NQ, d = (i - r * NQ) * 4;
+      f32x4_t x = {0.f, 0.f, 0.f, 0.f};
+      if (r < steps && d < D) {
+        const float* p = src + (size_t)(row0 + t0 + r) * ld + col0 + d;
+        if (vec) {
+          x = *reinterpret_cast<const f32x4_t*>(p);
+        } else {
+#pragma unroll
+          for (int j = 0; j < 4; ++j) x[j] = d + j < D ? p[j] : 0.f;
+        }
+        x *= f;
+      }
+      *reinterpret_cast<f32x4_t*>(dst + r * LD + d) = x;
+    }
+  };
+
+  for (int t0 = t_begin; t0 < t_end; t0 += QC) {
+    const int steps = min(QC, t_end - t0);
+    __syncthreads();                        // the chunk before is done with
+    load_rows(Ks, A.k, A.ldk, g * D, 1.f, t0, steps);
+    if (FINAL) load_rows(Qs, A.q, A.ldq, g * D, A.qscale, t0, steps);
+    // (rows past the end keep what is there: their decay is taken as one, below)
+    if (MODE == MODE_CHANNEL) load_rows(As, A.decay, A.lda, h * D, 1.f, t0, steps);
+    for (int i = tid; i < QC * 16; i += 256) {
+      const int r = i >> 4, x0 = (i & 15) * 4;
+      f32x4_t x = {0.f, 0.f, 0.f, 0.f};
+      if (r < steps && c0 + x0 < Dv) {
+        const float* p = A.v + (size_t)(row0 + t0 + r) * A.ldv + (size_t)h * Dv + c0 + x0;
+        if (vec) {
+          x = *reinterpret_cast<const f32x4_t*>(p);
+        } else {
+#pragma unroll
+          for (int j = 0; j < 4; ++j) x[j] = c0 + x0 + j < Dv ? p[j] : 0.f;
+        }
+      }
+      *reinterpret_cast<f32x4_t*>(Xs + r * XLD + x0) = x;
+    }
+    if (MODE == MODE_SCALAR && tid < 64) {  // one wave; its upper half repeats the last token
+      const int r = min(tid, QC - 1);
+      float step = 0.f;
+      if (r < steps) step = softplus_f(A.dt[(size_t)(row0 + t0 + r) * A.ldt + h] + dt_bias);
+      double s = tid < QC ? (double)(neg_A * step) : 0.0;
+#pragma unroll
+      for (int o = 1; o < QC; o <<= 1) {
+        const double up = __shfl_up(s, o, 64);
+        if (tid >= o) s += up;
+      }
+      const double all = __shfl(s, QC - 1, 64);
+      if (tid < QC) {
+        cum[tid] = s;
+        dts[tid] = step;
+        es[tid] = expf((float)s);
+        ws[tid] = step * expf((float)(all - s));
+      }
+    }
+    __syncthreads();
+
+    if (MODE == MODE_CHANNEL) {
+      // The two diagonal tiles: lane (t, lg) walks s from t down, w = q_t times the decays of
+      // s + 1 .. t; wave w takes tile w % 2 and half of the key channels, a lane every fourth float4.
+      if (FINAL) {
+        const int base = 16 * (wave & 1), half = wave >> 1;
+        float acc[16];
+#pragma unroll
+        for (int s = 0; s < 16; ++s) acc[s] = 0.f;
+        for (int qd = half * (NQ / 2) + lg; qd < (half + 1) * (NQ / 2); qd += 4) {
+          const f32x4_t qt = *reinterpret_cast<const f32x4_t*>(Qs + (base + ln) * LD + 4 * qd);
+          f32x4_t w = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int s = 15; s >= 0; --s) {
+            if (s < 15) w *= *reinterpret_cast<const f32x4_t*>(As + (base + s + 1) * LD + 4 * qd);
+            if (s == ln) w = qt;
+            const f32x4_t ks = *reinterpret_cast<const f32x4_t*>(Ks + (base + s) * LD + 4 * qd);
+            acc[s] += (w[0] * ks[0] + w[1] * ks[1]) + (w[2] * ks[2] + w[3] * ks[3]);
+          }
+        }
+#pragma unroll
+        for (int s = 0; s < 16; ++s) {
+          acc[s] += __shfl_xor(acc[s], 16, 64);
+          acc[s] += __shfl_xor(acc[s], 32, 64);
+        }
+        // lane (t, lg) keeps columns 4 lg .. 4 lg + 3 (zero right of the diagonal: w was zero there)
+        f32x4_t mine;
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          mine[i] = lg == 0 ? acc[i] : (lg == 1 ? acc[4 + i] : (lg == 2 ? acc[8 + i] : acc[12 + i]));
+        if (half == 0) *reinterpret_cast<f32x4_t*>(Ps + (base + ln) * PLD + base + 4 * lg) = mine;
+        else *reinterpret_cast<f32x4_t*>(Pd + (base + ln) * 20 + 4 * lg) = mine;
+        __syncthreads();
+      }
+      // q_t times the decays from the start of its block of 16, k_s times those to the block's end
+      for (int i = tid; i < 2 * DP; i += 256) {
+        const int b = i / DP, d = i - b * DP;
+        float* a = As + 16 * b * LD + d;
+        if (FINAL) {
+          float e = 1.f;
+          float* q = Qs + 16 * b * LD + d;
+#pragma unroll
+          for (int t = 0; t < 16; ++t) {
+            e *= 16 * b + t < steps ? a[t * LD] : 1.f;
+            q[t * LD] *= e;
+          }
+        }
+        float f = 1.f;
+        float* k = Ks + 16 * b * LD + d;
+#pragma unroll
+        for (int t = 15; t >= 0; --t) {
+          k[t * LD] *= f;
+          f *= 16 * b + t < steps ? a[t * LD] : 1.f;
+        }
+        tot[i] = f;
+      }
+      __syncthreads();
+    }
+
+    if (FINAL) {
+      // P: tiles (t, s) = (0, 0), (1, 0), (1, 1), one a wave (channel: the second one is left)
+      if (MODE == MODE_SCALAR ? wave < 3 : wave == 3) {
+        const int tt = MODE == MODE_SCALAR ? (wave > 0) : 1, ts = MODE == MODE_SCALAR ? (wave == 2) : 0;
+        f32x4_t p = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int dt = 0; dt < NDT; ++dt) {
+          const f32x4_t ka = *reinterpret_cast<const f32x4_t*>(Ks + (16 * ts + ln) * LD + 16 * dt + 4 * lg);
+          const f32x4_t qb = *reinterpret_cast<const f32x4_t*>(Qs + (16 * tt + ln) * LD + 16 * dt + 4 * lg);
+#pragma unroll
+          for (int m = 0; m < 4; ++m) p = __builtin_amdgcn_mfma_f32_16x16x4f32(ka[m], qb[m], p, 0, 0, 0);
+        }
+        if (MODE == MODE_SCALAR) {
+          const int t = 16 * tt + ln;
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int s = 16 * ts + 4 * lg + i;
+            p[i] = s <= t ? p[i] * (dts[s] * expf((float)(cum[t] - cum[s]))) : 0.f;
+          }
+        }
+        *reinterpret_cast<f32x4_t*>(Ps + (16 * tt + ln) * PLD + 16 * ts + 4 * lg) = p;
+      }
+      f32x4_t O[2];
+      if (wave_live) {
+#pragma unroll
+        for (int tt = 0; tt < 2; ++tt) {
+          O[tt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int dt = 0; dt < NDT; ++dt) {
+            f32x4_t qa = *reinterpret_cast<const f32x4_t*>(Qs + (16 * tt + ln) * LD + 16 * dt + 4 * lg);
+            if (MODE == MODE_CHANNEL && tt == 1) qa *= *reinterpret_cast<const f32x4_t*>(tot + 16 * dt + 4 * lg);
+#pragma unroll
+            for (int m = 0; m < 4; ++m) O[tt] = __builtin_amdgcn_mfma_f32_16x16x4f32(qa[m], S[dt][m], O[tt], 0, 0, 0);
+          }
+          if (MODE == MODE_SCALAR) O[tt] *= *reinterpret_cast<const f32x4_t*>(es + 16 * tt + 4 * lg);
+        }
+      }
+      __syncthreads();                      // P is there
+      if (wave_live) {
+#pragma unroll
+        for (int tt = 0; tt < 2; ++tt) {
+#pragma unroll
+          for (int ts = 0; ts <= tt; ++ts) {
+            f32x4_t pa = *reinterpret_cast<const f32x4_t*>(Ps + (16 * tt + ln) * PLD + 16 * ts + 4 * lg);
+            if (MODE == MODE_CHANNEL && ts == tt) pa += *reinterpret_cast<const f32x4_t*>(Pd + (16 * tt + ln) * 20 + 4 * lg);
+#pragma unroll
+            for (int m = 0; m < 4; ++m)
+              O[tt] = __builtin_amdgcn_mfma_f32_16x16x4f32(pa[m], Xs[(16 * ts + 4 * lg + m) * XLD + 16 * wave + ln], O[tt], 0, 0, 0);
+          }
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int t = 16 * tt + 4 * lg + i;
+            float o = O[tt][i];
+            if (MODE == MODE_SCALAR) o = fmaf(skip, Xs[t * XLD + 16 * wave + ln], o);
+            if (live && t < steps) A.out[((size_t)(row0 + t0 + t) * A.H + h) * Dv + c] = o;
+          }
+        }
+      }
+    }
+    // S
+    if (wave_live) {
+      if (MODE == MODE_SCALAR) {
+        const float e = es[QC - 1];
+#pragma unroll
+        for (int dt = 0; dt < NDT; ++dt) S[dt] *= e;
+      } else {
+#pragma unroll
+        for (int dt = 0; dt < NDT; ++dt)
+          S[dt] *= *reinterpret_cast<const f32x4_t*>(tot + 16 * dt + 4 * lg) *
+                   *reinterpret_cast<const f32x4_t*>(tot + DP + 16 * dt + 4 * lg);
+      }
+#pragma unroll
+      for (int ts = 0; ts < 2; ++ts) {
+        float x[4];
+#pragma unroll
+        for (int m = 0; m < 4; ++m) {
+          const int s = 16 * ts + 4 * lg + m;
+          x[m] = Xs[s * XLD + 16 * wave + ln];
+          if (MODE == MODE_SCALAR) x[m] *= ws[s];
+        }
+#pragma unroll
+        for (int dt = 0; dt < NDT; ++dt) {
+          const float f = MODE == MODE_CHANNEL && ts == 0 ? tot[DP + 16 * dt + ln] : 1.f;
+#pragma unroll
+          for (int m = 0; m < 4; ++m) {
+            float ka = Ks[(16 * ts + 4 * lg + m) * LD + 16 * dt + ln];
+            if (MODE == MODE_CHANNEL && ts == 0) ka *= f;
+            S[dt] = __builtin_amdgcn_mfma_f32_16x16x4f32(ka, x[m], S[dt], 0, 0, 0);
+          }
+        }
+      }
+    }
+    if (!FINAL) {
+      if (MODE == MODE_SCALAR) log_total += cum[QC - 1];
+      else if (tid < DP) my_total *= tot[tid] * tot[DP + tid];
+    }
+  }
+
+  float* to = !FINAL ? work_at(seg + 1) : (seg == nseg - 1 ? slot : nullptr);
+  if (to) {
+#pragma unroll
+    for (int dt = 0; dt < NDT; ++dt) {
+      const int d = 16 * dt + 4 * lg;
+      if (live && d < DS) *reinterpret_cast<f32x4_t*>(column(to) + d) = S[dt];
+    }
+  }
+  if (!FINAL && blockIdx.x == 0) {
+    float* decays = work_at(seg + 1) + (size_t)A.H * Dv * DS;
+    if (MODE == MODE_SCALAR) {
+      if (tid == 0) decays[h] = expf((float)log_total);
+    } else if (tid < DS) {
+      decays[(size_t)h * DS + tid] = my_total;
+    }
+  }
+}
+
+// start(0) = the slot's state; start(p + 1) = decays(p) start(p) + what segment p added. A thread takes
+// four key channels of one column through the sequence's segments.
+template <int MODE>
+__global__ void __launch_bounds__(256) linear_combine_kernel(LinArgs A) {
+  const int seq = blockIdx.y;
+  const int qlen = A.q_start[seq + 1] - A.q_start[seq];
+  if (qlen <= 0) return;
+  const int nseg = (qlen + A.seg_len - 1) / A.seg_len;
+  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  const int nq = A.DS / 4;
+  if (i >= (size_t)A.H * A.Dv * nq) return;
+  const int dq = (int)(i % nq), h = (int)(i / nq / A.Dv);
+  const size_t wsize = work_floats(A, MODE), decays = (size_t)A.H * A.Dv * A.DS;
+  float* w = A.work + (size_t)seq * A.P * wsize;
+  f32x4_t cur = *reinterpret_cast<const f32x4_t*>(A.state + (size_t)A.state_slots[seq] * A.slot_stride + 4 * i);
+  *reinterpret_cast<f32x4_t*>(w + 4 * i) = cur;
+  constexpr int AHEAD = 8;                  // segments whose loads are under way together
+  for (int p0 = 1; p0 < nseg; p0 += AHEAD) {
+    f32x4_t u[AHEAD], f[AHEAD];
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j) {
+      if (p0 + j < nseg) {
+        const float* at = w + (size_t)(p0 + j) * wsize;
+        u[j] = *reinterpret_cast<const f32x4_t*>(at + 4 * i);
+        if (MODE == MODE_SCALAR) {
+          const float e = at[decays + h];
+          f[j] = f32x4_t{e, e, e, e};
+        } else {
+          f[j] = *reinterpret_cast<const f32x4_t*>(at + decays + (size_t)h * A.DS + 4 * dq);
+        }
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j) {
+      if (p0 + j < nseg) {
+        cur = f[j] * cur + u[j];
+        *reinterpret_cast<f32x4_t*>(w + (size_t)(p0 + j) * wsize + 4 * i) = cur;
+      }
+    }
+  }
+}
+
+template <int NDT, int MODE, bool FINAL>
+static int launch_chunks(const LinArgs& A, int vec, int n_seqs, hipStream_t st) {
+  constexpr size_t lds = chunk_lds_floats<NDT, MODE, FINAL>() * sizeof(float);
+  static bool raised = false;               // (per instantiation)
+  if (lds > 48 * 1024 && !raised) {
+    if (hipFuncSetAttribute(reinterpret_cast<const void*>(&linear_chunk_kernel<NDT, MODE, FINAL>),
+                            hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) {
+      (void)hipGetLastError();
+      return PTL_ERR_LAUNCH;
+    }
+    raised = true;
+  }
+  linear_chunk_kernel<NDT, MODE, FINAL><<<dim3((A.Dv + 63) / 64, A.H, n_seqs * A.P), 256, lds, st>>>(A, vec);
+  return ptl_launch_status();
+}
+
+template <int MODE>
+static int launch_scan(const LinArgs& A, int n_seqs, hipStream_t st) {
+  if (A.D <= 0 || A.D > 256 || A.Dv <= 0 || A.H <= 0 || A.H > 65535 || A.heads_per_qk <= 0 ||
+      A.H % A.heads_per_qk || A.P < 1 || (long)n_seqs * A.P > 65535 || A.seg_len < 1 || (A.P > 1 && !A.work) ||
+      A.slot_stride < (long)A.H * A.Dv * A.DS || A.slot_stride % 4 || ((uintptr_t)A.state & 15) ||
+      ((uintptr_t)A.work & 15))
+    return PTL_ERR_ARG;
+  auto aligned = [](const float* p, long ld) { return ld % 4 == 0 && ((uintptr_t)p & 15) == 0; };
+  const int vec = A.D % 4 == 0 && A.Dv % 4 == 0 && aligned(A.q, A.ldq) && aligned(A.k, A.ldk) && aligned(A.v, A.ldv) &&
+                  (MODE == MODE_SCALAR || aligned(A.decay, A.lda));
+  const int tiles = (A.D + 15) / 16;
+#define GO(N)                                                                                      \
+  if (tiles <= N) {                                                                                \
+    if (A.P > 1) {                                                                                 \
+      if (int e = launch_chunks<N, MODE, false>(A, vec, n_seqs, st)) return e;                     \
+      const size_t quads = (size_t)A.H * A.Dv * (A.DS / 4);                                        \
+      linear_combine_kernel<MODE><<<dim3((unsigned)((quads + 255) / 256), n_seqs), 256, 0, st>>>(A); \
+      if (int e = ptl_launch_status()) return e;                                                   \
+    }                                                                                              \
+    return launch_chunks<N, MODE, true>(A, vec, n_seqs, st);                                       \
+  }
+  GO(1) GO(2) GO(3) GO(4) GO(6) GO(8) GO(12) GO(16)
+#undef GO
+  return PTL_ERR_ARG;
+}
+
+// Floats of the workspace that ptl_linear_scan wants when P > 1.
+extern "C" long ptl_linear_work_floats(int mode, int n_seqs, int P, int H, int D, int Dv) {
+  LinArgs A{};
+  A.H = H; A.Dv = Dv; A.DS = (D + 3) / 4 * 4;
+  return (long)(work_floats(A, mode) * n_seqs * P);
+}
+
+// Portions of n_seqs sequences. mode 0 (scalar): dt, A_log, dt_bias, skip; mode 1
+// (channel): decay. P: the most segments of seg_len rows that one of the sequences has.
+extern "C" int ptl_linear_scan(int mode, float* out, const float* q, long ldq, const float* k, long ldk,
+                               const float* v, long ldv, float qscale, const float* dt, long ldt,
+                               const float* A_log, const float* dt_bias, const float* skip, const float* decay,
+                               long lda, float* state, long slot_stride, float* work, int P, int seg_len,
+                               const int32_t* q_start, const int32_t* state_slots, int n_seqs, int H,
+                               int G, int D, int Dv, hipStream_t st) {
+  if (n_seqs <= 0) return PTL_OK;
+  if (G <= 0 || H % G) return PTL_ERR_ARG;
+  LinArgs A{out, q, ldq, k, ldk, v, ldv, qscale, dt, ldt, A_log, dt_bias, skip, decay, lda, state, slot_stride, work,
+            q_start, state_slots, H, H / G, D, (D + 3) / 4 * 4, Dv, P, seg_len};
+  if (mode == MODE_SCALAR) {
+    if (!dt || !A_log || !dt_bias || !skip) return PTL_ERR_ARG;
+    return launch_scan<MODE_SCALAR>(A, n_seqs, st);
+  }
+  if (mode != MODE_CHANNEL || !decay) return PTL_ERR_ARG;
+  return launch_scan<MODE_CHANNEL>(A, n_seqs, st);
+}
+
+// ---- the low-rank decays of all rows ---------------------------------------------------------------
+// grid (blocks of 256 channels, blocks of ROWS rows): a thread keeps its channel's row of W2 in
+// registers (up to 32 entries; a longer one is read again for every row), the rows of r go through LDS
+#define DECAY_ROWS 8
+template <int RM>
+__global__ void __launch_bounds__(256)
+lowrank_decay_kernel(float* __restrict__ out, const float* __restrict__ r, long ldr, const float* __restrict__ w,
+                     const float* __restrict__ b, float inv_tau, int T, int C, int R) {
+  extern __shared__ float rs[];             // [DECAY_ROWS][R]
+  const int t0 = blockIdx.y * DECAY_ROWS, rows = min(DECAY_ROWS, T - t0);
+  for (int i = threadIdx.x; i < rows * R; i += 256) rs[i] = r[(size_t)(t0 + i / R) * ldr + i % R];
+  __syncthreads();
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= C) return;
+  const float* wr = w + (size_t)c * R;
+  float wv[RM > 0 ? RM : 1];
+  if (RM > 0) {
+#pragma unroll
+    for (int j = 0; j < RM; ++j) wv[j] = j < R ? wr[j] : 0.f;
+  }
+  const float bias = b[c];
+  for (int t = 0; t < rows; ++t) {
+    float z = bias;
+    if (RM > 0) {
+#pragma unroll
+      for (int j = 0; j < RM; ++j) z = fmaf(wv[j], rs[t * R + min(j, R - 1)], z);
+    } else {
+      for (int j = 0; j < R; ++j) z = fmaf(wr[j], rs[t * R + j], z);
+    }
+    out[(size_t)(t0 + t) * C + c] = sigmoid_power(z, inv_tau);
+  }
+}
+
+extern "C" int ptl_lowrank_decay(float* out, const float* r, long ldr, const float* w, const float* b,
+                                 float inv_tau, int T_, int C, int R, hipStream_t st) {
+  if (T_ <= 0) return PTL_OK;
+  const size_t lds = (size_t)DECAY_ROWS * R * sizeof(float);
+  if (C <= 0 || R <= 0 || lds > 48 * 1024 || (T_ + DECAY_ROWS - 1) / DECAY_ROWS > 65535) return PTL_ERR_ARG;
+  const dim3 grid((C + 255) / 256, (T_ + DECAY_ROWS - 1) / DECAY_ROWS);
+  if (R <= 16) lowrank_decay_kernel<16><<<grid, 256, lds, st>>>(out, r, ldr, w, b, inv_tau, T_, C, R);
+  else if (R <= 32) lowrank_decay_kernel<32><<<grid, 256, lds, st>>>(out, r, ldr, w, b, inv_tau, T_, C, R);
+  else lowrank_decay_kernel<0><<<grid, 256, lds, st>>>(out, r, ldr, w, b, inv_tau, T_, C, R);
+  return ptl_launch_status();
+}
+
+// ---- one token -------------------------------------------------------------------------------------
+struct DecodeArgs {
+  float* out;                               // [T, H, Dv]
+  const float* p; long ldp;                 // the float32 projection
+  int q_off, k_off, v_off;                  // columns of q [G, D], k [G, D] and v [H, Dv] (before the convolution)
+  float qscale;
+  // scalar form
+  int dt_off;
+  const float* A_log; const float* dt_bias; const float* skip;     // [H]
+  const float* cw; const float* cb; int taps; long tail_off;       // convolution [C, taps], [C]; channel of a
+  int conv_off, C;                                                 // column: column - conv_off; tail [taps - 1, C]
+  // channel form
+  int a_off;
+  const float* w2; const float* b2; int R; float inv_tau;          // [H * D, R], [H * D]
+  float* state; long slot_stride;
+  const int32_t* q_start; const int32_t* state_slots;
+  int H, heads_per_qk, D, DS, Dv;
+};
+
+template <int J, int MODE>
+__global__ void __launch_bounds__(256) linear_decode_kernel(DecodeArgs A) {
+  __shared__ __attribute__((aligned(16))) float ks[64 * J], qs[64 * J], as[MODE == MODE_CHANNEL ? 64 * J : 4], xs[16];
+  const int tid = threadIdx.x, cg = tid >> 4, l = tid & 15;
+  const int h = blockIdx.y, seq = blockIdx.z, g = h / A.heads_per_qk;
+  const int row = A.q_start[seq];
+  if (A.q_start[seq + 1] <= row) return;
+  const int D = A.D, DS = A.DS, Dv = A.Dv;
+  const int c = blockIdx.x * 16 + cg;
+  const bool live = c < Dv;
+  float* slot = A.state + (size_t)A.state_slots[seq] * A.slot_stride;
+  float* st = slot + ((size_t)h * Dv + c) * DS;
+  f32x4_t S[J];
+#pragma unroll
+  for (int j = 0; j < J; ++j) {
+    const int d = 4 * (l + 16 * j);
+    S[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    if (live && d < DS) S[j] = __builtin_nontemporal_load(reinterpret_cast<const f32x4_t*>(st + d));
+  }
+  const float* p = A.p + (size_t)row * A.ldp;
+  // what the columns of the projection hold for this workgroup: k and q of the head (group), 16 values
+  auto value = [&](int col) {
+    float x = p[col];
+    if (MODE == MODE_SCALAR) {
+      const int ch = col - A.conv_off;
+      float s = A.cb ? A.cb[ch] : 0.f;
+      const float* w = A.cw + (size_t)ch * A.taps;
+      const float* tail = slot + A.tail_off + ch;
+      for (int j = 0; j < A.taps - 1; ++j) s = fmaf(w[j], tail[(size_t)j * A.C], s);
+      x = silu_f(fmaf(w[A.taps - 1], x, s));
+    }
+    return x;
+  };
+  const int DP = 64 * J;
+  for (int i = tid; i < 2 * DP + 16; i += 256) {
+    if (i < DP) {
+      ks[i] = i < D ? value(A.k_off + g * D + i) : 0.f;
+    } else if (i < 2 * DP) {
+      const int d = i - DP;
+      qs[d] = d < D ? value(A.q_off + g * D + d) * A.qscale : 0.f;
+    } else {
+      const int cc = blockIdx.x * 16 + i - 2 * DP;
+      xs[i - 2 * DP] = cc < Dv ? value(A.v_off + h * Dv + cc) : 0.f;
+    }
+  }
+  float decay = 1.f, step = 1.f;
+  if (MODE == MODE_SCALAR) {
+    step = softplus_f(p[A.dt_off + h] + A.dt_bias[h]);
+    decay = expf(-expf(A.A_log[h]) * step);
+  } else {
+    for (int d = tid; d < DP; d += 256) {
+      float a = 1.f;
+      if (d < D) {
+        const int ch = h * D + d;
+        const float* w = A.w2 + (size_t)ch * A.R;
+        const float* r = p + A.a_off;
+        float z = A.b2[ch];
+        for (int j = 0; j < A.R; ++j) z = fmaf(w[j], r[j], z);
+        a = sigmoid_power(z, A.inv_tau);
+      }
+      as[d] = a;
+    }
+  }
+  __syncthreads();
+  const float x = xs[cg], v = x * step;
+  float o = 0.f;
+#pragma unroll
+  for (int j = 0; j < J; ++j) {
+    const int d = 4 * (l + 16 * j);
+    const f32x4_t k4 = *reinterpret_cast<const f32x4_t*>(ks + d), q4 = *reinterpret_cast<const f32x4_t*>(qs + d);
+    if (MODE == MODE_CHANNEL) S[j] *= *reinterpret_cast<const f32x4_t*>(as + d);
+    else S[j] *= decay;
+    S[j] += k4 * v;
+    o += (S[j][0] * q4[0] + S[j][1] * q4[1]) + (S[j][2] * q4[2] + S[j][3] * q4[3]);
+    if (live && d < DS) __builtin_nontemporal_store(S[j], reinterpret_cast<f32x4_t*>(st + d));
+  }
+  o = row16_sum(o);
+  if (MODE == MODE_SCALAR) o = fmaf(A.skip[h], x, o);
+  if (live && l == 0) A.out[((size_t)row * A.H + h) * Dv + c] = o;
+}
+
+template <int MODE>
+static int launch_decode(const DecodeArgs& A, int n_seqs, hipStream_t st) {
+  if (A.D <= 0 || A.D > 256 || A.Dv <= 0 || A.H <= 0 || A.H > 65535 || n_seqs > 65535 || A.heads_per_qk <= 0 ||
+      A.slot_stride < (long)A.H * A.Dv * A.DS || A.slot_stride % 4 || ((uintptr_t)A.state & 15))
+    return PTL_ERR_ARG;
+  const dim3 grid((A.Dv + 15) / 16, A.H, n_seqs);
+  switch ((A.DS + 63) / 64) {
+    case 1: linear_decode_kernel<1, MODE><<<grid, 256, 0, st>>>(A); break;
+    case 2: linear_decode_kernel<2, MODE><<<grid, 256, 0, st>>>(A); break;
+    case 3: linear_decode_kernel<3, MODE><<<grid, 256, 0, st>>>(A); break;
+    default: linear_decode_kernel<4, MODE><<<grid, 256, 0, st>>>(A); break;
+  }
+  return ptl_launch_status();
+}
+
+// Sequences 0 .. n_seqs - 1, one token each, scalar form behind a short convolution. p float32 [T,
+// ldp] with the raw x (H heads of Dv), B and C (G groups of D) and step sizes at their columns;
+// conv_off: the column of the convolution's channel 0. The tails are read, not advanced.
+extern "C" int ptl_linear_decode_conv(float* out, const float* p, long ldp, int x_off, int b_off, int c_off,
+                                      int dt_off, const float* A_log, const float* dt_bias, const float* skip,
+                                      const float* cw, const float* cb, int taps, int conv_off, int C,
+                                      long tail_off, float* state, long slot_stride, const int32_t* q_start,
+                                      const int32_t* state_slots, int n_seqs, int H, int G, int D, int Dv,
+                                      hipStream_t st) {
+  if (n_seqs <= 0) return PTL_OK;
+  if (G <= 0 || H % G || taps < 1 || !cw || tail_off < (long)H * Dv * ((D + 3) / 4 * 4)) return PTL_ERR_ARG;
+  DecodeArgs A{};
+  A.out = out; A.p = p; A.ldp = ldp; A.q_off = c_off; A.k_off = b_off; A.v_off = x_off; A.qscale = 1.f;
+  A.dt_off = dt_off; A.A_log = A_log; A.dt_bias = dt_bias; A.skip = skip;
+  A.cw = cw; A.cb = cb; A.taps = taps; A.tail_off = tail_off; A.conv_off = conv_off; A.C = C;
+  A.state = state; A.slot_stride = slot_stride; A.q_start = q_start; A.state_slots = state_slots;
+  A.H = H; A.heads_per_qk = H / G; A.D = D; A.DS = (D + 3) / 4 * 4; A.Dv = Dv;
+  return launch_decode<MODE_SCALAR>(A, n_seqs, st);
+}
+
+// The channel form: q, k (H heads of D), v (H of Dv) and the decays' low-rank input r [R] at columns of p;
+// w2 [H * D, R], b2 [H * D].
+extern "C" int ptl_linear_decode_lowrank(float* out, const float* p, long ldp, int q_off, int k_off, int v_off,
+                                         int a_off, float qscale, const float* w2, const float* b2, int R,
+                                         float inv_tau, float* state, long slot_stride, const int32_t* q_start,
+                                         const int32_t* state_slots, int n_seqs, int H, int D, int Dv,
+                                         hipStream_t st) {
+  if (n_seqs <= 0) return PTL_OK;
+  if (R <= 0 || !w2 || !b2) return PTL_ERR_ARG;
+  DecodeArgs A{};
+  A.out = out; A.p = p; A.ldp = ldp; A.q_off = q_off; A.k_off = k_off; A.v_off = v_off; A.qscale = qscale;
+  A.a_off = a_off; A.w2 = w2; A.b2 = b2; A.R = R; A.inv_tau = inv_tau;
+  A.state = state; A.slot_stride = slot_stride; A.q_start = q_start; A.state_slots = state_slots;
+  A.H = H; A.heads_per_qk = 1; A.D = D; A.DS = (D + 3) / 4 * 4; A.Dv = Dv;
+  return launch_decode<MODE_CHANNEL>(A, n_seqs, st);
+}

@@ -17,6 +17,12 @@
 //   constant, times act(gate) with the gate read from a float32 matrix at given columns
 //   (sigmoid, SiLU, or none). The result [T, H * Dv] is in the engine's type.
 //
+// ptl_gate_group_norm: one workgroup a (token, group of columns). y float32 [T, n] times silu(gate),
+//   then every one of the equal groups of neighbouring columns divided by its own root mean square,
+//   times a weight [n]; the result is in the engine's type. For the leading rows of a step that are
+//   sequences of one token it also advances the inputs that a short convolution keeps in the state
+//   slot (the recurrence in front of it has read the old ones).
+//
 // All arithmetic is float32: the angle is float(position) * frequency, sinf / cosf / expf are the
 // accurate ones.
 #include "common.h"
@@ -218,4 +224,68 @@ extern "C" int ptl_head_norm_gate(void* out, long ldo, const float* a, int maps,
   if (dtype == PTL_DTYPE_BF16) GO(bf16_t)
 #undef GO
   return PTL_ERR_ARG;
+}
+
+// The kept inputs of a short convolution of the first n_rows rows, each a sequence of one token:
+// tail [taps - 1, C] at tail_off of the sequence's slot; x[t * ldx + c] the token's input.
+struct TailArgs {
+  float* state; long slot_stride; long tail_off;
+  const float* x; long ldx;
+  const int32_t* state_slots;
+  int n_rows, C, taps;
+};
+
+template <typename TO>
+__global__ void __launch_bounds__(256)
+gate_group_norm_kernel(TO* __restrict__ out, const float* __restrict__ y, const float* __restrict__ z, long ldz,
+                       const float* __restrict__ w, int n, int groups, float eps, TailArgs tail) {
+  extern __shared__ float us[];
+  __shared__ float scratch[16];
+  const int t = blockIdx.x, part = blockIdx.y, tid = threadIdx.x, nt = blockDim.x;
+  const int size = n / groups, c0 = part * size;
+  const float* yr = y + (size_t)t * n + c0;
+  const float* zr = z + (size_t)t * ldz + c0;
+  float ss = 0.f;
+  for (int c = tid; c < size; c += nt) {
+    const float g = zr[c];
+    const float u = yr[c] * (g / (1.0f + expf(-g)));
+    us[c] = u;
+    ss = fmaf(u, u, ss);
+  }
+  ss = block_sum(ss, scratch);
+  const float r = 1.0f / sqrtf(ss / (float)size + eps);
+  TO* dst = out + (size_t)t * n + c0;
+  for (int c = tid; c < size; c += nt) dst[c] = from_float<TO>(us[c] * r * w[c0 + c]);
+  if (t < tail.n_rows) {
+    float* kept = tail.state + (size_t)tail.state_slots[t] * tail.slot_stride + tail.tail_off;
+    const int per = (tail.C + groups - 1) / groups;
+    for (int c = part * per + tid; c < min(tail.C, (part + 1) * per); c += nt) {
+      for (int i = 0; i + 2 < tail.taps; ++i) kept[(size_t)i * tail.C + c] = kept[(size_t)(i + 1) * tail.C + c];
+      kept[(size_t)(tail.taps - 2) * tail.C + c] = tail.x[(size_t)t * tail.ldx + c];
+    }
+  }
+}
+
+// y float32 [T, n] dense, z float32 [T, ldz] (its first n columns), w float32 [n], out [T, n] dense.
+// tail_rows > 0 and taps > 1: rows 0 .. tail_rows - 1 also advance the kept inputs of their slots.
+extern "C" int ptl_gate_group_norm(void* out, const float* y, const float* z, long ldz, const float* w, int groups,
+                                   float eps, int T_, int n, float* state, long slot_stride, long tail_off,
+                                   const float* x, long ldx, const int32_t* state_slots, int tail_rows, int C,
+                                   int taps, int dtype, hipStream_t st) {
+  if (T_ <= 0) return PTL_OK;
+  if (n <= 0 || groups <= 0 || n % groups || groups > 65535 || (size_t)(n / groups) * sizeof(float) > 60 * 1024 ||
+      tail_rows > T_ || (tail_rows > 0 && taps > 1 && (!state || !x || !state_slots || C <= 0)))
+    return PTL_ERR_ARG;
+  const TailArgs tail{state, slot_stride, tail_off, x, ldx, state_slots, taps > 1 ? tail_rows : 0, C, taps};
+  const int size = n / groups;
+  const int threads = size >= 256 ? 256 : (size + 63) / 64 * 64;
+  const size_t lds = (size_t)size * sizeof(float);
+  if (dtype == PTL_DTYPE_F32)
+    gate_group_norm_kernel<float><<<dim3(T_, groups), threads, lds, st>>>((float*)out, y, z, ldz, w, n, groups, eps, tail);
+  else if (dtype == PTL_DTYPE_BF16)
+    gate_group_norm_kernel<bf16_t><<<dim3(T_, groups), threads, lds, st>>>((bf16_t*)out, y, z, ldz, w, n, groups, eps,
+                                                                           tail);
+  else
+    return PTL_ERR_ARG;
+  return ptl_launch_status();
 }

@@ -10,10 +10,14 @@
 //   of the new stream in the engine's dtype for a product that reads the stream itself.
 // ptl_stream_add_rmsnorm: stream += rmsnorm(y) * w, the same with a norm that needs the row.
 // ptl_stream_add_rmsnorm_sum: the same for a result that is a weighted sum of two and a bias.
+// ptl_stream_postnorm: stream = rmsnorm(alpha stream + y) * w, the norm behind the residual sum, with y a
+//   weighted sum of up to two results each of which may be RMS-normed first (where it stands, below).
 // ptl_stream_rmsnorm: the RMS norm of rows of the stream, in the engine's type.
 // ptl_dyt: the norm alone, for rows that are no stream (the rows picked for the head).
 // ptl_embedding_scaled: stream[t] = table[ids[t]] * scale, in float32 (``copies`` times side by side in
-//   a row, for a model that keeps several streams).
+//   a row, for a model that keeps several streams). ptl_embedding_positions: the same with a sinusoidal
+//   vector of the token's position added.
+// ptl_softcap: cap * tanh(x / cap) on float32 logits.
 // ptl_hyper_mix: several residual streams a token (hyper-connections): the streams' update behind a
 //   sublayer and the read-out with its RMS norm in front of the next one (where it stands, below).
 // ptl_gelu_gather_mul: out[t, j] = gelu_tanh(z[t, j]) * table[ids[t], col0 + j]: a gate on a
@@ -22,6 +26,7 @@
 // All arithmetic is float32; tanhf / expf are the accurate ones.
 #include "common.h"
 #include <math.h>
+#include <type_traits>
 
 struct DytArgs {
   const float* w;     // [H]; null: the norm is absent
@@ -200,6 +205,147 @@ extern "C" int ptl_stream_add_rmsnorm_sum(float* stream, const void* y1, float a
   return PTL_ERR_ARG;
 }
 
+// The norm behind the residual sum: stream <- u * rsqrt(mean(u^2) + eps) * w with
+//   u = alpha stream + a n1(y1) + b n2(y2) + c bias,    n(y) = y * rsqrt(mean(y^2) + n_eps) * nw, or y
+// (y2, the bias and both inner norms are optional), and a copy of the new stream in the engine's
+// type. One workgroup a row; a thread keeps its VPT groups of VEC neighbouring entries of y1, y2 and
+// the stream in registers from the one pass over memory to the last use.
+struct PostNormArgs {
+  float* stream; float alpha;
+  const void* y1; float a; const float* n1;
+  const void* y2; float b; const float* n2;
+  const float* bias; float c;
+  float n_eps;
+  const float* w; float eps;
+  void* copy;
+  int H;
+};
+
+template <int NT, int VPT, int VEC, typename TY, typename TO>
+__global__ void __launch_bounds__(NT) stream_postnorm_kernel(PostNormArgs A) {
+  __shared__ float scratch[16];
+  const size_t row = (size_t)blockIdx.x * A.H;
+  const TY* y1 = (const TY*)A.y1 + row;
+  const TY* y2 = A.y2 ? (const TY*)A.y2 + row : nullptr;
+  float* stream = A.stream + row;
+  float v1[VPT][VEC], v2[VPT][VEC], u[VPT][VEC];
+  float s1 = 0.f, s2 = 0.f;
+  auto read = [&](const auto* p, int i0, float (&v)[VEC]) {
+    typedef typename std::remove_cv<typename std::remove_pointer<decltype(p)>::type>::type T;
+    if (VEC == 1) {
+      v[0] = to_float<T>(p[i0]);
+    } else if (sizeof(T) == 4) {
+      const float4 x = *reinterpret_cast<const float4*>(p + i0);
+      v[0] = x.x; v[VEC > 1 ? 1 : 0] = x.y; v[VEC > 2 ? 2 : 0] = x.z; v[VEC > 3 ? 3 : 0] = x.w;
+    } else {
+      const uint2 x = *reinterpret_cast<const uint2*>(p + i0);
+      v[0] = __uint_as_float(x.x << 16); v[VEC > 1 ? 1 : 0] = __uint_as_float(x.x & 0xffff0000u);
+      v[VEC > 2 ? 2 : 0] = __uint_as_float(x.y << 16); v[VEC > 3 ? 3 : 0] = __uint_as_float(x.y & 0xffff0000u);
+    }
+  };
+#pragma unroll
+  for (int k = 0; k < VPT; ++k) {
+    const int i = (k * NT + threadIdx.x) * VEC;
+    if (i >= A.H) {
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) v1[k][j] = v2[k][j] = u[k][j] = 0.f;
+      continue;
+    }
+    read(y1, i, v1[k]);
+    if (y2) read(y2, i, v2[k]);
+    read((const float*)stream, i, u[k]);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      if (!y2) v2[k][j] = 0.f;
+      s1 = fmaf(v1[k][j], v1[k][j], s1);
+      s2 = fmaf(v2[k][j], v2[k][j], s2);
+    }
+  }
+  float f1 = A.a, f2 = A.b;
+  if (A.n1) f1 *= 1.0f / sqrtf(block_sum(s1, scratch) / (float)A.H + A.n_eps);
+  if (A.n2) f2 *= 1.0f / sqrtf(block_sum(s2, scratch) / (float)A.H + A.n_eps);
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < VPT; ++k) {
+    const int i = (k * NT + threadIdx.x) * VEC;
+    if (i >= A.H) continue;
+    float w1[VEC], w2[VEC], bs[VEC];
+    if (A.n1) read(A.n1, i, w1);
+    if (A.n2) read(A.n2, i, w2);
+    if (A.bias) read(A.bias, i, bs);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      float x = A.alpha * u[k][j];
+      x = fmaf(f1, A.n1 ? v1[k][j] * w1[j] : v1[k][j], x);
+      if (y2) x = fmaf(f2, A.n2 ? v2[k][j] * w2[j] : v2[k][j], x);
+      if (A.bias) x = fmaf(A.c, bs[j], x);
+      u[k][j] = x;
+      ss = fmaf(x, x, ss);
+    }
+  }
+  const float r = 1.0f / sqrtf(block_sum(ss, scratch) / (float)A.H + A.eps);
+  TO* copy = A.copy ? (TO*)A.copy + row : nullptr;
+#pragma unroll
+  for (int k = 0; k < VPT; ++k) {
+    const int i = (k * NT + threadIdx.x) * VEC;
+    if (i >= A.H) continue;
+    float w[VEC];
+    read(A.w, i, w);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) u[k][j] = u[k][j] * r * w[j];
+    if (VEC == 1) {
+      stream[i] = u[k][0];
+      if (copy) copy[i] = from_float<TO>(u[k][0]);
+    } else {
+      *reinterpret_cast<float4*>(stream + i) = make_float4(u[k][0], u[k][VEC > 1 ? 1 : 0], u[k][VEC > 2 ? 2 : 0], u[k][VEC > 3 ? 3 : 0]);
+      if (copy) {
+        TO e[VEC];
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) e[j] = from_float<TO>(u[k][j]);
+        if (sizeof(TO) == 2) *reinterpret_cast<uint2*>(copy + i) = *reinterpret_cast<const uint2*>(e);
+        else *reinterpret_cast<float4*>(copy + i) = *reinterpret_cast<const float4*>(e);
+      }
+    }
+  }
+}
+
+template <typename TY, typename TO>
+static int launch_postnorm(const PostNormArgs& A, int T_, hipStream_t st) {
+  auto odd = [](const void* p) { return ((uintptr_t)p & 15) != 0; };
+  const bool vec = A.H % 4 == 0 && !odd(A.stream) && !odd(A.y1) && !odd(A.y2) && !odd(A.n1) && !odd(A.n2) &&
+                   !odd(A.bias) && !odd(A.w) && !odd(A.copy);
+  const int n = vec ? A.H / 4 : A.H;         // groups of entries of a row
+  // few rows: a row over 1,024 threads, so that a thread's loads are one or two deep
+  const bool few = T_ <= 512 && n > 256;
+#define GO(NT, VPT)                                                                  \
+  if (n <= NT * VPT) {                                                               \
+    if (vec) stream_postnorm_kernel<NT, VPT, 4, TY, TO><<<T_, NT, 0, st>>>(A);       \
+    else stream_postnorm_kernel<NT, VPT, 1, TY, TO><<<T_, NT, 0, st>>>(A);           \
+    return ptl_launch_status();                                                      \
+  }
+  if (!few) { GO(256, 1) GO(256, 2) GO(256, 4) }
+  GO(1024, 1) GO(1024, 2) GO(1024, 4)
+  if (!vec) { GO(1024, 16) }
+#undef GO
+  return PTL_ERR_ARG;
+}
+
+// stream float32 [T, H], in place; y1, y2 [T, H] of y_dtype; n1, n2, bias, w float32 [H]; copy [T, H] of
+// out_dtype or null. H up to 16,384.
+extern "C" int ptl_stream_postnorm(float* stream, float alpha, const void* y1, float a, const float* n1,
+                                   const void* y2, float b, const float* n2, int y_dtype, const float* bias, float c,
+                                   float n_eps, const float* w, float eps, void* copy, int out_dtype, int T_, int H,
+                                   hipStream_t st) {
+  if (T_ <= 0) return PTL_OK;
+  if (H <= 0 || !stream || !y1 || !w || (n2 && !y2)) return PTL_ERR_ARG;
+  const PostNormArgs A{stream, alpha, y1, a, n1, y2, b, n2, bias, c, n_eps, w, eps, copy, H};
+  if (y_dtype == PTL_DTYPE_F32 && out_dtype == PTL_DTYPE_F32) return launch_postnorm<float, float>(A, T_, st);
+  if (y_dtype == PTL_DTYPE_F32 && out_dtype == PTL_DTYPE_BF16) return launch_postnorm<float, bf16_t>(A, T_, st);
+  if (y_dtype == PTL_DTYPE_BF16 && out_dtype == PTL_DTYPE_BF16) return launch_postnorm<bf16_t, bf16_t>(A, T_, st);
+  if (y_dtype == PTL_DTYPE_BF16 && out_dtype == PTL_DTYPE_F32) return launch_postnorm<bf16_t, float>(A, T_, st);
+  return PTL_ERR_ARG;
+}
+
 // out = x * rsqrt(mean(x^2) + eps) * w for rows of a float32 stream, in the engine's type (the rows
 // picked for the head).
 template <typename TO>
@@ -257,6 +403,58 @@ extern "C" int ptl_embedding_scaled(float* out, const void* table, const int32_t
   return ptl_launch_status();
 }
 
+// out[t, j] = table[ids[t], j] * scale + sin or cos (j even or odd) of positions[t] * freq[j / 2]
+template <typename T>
+__global__ void __launch_bounds__(256)
+embedding_positions_kernel(float* __restrict__ out, const T* __restrict__ table, const int32_t* __restrict__ ids,
+                           const int32_t* __restrict__ positions, const float* __restrict__ freq, int H, int V,
+                           float scale) {
+  const int t = blockIdx.x;
+  int id = ids[t];
+  if (id < 0 || id >= V) id = 0;          // checked on the host; never read out of bounds
+  const T* src = table + (size_t)id * H;
+  float* dst = out + (size_t)t * H;
+  const float pos = (float)positions[t];
+  for (int i = threadIdx.x; 2 * i < H; i += blockDim.x) {
+    float s, c;
+    sincosf(pos * freq[i], &s, &c);
+    dst[2 * i] = fmaf(to_float<T>(src[2 * i]), scale, s);
+    if (2 * i + 1 < H) dst[2 * i + 1] = fmaf(to_float<T>(src[2 * i + 1]), scale, c);
+  }
+}
+
+extern "C" int ptl_embedding_positions(float* out, const void* table, const int32_t* ids, const int32_t* positions,
+                                       const float* freq, int T_, int H, int V, float scale, int dtype,
+                                       hipStream_t st) {
+  if (T_ <= 0) return PTL_OK;
+  if (H <= 0 || V <= 0 || !positions || !freq) return PTL_ERR_ARG;
+  const int threads = H >= 512 ? 256 : (H >= 256 ? 128 : 64);
+  if (dtype == PTL_DTYPE_F32)
+    embedding_positions_kernel<float><<<T_, threads, 0, st>>>(out, (const float*)table, ids, positions, freq, H, V, scale);
+  else if (dtype == PTL_DTYPE_BF16)
+    embedding_positions_kernel<bf16_t><<<T_, threads, 0, st>>>(out, (const bf16_t*)table, ids, positions, freq, H, V,
+                                                               scale);
+  else
+    return PTL_ERR_ARG;
+  return ptl_launch_status();
+}
+
+// logits <- cap * tanh(logits / cap), in place
+__global__ void __launch_bounds__(256) softcap_kernel(float* __restrict__ x, float cap, size_t total) {
+  size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  const size_t step = (size_t)gridDim.x * 256;
+  for (; i < total; i += step) x[i] = cap * tanhf(x[i] / cap);
+}
+
+extern "C" int ptl_softcap(float* x, float cap, long total, hipStream_t st) {
+  if (total <= 0) return PTL_OK;
+  if (!x || !(cap > 0.f)) return PTL_ERR_ARG;
+  long blocks = (total + 255) / 256;
+  if (blocks > 16384) blocks = 16384;
+  softcap_kernel<<<(int)blocks, 256, 0, st>>>(x, cap, (size_t)total);
+  return ptl_launch_status();
+}
+
 // out[t] = e * rsqrt(mean(e^2) + eps) * w with e = table[ids[t]] * scale, as float32: a residual
 // stream that starts from the normed embedding, in one pass over the row.
 template <typename T>
@@ -290,10 +488,6 @@ extern "C" int ptl_embedding_rmsnorm(float* out, const void* table, const int32_
   else
     return PTL_ERR_ARG;
   return ptl_launch_status();
-}
-
-__device__ __forceinline__ float gelu_tanh(float z) {
-  return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
 
 template <typename T>

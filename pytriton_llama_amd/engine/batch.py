@@ -279,7 +279,7 @@ class StepLayout:
             for i, d in enumerate(decode):
                 table = group.tables[d.request]
                 slots[i] = table[d.start // P] * P + d.start % P
-                self._table_row(table_np, owner, i, table, group.spec.window is None)
+                self._table_row(table_np, owner, i, table, not group.spec.gives_back)
             slots[k:B] = -1
             row = B
             for j, s in enumerate(multi):

@@ -71,7 +71,7 @@ class Scheduler:
                              f"({req.params.max_new_tokens}) exceeds max_model_len {self.max_model_len}")
         P = self.manager.page_size
         for g in self.manager.paged:
-            if -(-total // P) > g.pool.num_pages and g.spec.window is None:
+            if -(-total // P) > g.pool.num_pages and not g.spec.gives_back:
                 raise ValueError(f"request {req.id!r} needs {-(-total // P)} pages, the pool has "
                                  f"{g.pool.num_pages}: it can never fit")
         req.status = WAITING

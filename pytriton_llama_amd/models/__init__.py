@@ -4,3 +4,4 @@ from .rubasun import build_rubasun
 from .virusun import build_virusun
 from .matusun import build_matusun
 from .senavik import build_senavik
+from .bimopel import build_bimopel

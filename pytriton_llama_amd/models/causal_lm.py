@@ -48,8 +48,9 @@ class CausalLM:
         self.schedule = list(schedule)
         self.prefixes = list(prefixes)
         self.ignorable = tuple(ignorable)
-        # called by the loader with the names of the checkpoint's tensors before it asks for
-        # expected_tensors(): for what config.json leaves open and the file settles
+        # called by the loader with the names of the checkpoint's tensors and a function from a name
+        # to its shape before it asks for expected_tensors(): for what config.json leaves open and
+        # the file settles
         self.before_load = None
         for call in self.schedule:
             if not 0 <= call.block < len(self.blocks):
@@ -131,7 +132,10 @@ class CausalLM:
     # ---- the forward pass of one step ------------------------------------------
     def forward(self, ctx, storage) -> torch.Tensor:
         """Float32 logits [len(ctx.logit_rows), vocab] for the flat batch ``ctx``."""
-        h = self.embedding.forward(ctx.token_ids)
+        if getattr(self.embedding, "takes_positions", False):
+            h = self.embedding.forward(ctx.token_ids, ctx.positions)
+        else:
+            h = self.embedding.forward(ctx.token_ids)
         residual = None
         last = len(self.schedule) - 1
         for i, call in enumerate(self.schedule):

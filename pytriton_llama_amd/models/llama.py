@@ -85,7 +85,7 @@ def build_llama(cfg: LlamaConfig) -> CausalLM:
         # config.json does not say: tied is the reference's default
         # (lite_llama/models/model_config.py:30), but a file that brings a head of its own is an
         # untied model, and running it with the embedding table would give wrong logits quietly
-        def the_file_decides(names):
+        def the_file_decides(names, shape_of):
             head.tied_to = None if "lm_head.weight" in names else embedding
         model.before_load = the_file_decides
     return model

@@ -143,15 +143,19 @@ def rmsnorm_cols(x: torch.Tensor, weight: torch.Tensor, eps: float) -> torch.Ten
     return y
 
 
-def silu_mul(gate_up: torch.Tensor) -> torch.Tensor:
-    """out[:, i] = silu(gate_up[:, i]) * gate_up[:, I + i] for a [T, 2I] input."""
+GLU_SILU, GLU_GELU_TANH = 0, 1        # activations of a gated feed-forward's gate
+
+
+def silu_mul(gate_up: torch.Tensor, act: int = GLU_SILU) -> torch.Tensor:
+    """out[:, i] = act(gate_up[:, i]) * gate_up[:, I + i] for a [T, 2I] input, act SiLU or the tanh
+    form of GELU."""
     _need_gpu(gate_up)
     if gate_up.dim() != 2 or not gate_up.is_contiguous() or gate_up.shape[1] % 2:
         raise KernelError("silu_mul: input must be a contiguous [T, 2I] matrix")
     T, I2 = gate_up.shape
     out = torch.empty((T, I2 // 2), dtype=gate_up.dtype, device=gate_up.device)
     lib = library.load("activation")
-    _check(lib.ptl_silu_mul(_ptr(out), _ptr(gate_up), T, I2 // 2, _dtype_code(gate_up), _stream()),
+    _check(lib.ptl_silu_mul(_ptr(out), _ptr(gate_up), T, I2 // 2, int(act), _dtype_code(gate_up), _stream()),
            "silu_mul")
     return out
 
@@ -545,8 +549,8 @@ def gate_up_silu_fits(x: torch.Tensor, w: torch.Tensor, blocked: Optional[torch.
 
 
 def gate_up_silu(x: torch.Tensor, w: torch.Tensor, scale: Optional[RowScale] = None,
-                 blocked: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """silu(x Wg^T) * (x Wu^T) for w = [Wg; Wu] ([2I, K]) in one kernel: for at most 16 rows
+                 blocked: Optional[torch.Tensor] = None, act: int = GLU_SILU) -> torch.Tensor:
+    """act(x Wg^T) * (x Wu^T) for w = [Wg; Wu] ([2I, K]) in one kernel (act as for silu_mul): for at most 16 rows
     of bfloat16 x the one of csrc/gemm.hip, from ROWS_MIN rows on, with the blocked copy of w,
     the one of csrc/gemm_rows.hip. ``scale``: the factor that the rows of x still lack (at most
     16 rows); it is applied to both products."""
@@ -561,14 +565,14 @@ def gate_up_silu(x: torch.Tensor, w: torch.Tensor, scale: Optional[RowScale] = N
     if rows:
         _check(library.load("gemm_rows").ptl_rows_gate_up_silu(
             _ptr(out), _ptr(x), _rows_weight(w, blocked, "gate_up_silu"), M, I, K,
-            ctypes.c_long(x.stride(0)), _stream()), "gate_up_silu")
+            ctypes.c_long(x.stride(0)), int(act), _stream()), "gate_up_silu")
         return out
     lib = library.load("gemm")
     pp, count, eps = scale.args(M, K, "gate_up_silu") if scale is not None else _NO_SCALE
     wp, wb = _weight_arg(w, blocked, M, "gate_up_silu")
     _check(lib.ptl_gate_up_silu_bf16(_ptr(out), _ptr(x), wp, wb, M, I, K,
                                      ctypes.c_long(x.stride(0) if M > 1 else max(K, 8)),
-                                     pp, count, eps, _stream()),
+                                     pp, count, eps, int(act), _stream()),
            "gate_up_silu")
     return out
 
@@ -637,28 +641,41 @@ def qkv_rope_store(x: torch.Tensor, w: torch.Tensor, positions: torch.Tensor,
     return q
 
 
-def _mask_extras(what: str, Hq: int, window: int, keep_first: int, sink: Optional[torch.Tensor]):
-    """The two optional pieces every attention kernel takes: ``keep_first`` (with a window: the
-    keys at positions below it stay visible to every later query) and ``sink`` (float32 [Hq]: the
-    softmax denominator of head h also holds exp(sink[h]), a term without key and value)."""
+def _mask_extras(what: str, T: int, Hq: int, window: int, keep_first: int, chunk: int,
+                 sink: Optional[torch.Tensor], gate: Optional[torch.Tensor]):
+    """The optional pieces every attention kernel takes, as kernel arguments: ``window`` (a query
+    sees its own key and the window - 1 before it), ``keep_first`` (with a window: the keys at
+    positions below it stay visible to every later query), ``chunk`` (a query sees the keys of its
+    own chunk of so many positions), ``sink`` (float32 [Hq]: the softmax denominator of head h also
+    holds exp(sink[h]), a term without key and value), ``gate`` (float32 [T, >= Hq], rows may be
+    strided: head h's result of row t is multiplied by sigmoid(gate[t, h]))."""
     if keep_first < 0 or (keep_first and window <= 0):
         raise KernelError(f"{what}: keep_first goes with a window, and is not negative")
+    if chunk < 0 or (chunk and window > 0):
+        raise KernelError(f"{what}: a query sees a window or a chunk, not both")
     if sink is not None and (not sink.is_cuda or sink.dtype != torch.float32 or sink.shape != (Hq,)
                              or not sink.is_contiguous()):
         raise KernelError(f"{what}: sink must be a contiguous float32 GPU tensor [{Hq}]")
-    return int(keep_first), _ptr(sink)
+    stride = 0
+    if gate is not None:
+        if not gate.is_cuda or gate.dim() != 2 or gate.dtype != torch.float32 or gate.stride(1) != 1 \
+                or gate.shape[0] != T or gate.shape[1] < Hq:
+            raise KernelError(f"{what}: gate must be a float32 GPU matrix [{T}, >= {Hq}] with dense rows")
+        stride = gate.stride(0)
+    return int(window), int(keep_first), int(chunk), _ptr(sink), _ptr(gate), ctypes.c_long(stride)
 
 
 def attention_generic(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
                       v_cache: torch.Tensor, q_start: torch.Tensor, ctx_len: torch.Tensor,
                       block_table: torch.Tensor, work_seq: torch.Tensor, work_qoff: torch.Tensor,
                       scale: float, window: int = 0, keep_first: int = 0,
-                      sink: Optional[torch.Tensor] = None) -> None:
+                      sink: Optional[torch.Tensor] = None, chunk: int = 0,
+                      gate: Optional[torch.Tensor] = None) -> None:
     """Attention of a mixed batch over the paged cache (see csrc/attention.hip).
     q [T, Hq, D] (rows may be strided), out [T, Hq, D], caches
     [pages, Hkv, page_size, D], q_start [n+1], ctx_len [n], block_table [n, max_pages],
-    work_seq / work_qoff: the list of 16-row query blocks. ``keep_first``, ``sink``: see
-    _mask_extras."""
+    work_seq / work_qoff: the list of 16-row query blocks. ``window`` and
+    what follows it: see _mask_extras."""
     _need_gpu(out, q, k_cache, v_cache, q_start, ctx_len, block_table, work_seq, work_qoff)
     T, Hq, D = q.shape
     if k_cache.dim() != 4 or k_cache.shape != v_cache.shape or k_cache.shape[3] != D:
@@ -683,13 +700,13 @@ def attention_generic(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
     if block_table.dtype != torch.int32 or block_table.dim() != 2 or block_table.shape[0] < n \
             or block_table.stride(1) != 1:
         raise KernelError("attention: block_table must be int32 [n, max_pages]")
-    keep, sk = _mask_extras("attention", Hq, window, keep_first, sink)
+    extras = _mask_extras("attention", T, Hq, window, keep_first, chunk, sink, gate)
     lib = library.load("attention")
     _check(lib.ptl_attention_generic(
         _ptr(out), ctypes.c_long(out.stride(0)), _ptr(q), ctypes.c_long(q.stride(0)),
         _ptr(k_cache), _ptr(v_cache), _ptr(q_start), _ptr(ctx_len), _ptr(block_table),
         int(block_table.stride(0)), _ptr(work_seq), _ptr(work_qoff), int(work_seq.numel()),
-        Hq, Hkv, D, page_size, int(window), keep, sk, ctypes.c_float(scale), _dtype_code(q), _stream()),
+        Hq, Hkv, D, page_size, *extras, ctypes.c_float(scale), _dtype_code(q), _stream()),
         "attention")
 
 
@@ -727,7 +744,8 @@ def attention_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
                      v_cache: torch.Tensor, q_start: torch.Tensor, ctx_len: torch.Tensor,
                      block_table: torch.Tensor, n_seq: int, scale: float, window: int = 0,
                      num_splits: int = 1, matrix_cores: bool = False, unroll: int = 0,
-                     keep_first: int = 0, sink: Optional[torch.Tensor] = None) -> None:
+                     keep_first: int = 0, sink: Optional[torch.Tensor] = None, chunk: int = 0,
+                     gate: Optional[torch.Tensor] = None) -> None:
     """Split-KV attention of the first ``n_seq`` sequences of the tables, each of
     which brings exactly one query token (see csrc/attention.hip). Head sizes in
     steps of 16 up to 256, float32 or bfloat16. ``matrix_cores``: the MFMA
@@ -742,7 +760,7 @@ def attention_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
         raise KernelError("attention_decode: tables are shorter than n_seq")
     if num_splits < 1:
         raise KernelError("attention_decode: num_splits must be >= 1")
-    keep, sk = _mask_extras("attention_decode", Hq, window, keep_first, sink)
+    extras = _mask_extras("attention_decode", T, Hq, window, keep_first, chunk, sink, gate)
     part_acc = part_ml = None
     if num_splits > 1:
         part_acc = torch.empty((n_seq, Hq, num_splits, D), dtype=torch.float32, device=q.device)
@@ -758,14 +776,14 @@ def attention_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
             _ptr(out), ctypes.c_long(out.stride(0)), _ptr(q), ctypes.c_long(q.stride(0)),
             _ptr(k_cache), _ptr(v_cache), _ptr(q_start), _ptr(ctx_len), _ptr(block_table),
             int(block_table.stride(0)), _ptr(part_acc), _ptr(part_ml), int(n_seq), Hq, Hkv, D,
-            page_size, int(window), keep, sk, ctypes.c_float(scale), int(num_splits), int(unroll),
+            page_size, *extras, ctypes.c_float(scale), int(num_splits), int(unroll),
             _stream()), "attention_decode_mfma")
         return
     _check(lib.ptl_attention_decode(
         _ptr(out), ctypes.c_long(out.stride(0)), _ptr(q), ctypes.c_long(q.stride(0)),
         _ptr(k_cache), _ptr(v_cache), _ptr(q_start), _ptr(ctx_len), _ptr(block_table),
         int(block_table.stride(0)), _ptr(part_acc), _ptr(part_ml), int(n_seq), Hq, Hkv, D, page_size,
-        int(window), keep, sk, ctypes.c_float(scale), int(num_splits), _dtype_code(q), _stream()),
+        *extras, ctypes.c_float(scale), int(num_splits), _dtype_code(q), _stream()),
         "attention_decode")
 
 
@@ -815,7 +833,8 @@ def attention_prefill_mfma(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Te
                            block_table: torch.Tensor, work_seq: torch.Tensor,
                            work_qoff: torch.Tensor, scale: float, window: int = 0,
                            block_rows: int = 64, groups: int = 0, keep_first: int = 0,
-                           sink: Optional[torch.Tensor] = None) -> None:
+                           sink: Optional[torch.Tensor] = None, chunk: int = 0,
+                           gate: Optional[torch.Tensor] = None) -> None:
     """bfloat16 attention of prompt portions on the matrix cores; the work list
     names query blocks of ``block_rows`` (64 or 128) rows, those with the most
     keys first. ``groups`` workgroups a head share the list (0: one for every
@@ -838,7 +857,7 @@ def attention_prefill_mfma(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Te
         raise KernelError("attention_prefill_mfma: query blocks are 64 or 128 rows")
     if q.stride(0) % 8 or out.stride(0) % 4 or q.data_ptr() % 16 or out.data_ptr() % 8:
         raise KernelError("attention_prefill_mfma: q rows must be 16-byte aligned, out rows 8-byte")
-    keep, sk = _mask_extras("attention_prefill_mfma", Hq, window, keep_first, sink)
+    extras = _mask_extras("attention_prefill_mfma", T, Hq, window, keep_first, chunk, sink, gate)
     lib = library.load("attention_prefill")
     n_work = int(work_seq.numel())
     _check(lib.ptl_attention_prefill_mfma(
@@ -846,7 +865,7 @@ def attention_prefill_mfma(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Te
         _ptr(k_cache), _ptr(v_cache), _ptr(q_start), _ptr(ctx_len), _ptr(block_table),
         int(block_table.stride(0)), _ptr(work_seq), _ptr(work_qoff), n_work,
         min(n_work, int(groups)) if groups > 0 else n_work, int(block_rows), Hq, Hkv, D, page_size,
-        int(window), keep, sk, ctypes.c_float(scale), _stream()), "attention_prefill_mfma")
+        *extras, ctypes.c_float(scale), _stream()), "attention_prefill_mfma")
 
 
 def argmax(logits: torch.Tensor, host_out: Optional[torch.Tensor] = None) -> torch.Tensor:
@@ -991,6 +1010,37 @@ def embedding_scaled(table: torch.Tensor, ids: torch.Tensor, scale: float, copie
                                                        ctypes.c_float(scale), int(copies), _dtype_code(table),
                                                        _stream()), "embedding_scaled")
     return out
+
+
+def embedding_positions(table: torch.Tensor, ids: torch.Tensor, positions: torch.Tensor, freq: torch.Tensor,
+                        scale: float = 1.0) -> torch.Tensor:
+    """out[t, j] = table[ids[t], j] * scale + sin (j even) or cos (j odd) of positions[t] *
+    freq[j // 2], as float32: a float32 residual stream that starts with a sinusoidal position."""
+    _need_gpu(table, ids, positions, freq)
+    _i32(ids, "ids")
+    _i32(positions, "positions")
+    if table.dim() != 2 or not table.is_contiguous():
+        raise KernelError("embedding table must be a contiguous [V, H] matrix")
+    V, H = table.shape
+    T = ids.numel()
+    if positions.numel() != T:
+        raise KernelError("embedding_positions: one position a token")
+    _f32_vec(freq, -(-H // 2), "embedding_positions: freq")
+    out = torch.empty((T, H), dtype=torch.float32, device=table.device)
+    _check(library.load("stream").ptl_embedding_positions(
+        _ptr(out), _ptr(table), _ptr(ids), _ptr(positions), _ptr(freq), T, H, V, ctypes.c_float(scale),
+        _dtype_code(table), _stream()), "embedding_positions")
+    return out
+
+
+def softcap_(logits: torch.Tensor, cap: float) -> torch.Tensor:
+    """logits <- cap * tanh(logits / cap) in place, for contiguous float32 logits."""
+    _need_gpu(logits)
+    if logits.dtype != torch.float32 or not logits.is_contiguous() or cap <= 0:
+        raise KernelError("softcap: contiguous float32 logits and a positive cap")
+    _check(library.load("stream").ptl_softcap(_ptr(logits), ctypes.c_float(cap), ctypes.c_long(logits.numel()),
+                                              _stream()), "softcap")
+    return logits
 
 
 def embedding_rmsnorm(table: torch.Tensor, ids: torch.Tensor, weight: torch.Tensor, eps: float,
@@ -1206,7 +1256,8 @@ def gemm_heads_nt(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor,
 def attention_generic_kv(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                          q_start: torch.Tensor, ctx_len: torch.Tensor, block_table: torch.Tensor,
                          work_seq: torch.Tensor, work_qoff: torch.Tensor, scale: float, maps: int = 1,
-                         window: int = 0, keep_first: int = 0, sink: Optional[torch.Tensor] = None) -> None:
+                         window: int = 0, keep_first: int = 0, sink: Optional[torch.Tensor] = None,
+                         chunk: int = 0, gate: Optional[torch.Tensor] = None) -> None:
     """The vector-FMA attention kernel in its general form (csrc/attention.hip): q [T, Hq, Dk]
     with Hq = heads * maps (head after head, map after map), k_cache [pages, Hkv * maps, page_size,
     Dk], v_cache [pages, Hkv, page_size, Dv], out [T, Hq, Dv] in the caches' dtype or float32.
@@ -1238,12 +1289,12 @@ def attention_generic_kv(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tens
     if block_table.dtype != torch.int32 or block_table.dim() != 2 or block_table.shape[0] < n \
             or block_table.stride(1) != 1:
         raise KernelError("attention: block_table must be int32 [n, max_pages]")
-    keep, sk = _mask_extras("attention", Hq, window, keep_first, sink)
+    extras = _mask_extras("attention", T, Hq, window, keep_first, chunk, sink, gate)
     _check(library.load("attention").ptl_attention_generic_kv(
         _ptr(out), ctypes.c_long(out.stride(0)), int(out.dtype == torch.float32 and q.dtype != torch.float32),
         _ptr(q), ctypes.c_long(q.stride(0)), _ptr(k_cache), _ptr(v_cache), _ptr(q_start), _ptr(ctx_len),
         _ptr(block_table), int(block_table.stride(0)), _ptr(work_seq), _ptr(work_qoff),
-        int(work_seq.numel()), Hq, Hkv, int(maps), Dk, Dv, page_size, int(window), keep, sk,
+        int(work_seq.numel()), Hq, Hkv, int(maps), Dk, Dv, page_size, *extras,
         ctypes.c_float(scale), _dtype_code(q), _stream()), "attention")
 
 
@@ -1261,7 +1312,8 @@ def attention_prefill_mfma_kv(out: torch.Tensor, q: torch.Tensor, k_cache: torch
                               q_start: torch.Tensor, ctx_len: torch.Tensor, block_table: torch.Tensor,
                               work_seq: torch.Tensor, work_qoff: torch.Tensor, scale: float, maps: int = 1,
                               groups: int = 1, window: int = 0, keep_first: int = 0,
-                              sink: Optional[torch.Tensor] = None) -> None:
+                              sink: Optional[torch.Tensor] = None, chunk: int = 0,
+                              gate: Optional[torch.Tensor] = None) -> None:
     """The matrix-core kernel for prompt portions in its general form (csrc/attention_prefill.hip):
     shapes as for attention_generic_kv, bfloat16 q and caches, out bfloat16 or float32; the work
     list names 64-row blocks, ``groups`` workgroups a head share it."""
@@ -1293,12 +1345,12 @@ def attention_prefill_mfma_kv(out: torch.Tensor, q: torch.Tensor, k_cache: torch
     n_work = int(work_seq.numel())
     if n_work == 0:
         return
-    keep, sk = _mask_extras("attention_prefill_mfma_kv", Hq, window, keep_first, sink)
+    extras = _mask_extras("attention_prefill_mfma_kv", T, Hq, window, keep_first, chunk, sink, gate)
     _check(library.load("attention_prefill").ptl_attention_prefill_mfma_kv(
         _ptr(out), ctypes.c_long(out.stride(0)), int(out.dtype == torch.float32), _ptr(q),
         ctypes.c_long(q.stride(0)), _ptr(k_cache), _ptr(v_cache), _ptr(q_start), _ptr(ctx_len),
         _ptr(block_table), int(block_table.stride(0)), _ptr(work_seq), _ptr(work_qoff), n_work,
-        max(1, min(int(groups), n_work)), Hq, Hkv, int(maps), Dk, Dv, page_size, int(window), keep, sk,
+        max(1, min(int(groups), n_work)), Hq, Hkv, int(maps), Dk, Dv, page_size, *extras,
         ctypes.c_float(scale), _stream()), "attention_prefill_mfma_kv")
 
 
@@ -1310,7 +1362,8 @@ def attention_decode_kv_fits(Dk: int, Dv: int) -> bool:
 def attention_decode_kv(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                         q_start: torch.Tensor, ctx_len: torch.Tensor, block_table: torch.Tensor, n_seq: int,
                         scale: float, maps: int = 1, num_splits: int = 1, window: int = 0,
-                        keep_first: int = 0, sink: Optional[torch.Tensor] = None) -> None:
+                        keep_first: int = 0, sink: Optional[torch.Tensor] = None, chunk: int = 0,
+                        gate: Optional[torch.Tensor] = None) -> None:
     """Split-KV attention of the first ``n_seq`` sequences of the tables, each of which brings one
     query token, with keys and values of different sizes and ``maps`` score maps a head (shapes as
     for attention_generic_kv; sizes in steps of 16 up to 256)."""
@@ -1337,7 +1390,7 @@ def attention_decode_kv(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tenso
         raise KernelError("attention_decode_kv: block_table must be int32 [n, max_pages]")
     if n_seq > ctx_len.numel() or q_start.numel() < n_seq + 1 or block_table.shape[0] < n_seq or num_splits < 1:
         raise KernelError("attention_decode_kv: tables are shorter than n_seq, or no splits")
-    keep, sk = _mask_extras("attention_decode_kv", Hq, window, keep_first, sink)
+    extras = _mask_extras("attention_decode_kv", T, Hq, window, keep_first, chunk, sink, gate)
     part_acc = part_ml = None
     if num_splits > 1:
         part_acc = torch.empty((n_seq, Hq, num_splits, Dv), dtype=torch.float32, device=q.device)
@@ -1346,7 +1399,7 @@ def attention_decode_kv(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tenso
         _ptr(out), ctypes.c_long(out.stride(0)), int(out.dtype == torch.float32 and q.dtype != torch.float32),
         _ptr(q), ctypes.c_long(q.stride(0)), _ptr(k_cache), _ptr(v_cache), _ptr(q_start), _ptr(ctx_len),
         _ptr(block_table), int(block_table.stride(0)), _ptr(part_acc), _ptr(part_ml), int(n_seq), Hq, Hkv,
-        int(maps), Dk, Dv, page_size, int(window), keep, sk, ctypes.c_float(scale), int(num_splits),
+        int(maps), Dk, Dv, page_size, *extras, ctypes.c_float(scale), int(num_splits),
         _dtype_code(q), _stream()), "attention_decode_kv")
 
 
@@ -1466,6 +1519,33 @@ def stream_add_rmsnorm_sum(stream: torch.Tensor, y1: torch.Tensor, a: float, y2:
         _ptr(stream), _ptr(y1), ctypes.c_float(a), _ptr(y2), ctypes.c_float(b), _dtype_code(y1), _ptr(bias),
         ctypes.c_float(c), _ptr(weight), ctypes.c_float(eps), _ptr(copy),
         _F32 if out_dtype == torch.float32 else _BF16, T, H, _stream()), "stream_add_rmsnorm_sum")
+    return copy
+
+
+def stream_postnorm(stream: torch.Tensor, alpha: float, y1: torch.Tensor, a: float, norm1: Optional[torch.Tensor],
+                    y2: Optional[torch.Tensor], b: float, norm2: Optional[torch.Tensor],
+                    bias: Optional[torch.Tensor], c: float, norm_eps: float, weight: torch.Tensor, eps: float,
+                    out_dtype: Optional[torch.dtype] = None, want_copy: bool = False):
+    """stream <- rmsnorm(alpha stream + a n1(y1) + b n2(y2) + c bias) * weight in place, where n(y) is
+    rmsnorm(y) * norm (with norm_eps), or y when its norm is None; y2 and bias are optional. Returns a
+    copy of the new stream in ``out_dtype`` when asked, else None."""
+    T, H = _check_stream(stream, "stream_postnorm")
+    _need_gpu(y1, y2, norm1, norm2, bias, weight)
+    for y in (y1, y2):
+        if y is not None and (y.shape != stream.shape or not y.is_contiguous() or y.dtype != y1.dtype):
+            raise KernelError("stream_postnorm: the terms must be contiguous matrices of the stream's shape and "
+                              "of one dtype")
+    if H > 16384:
+        raise KernelError(f"stream_postnorm: rows of up to 16384 entries, got {H}")
+    for v, what in ((norm1, "norm1"), (norm2, "norm2"), (bias, "bias"), (weight, "weight")):
+        _f32_vec(v, H, f"stream_postnorm: {what}")
+    out_dtype = out_dtype or torch.float32
+    copy = torch.empty((T, H), dtype=out_dtype, device=stream.device) if want_copy else None
+    _check(library.load("stream").ptl_stream_postnorm(
+        _ptr(stream), ctypes.c_float(alpha), _ptr(y1), ctypes.c_float(a), _ptr(norm1), _ptr(y2), ctypes.c_float(b),
+        _ptr(norm2) if y2 is not None else None, _dtype_code(y1), _ptr(bias), ctypes.c_float(c),
+        ctypes.c_float(norm_eps), _ptr(weight), ctypes.c_float(eps), _ptr(copy),
+        _F32 if out_dtype == torch.float32 else _BF16, T, H, _stream()), "stream_postnorm")
     return copy
 
 
@@ -1910,4 +1990,212 @@ def selective_scan(xc: torch.Tensor, p: torch.Tensor, z_off: int, r: torch.Tenso
         ctypes.c_long(r.stride(0)), int(b_off), int(c_off), _ptr(w_dt), _ptr(dt_bias), _ptr(A_log), _ptr(D),
         _ptr(state), ctypes.c_long(state.stride(0)), _ptr(q_start), _ptr(state_slots), n, int(max_q_len), C, N, R,
         _stream()), "selective_scan")
+    return out
+
+
+# ---------------------------------------------------------------------------
+# Linear recurrences with a decay a head or a key channel (csrc/linear_scan.hip)
+LINEAR_CHUNK = 32                 # tokens whose products run on the matrix cores together
+LINEAR_WORKGROUPS_PER_CU = 3      # workgroups of the final pass that fill the chip
+LINEAR_MAX_KEYS = 256
+
+
+def linear_state_floats(H: int, D: int, Dv: int) -> int:
+    """Floats of the matrices of all heads in a state slot: [H][Dv][D rounded up to 4]."""
+    return H * Dv * (-(-D // 4) * 4)
+
+
+def linear_segment(n_seqs: int, max_q_len: int, H: int, Dv: int, compute_units_: int) -> int:
+    """Rows of a segment of a step's long portions: a multiple of LINEAR_CHUNK, at least two of them,
+    as long as LINEAR_WORKGROUPS_PER_CU workgroups a compute unit allow (a workgroup takes 64 columns
+    of a head in a segment). max_q_len itself when one segment fills the chip."""
+    blocks = max(1, n_seqs) * H * -(-Dv // 64)
+    want = -(-LINEAR_WORKGROUPS_PER_CU * compute_units_ // blocks)
+    if want <= 1 or max_q_len <= 4 * LINEAR_CHUNK:
+        return max(1, max_q_len)
+    rows = -(-max_q_len // want)
+    return max(2 * LINEAR_CHUNK, -(-rows // LINEAR_CHUNK) * LINEAR_CHUNK)
+
+
+def _linear_state(state, q_start, state_slots, H, D, Dv, extra, what):
+    _need_gpu(state, q_start, state_slots)
+    _i32(q_start, "q_start")
+    _i32(state_slots, "state_slots")
+    need = linear_state_floats(H, D, Dv) + extra
+    if state.dim() != 2 or state.dtype != torch.float32 or not state.is_contiguous() or state.shape[1] < need \
+            or state.shape[1] % 4:
+        raise KernelError(f"{what}: state must be contiguous float32 [slots, >= {need}], rows of a multiple of 4")
+    if q_start.numel() != state_slots.numel() + 1:
+        raise KernelError(f"{what}: q_start has one entry more than there are sequences")
+    if D > LINEAR_MAX_KEYS:
+        raise KernelError(f"{what}: key sizes up to {LINEAR_MAX_KEYS}, got {D}")
+    return state_slots.numel()
+
+
+def _linear_columns(m, width, what):
+    if m.dim() != 2 or m.dtype != torch.float32 or not m.is_cuda or m.stride(1) != 1 or m.shape[1] < width:
+        raise KernelError(f"{what}: float32 [T, >= {width}] with dense rows")
+
+
+def linear_scan(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, G: int, D: int,
+                state: torch.Tensor, q_start: torch.Tensor, state_slots: torch.Tensor, max_q_len: int,
+                qscale: float = 1.0, dt: Optional[torch.Tensor] = None, A_log: Optional[torch.Tensor] = None,
+                dt_bias: Optional[torch.Tensor] = None, skip: Optional[torch.Tensor] = None,
+                decay: Optional[torch.Tensor] = None, seg_len: int = 0) -> None:
+    """S <- diag(a) S + k v^T, o = S^T (qscale q) over the rows of every sequence named by q_start and
+    state_slots, from and to the state slots; out float32 [T, H, Dv] receives their rows. q, k:
+    float32 matrices whose first G * D columns are the heads' (head h uses q/k head h / (H / G)); v:
+    H * Dv columns. Either ``decay`` float32 [T, >= H * D] (a decay a key channel), or dt (raw step
+    sizes, H columns), A_log, dt_bias, skip [H]: step = softplus(dt + dt_bias), a = exp(-exp(A_log)
+    step), the value is step * v and skip * v is added to the result. ``max_q_len``: the rows of the
+    longest sequence (or a bound); ``seg_len``: rows of the segments that are walked side by side (0:
+    chosen by linear_segment)."""
+    if out.dim() != 3 or out.dtype != torch.float32 or not out.is_contiguous() or not out.is_cuda:
+        raise KernelError("linear_scan: out must be contiguous float32 [T, H, Dv]")
+    T, H, Dv = out.shape
+    n = _linear_state(state, q_start, state_slots, H, D, Dv, 0, "linear_scan")
+    if n == 0 or T == 0:
+        return
+    if H % G:
+        raise KernelError(f"linear_scan: {H} heads are not a multiple of {G} q/k heads")
+    for m, width in ((q, G * D), (k, G * D), (v, H * Dv)):
+        _linear_columns(m, width, "linear_scan: q, k, v")
+        if m.shape[0] != T:
+            raise KernelError("linear_scan: q, k, v and out have one row a token")
+    scalar = decay is None
+    if scalar:
+        if dt is None or A_log is None or dt_bias is None or skip is None:
+            raise KernelError("linear_scan: decays, or step sizes with A_log, dt_bias and skip")
+        _linear_columns(dt, H, "linear_scan: dt")
+        for t, what in ((A_log, "A_log"), (dt_bias, "dt_bias"), (skip, "skip")):
+            _f32_vec(t, H, f"linear_scan: {what}")
+    else:
+        if G != H:
+            raise KernelError("linear_scan: decays a key channel come with a q/k head a head")
+        _linear_columns(decay, H * D, "linear_scan: decay")
+    max_q_len = max(1, min(int(max_q_len), T))
+    seg_len = int(seg_len) or linear_segment(n, max_q_len, H, Dv, compute_units(out.device))
+    P = -(-max_q_len // seg_len)
+    lib = library.load("linear_scan")
+    work = None
+    if P > 1:
+        lib.ptl_linear_work_floats.restype = ctypes.c_long
+        floats = lib.ptl_linear_work_floats(0 if scalar else 1, n, P, H, D, Dv)
+        if n * P > 65535 or floats > 1 << 28:       # too much to keep: one segment a sequence
+            seg_len, P = max_q_len, 1
+        else:
+            work = torch.empty((floats,), dtype=torch.float32, device=out.device)
+    _check(lib.ptl_linear_scan(
+        0 if scalar else 1, _ptr(out), _ptr(q), ctypes.c_long(q.stride(0)), _ptr(k), ctypes.c_long(k.stride(0)),
+        _ptr(v), ctypes.c_long(v.stride(0)), ctypes.c_float(qscale), _ptr(dt),
+        ctypes.c_long(dt.stride(0) if scalar else 0), _ptr(A_log), _ptr(dt_bias), _ptr(skip), _ptr(decay),
+        ctypes.c_long(0 if scalar else decay.stride(0)), _ptr(state), ctypes.c_long(state.stride(0)), _ptr(work),
+        int(P), int(seg_len), _ptr(q_start), _ptr(state_slots), n, H, G, D, Dv, _stream()), "linear_scan")
+
+
+def lowrank_decay(r: torch.Tensor, w: torch.Tensor, bias: torch.Tensor, tau: float) -> torch.Tensor:
+    """sigmoid(w . r + bias)^(1 / tau): float32 [T, C] from r (float32, the first R columns of its
+    rows), w float32 [C, R], bias [C]."""
+    C, R = w.shape
+    _linear_columns(r, R, "lowrank_decay: r")
+    _f32_vec(w, C * R, "lowrank_decay: w")
+    _f32_vec(bias, C, "lowrank_decay: bias")
+    if R > 1536:
+        raise KernelError(f"lowrank_decay: ranks up to 1536, got {R}")
+    T = r.shape[0]
+    out = torch.empty((T, C), dtype=torch.float32, device=r.device)
+    _check(library.load("linear_scan").ptl_lowrank_decay(
+        _ptr(out), _ptr(r), ctypes.c_long(r.stride(0)), _ptr(w), _ptr(bias), ctypes.c_float(1.0 / tau), T, C, R,
+        _stream()), "lowrank_decay")
+    return out
+
+
+def linear_decode_conv(out: torch.Tensor, p: torch.Tensor, x_off: int, b_off: int, c_off: int, dt_off: int,
+                       A_log: torch.Tensor, dt_bias: torch.Tensor, skip: torch.Tensor, conv_weight: torch.Tensor,
+                       conv_bias: Optional[torch.Tensor], tail_off: int, state: torch.Tensor, q_start: torch.Tensor,
+                       state_slots: torch.Tensor, G: int, D: int) -> None:
+    """One token of every sequence named by q_start and state_slots (the first rows of the step): the
+    short convolution with SiLU on the columns x (H heads of Dv), B and C (G groups of D) of the float32
+    matrix p, then the recurrence of linear_scan with a decay a head (k = B, q = C, v = x). The
+    convolution's channel 0 is column x_off, its kept inputs [taps - 1, C] lie at tail_off of a slot and
+    are read, not advanced (gate_group_norm does that behind this)."""
+    _f32_rows(p, "linear_decode_conv: p")
+    T, H, Dv = out.shape
+    C, taps = conv_weight.shape
+    n = _linear_state(state, q_start, state_slots, H, D, Dv, 0, "linear_decode_conv")
+    if out.dtype != torch.float32 or not out.is_contiguous() or p.shape[0] != T or H % G:
+        raise KernelError("linear_decode_conv: out must be contiguous float32 [T, H, Dv], G must divide H")
+    if tail_off < linear_state_floats(H, D, Dv) or tail_off + (taps - 1) * C > state.shape[1]:
+        raise KernelError("linear_decode_conv: the tail lies outside the state, or inside the matrices")
+    for off, width in ((x_off, H * Dv), (b_off, G * D), (c_off, G * D)):
+        if off < x_off or off + width > min(p.shape[1], x_off + C):
+            raise KernelError("linear_decode_conv: columns outside p, or outside the convolution's channels")
+    if dt_off < 0 or dt_off + H > p.shape[1]:
+        raise KernelError("linear_decode_conv: step sizes outside p")
+    _f32_vec(conv_weight, C * taps, "linear_decode_conv: conv_weight")
+    _f32_vec(conv_bias, C, "linear_decode_conv: conv_bias")
+    for t, what in ((A_log, "A_log"), (dt_bias, "dt_bias"), (skip, "skip")):
+        _f32_vec(t, H, f"linear_decode_conv: {what}")
+    _check(library.load("linear_scan").ptl_linear_decode_conv(
+        _ptr(out), _ptr(p), ctypes.c_long(p.stride(0)), int(x_off), int(b_off), int(c_off), int(dt_off), _ptr(A_log),
+        _ptr(dt_bias), _ptr(skip), _ptr(conv_weight), _ptr(conv_bias), int(taps), int(x_off), int(C),
+        ctypes.c_long(tail_off), _ptr(state), ctypes.c_long(state.stride(0)), _ptr(q_start), _ptr(state_slots), n,
+        H, G, D, Dv, _stream()), "linear_decode_conv")
+
+
+def linear_decode_lowrank(out: torch.Tensor, p: torch.Tensor, q_off: int, k_off: int, v_off: int, a_off: int,
+                          qscale: float, w: torch.Tensor, bias: torch.Tensor, tau: float, state: torch.Tensor,
+                          q_start: torch.Tensor, state_slots: torch.Tensor, D: int) -> None:
+    """One token of every sequence named by q_start and state_slots: the recurrence of linear_scan with
+    a decay a key channel, sigmoid(w . r + bias)^(1 / tau), r the columns of p from a_off on."""
+    _f32_rows(p, "linear_decode_lowrank: p")
+    T, H, Dv = out.shape
+    n = _linear_state(state, q_start, state_slots, H, D, Dv, 0, "linear_decode_lowrank")
+    if out.dtype != torch.float32 or not out.is_contiguous() or p.shape[0] != T:
+        raise KernelError("linear_decode_lowrank: out must be contiguous float32 [T, H, Dv]")
+    C, R = w.shape
+    if C != H * D:
+        raise KernelError(f"linear_decode_lowrank: w must have {H * D} rows")
+    for off, width in ((q_off, H * D), (k_off, H * D), (v_off, H * Dv), (a_off, R)):
+        if off < 0 or off + width > p.shape[1]:
+            raise KernelError("linear_decode_lowrank: columns outside p")
+    _f32_vec(w, C * R, "linear_decode_lowrank: w")
+    _f32_vec(bias, C, "linear_decode_lowrank: bias")
+    _check(library.load("linear_scan").ptl_linear_decode_lowrank(
+        _ptr(out), _ptr(p), ctypes.c_long(p.stride(0)), int(q_off), int(k_off), int(v_off), int(a_off),
+        ctypes.c_float(qscale), _ptr(w), _ptr(bias), R, ctypes.c_float(1.0 / tau), _ptr(state),
+        ctypes.c_long(state.stride(0)), _ptr(q_start), _ptr(state_slots), n, H, D, Dv, _stream()),
+        "linear_decode_lowrank")
+
+
+def gate_group_norm(y: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, groups: int, eps: float,
+                    out_dtype: torch.dtype, tail=None) -> torch.Tensor:
+    """y * silu(gate), then each of ``groups`` equal groups of neighbouring columns divided by its root
+    mean square, times weight: y float32 [T, n] contiguous, gate float32 (the first n columns of its
+    rows), weight float32 [n]; the result [T, n] in ``out_dtype``. ``tail``: (state, tail_off, x, C,
+    taps, state_slots, rows): the first ``rows`` rows are sequences of one token whose slots' kept
+    inputs of a short convolution [taps - 1, C] at tail_off advance by x[t, :C]."""
+    _need_gpu(y, gate, weight)
+    if y.dim() != 2 or y.dtype != torch.float32 or not y.is_contiguous():
+        raise KernelError("gate_group_norm: y must be a contiguous float32 [T, n] matrix")
+    T, n = y.shape
+    _linear_columns(gate, n, "gate_group_norm: gate")
+    _f32_vec(weight, n, "gate_group_norm: weight")
+    if groups <= 0 or n % groups or gate.shape[0] != T or n // groups > 15360:
+        raise KernelError(f"gate_group_norm: {groups} groups of {n} columns (of up to 15360), one gate row a row")
+    state = x = slots = None
+    tail_off, stride, ldx, C, taps, rows = 0, 0, 0, 0, 1, 0
+    if tail is not None:
+        state, tail_off, x, C, taps, slots, rows = tail
+        _linear_columns(x, C, "gate_group_norm: the convolution's inputs")
+        _i32(slots, "state_slots")
+        if state.dim() != 2 or state.dtype != torch.float32 or not state.is_contiguous() or rows > T \
+                or rows > slots.numel() or x.shape[0] != T or tail_off + (taps - 1) * C > state.shape[1]:
+            raise KernelError("gate_group_norm: the tail lies outside the state, or too many rows")
+        stride, ldx = state.stride(0), x.stride(0)
+    out = torch.empty((T, n), dtype=out_dtype, device=y.device)
+    _check(library.load("prepare").ptl_gate_group_norm(
+        _ptr(out), _ptr(y), _ptr(gate), ctypes.c_long(gate.stride(0)), _ptr(weight), int(groups), ctypes.c_float(eps),
+        T, n, _ptr(state), ctypes.c_long(stride), ctypes.c_long(tail_off), _ptr(x), ctypes.c_long(ldx), _ptr(slots),
+        int(rows), int(C), int(taps), _dtype_code(out), _stream()), "gate_group_norm")
     return out

@@ -28,7 +28,7 @@ HIPCC_FLAGS = ["--offload-arch=" + ARCH, "-O3", "-fPIC", "-shared", "-std=c++17"
 
 KERNEL_LIBRARIES = ("embedding", "norm", "rope", "attention", "attention_prefill", "activation",
                     "gemm", "gemm_rows", "blaslt", "sampling", "probe", "stream", "latent", "moe", "prepare",
-                    "recurrent", "selective")
+                    "recurrent", "selective", "linear_scan")
 # options of single sources. attention_prefill: no value there is a NaN unless an input is, and
 # without the promise every maximum of scores is preceded by instructions that quiet its inputs
 EXTRA_FLAGS = {"attention_prefill": ["-fno-honor-nans"]}

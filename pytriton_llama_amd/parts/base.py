@@ -20,7 +20,8 @@ mixer:           cache_spec() -> PagedSpec | StateSpec | None
                  work_lists() -> WorkList, ...   (optional) how its kernels cut the query rows
 feed-forward:    forward(x) -> y
 position:        rotary_inv_freq() -> float32 [D/2] or None;  apply(q, k, positions) in place
-embedding:       forward(token_ids int32 [T]) -> [T, hidden]
+embedding:       forward(token_ids int32 [T]) -> [T, hidden]; one whose class says
+                 takes_positions gets the positions int32 [T] as well
 head:            forward(x [R, hidden]) -> float32 logits [R, vocab]
 block:           forward(h, residual, ctx, cache) -> (h, residual); may set the flags
                  can_defer_output (forward then takes defer_output=True and may return a
@@ -99,11 +100,13 @@ class PagedSpec:
     """What a mixer keeps for every token, in pages: any number of named tensors. ``window``:
     only the last ``window`` positions are ever read again, older pages can be given back;
     ``keep_first``: except the first so many positions of a sequence, which every later query
-    reads (their pages stay). Cache layers with equal specs share a page pool and a block table
-    per request."""
+    reads (their pages stay). ``chunk``: the positions form chunks of so many, counted from the
+    sequence's start, and a query reads its own chunk only; pages of chunks that are over can be
+    given back. Cache layers with equal specs share a page pool and a block table per request."""
     tensors: Tuple[PagedTensor, ...]
     window: Optional[int] = None
     keep_first: int = 0
+    chunk: Optional[int] = None
 
     def __post_init__(self):
         names = [t.name for t in self.tensors]
@@ -111,6 +114,22 @@ class PagedSpec:
             raise ValueError(f"a paged cache spec needs tensors with names of their own, got {names}")
         if self.keep_first < 0:
             raise ValueError("keep_first is a number of positions")
+        if self.chunk is not None and (self.chunk <= 0 or self.window is not None):
+            raise ValueError("a chunk holds at least one position, and goes without a window")
+
+    @property
+    def gives_back(self) -> bool:
+        """Whether later queries leave pages behind (else a request keeps all of them)."""
+        return self.window is not None or self.chunk is not None
+
+    def first_needed(self, position: int) -> int:
+        """The first position that a query at ``position``, or any later one, reads (beside the
+        kept first ones)."""
+        if self.window is not None:
+            return max(0, position - self.window + 1)
+        if self.chunk is not None:
+            return max(0, position) // self.chunk * self.chunk
+        return 0
 
 
 def paged_kv_spec(num_kv_heads: int, head_dim: int, window: Optional[int] = None) -> PagedSpec:
@@ -178,22 +197,30 @@ class PendingSum:
     """a y1 + b y2 + c bias that has not been added up: what a mixer returns whose result is a
     weighted sum (two mixers side by side, an output projection with a bias). ``terms``: one or two
     (matrix [T, hidden], factor); ``bias``: (float32 vector [hidden], factor) or None. A block
-    whose next kernel reads the result anyway (a norm on the sublayer's output) adds it up there."""
-    __slots__ = ("terms", "bias")
+    whose next kernel reads the result anyway (a norm on the sublayer's output) adds it up there.
+    ``norms``: None, or for every term (float32 weight [hidden], eps): the term is then rmsnorm(y) *
+    weight, also not computed yet (all with one eps)."""
+    __slots__ = ("terms", "bias", "norms")
 
-    def __init__(self, terms, bias=None):
+    def __init__(self, terms, bias=None, norms=None):
         if not 1 <= len(terms) <= 2:
             raise ValueError("a pending sum has one or two terms")
-        self.terms, self.bias = list(terms), bias
+        if norms is not None and (len(norms) != len(terms) or len({n[1] for n in norms}) != 1):
+            raise ValueError("a norm for every term, all with one eps")
+        self.terms, self.bias, self.norms = list(terms), bias, norms
 
     @property
     def shape(self):
         return self.terms[0][0].shape
 
     def tensor(self) -> torch.Tensor:
-        out = self.terms[0][0].float() * self.terms[0][1]
-        for y, f in self.terms[1:]:
-            out = out + y.float() * f
+        out = 0.0
+        for i, (y, f) in enumerate(self.terms):
+            y = y.float()
+            if self.norms is not None:
+                w, eps = self.norms[i]
+                y = y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + eps) * w
+            out = out + y * f
         if self.bias is not None:
             out = out + self.bias[0] * self.bias[1]
         return out.to(self.terms[0][0].dtype)

@@ -240,12 +240,11 @@ class OutputNormBlock(Part):
     def graph_capturable(self) -> bool:
         return all(getattr(p, "graph_capturable", True) for p in self.children().values())
 
-    @staticmethod
-    def _add(stream, y, norm, dtype, want_copy):
+    def _add(self, stream, y, norm, dtype, want_copy):
         """stream += norm(y); returns the new stream in ``dtype`` when asked (the stream itself
         when that is float32)."""
         copy = want_copy and dtype != torch.float32
-        if isinstance(y, PendingSum):
+        if isinstance(y, PendingSum) and y.norms is None:
             (y1, a), (y2, b) = y.terms[0], (y.terms[1] if len(y.terms) > 1 else (None, 0.0))
             bias, c = y.bias if y.bias is not None else (None, 0.0)
             out = ops.stream_add_rmsnorm_sum(stream, y1, a, y2, b, bias, c, norm.weight, norm.eps, dtype, copy)
@@ -266,6 +265,38 @@ class OutputNormBlock(Part):
         a = self._add(stream, y, self.norm1, dtype, True)
         y = self.feed_forward.forward(a)
         return stream, self._add(stream, y, self.norm2, dtype, not self.last)
+
+
+@register_part("block", "post_norm")
+class PostNormBlock(OutputNormBlock):
+    """A norm behind every residual sum, on a stream kept in float32 whose old value is scaled first:
+
+        x <- norm1(alpha x + mixer(x));   x <- norm2(alpha x + ffn(x))
+
+    The sublayers read x itself (in the engine's dtype); the feed-forward with its norm is optional.
+    The norms are RMS norms; the sum, the norm and the copy of the new stream for the next sublayer
+    are one kernel, which also finishes a sublayer's result that arrives as a weighted sum not yet
+    made, of terms that may each lack a norm of their own (parts.base.PendingSum)."""
+
+    def __init__(self, mixer: Part, mixer_norm: Part, feed_forward: Part = None, ffn_norm: Part = None,
+                 alpha: float = 1.0):
+        super().__init__(mixer, mixer_norm, feed_forward, ffn_norm)
+        self.alpha = float(alpha)
+
+    def _add(self, stream, y, norm, dtype, want_copy):
+        """stream = norm(alpha stream + y); returns the new stream in ``dtype`` when asked (the stream
+        itself when that is float32)."""
+        copy = want_copy and dtype != torch.float32
+        if not isinstance(y, PendingSum):
+            y = PendingSum([(as_tensor(y), 1.0)])
+        (y1, a), (y2, b) = y.terms[0], (y.terms[1] if len(y.terms) > 1 else (None, 0.0))
+        norms = y.norms or [(None, 0.0)] * 2
+        n1, n_eps = norms[0]
+        n2 = norms[1][0] if y2 is not None else None
+        bias, c = y.bias if y.bias is not None else (None, 0.0)
+        out = ops.stream_postnorm(stream, self.alpha, y1, a, n1, y2, b, n2, bias, c, n_eps, norm.weight, norm.eps,
+                                  dtype, copy)
+        return out if copy else (stream if want_copy else None)
 
 
 @register_part("block", "hyper_connections")

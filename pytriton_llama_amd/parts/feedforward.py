@@ -12,17 +12,21 @@ from .linear import LINEAR_LIBRARIES, decode_copy, linear
 
 @register_part("feed_forward", "swiglu")
 class SwiGLU(Part):
-    """down(silu(gate(x)) * up(x)), three matrices without bias
-    (lite_llama/models/llama.py:107-120, lite_llama/kernels/swiglu.py:44-67).
+    """down(act(gate(x)) * up(x)), three matrices without bias, act SiLU
+    (lite_llama/models/llama.py:107-120, lite_llama/kernels/swiglu.py:44-67) or, with
+    ``activation`` "gelu_tanh", the tanh form of GELU.
     gate and up are concatenated at load into one [2I, hidden] matrix (rows
-    gate | up) so that one product feeds the SiLU-multiply kernel."""
+    gate | up) so that one product feeds the activation-multiply kernel."""
     kernel_libraries = ("activation", "norm") + LINEAR_LIBRARIES
     takes_pending_scale = True
     can_defer_output = True
 
     def __init__(self, hidden_size: int, intermediate_size: int,
                  gate_name: str = "gate_proj.weight", up_name: str = "up_proj.weight",
-                 down_name: str = "down_proj.weight"):
+                 down_name: str = "down_proj.weight", activation: str = "silu"):
+        if activation not in ("silu", "gelu_tanh"):
+            raise ValueError(f"unknown gated activation {activation!r} (known: 'silu', 'gelu_tanh')")
+        self.act = ops.GLU_GELU_TANH if activation == "gelu_tanh" else ops.GLU_SILU
         self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
         self.names = (gate_name, up_name, down_name)
         self.gate_up: Optional[torch.Tensor] = None
@@ -52,12 +56,12 @@ class SwiGLU(Part):
             x, scale = x.values, x.scale
         x = as_tensor(x)
         if ops.gate_up_silu_fits(x, self.gate_up, self.gate_up_blocked):
-            # the few rows of a decode step: product and SiLU-multiply in one kernel
-            a = ops.gate_up_silu(x, self.gate_up, scale, blocked=self.gate_up_blocked)
+            # the few rows of a decode step: product and activation-multiply in one kernel
+            a = ops.gate_up_silu(x, self.gate_up, scale, blocked=self.gate_up_blocked, act=self.act)
             if defer_output:
                 return PendingProduct(a, self.down, self.down_blocked)
             return linear(a, self.down, blocked=self.down_blocked)
-        a = ops.silu_mul(linear(x, self.gate_up, blocked=self.gate_up_blocked))
+        a = ops.silu_mul(linear(x, self.gate_up, blocked=self.gate_up_blocked), self.act)
         if defer_output:                    # (the norm that follows picks the kernels by the rows)
             return PendingProduct(a, self.down, self.down_blocked)
         return linear(a, self.down, blocked=self.down_blocked)

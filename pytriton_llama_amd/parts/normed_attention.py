@@ -37,7 +37,10 @@ class NormedAttention(Part):
                 ``keep_first``: and over the keys at positions below it, which stay where they
                 are and are never given back. ``sink_name``: a vector of the checkpoint, one
                 number a head; the softmax denominator of head h also holds exp(sink_h), a term
-                without key and value that the scale does not touch)
+                without key and value that the scale does not touch; ``sink``: the same with one
+                fixed number for all heads. ``chunk``: over the keys of the query's own chunk, the
+                positions cut into chunks of so many from the sequence's start; pages of chunks that
+                are over are given back)
 
     maps = 1: out = W_o concat_h a + b_o.
     maps = 2 (differential attention: the second map is subtracted so that what both maps give
@@ -45,11 +48,13 @@ class NormedAttention(Part):
     for the layer, from four vectors of the checkpoint), o = a_1 - lam a_2, divided by its root mean
     square over vdim (no weight), times (1 - diff).
     ``gated``: the concatenated heads times sigmoid(W_g x) before the output projection.
+    ``head_gated`` (maps = 1): head h's result times sigmoid(W_g x)_h, W_g [heads, hidden], where the
+    attention kernel finishes its rows.
 
     The cache keeps the normed and rotated keys [kv_heads * maps, dim] and the values [kv_heads,
     vdim] of every token. ``own_kv`` False: the layer has no key and value tensors and reads the
     cache layer of another one (the run order hands it over, not writable); sizes and rotation
-    are the owner's. Scores, softmax, norms, angles and lam are float32; the projection's result is
+    are the owner's. ``o_bias`` False: the output projection has no bias even with ``bias``. Scores, softmax, norms, angles and lam are float32; the projection's result is
     taken in float32 so that bias and norm see it unrounded. Tensor names are parameters; biases
     are the projection's name with ".b" added. ``rot_scaling``: None, or the numbers of a
     frequency scaling: factor, original, fast, slow (a ramp between the entries that turn fast and
@@ -61,7 +66,8 @@ class NormedAttention(Part):
                  maps: int = 1, diff: float = 0.0, bias: bool = True, gated: bool = False,
                  rot_dims: int = 0, rot_base: float = 10000.0, rot_scaling: Optional[dict] = None,
                  own_kv: bool = True, window: Optional[int] = None, keep_first: int = 0,
-                 sink_name: Optional[str] = None, q_name: str = "q", k_name: str = "k", v_name: str = "v",
+                 sink_name: Optional[str] = None, sink: Optional[float] = None, chunk: Optional[int] = None,
+                 head_gated: bool = False, o_bias: bool = True, q_name: str = "q", k_name: str = "k", v_name: str = "v",
                  g_name: str = "g", o_name: str = "o", lambda_names=("lq1", "lk1", "lq2", "lk2")):
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} heads are not a multiple of {num_kv_heads} kv heads")
@@ -70,6 +76,8 @@ class NormedAttention(Part):
         if gated and maps == 1:
             raise ValueError("the output gate is built for two maps a head (it is applied where the maps "
                              "are combined)")
+        if head_gated and (maps != 1 or gated):
+            raise ValueError("a gate a head is built for one map a head, and is the only gate")
         if qk_norm not in (None, "head", "whole"):
             raise ValueError(f"unknown query/key norm {qk_norm!r} (known: 'head', 'whole', None)")
         if rot_dims % 2 or not 0 <= rot_dims <= dim:
@@ -82,6 +90,7 @@ class NormedAttention(Part):
         self.eps, self.diff = float(eps), float(diff)
         self.norm_mode = {None: ops.NORM_NONE, "head": ops.NORM_HEAD, "whole": ops.NORM_WHOLE}[qk_norm]
         self.bias, self.gated, self.own_kv = bool(bias), bool(gated), bool(own_kv)
+        self.head_gated, self.has_o_bias = bool(head_gated), bool(bias) and bool(o_bias)
         self.rot_dims = int(rot_dims)
         if window is not None and window <= 0:
             raise ValueError("a window holds at least the query's own position")
@@ -89,9 +98,14 @@ class NormedAttention(Part):
         if keep_first < 0 or (keep_first and not self.window):
             raise ValueError("first positions are kept beside a window, and their number is not negative")
         self.keep_first = int(keep_first)
-        if sink_name and maps != 1:
+        if chunk is not None and (chunk <= 0 or self.window):
+            raise ValueError("a chunk holds at least one position, and goes without a window")
+        self.chunk = int(chunk) if chunk else None
+        if (sink_name or sink is not None) and maps != 1:
             raise ValueError("a term of the denominator without a key is built for one score map a head")
-        self.sink_name = sink_name or None
+        if sink_name and sink is not None:
+            raise ValueError("the term without a key is learned or fixed, not both")
+        self.sink_name, self.sink_value = sink_name or None, sink
         self.sink = None
         self.mag = 1.0
         self.inv_freq_host = None
@@ -140,6 +154,8 @@ class NormedAttention(Part):
         span = max(ctx.ctx_lens[:n_dec])
         if self.window:
             span = min(span, self.window + self.keep_first)
+        if self.chunk:
+            span = min(span, self.chunk)
         cus = ops.compute_units(device)
         if matrix_cores:
             base = max(1, n_dec * self.num_kv_heads)
@@ -154,14 +170,14 @@ class NormedAttention(Part):
         want = -(-2 * cus // base)
         return max(1, min(want, -(-span // turn), 64))
 
-    def attend(self, a, q, cache, ctx, group) -> None:
+    def attend(self, a, q, cache, ctx, group, gate=None) -> None:
         """Leading sequences of one token: the split-KV kernel (its matrix-core form where one
         map reads keys and values of one size that it takes); the rest: the matrix-core kernel in
         64-row blocks (bfloat16, sizes that are multiples of 32 up to 128) or the vector kernel in
-        16-row blocks."""
+        16-row blocks. ``gate``: float32 [T, >= heads], a factor sigmoid(gate) a row and head."""
         n_dec = ctx.num_decode_seqs if ops.attention_decode_kv_fits(self.dim, self.vdim) else 0
         window = self.window or 0
-        extras = dict(keep_first=self.keep_first, sink=self.sink)
+        extras = dict(keep_first=self.keep_first, sink=self.sink, chunk=self.chunk or 0, gate=gate)
         # one map and keys as large as values: the matrix-core form of the split-KV kernel takes them
         mfma = (n_dec and self.maps == 1 and self.dim == self.vdim and q.stride(0) % 8 == 0
                 and ops.attention_decode_mfma_fits(q.dtype, self.num_heads, self.num_kv_heads, self.dim,
@@ -196,7 +212,7 @@ class NormedAttention(Part):
             return None
         return PagedSpec((PagedTensor("k", (self.num_kv_heads * self.maps, self.dim), 1),
                           PagedTensor("v", (self.num_kv_heads, self.vdim), 1)), self.window,
-                         self.keep_first)
+                         self.keep_first, self.chunk)
 
     def _norm_sizes(self):
         if self.norm_mode == ops.NORM_WHOLE:
@@ -224,10 +240,12 @@ class NormedAttention(Part):
             out += [ParamSource(x, (self.dim,), "vector", init=("normal", 0.0, 0.1)) for x in self.lambda_names]
         if self.gated:
             out.append(ParamSource(n["g"], (self.o_size, W)))
+        if self.head_gated:
+            out.append(ParamSource(n["g"], (self.num_heads, W)))
         if self.sink_name:
             out.append(ParamSource(self.sink_name, (self.num_heads,), "vector", init=("normal", 0.0, 1.0)))
         out.append(ParamSource(n["o"], (W, self.o_size)))
-        if self.bias:
+        if self.has_o_bias:
             out.append(ParamSource(n["o"] + ".b", (W,), "vector", init=small))
         return out
 
@@ -236,13 +254,14 @@ class NormedAttention(Part):
         rows = [tensors[n["q"]]]
         if self.own_kv:
             rows += [tensors[n["k"]], tensors[n["v"]]]
-        if self.gated:
+        if self.gated or self.head_gated:
             rows.append(tensors[n["g"]])
         self.proj = place(pad_rows(torch.cat(rows, dim=0)), "matrix", dtype, device)
         self.o = place(tensors[n["o"]], "matrix", dtype, device)
         if self.bias:
             self.q_bias = place(tensors[n["q"] + ".b"], "vector", dtype, device)
-            self.o_bias = place(tensors[n["o"] + ".b"], "vector", dtype, device)
+            if self.has_o_bias:
+                self.o_bias = place(tensors[n["o"] + ".b"], "vector", dtype, device)
             if self.own_kv:
                 self.k_bias = place(tensors[n["k"] + ".b"], "vector", dtype, device)
                 self.v_bias = place(tensors[n["v"] + ".b"], "vector", dtype, device)
@@ -257,6 +276,8 @@ class NormedAttention(Part):
             self.inv_freq = self.inv_freq_host.to(device)
         if self.sink_name:
             self.sink = place(tensors[self.sink_name], "vector", dtype, device)
+        elif self.sink_value is not None:
+            self.sink = torch.full((self.num_heads,), float(self.sink_value), dtype=torch.float32, device=device)
 
     def make_decode_copies(self) -> int:
         self.proj_blocked, self.o_blocked = decode_copy(self.proj), decode_copy(self.o)
@@ -279,7 +300,7 @@ class NormedAttention(Part):
                         H * M, G * M, G, Dk, Dv, cache.page_size)
         plain = M == 1
         a = torch.empty((T, H * M, Dv), dtype=x.dtype if plain else torch.float32, device=x.device)
-        self.attend(a, q, cache, ctx, group)
+        self.attend(a, q, cache, ctx, group, p[:, self.g_off:] if self.head_gated else None)
         if plain:
             return a.view(T, H * Dv)
         out = torch.empty((T, H * Dv), dtype=x.dtype, device=x.device)
@@ -291,4 +312,4 @@ class NormedAttention(Part):
     def forward(self, x, ctx, cache):
         heads = self.heads_output(x, ctx, cache)
         y = linear(heads, self.o, out_dtype=torch.float32, blocked=self.o_blocked)
-        return PendingSum([(y, 1.0)], (self.o_bias, 1.0) if self.bias else None)
+        return PendingSum([(y, 1.0)], (self.o_bias, 1.0) if self.has_o_bias else None)

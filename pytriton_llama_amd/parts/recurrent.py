@@ -254,11 +254,19 @@ class ParallelMixers(Part):
     """Two mixers side by side on one input: left_scale * left(x) + right_scale * right(x). Each
     keeps a cache of its own kind: ``cache_spec`` is a pair, and the model's run order hands the
     mixer a pair of cache layers. The sum is not made here: it is handed on (parts.base.PendingSum)
-    to whoever reads the result next."""
+    to whoever reads the result next. ``left_norm``, ``right_norm``: RMS norm parts (both or neither)
+    applied to the two results before they are scaled and added; they are handed on with the sum."""
 
-    def __init__(self, left: Part, right: Part, left_scale: float = 1.0, right_scale: float = 1.0):
+    def __init__(self, left: Part, right: Part, left_scale: float = 1.0, right_scale: float = 1.0,
+                 left_norm: Part = None, right_norm: Part = None):
         self.left, self.right = left, right
         self.left_scale, self.right_scale = float(left_scale), float(right_scale)
+        if (left_norm is None) != (right_norm is None):
+            raise ValueError("a norm for both results, or for neither")
+        self.norms = None if left_norm is None else {"left.": left_norm, "right.": right_norm}
+        for n in (left_norm, right_norm):
+            if n is not None and not (hasattr(n, "weight") and hasattr(n, "eps")):
+                raise ValueError("the norms of the results are RMS norms (a weight and an eps)")
         self.kernel_libraries = tuple(dict.fromkeys(tuple(left.kernel_libraries) + tuple(right.kernel_libraries)))
 
     def children(self):
@@ -283,13 +291,16 @@ class ParallelMixers(Part):
     def param_sources(self) -> List[ParamSource]:
         out = []
         for prefix, m in self.children().items():
-            for s in m.param_sources():
+            for s in m.param_sources() + (self.norms[prefix].param_sources() if self.norms else []):
                 out.append(ParamSource(prefix + s.name, s.shape, s.kind, s.init))
         return out
 
     def load(self, tensors, dtype, device) -> None:
         for prefix, m in self.children().items():
-            m.load({k[len(prefix):]: v for k, v in tensors.items() if k.startswith(prefix)}, dtype, device)
+            own = {k[len(prefix):]: v for k, v in tensors.items() if k.startswith(prefix)}
+            m.load(own, dtype, device)
+            if self.norms:
+                self.norms[prefix].load(own, dtype, device)
 
     def make_decode_copies(self) -> int:
         return sum(m.make_decode_copies() for m in (self.left, self.right) if hasattr(m, "make_decode_copies"))
@@ -298,10 +309,19 @@ class ParallelMixers(Part):
         x = as_tensor(x)
         if not isinstance(cache, tuple) or len(cache) != 2:
             raise RuntimeError("two mixers side by side need a pair of cache layers")
+        if self.norms:
+            terms = []
+            for m, c, scale in ((self.left, cache[0], self.left_scale), (self.right, cache[1], self.right_scale)):
+                y = m.forward(x, ctx, c)
+                plain = isinstance(y, PendingSum) and len(y.terms) == 1 and y.terms[0][1] == 1.0 and y.bias is None
+                terms.append((y.terms[0][0] if plain and y.norms is None else as_tensor(y), scale))
+            if terms[0][0].dtype != terms[1][0].dtype:
+                terms = [(t.float(), s) for t, s in terms]
+            return PendingSum(terms, None, [(n.weight, n.eps) for n in self.norms.values()])
         terms, bias = [], None
         for m, c, scale in ((self.left, cache[0], self.left_scale), (self.right, cache[1], self.right_scale)):
             y = m.forward(x, ctx, c)
-            if isinstance(y, PendingSum) and len(y.terms) == 1 and (y.bias is None or bias is None):
+            if isinstance(y, PendingSum) and len(y.terms) == 1 and y.norms is None and (y.bias is None or bias is None):
                 terms.append((y.terms[0][0], y.terms[0][1] * scale))
                 if y.bias is not None:
                     bias = (y.bias[0], y.bias[1] * scale)

@@ -70,11 +70,6 @@ def load_weights(model, folder: str, dtype: torch.dtype, device) -> None:
     from safetensors import safe_open
 
     files = _tensor_files(folder)
-    if getattr(model, "before_load", None) is not None:
-        model.before_load(set(files))
-    expected = model.expected_tensors()
-    missing = sorted(n for n in expected if n not in files)
-    unexpected = sorted(n for n in files if n not in expected and not model.is_ignorable(n))
     handles = {}
 
     def handle(path):
@@ -82,13 +77,21 @@ def load_weights(model, folder: str, dtype: torch.dtype, device) -> None:
             handles[path] = safe_open(path, framework="pt")
         return handles[path]
 
+    def shape_of(name):
+        return tuple(handle(files[name]).get_slice(name).get_shape())
+
+    if getattr(model, "before_load", None) is not None:
+        model.before_load(set(files), shape_of)
+    expected = model.expected_tensors()
+    missing = sorted(n for n in expected if n not in files)
+    unexpected = sorted(n for n in files if n not in expected and not model.is_ignorable(n))
+
     wrong: List[Tuple[str, tuple, tuple]] = []
     other: List[str] = []
     for name, (_, src) in expected.items():
         if name not in files:
             continue
-        sl = handle(files[name]).get_slice(name)
-        shape = tuple(sl.get_shape())
+        shape = shape_of(name)
         if shape != tuple(src.shape):
             wrong.append((name, shape, tuple(src.shape)))
     if missing or unexpected or wrong or other:
