@@ -345,6 +345,42 @@ SENAVIK_SIZES = {
 }
 
 
+def bimopel_shape(width, layers, heads, kv_heads, dim, chunk, linear_heads, linear_dim, linear_vdim, mamba_heads,
+                  mamba_vdim, state, groups, norm_groups, ff, vocab):
+    """A Bimopel config.json of a real model's layer sizes: three layers of Mamba-2 without a
+    feed-forward, then one with attention inside chunks beside gated linear attention and a dense
+    feed-forward, in turn."""
+    mamba = {"heads": mamba_heads, "vdim": mamba_vdim, "state": state, "groups": groups, "conv": 4,
+             "norm_groups": norm_groups}
+    left = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+            "mask": {"size": chunk}}
+    right = {"heads": linear_heads, "dim": linear_dim, "vdim": linear_vdim, "tau": 16.0, "rank": 16}
+    out = []
+    for i in range(layers):
+        if i % 4 == 3:
+            out.append({"type": "parallel", "mixer": {"left": left, "right": right}, "mlp": {"kind": "dense", "ff": ff}})
+        else:
+            out.append({"type": "mamba2", "mixer": mamba, "mlp": None})
+    return {"architecture": "Bimopel", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+            "embedding": {"scale": width ** 0.5}, "postln_alpha": 2.0, "logit_softcap": 30.0, "layers": out,
+            "initializer_range": 0.02}
+
+
+# name -> (Bimopel sizes, the Llama shape of equal width, depth, heads and feed-forward width)
+BIMOPEL_SIZES = {
+    "2048": (dict(width=2048, layers=8, heads=16, kv_heads=4, dim=128, chunk=1024, linear_heads=8, linear_dim=128,
+                  linear_vdim=128, mamba_heads=64, mamba_vdim=64, state=128, groups=8, norm_groups=8, ff=8192,
+                  vocab=32000),
+             dict(num_hidden_layers=8, hidden_size=2048, num_attention_heads=16, num_key_value_heads=4,
+                  head_dim=128, intermediate_size=8192, vocab_size=32000, tie_word_embeddings=False)),
+    "4096": (dict(width=4096, layers=4, heads=32, kv_heads=8, dim=128, chunk=2048, linear_heads=16, linear_dim=128,
+                  linear_vdim=128, mamba_heads=128, mamba_vdim=64, state=128, groups=8, norm_groups=8, ff=14336,
+                  vocab=32000),
+             dict(num_hidden_layers=4, hidden_size=4096, num_attention_heads=32, num_key_value_heads=8,
+                  head_dim=128, intermediate_size=14336, vocab_size=32000, tie_word_embeddings=False)),
+}
+
+
 def engine_rates(cfg, dtype, S, batch, steps, warmup):
     """Prefill of one S-token prompt (one step) and decode steps of ``batch`` requests behind
     S-token prompts, through the whole engine, for any architecture."""
@@ -449,6 +485,14 @@ def senavik_beside_llama(args):
                         others=(("matusun", MATUSUN_SIZES, matusun_shape),))
 
 
+def bimopel_beside_llama(args):
+    """Bimopel beside Llama and, with 'virusun' or 'matusun' among --bimopel-models, beside the designs
+    whose layers are closest to its own (attention beside a recurrence and norms on a float32
+    stream; the selective scan)."""
+    return beside_llama(args, "bimopel", args.bimopel, args.bimopel_models, BIMOPEL_SIZES, bimopel_shape,
+                        others=(("virusun", VIRUSUN_SIZES, virusun_shape), ("matusun", MATUSUN_SIZES, matusun_shape)))
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -497,6 +541,11 @@ def main():
     ap.add_argument("--senavik-models", default="senavik,llama",
                     help="with --senavik: which models to run, of senavik, llama and matusun (the design with "
                          "the closest layers, at the same named size)")
+    ap.add_argument("--bimopel", default="", metavar="SIZES",
+                    help="the same for the Bimopel design (sizes of: 2048, 4096)")
+    ap.add_argument("--bimopel-models", default="bimopel,llama",
+                    help="with --bimopel: which models to run, of bimopel, llama, virusun and matusun (the designs "
+                         "with the closest layers, at the same named size)")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py measures one GPU: this engine has no multi-GPU path, --gpus {args.gpus} is not run")
@@ -529,6 +578,8 @@ def main():
         return matusun_beside_llama(args)
     if args.senavik:
         return senavik_beside_llama(args)
+    if args.bimopel:
+        return bimopel_beside_llama(args)
     if args.mixed:
         return mixed_workload(args, cfg, short)
     if args.like_reference:

@@ -12,8 +12,8 @@
 // Everything is float32. Query head h uses q/k head h / heads_per_qk. S lives in the request's state
 // slot as [H][Dv][DS] floats (a column of S after the other, DS = D rounded up to a multiple of 4).
 //
-// ptl_linear_decode: sequences of one token. A workgroup takes 16 columns of a head of a sequence, a
-//   column in 16 lanes (one row of a wave for the data-parallel lane moves); what is in front of the
+// ptl_linear_decode_conv, ptl_linear_decode_lowrank: sequences of one token. A workgroup takes 16 to 64
+//   columns of a head of a sequence, a column in 16 lanes (one row of a wave for the data-parallel lane moves); what is in front of the
 //   recurrence is done by the workgroup itself: the short causal convolution with SiLU (scalar form)
 //   or the low-rank decays (channel form). Bound by reading and writing S once.
 // ptl_linear_scan: portions. The rows of a sequence are walked in chunks of 32 tokens whose products
@@ -83,11 +83,20 @@ constexpr size_t chunk_lds_floats() {
   constexpr size_t rows = (size_t)QC * (16 * NDT + 4);
   return rows * (1 + (FINAL ? 1 : 0) + (MODE == MODE_CHANNEL ? 1 : 0)) + (size_t)QC * XLD +
          (FINAL ? (size_t)QC * PLD : 0) + (MODE == MODE_CHANNEL && FINAL ? (size_t)QC * 20 : 0) +
-         (MODE == MODE_CHANNEL ? 2 * 16 * NDT : 0) + 5 * QC;
+         (MODE == MODE_CHANNEL ? 2 * 16 * NDT : 2 * 5 * QC);
+}
+
+// waves a SIMD that the registers are shared out for
+constexpr int chunk_waves(int ndt, bool final) {
+#ifdef CHUNK_WAVES
+  return ndt > 8 && final ? 1 : CHUNK_WAVES;
+#else
+  return ndt > 8 && final ? 1 : 2;
+#endif
 }
 
 template <int NDT, int MODE, bool FINAL>
-__global__ void __launch_bounds__(256) linear_chunk_kernel(LinArgs A, int vec) {
+__global__ void __launch_bounds__(256, chunk_waves(NDT, FINAL)) linear_chunk_kernel(LinArgs A, int vec) {
   constexpr int DP = 16 * NDT;              // key channels, padded
   constexpr int LD = DP + 4;                // row stride of q, k and the decays in LDS
   constexpr int NQ = DP / 4;                // float4 of a row
@@ -100,10 +109,12 @@ __global__ void __launch_bounds__(256) linear_chunk_kernel(LinArgs A, int vec) {
   float* Pd = Ps + (FINAL ? QC * PLD : 0);                      // channel, FINAL: [QC][20], second halves of the
                                                                 // sums over d of the two diagonal tiles
   float* tot = Pd + (MODE == MODE_CHANNEL && FINAL ? QC * 20 : 0);   // channel: [2][DP]
-  double* cum = reinterpret_cast<double*>(tot + (MODE == MODE_CHANNEL ? 2 * DP : 0));     // scalar: [QC]
-  float* dts = reinterpret_cast<float*>(cum + QC);              // scalar: [QC] step sizes
-  float* es = dts + QC;                                         // scalar: [QC] decays from the chunk's start
-  float* ws = es + QC;                                          // scalar: [QC] dt x the decay to its end
+  // scalar, twice (this chunk's and the next one's): [QC] each of the sums of the log decays from the
+  // chunk's start, the step sizes, the decays from the chunk's start, the step sizes x decays to its end
+  double* cums = reinterpret_cast<double*>(tot);
+  float* dtss = reinterpret_cast<float*>(cums + 2 * QC);
+  float* ess = dtss + 2 * QC;
+  float* wss = ess + 2 * QC;
 
   const int tid = threadIdx.x, lane = tid & 63, ln = lane & 15, lg = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -139,64 +150,97 @@ __global__ void __launch_bounds__(256) linear_chunk_kernel(LinArgs A, int vec) {
     skip = A.skip[h];
   }
 
-  auto load_rows = [&](float* dst, const float* src, long ld, int col0, float f, int t0, int steps) {
-    for (int i = tid; i < QC * NQ; i += 256) {
-      const int r = i / NQ, d = (i - r * NQ) * 4;
-      f32x4_t x = {0.f, 0.f, 0.f, 0.f};
-      if (r < steps && d < D) {
-        const float* p = src + (size_t)(row0 + t0 + r) * ld + col0 + d;
-        if (vec) {
-          x = *reinterpret_cast<const f32x4_t*>(p);
-        } else {
+  // The rows of the next chunk are on their way from global memory into registers while the current
+  // one is worked on from LDS: a thread holds NR float4 of k (and of q and the decays) and two of v.
+  constexpr int NR = (QC * NQ + 255) / 256;
+  f32x4_t fk[NR], fq[FINAL ? NR : 1], fa[MODE == MODE_CHANNEL ? NR : 1], fv[2];
+  float fdt = 0.f;                          // scalar: a token's raw step size
+  auto fetch4 = [&](const float* p, int col, int most) {
+    f32x4_t x = {0.f, 0.f, 0.f, 0.f};
+    if (vec) {
+      x = *reinterpret_cast<const f32x4_t*>(p + col);
+    } else {
 #pragma unroll
-          for (int j = 0; j < 4; ++j) x[j] = d + j < D ? p[j] : 0.f;
-        }
-        x *= f;
-      }
-      *reinterpret_cast<f32x4_t*>(dst + r * LD + d) = x;
+      for (int j = 0; j < 4; ++j) x[j] = col + j < most ? p[col + j] : 0.f;
+    }
+    return x;
+  };
+  auto fetch = [&](int t0) {
+    const int steps = min(QC, t_end - t0);
+#pragma unroll
+    for (int n = 0; n < NR; ++n) {
+      const int i = tid + 256 * n, r = i / NQ, d = (i - r * NQ) * 4;
+      const f32x4_t zero = {0.f, 0.f, 0.f, 0.f};
+      const size_t row = (size_t)(row0 + t0 + r);
+      const bool in = r < steps && d < D;
+      fk[n] = in ? fetch4(A.k + row * A.ldk + g * D, d, D) : zero;
+      if (FINAL) fq[n] = in ? fetch4(A.q + row * A.ldq + g * D, d, D) : zero;
+      if (MODE == MODE_CHANNEL) fa[n] = in ? fetch4(A.decay + row * A.lda + h * D, d, D) : zero;
+    }
+#pragma unroll
+    for (int n = 0; n < 2; ++n) {
+      const int i = tid + 256 * n, r = i >> 4, x0 = (i & 15) * 4;
+      fv[n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      if (r < steps && c0 + x0 < Dv) fv[n] = fetch4(A.v + (size_t)(row0 + t0 + r) * A.ldv + (size_t)h * Dv, c0 + x0, Dv);
+    }
+  };
+  auto put = [&]() {
+#pragma unroll
+    for (int n = 0; n < NR; ++n) {
+      const int i = tid + 256 * n, r = i / NQ, d = (i - r * NQ) * 4;
+      if (QC * NQ % 256 != 0 && i >= QC * NQ) break;
+      *reinterpret_cast<f32x4_t*>(Ks + r * LD + d) = fk[n];
+      if (FINAL) *reinterpret_cast<f32x4_t*>(Qs + r * LD + d) = fq[n] * A.qscale;
+      // (rows past the end: zeros; their decay is taken as one where it matters, below)
+      if (MODE == MODE_CHANNEL) *reinterpret_cast<f32x4_t*>(As + r * LD + d) = fa[n];
+    }
+#pragma unroll
+    for (int n = 0; n < 2; ++n) {
+      const int i = tid + 256 * n;
+      *reinterpret_cast<f32x4_t*>(Xs + (i >> 4) * XLD + (i & 15) * 4) = fv[n];
     }
   };
 
-  for (int t0 = t_begin; t0 < t_end; t0 += QC) {
+  // Scalar: the last wave, a lane a token, works the next chunk's scalars out while the others make P;
+  // the raw step sizes are read a chunk earlier still.
+  const bool scalar_wave = MODE == MODE_SCALAR && wave == 3;
+  auto fetch_dt = [&](int t0) {
+    if (scalar_wave && t0 + lane < t_end && lane < QC) fdt = A.dt[(size_t)(row0 + t0 + lane) * A.ldt + h];
+  };
+  auto scalars = [&](int t0, int buf) {
+    const float step = t0 + lane < t_end && lane < QC ? softplus_f(fdt + dt_bias) : 0.f;
+    double s = (double)(neg_A * step);
+#pragma unroll
+    for (int o = 1; o < QC; o <<= 1) {
+      const double up = __shfl_up(s, o, 64);
+      if (lane >= o) s += up;
+    }
+    const double all = __shfl(s, QC - 1, 64);
+    if (lane < QC) {
+      cums[buf * QC + lane] = s;
+      dtss[buf * QC + lane] = step;
+      ess[buf * QC + lane] = expf((float)s);
+      wss[buf * QC + lane] = step * expf((float)(all - s));
+    }
+  };
+
+  fetch(t_begin);
+  fetch_dt(t_begin);
+  if (scalar_wave) scalars(t_begin, 0);
+  fetch_dt(t_begin + QC);
+  int buf = 0;
+  for (int t0 = t_begin; t0 < t_end; t0 += QC, buf ^= 1) {
     const int steps = min(QC, t_end - t0);
+    const double* cum = cums + buf * QC;
+    const float *dts = dtss + buf * QC, *es = ess + buf * QC, *ws = wss + buf * QC;
     __syncthreads();                        // the chunk before is done with
-    load_rows(Ks, A.k, A.ldk, g * D, 1.f, t0, steps);
-    if (FINAL) load_rows(Qs, A.q, A.ldq, g * D, A.qscale, t0, steps);
-    // (rows past the end keep what is there: their decay is taken as one, below)
-    if (MODE == MODE_CHANNEL) load_rows(As, A.decay, A.lda, h * D, 1.f, t0, steps);
-    for (int i = tid; i < QC * 16; i += 256) {
-      const int r = i >> 4, x0 = (i & 15) * 4;
-      f32x4_t x = {0.f, 0.f, 0.f, 0.f};
-      if (r < steps && c0 + x0 < Dv) {
-        const float* p = A.v + (size_t)(row0 + t0 + r) * A.ldv + (size_t)h * Dv + c0 + x0;
-        if (vec) {
-          x = *reinterpret_cast<const f32x4_t*>(p);
-        } else {
-#pragma unroll
-          for (int j = 0; j < 4; ++j) x[j] = c0 + x0 + j < Dv ? p[j] : 0.f;
-        }
-      }
-      *reinterpret_cast<f32x4_t*>(Xs + r * XLD + x0) = x;
-    }
-    if (MODE == MODE_SCALAR && tid < 64) {  // one wave; its upper half repeats the last token
-      const int r = min(tid, QC - 1);
-      float step = 0.f;
-      if (r < steps) step = softplus_f(A.dt[(size_t)(row0 + t0 + r) * A.ldt + h] + dt_bias);
-      double s = tid < QC ? (double)(neg_A * step) : 0.0;
-#pragma unroll
-      for (int o = 1; o < QC; o <<= 1) {
-        const double up = __shfl_up(s, o, 64);
-        if (tid >= o) s += up;
-      }
-      const double all = __shfl(s, QC - 1, 64);
-      if (tid < QC) {
-        cum[tid] = s;
-        dts[tid] = step;
-        es[tid] = expf((float)s);
-        ws[tid] = step * expf((float)(all - s));
-      }
-    }
+    put();
     __syncthreads();
+    if (t0 + QC < t_end) fetch(t0 + QC);
+    if (scalar_wave) {
+      if (t0 + QC < t_end) scalars(t0 + QC, buf ^ 1);
+      fetch_dt(t0 + 2 * QC);
+    }
 
     if (MODE == MODE_CHANNEL) {
       // The two diagonal tiles: lane (t, lg) walks s from t down, w = q_t times the decays of
@@ -280,17 +324,21 @@ __global__ void __launch_bounds__(256) linear_chunk_kernel(LinArgs A, int vec) {
       }
       f32x4_t O[2];
       if (wave_live) {
+        O[0] = O[1] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int tt = 0; tt < 2; ++tt) {
-          O[tt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        for (int dt = 0; dt < NDT; ++dt) {
+          const f32x4_t q0 = *reinterpret_cast<const f32x4_t*>(Qs + ln * LD + 16 * dt + 4 * lg);
+          f32x4_t q1 = *reinterpret_cast<const f32x4_t*>(Qs + (16 + ln) * LD + 16 * dt + 4 * lg);
+          if (MODE == MODE_CHANNEL) q1 *= *reinterpret_cast<const f32x4_t*>(tot + 16 * dt + 4 * lg);
 #pragma unroll
-          for (int dt = 0; dt < NDT; ++dt) {
-            f32x4_t qa = *reinterpret_cast<const f32x4_t*>(Qs + (16 * tt + ln) * LD + 16 * dt + 4 * lg);
-            if (MODE == MODE_CHANNEL && tt == 1) qa *= *reinterpret_cast<const f32x4_t*>(tot + 16 * dt + 4 * lg);
-#pragma unroll
-            for (int m = 0; m < 4; ++m) O[tt] = __builtin_amdgcn_mfma_f32_16x16x4f32(qa[m], S[dt][m], O[tt], 0, 0, 0);
+          for (int m = 0; m < 4; ++m) {
+            O[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(q0[m], S[dt][m], O[0], 0, 0, 0);
+            O[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(q1[m], S[dt][m], O[1], 0, 0, 0);
           }
-          if (MODE == MODE_SCALAR) O[tt] *= *reinterpret_cast<const f32x4_t*>(es + 16 * tt + 4 * lg);
+        }
+        if (MODE == MODE_SCALAR) {
+          O[0] *= *reinterpret_cast<const f32x4_t*>(es + 4 * lg);
+          O[1] *= *reinterpret_cast<const f32x4_t*>(es + 16 + 4 * lg);
         }
       }
       __syncthreads();                      // P is there
@@ -336,13 +384,15 @@ __global__ void __launch_bounds__(256) linear_chunk_kernel(LinArgs A, int vec) {
           x[m] = Xs[s * XLD + 16 * wave + ln];
           if (MODE == MODE_SCALAR) x[m] *= ws[s];
         }
+        float f[NDT];                       // channel: the second block's decays on top of the first's
 #pragma unroll
-        for (int dt = 0; dt < NDT; ++dt) {
-          const float f = MODE == MODE_CHANNEL && ts == 0 ? tot[DP + 16 * dt + ln] : 1.f;
+        for (int dt = 0; dt < NDT; ++dt) f[dt] = MODE == MODE_CHANNEL && ts == 0 ? tot[DP + 16 * dt + ln] : 1.f;
 #pragma unroll
-          for (int m = 0; m < 4; ++m) {
+        for (int m = 0; m < 4; ++m) {
+#pragma unroll
+          for (int dt = 0; dt < NDT; ++dt) {
             float ka = Ks[(16 * ts + 4 * lg + m) * LD + 16 * dt + ln];
-            if (MODE == MODE_CHANNEL && ts == 0) ka *= f;
+            if (MODE == MODE_CHANNEL && ts == 0) ka *= f[dt];
             S[dt] = __builtin_amdgcn_mfma_f32_16x16x4f32(ka, x[m], S[dt], 0, 0, 0);
           }
         }
@@ -547,27 +597,30 @@ struct DecodeArgs {
   int H, heads_per_qk, D, DS, Dv;
 };
 
-template <int J, int MODE>
+// NB: blocks of 16 columns a workgroup takes (what is in front of the recurrence is then done less often)
+template <int J, int NB, int MODE>
 __global__ void __launch_bounds__(256) linear_decode_kernel(DecodeArgs A) {
-  __shared__ __attribute__((aligned(16))) float ks[64 * J], qs[64 * J], as[MODE == MODE_CHANNEL ? 64 * J : 4], xs[16];
+  __shared__ __attribute__((aligned(16))) float ks[64 * J], qs[64 * J], as[MODE == MODE_CHANNEL ? 64 * J : 4], xs[16 * NB];
   const int tid = threadIdx.x, cg = tid >> 4, l = tid & 15;
   const int h = blockIdx.y, seq = blockIdx.z, g = h / A.heads_per_qk;
   const int row = A.q_start[seq];
   if (A.q_start[seq + 1] <= row) return;
   const int D = A.D, DS = A.DS, Dv = A.Dv;
-  const int c = blockIdx.x * 16 + cg;
-  const bool live = c < Dv;
+  const int c0 = blockIdx.x * 16 * NB;
   float* slot = A.state + (size_t)A.state_slots[seq] * A.slot_stride;
-  float* st = slot + ((size_t)h * Dv + c) * DS;
-  f32x4_t S[J];
+  auto column = [&](int b) { return slot + ((size_t)h * Dv + c0 + 16 * b + cg) * DS; };
+  f32x4_t S[NB][J];
 #pragma unroll
-  for (int j = 0; j < J; ++j) {
-    const int d = 4 * (l + 16 * j);
-    S[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    if (live && d < DS) S[j] = __builtin_nontemporal_load(reinterpret_cast<const f32x4_t*>(st + d));
-  }
+  for (int b = 0; b < NB; ++b)
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+      const int d = 4 * (l + 16 * j);
+      S[b][j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      if (c0 + 16 * b + cg < Dv && d < DS)
+        S[b][j] = __builtin_nontemporal_load(reinterpret_cast<const f32x4_t*>(column(b) + d));
+    }
   const float* p = A.p + (size_t)row * A.ldp;
-  // what the columns of the projection hold for this workgroup: k and q of the head (group), 16 values
+  // what the columns of the projection hold for this workgroup: k and q of the head (group), its values
   auto value = [&](int col) {
     float x = p[col];
     if (MODE == MODE_SCALAR) {
@@ -581,14 +634,14 @@ __global__ void __launch_bounds__(256) linear_decode_kernel(DecodeArgs A) {
     return x;
   };
   const int DP = 64 * J;
-  for (int i = tid; i < 2 * DP + 16; i += 256) {
+  for (int i = tid; i < 2 * DP + 16 * NB; i += 256) {
     if (i < DP) {
       ks[i] = i < D ? value(A.k_off + g * D + i) : 0.f;
     } else if (i < 2 * DP) {
       const int d = i - DP;
       qs[d] = d < D ? value(A.q_off + g * D + d) * A.qscale : 0.f;
     } else {
-      const int cc = blockIdx.x * 16 + i - 2 * DP;
+      const int cc = c0 + i - 2 * DP;
       xs[i - 2 * DP] = cc < Dv ? value(A.v_off + h * Dv + cc) : 0.f;
     }
   }
@@ -611,21 +664,26 @@ __global__ void __launch_bounds__(256) linear_decode_kernel(DecodeArgs A) {
     }
   }
   __syncthreads();
-  const float x = xs[cg], v = x * step;
-  float o = 0.f;
+  const float skip = MODE == MODE_SCALAR ? A.skip[h] : 0.f;
 #pragma unroll
-  for (int j = 0; j < J; ++j) {
-    const int d = 4 * (l + 16 * j);
-    const f32x4_t k4 = *reinterpret_cast<const f32x4_t*>(ks + d), q4 = *reinterpret_cast<const f32x4_t*>(qs + d);
-    if (MODE == MODE_CHANNEL) S[j] *= *reinterpret_cast<const f32x4_t*>(as + d);
-    else S[j] *= decay;
-    S[j] += k4 * v;
-    o += (S[j][0] * q4[0] + S[j][1] * q4[1]) + (S[j][2] * q4[2] + S[j][3] * q4[3]);
-    if (live && d < DS) __builtin_nontemporal_store(S[j], reinterpret_cast<f32x4_t*>(st + d));
+  for (int b = 0; b < NB; ++b) {
+    const bool live = c0 + 16 * b + cg < Dv;
+    const float x = xs[16 * b + cg], v = x * step;
+    float o = 0.f;
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+      const int d = 4 * (l + 16 * j);
+      const f32x4_t k4 = *reinterpret_cast<const f32x4_t*>(ks + d), q4 = *reinterpret_cast<const f32x4_t*>(qs + d);
+      f32x4_t s = S[b][j];
+      if (MODE == MODE_CHANNEL) s *= *reinterpret_cast<const f32x4_t*>(as + d);
+      else s *= decay;
+      s += k4 * v;
+      o += (s[0] * q4[0] + s[1] * q4[1]) + (s[2] * q4[2] + s[3] * q4[3]);
+      if (live && d < DS) __builtin_nontemporal_store(s, reinterpret_cast<f32x4_t*>(column(b) + d));
+    }
+    o = row16_sum(o);
+    if (live && l == 0) A.out[((size_t)row * A.H + h) * Dv + c0 + 16 * b + cg] = fmaf(skip, x, o);
   }
-  o = row16_sum(o);
-  if (MODE == MODE_SCALAR) o = fmaf(A.skip[h], x, o);
-  if (live && l == 0) A.out[((size_t)row * A.H + h) * Dv + c] = o;
 }
 
 template <int MODE>
@@ -633,14 +691,25 @@ static int launch_decode(const DecodeArgs& A, int n_seqs, hipStream_t st) {
   if (A.D <= 0 || A.D > 256 || A.Dv <= 0 || A.H <= 0 || A.H > 65535 || n_seqs > 65535 || A.heads_per_qk <= 0 ||
       A.slot_stride < (long)A.H * A.Dv * A.DS || A.slot_stride % 4 || ((uintptr_t)A.state & 15))
     return PTL_ERR_ARG;
-  const dim3 grid((A.Dv + 15) / 16, A.H, n_seqs);
-  switch ((A.DS + 63) / 64) {
-    case 1: linear_decode_kernel<1, MODE><<<grid, 256, 0, st>>>(A); break;
-    case 2: linear_decode_kernel<2, MODE><<<grid, 256, 0, st>>>(A); break;
-    case 3: linear_decode_kernel<3, MODE><<<grid, 256, 0, st>>>(A); break;
-    default: linear_decode_kernel<4, MODE><<<grid, 256, 0, st>>>(A); break;
+  // as many columns a workgroup as leave about two workgroups a compute unit (of 256)
+  const int blocks = (A.Dv + 15) / 16;
+  const long all = (long)blocks * A.H * n_seqs;
+  const int nb = blocks >= 4 && all >= 4 * 512 ? 4 : (blocks >= 2 && all >= 2 * 512 ? 2 : 1);
+  const dim3 grid((blocks + nb - 1) / nb, A.H, n_seqs);
+#define GO(J)                                                                       \
+  {                                                                                 \
+    if (nb == 4) linear_decode_kernel<J, 4, MODE><<<grid, 256, 0, st>>>(A);         \
+    else if (nb == 2) linear_decode_kernel<J, 2, MODE><<<grid, 256, 0, st>>>(A);    \
+    else linear_decode_kernel<J, 1, MODE><<<grid, 256, 0, st>>>(A);                 \
+    return ptl_launch_status();                                                     \
   }
-  return ptl_launch_status();
+  switch ((A.DS + 63) / 64) {
+    case 1: GO(1)
+    case 2: GO(2)
+    case 3: GO(3)
+    default: GO(4)
+  }
+#undef GO
 }
 
 // Sequences 0 .. n_seqs - 1, one token each, scalar form behind a short convolution. p float32 [T,

@@ -17,7 +17,8 @@
 //   constant, times act(gate) with the gate read from a float32 matrix at given columns
 //   (sigmoid, SiLU, or none). The result [T, H * Dv] is in the engine's type.
 //
-// ptl_gate_group_norm: one workgroup a (token, group of columns). y float32 [T, n] times silu(gate),
+// ptl_gate_group_norm: one workgroup a (token, group of columns), or one wave where a group's columns
+//   fit its registers. y float32 [T, n] times silu(gate),
 //   then every one of the equal groups of neighbouring columns divided by its own root mean square,
 //   times a weight [n]; the result is in the engine's type. For the leading rows of a step that are
 //   sequences of one token it also advances the inputs that a short convolution keeps in the state
@@ -266,6 +267,73 @@ gate_group_norm_kernel(TO* __restrict__ out, const float* __restrict__ y, const 
   }
 }
 
+// A wave a (token, group): the group's columns as NV float4 a lane, nothing through LDS.
+template <int NV, typename TO>
+__global__ void __launch_bounds__(256)
+gate_group_norm_wave_kernel(TO* __restrict__ out, const float* __restrict__ y, const float* __restrict__ z, long ldz,
+                            const float* __restrict__ w, int n, int groups, float eps, long items) {
+  const long item = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (item >= items) return;
+  const int lane = threadIdx.x & 63;
+  const long t = item / groups;
+  const int size = n / groups, c0 = (int)(item - t * groups) * size;
+  const float* yr = y + (size_t)t * n + c0;
+  const float* zr = z + (size_t)t * ldz + c0;
+  float4 a[NV], b[NV];
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int c = 4 * (lane + 64 * k);
+    a[k] = b[k] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (c < size) {
+      a[k] = *reinterpret_cast<const float4*>(yr + c);
+      b[k] = *reinterpret_cast<const float4*>(zr + c);
+    }
+  }
+  auto gated = [](float v, float g) { return v * (g / (1.0f + expf(-g))); };
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    a[k] = make_float4(gated(a[k].x, b[k].x), gated(a[k].y, b[k].y), gated(a[k].z, b[k].z), gated(a[k].w, b[k].w));
+    ss = fmaf(a[k].x, a[k].x, fmaf(a[k].y, a[k].y, fmaf(a[k].z, a[k].z, fmaf(a[k].w, a[k].w, ss))));
+  }
+  const float r = 1.0f / sqrtf(wave_sum(ss) / (float)size + eps);
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int c = 4 * (lane + 64 * k);
+    if (c >= size) continue;
+    const float4 ww = *reinterpret_cast<const float4*>(w + c0 + c);
+    const float v[4] = {a[k].x * r * ww.x, a[k].y * r * ww.y, a[k].z * r * ww.z, a[k].w * r * ww.w};
+    TO* dst = out + (size_t)t * n + c0 + c;
+    if (sizeof(TO) == 2) {
+      union { uint2 u; bf16_t e[4]; } o;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) o.e[j] = float_to_bf16(v[j]);
+      *reinterpret_cast<uint2*>(dst) = o.u;
+    } else {
+      *reinterpret_cast<float4*>(dst) = make_float4(v[0], v[1], v[2], v[3]);
+    }
+  }
+}
+
+template <typename TO>
+static bool gate_group_norm_waves(void* out, const float* y, const float* z, long ldz, const float* w, int groups,
+                                  float eps, int T_, int n, hipStream_t st) {
+  const int size = n / groups;
+  const long items = (long)T_ * groups;
+  if (size % 4 || ldz % 4 || size > 2048 || (((uintptr_t)y | (uintptr_t)z | (uintptr_t)w | (uintptr_t)out) & 15) ||
+      items > 4L * 0x7fffffff)
+    return false;
+  const int blocks = (int)((items + 3) / 4);
+#define GO(NV)                                                                                                       \
+  if (size <= 256 * NV) {                                                                                            \
+    gate_group_norm_wave_kernel<NV, TO><<<blocks, 256, 0, st>>>((TO*)out, y, z, ldz, w, n, groups, eps, items);      \
+    return true;                                                                                                     \
+  }
+  GO(1) GO(2) GO(4) GO(8)
+#undef GO
+  return false;
+}
+
 // y float32 [T, n] dense, z float32 [T, ldz] (its first n columns), w float32 [n], out [T, n] dense.
 // tail_rows > 0 and taps > 1: rows 0 .. tail_rows - 1 also advance the kept inputs of their slots.
 extern "C" int ptl_gate_group_norm(void* out, const float* y, const float* z, long ldz, const float* w, int groups,
@@ -277,6 +345,13 @@ extern "C" int ptl_gate_group_norm(void* out, const float* y, const float* z, lo
       tail_rows > T_ || (tail_rows > 0 && taps > 1 && (!state || !x || !state_slots || C <= 0)))
     return PTL_ERR_ARG;
   const TailArgs tail{state, slot_stride, tail_off, x, ldx, state_slots, taps > 1 ? tail_rows : 0, C, taps};
+  // many rows, none of which advances a tail: a wave a (token, group)
+  if (tail.n_rows == 0) {
+    bool done = false;
+    if (dtype == PTL_DTYPE_F32) done = gate_group_norm_waves<float>(out, y, z, ldz, w, groups, eps, T_, n, st);
+    else if (dtype == PTL_DTYPE_BF16) done = gate_group_norm_waves<bf16_t>(out, y, z, ldz, w, groups, eps, T_, n, st);
+    if (done) return ptl_launch_status();
+  }
   const int size = n / groups;
   const int threads = size >= 256 ? 256 : (size + 63) / 64 * 64;
   const size_t lds = (size_t)size * sizeof(float);

@@ -1996,7 +1996,7 @@ def selective_scan(xc: torch.Tensor, p: torch.Tensor, z_off: int, r: torch.Tenso
 # ---------------------------------------------------------------------------
 # Linear recurrences with a decay a head or a key channel (csrc/linear_scan.hip)
 LINEAR_CHUNK = 32                 # tokens whose products run on the matrix cores together
-LINEAR_WORKGROUPS_PER_CU = 3      # workgroups of the final pass that fill the chip
+LINEAR_WORKGROUPS_PER_CU = 2      # workgroups of the final pass that fill the chip
 LINEAR_MAX_KEYS = 256
 
 
@@ -2010,7 +2010,7 @@ def linear_segment(n_seqs: int, max_q_len: int, H: int, Dv: int, compute_units_:
     as long as LINEAR_WORKGROUPS_PER_CU workgroups a compute unit allow (a workgroup takes 64 columns
     of a head in a segment). max_q_len itself when one segment fills the chip."""
     blocks = max(1, n_seqs) * H * -(-Dv // 64)
-    want = -(-LINEAR_WORKGROUPS_PER_CU * compute_units_ // blocks)
+    want = LINEAR_WORKGROUPS_PER_CU * compute_units_ // blocks
     if want <= 1 or max_q_len <= 4 * LINEAR_CHUNK:
         return max(1, max_q_len)
     rows = -(-max_q_len // want)
