@@ -388,7 +388,8 @@ def engine_rates(cfg, dtype, S, batch, steps, warmup):
     from pytriton_llama_amd.config import EngineConfig
     from pytriton_llama_amd.engine import Engine, SamplingParams
     page = 16
-    room = S + steps + warmup + 16
+    # requests whose prompt is in first go on decoding while the others' prompts are computed
+    room = S + steps + warmup + batch * -(-S // max(S, 2048)) + 16
     ec = EngineConfig(dtype=dtype, page_size=page, num_pages=-(-room // page) * batch + 8, max_num_seqs=batch,
                       max_num_batched_tokens=max(S, 2048), max_model_len=room, seed=0)
     engine = Engine(cfg, ec, random_seed=0)
@@ -406,7 +407,7 @@ def engine_rates(cfg, dtype, S, batch, steps, warmup):
         times.append(time.perf_counter() - t)
         engine.requests.pop(rid, None)
     pre = min(times[1:])
-    ids = [engine.add_request(prompt(), SamplingParams(temperature=0.0, max_new_tokens=steps + warmup,
+    ids = [engine.add_request(prompt(), SamplingParams(temperature=0.0, max_new_tokens=room - S - 8,
                                                        ignore_eos=True)) for _ in range(batch)]
     while any(engine.requests[i].num_computed < S for i in ids):
         engine.step()

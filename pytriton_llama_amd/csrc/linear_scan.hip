@@ -51,9 +51,13 @@ __device__ __forceinline__ float row16_sum(float v) {
 }
 __device__ __forceinline__ float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
 __device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
-// sigmoid(z)^p
+// sigmoid(z)^p = 2^(-p log2(1 + e^-z)), with log2(1 + e^-z) = log2(1 + e^-|z|) + max(-z, 0) log2 e: the
+// logarithm's argument lies in [1, 2], where the sum's rounding moves the logarithm by no more than
+// the result's own last place (p up to about 1)
 __device__ __forceinline__ float sigmoid_power(float z, float p) {
-  return expf((fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * p);
+  const float zl = z * 1.4426950408889634f;
+  const float l = __builtin_amdgcn_logf(1.0f + __builtin_amdgcn_exp2f(-fabsf(zl))) + fmaxf(-zl, 0.f);
+  return __builtin_amdgcn_exp2f(-p * l);
 }
 
 struct LinArgs {
@@ -86,17 +90,11 @@ constexpr size_t chunk_lds_floats() {
          (MODE == MODE_CHANNEL ? 2 * 16 * NDT : 2 * 5 * QC);
 }
 
-// waves a SIMD that the registers are shared out for
-constexpr int chunk_waves(int ndt, bool final) {
-#ifdef CHUNK_WAVES
-  return ndt > 8 && final ? 1 : CHUNK_WAVES;
-#else
-  return ndt > 8 && final ? 1 : 2;
-#endif
-}
+// workgroups a compute unit that the registers are shared out for (one where S takes many of them)
+constexpr int chunk_workgroups(int ndt, bool final) { return ndt > 8 && final ? 1 : 2; }
 
 template <int NDT, int MODE, bool FINAL>
-__global__ void __launch_bounds__(256, chunk_waves(NDT, FINAL)) linear_chunk_kernel(LinArgs A, int vec) {
+__global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chunk_kernel(LinArgs A, int vec) {
   constexpr int DP = 16 * NDT;              // key channels, padded
   constexpr int LD = DP + 4;                // row stride of q, k and the decays in LDS
   constexpr int NQ = DP / 4;                // float4 of a row
@@ -534,33 +532,43 @@ extern "C" int ptl_linear_scan(int mode, float* out, const float* q, long ldq, c
 }
 
 // ---- the low-rank decays of all rows ---------------------------------------------------------------
-// grid (blocks of 256 channels, blocks of ROWS rows): a thread keeps its channel's row of W2 in
-// registers (up to 32 entries; a longer one is read again for every row), the rows of r go through LDS
+// grid (blocks of 256 channels, blocks of DECAY_ROWS rows): a thread keeps its channel's row of W2 in
+// registers (up to 32 entries; a longer one is read again for every row), the rows of r go through LDS,
+// four entries a read
 #define DECAY_ROWS 8
 template <int RM>
 __global__ void __launch_bounds__(256)
 lowrank_decay_kernel(float* __restrict__ out, const float* __restrict__ r, long ldr, const float* __restrict__ w,
-                     const float* __restrict__ b, float inv_tau, int T, int C, int R) {
-  extern __shared__ float rs[];             // [DECAY_ROWS][R]
+                     const float* __restrict__ b, float inv_tau, int T, int C, int R, int RP) {
+  extern __shared__ __attribute__((aligned(16))) float rs[];       // [DECAY_ROWS][RP], zeros from R on
   const int t0 = blockIdx.y * DECAY_ROWS, rows = min(DECAY_ROWS, T - t0);
-  for (int i = threadIdx.x; i < rows * R; i += 256) rs[i] = r[(size_t)(t0 + i / R) * ldr + i % R];
-  __syncthreads();
   const int c = blockIdx.x * 256 + threadIdx.x;
-  if (c >= C) return;
-  const float* wr = w + (size_t)c * R;
-  float wv[RM > 0 ? RM : 1];
+  const float* wr = w + (size_t)min(c, C - 1) * R;
+  float wv[RM > 0 ? RM : 4];
   if (RM > 0) {
 #pragma unroll
     for (int j = 0; j < RM; ++j) wv[j] = j < R ? wr[j] : 0.f;
   }
-  const float bias = b[c];
+  const float bias = b[min(c, C - 1)];
+  for (int i = threadIdx.x; i < rows * RP; i += 256) {
+    const int t = i / RP, j = i - t * RP;
+    rs[i] = j < R ? r[(size_t)(t0 + t) * ldr + j] : 0.f;
+  }
+  __syncthreads();
+  if (c >= C) return;
   for (int t = 0; t < rows; ++t) {
+    const float* rr = rs + t * RP;
     float z = bias;
     if (RM > 0) {
 #pragma unroll
-      for (int j = 0; j < RM; ++j) z = fmaf(wv[j], rs[t * R + min(j, R - 1)], z);
+      for (int j = 0; j < RM; j += 4) {
+        if (j >= RP) break;
+        const f32x4_t x = *reinterpret_cast<const f32x4_t*>(rr + j);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) z = fmaf(wv[j + i], x[i], z);
+      }
     } else {
-      for (int j = 0; j < R; ++j) z = fmaf(wr[j], rs[t * R + j], z);
+      for (int j = 0; j < R; ++j) z = fmaf(wr[j], rr[j], z);
     }
     out[(size_t)(t0 + t) * C + c] = sigmoid_power(z, inv_tau);
   }
@@ -569,12 +577,13 @@ lowrank_decay_kernel(float* __restrict__ out, const float* __restrict__ r, long 
 extern "C" int ptl_lowrank_decay(float* out, const float* r, long ldr, const float* w, const float* b,
                                  float inv_tau, int T_, int C, int R, hipStream_t st) {
   if (T_ <= 0) return PTL_OK;
-  const size_t lds = (size_t)DECAY_ROWS * R * sizeof(float);
+  const int RP = (R + 3) / 4 * 4;
+  const size_t lds = (size_t)DECAY_ROWS * RP * sizeof(float);
   if (C <= 0 || R <= 0 || lds > 48 * 1024 || (T_ + DECAY_ROWS - 1) / DECAY_ROWS > 65535) return PTL_ERR_ARG;
   const dim3 grid((C + 255) / 256, (T_ + DECAY_ROWS - 1) / DECAY_ROWS);
-  if (R <= 16) lowrank_decay_kernel<16><<<grid, 256, lds, st>>>(out, r, ldr, w, b, inv_tau, T_, C, R);
-  else if (R <= 32) lowrank_decay_kernel<32><<<grid, 256, lds, st>>>(out, r, ldr, w, b, inv_tau, T_, C, R);
-  else lowrank_decay_kernel<0><<<grid, 256, lds, st>>>(out, r, ldr, w, b, inv_tau, T_, C, R);
+  if (R <= 16) lowrank_decay_kernel<16><<<grid, 256, lds, st>>>(out, r, ldr, w, b, inv_tau, T_, C, R, RP);
+  else if (R <= 32) lowrank_decay_kernel<32><<<grid, 256, lds, st>>>(out, r, ldr, w, b, inv_tau, T_, C, R, RP);
+  else lowrank_decay_kernel<0><<<grid, 256, lds, st>>>(out, r, ldr, w, b, inv_tau, T_, C, R, RP);
   return ptl_launch_status();
 }
 

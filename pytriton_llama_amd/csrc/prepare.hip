@@ -236,6 +236,22 @@ struct TailArgs {
   int n_rows, C, taps;
 };
 
+// Channels part * per .. of row t's kept inputs, the lanes of ``width`` threads side by side.
+__device__ __forceinline__ void advance_tail(const TailArgs& a, int t, int part, int parts, int lane, int width) {
+  float* kept = a.state + (size_t)a.state_slots[t] * a.slot_stride + a.tail_off;
+  const int per = (a.C + parts - 1) / parts;
+  for (int c = part * per + lane; c < min(a.C, (part + 1) * per); c += width) {
+    float v[4];                              // the first inputs read before any is written
+    const float x = a.x[(size_t)t * a.ldx + c];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = i + 2 < a.taps ? kept[(size_t)(i + 1) * a.C + c] : x;
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (i + 2 <= a.taps) kept[(size_t)i * a.C + c] = v[i];
+    for (int i = 4; i + 2 <= a.taps; ++i) kept[(size_t)i * a.C + c] = i + 2 < a.taps ? kept[(size_t)(i + 1) * a.C + c] : x;
+  }
+}
+
 template <typename TO>
 __global__ void __launch_bounds__(256)
 gate_group_norm_kernel(TO* __restrict__ out, const float* __restrict__ y, const float* __restrict__ z, long ldz,
@@ -257,26 +273,20 @@ gate_group_norm_kernel(TO* __restrict__ out, const float* __restrict__ y, const 
   const float r = 1.0f / sqrtf(ss / (float)size + eps);
   TO* dst = out + (size_t)t * n + c0;
   for (int c = tid; c < size; c += nt) dst[c] = from_float<TO>(us[c] * r * w[c0 + c]);
-  if (t < tail.n_rows) {
-    float* kept = tail.state + (size_t)tail.state_slots[t] * tail.slot_stride + tail.tail_off;
-    const int per = (tail.C + groups - 1) / groups;
-    for (int c = part * per + tid; c < min(tail.C, (part + 1) * per); c += nt) {
-      for (int i = 0; i + 2 < tail.taps; ++i) kept[(size_t)i * tail.C + c] = kept[(size_t)(i + 1) * tail.C + c];
-      kept[(size_t)(tail.taps - 2) * tail.C + c] = tail.x[(size_t)t * tail.ldx + c];
-    }
-  }
+  if (t < tail.n_rows) advance_tail(tail, t, part, groups, tid, nt);
 }
 
 // A wave a (token, group): the group's columns as NV float4 a lane, nothing through LDS.
 template <int NV, typename TO>
 __global__ void __launch_bounds__(256)
 gate_group_norm_wave_kernel(TO* __restrict__ out, const float* __restrict__ y, const float* __restrict__ z, long ldz,
-                            const float* __restrict__ w, int n, int groups, float eps, long items) {
+                            const float* __restrict__ w, int n, int groups, float eps, long items, TailArgs tail) {
   const long item = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (item >= items) return;
   const int lane = threadIdx.x & 63;
   const long t = item / groups;
-  const int size = n / groups, c0 = (int)(item - t * groups) * size;
+  const int part = (int)(item - t * groups);
+  const int size = n / groups, c0 = part * size;
   const float* yr = y + (size_t)t * n + c0;
   const float* zr = z + (size_t)t * ldz + c0;
   float4 a[NV], b[NV];
@@ -313,11 +323,12 @@ gate_group_norm_wave_kernel(TO* __restrict__ out, const float* __restrict__ y, c
       *reinterpret_cast<float4*>(dst) = make_float4(v[0], v[1], v[2], v[3]);
     }
   }
+  if (t < tail.n_rows) advance_tail(tail, (int)t, part, groups, lane, 64);
 }
 
 template <typename TO>
 static bool gate_group_norm_waves(void* out, const float* y, const float* z, long ldz, const float* w, int groups,
-                                  float eps, int T_, int n, hipStream_t st) {
+                                  float eps, int T_, int n, const TailArgs& tail, hipStream_t st) {
   const int size = n / groups;
   const long items = (long)T_ * groups;
   if (size % 4 || ldz % 4 || size > 2048 || (((uintptr_t)y | (uintptr_t)z | (uintptr_t)w | (uintptr_t)out) & 15) ||
@@ -326,7 +337,7 @@ static bool gate_group_norm_waves(void* out, const float* y, const float* z, lon
   const int blocks = (int)((items + 3) / 4);
 #define GO(NV)                                                                                                       \
   if (size <= 256 * NV) {                                                                                            \
-    gate_group_norm_wave_kernel<NV, TO><<<blocks, 256, 0, st>>>((TO*)out, y, z, ldz, w, n, groups, eps, items);      \
+    gate_group_norm_wave_kernel<NV, TO><<<blocks, 256, 0, st>>>((TO*)out, y, z, ldz, w, n, groups, eps, items, tail); \
     return true;                                                                                                     \
   }
   GO(1) GO(2) GO(4) GO(8)
@@ -345,11 +356,11 @@ extern "C" int ptl_gate_group_norm(void* out, const float* y, const float* z, lo
       tail_rows > T_ || (tail_rows > 0 && taps > 1 && (!state || !x || !state_slots || C <= 0)))
     return PTL_ERR_ARG;
   const TailArgs tail{state, slot_stride, tail_off, x, ldx, state_slots, taps > 1 ? tail_rows : 0, C, taps};
-  // many rows, none of which advances a tail: a wave a (token, group)
-  if (tail.n_rows == 0) {
+  // enough of them: a wave a (token, group)
+  if ((long)T_ * groups >= 1024) {
     bool done = false;
-    if (dtype == PTL_DTYPE_F32) done = gate_group_norm_waves<float>(out, y, z, ldz, w, groups, eps, T_, n, st);
-    else if (dtype == PTL_DTYPE_BF16) done = gate_group_norm_waves<bf16_t>(out, y, z, ldz, w, groups, eps, T_, n, st);
+    if (dtype == PTL_DTYPE_F32) done = gate_group_norm_waves<float>(out, y, z, ldz, w, groups, eps, T_, n, tail, st);
+    else if (dtype == PTL_DTYPE_BF16) done = gate_group_norm_waves<bf16_t>(out, y, z, ldz, w, groups, eps, T_, n, tail, st);
     if (done) return ptl_launch_status();
   }
   const int size = n / groups;

@@ -133,6 +133,6 @@ def drawn(seed):
         return parallel(left, gated(r.choice([1, 2, 3, 4]), r.choice([8, 15, 32, 48, 96]), r.choice([8, 20, 64, 66]),
                                     r.choice([1.0, 4.0, 16.0, 30.0]), r.choice([2, 8, 16, 17])))
     layers = [layer(r.choice([any_mamba2, any_parallel])(), r.choice([None, 32, 72])) for _ in range(r.randint(2, 5))]
-    return (model(r.choice([64, 101, 256]), r.choice([32, 56, 80, 128]), r.choice([1e-6, 1e-5, 1e-4]),
+    return (model(r.choice([64, 101, 256]), r.choice([32, 50, 56, 80, 100, 128]), r.choice([1e-6, 1e-5, 1e-4]),
                   r.choice([1.0, 4.0, 12.0]), r.choice([0.7, 1.0, 2.2]), r.choice([None, 8.0, 30.0]), layers),
             0.13, r.choice([4, 16, 32]))

@@ -41,7 +41,8 @@ def write_folder(tmp_path_factory, cfg, std, seed, edit=None, tame=False):
     ``tame``: gated linear attention's key projections are its query projections, so that a token's
     query is never at right angles to its own key: behind few tokens the read-out S^T q is then never
     the small rest of a cancellation whose sign the rounding of bfloat16 decides and the norm of the
-    heads blows up. The float32 tests run on the untamed weights."""
+    heads blows up. The float32 tests run on the untamed weights (but for the configurations drawn at random,
+    where rounding to float32 alone may be blown up to the tolerance)."""
     from safetensors.torch import load_file, save_file
     from pytriton_llama_amd.weights import write_random_model
     folder = str(tmp_path_factory.mktemp("bimopel"))
@@ -79,9 +80,9 @@ def skip_touchy(got, want, touchy):
             got[rid][t] = want[rid][t]
 
 
-def make_case(tmp_path_factory, cfg, std, page, lengths, seed):
-    folder = write_folder(tmp_path_factory, cfg, std, seed)
+def make_case(tmp_path_factory, cfg, std, page, lengths, seed, tame_both=False):
     tamed = write_folder(tmp_path_factory, cfg, std, seed, tame=True)
+    folder = tamed if tame_both else write_folder(tmp_path_factory, cfg, std, seed)
     seqs = random_sequences(cfg["vocab"], lengths, seed=seed + 3)
     touchy = {}
     want = {torch.float32: plain_logits(folder, seqs),
@@ -188,7 +189,7 @@ def test_a_batch_gives_what_each_request_gives_alone(cases, name):
 @pytest.mark.parametrize("seed", range(10))
 def test_configurations_drawn_at_random(tmp_path_factory, gpu_device, seed, dtype):
     cfg, std, page = drawn(seed)
-    case = make_case(tmp_path_factory, cfg, std, page, [3, 40, 101, 18], 300 + seed)
+    case = make_case(tmp_path_factory, cfg, std, page, [3, 40, 101, 18], 300 + seed, tame_both=True)
     for steps in (cuttings.tail_decode(case[2], 30), cuttings.portions(case[2], sizes=(19, 2, 33, 1, 5)),
                   cuttings.mixed(case[2], seed=seed, max_live=3)):
         run_steps(case, dtype, steps)
