@@ -443,7 +443,7 @@ def attend_plain(q, k, v, n, ql, chunk, window, scale, sink, gate):
 
 # (H, G, Dk, Dv, page size, chunk, window): chunks shorter than a page, equal to it, of one position,
 # longer than the context, borders inside 64-row blocks; a window beside the same extras
-CHUNK_CASES = [(4, 2, 32, 32, 16, 48, 0), (6, 1, 64, 64, 16, 96, 0), (4, 4, 128, 128, 32, 100, 0), (3, 3, 24, 40, 8, 5, 0),
+CHUNK_CASES = [(4, 2, 32, 32, 16, 48, 0), (5, 1, 64, 64, 16, 90, 0), (4, 4, 128, 128, 32, 100, 0), (3, 3, 24, 40, 8, 5, 0),
                (4, 1, 32, 64, 16, 16, 0), (8, 2, 64, 32, 4, 1, 0), (2, 2, 96, 96, 16, 1000, 0), (4, 2, 128, 128, 16, 37, 0),
                (2, 1, 18, 20, 4, 64, 0), (5, 5, 128, 64, 16, 130, 0), (4, 2, 64, 64, 16, 0, 70), (4, 2, 64, 64, 16, 0, 0)]
 
