@@ -10,6 +10,8 @@
 // sink (or null): one float a query head; the softmax denominator of that head holds exp(sink) once
 // more, a term without key and value that is not scaled. gate (or null): one float a row and query
 // head (row * gate_stride + head); the head's result is multiplied by sigmoid(gate).
+//
+// softcap > 0: a scaled score s becomes softcap * tanh(s / softcap) before the mask and the softmax.
 #pragma once
 #include "common.h"
 #include <math.h>
@@ -19,6 +21,7 @@ struct AttnExtras {
   const float* sink;
   const float* gate;
   long gate_stride;
+  float softcap;
 };
 
 // The first key that a query at position pos sees (of the window, for a window that keeps the
@@ -33,6 +36,16 @@ __device__ __forceinline__ float head_gate(const AttnExtras& ex, int row, int he
   return ex.gate ? 1.0f / (1.0f + expf(-ex.gate[(size_t)row * ex.gate_stride + head])) : 1.0f;
 }
 
+__device__ __forceinline__ float cap_score(const AttnExtras& ex, float s) {
+  return ex.softcap > 0.f ? ex.softcap * tanhf(s / ex.softcap) : s;
+}
+
+// tanh from the hardware's exp2 and reciprocal: 1 - 2 / (1 + e^(2x)), with x2 = 2 x log2 e. Absolute
+// error of a few 1e-7 (the result feeds the exponent of a softmax); saturates to -1 and 1.
+__device__ __forceinline__ float tanh_exp2(float x2) {
+  return fmaf(-2.0f, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x2)), 1.0f);
+}
+
 static inline bool extras_ok(const AttnExtras& ex) {
-  return !(ex.chunk > 0 && (ex.window > 0 || ex.keep_first > 0));
+  return ex.softcap >= 0.f && !(ex.chunk > 0 && (ex.window > 0 || ex.keep_first > 0));
 }

@@ -21,7 +21,8 @@
 // index v below n_kept is key v, index v from n_kept on is key v + shift).
 // chunk > 0: a query sees the keys of its own chunk only, chunks of so many positions counted from
 // position 0; pages of chunks before it may be gone too.
-// sink, gate: one more term of a head's denominator, and a factor on its result (attention.h).
+// sink, gate: one more term of a head's denominator, and a factor on its result; softcap: a bound on
+// the scores (attention.h).
 //
 // ptl_attention_generic: vector-FMA kernel, float32 math, storage type T
 // (float32 or bfloat16), any page size, any D up to 640 (beyond 256 with more LDS than a
@@ -132,7 +133,7 @@ attn_generic_kernel(TO* __restrict__ out, long out_stride, const T* __restrict__
       for (int d = 0; d < Dk; ++d) dot = fmaf(qr[d], kr[d], dot);
       const bool vis = row_valid && kw < n_walk && kp <= qpos &&
                        (kp >= row_lo || kp < ex.keep_first);
-      s[j] = vis ? dot * scale : -INFINITY;
+      s[j] = vis ? cap_score(ex, dot * scale) : -INFINITY;
       tmax = fmaxf(tmax, s[j]);
     }
 #pragma unroll
@@ -220,10 +221,10 @@ extern "C" int ptl_attention_generic_kv(void* out, long out_stride, int out_f32,
                                         const int32_t* work_seq, const int32_t* work_qoff, int n_work,
                                         int Hq, int Hkv, int maps, int Dk, int Dv, int page_size,
                                         int window, int keep_first, int chunk, const float* sink,
-                                        const float* gate, long gate_stride, float scale, int dtype,
+                                        const float* gate, long gate_stride, float softcap, float scale, int dtype,
                                         hipStream_t stream) {
   if (n_work <= 0) return PTL_OK;
-  const AttnExtras ex{window, keep_first, chunk, sink, gate, gate_stride};
+  const AttnExtras ex{window, keep_first, chunk, sink, gate, gate_stride, softcap};
   if (Hq <= 0 || Hkv <= 0 || maps <= 0 || Hq % maps || (Hq / maps) % Hkv || Dk <= 0 || Dv <= 0 ||
       Dk > 640 || Dv > 640 || page_size <= 0 || Hq > 65535 || !extras_ok(ex))
     return PTL_ERR_ARG;
@@ -255,11 +256,11 @@ extern "C" int ptl_attention_generic(void* out, long out_stride, const void* q, 
                                      const int32_t* work_seq, const int32_t* work_qoff, int n_work,
                                      int Hq, int Hkv, int D, int page_size, int window,
                                      int keep_first, int chunk, const float* sink, const float* gate,
-                                     long gate_stride, float scale, int dtype, hipStream_t stream) {
+                                     long gate_stride, float softcap, float scale, int dtype, hipStream_t stream) {
   return ptl_attention_generic_kv(out, out_stride, 0, q, q_stride, k_cache, v_cache, q_start, ctx_len,
                                   block_table, bt_stride, work_seq, work_qoff, n_work, Hq, Hkv, 1, D,
-                                  D, page_size, window, keep_first, chunk, sink, gate, gate_stride, scale,
-                                  dtype, stream);
+                                  D, page_size, window, keep_first, chunk, sink, gate, gate_stride, softcap,
+                                  scale, dtype, stream);
 }
 
 // ===========================================================================
@@ -392,6 +393,7 @@ attn_decode_kernel(TO* __restrict__ out, long out_stride, const T* __restrict__ 
       for (int j = 0; j < DEC_CHUNK; ++j) s = fmaf(qf[h][j], kf[j], s);
 #pragma unroll
       for (int o = 1; o < LPK; o <<= 1) s += __shfl_xor(s, o, 64);
+      s = cap_score(ex, s);
       if (valid) {
         if (s > m[h]) {
           const float alpha = expf(m[h] - s);     // exp(-inf) = 0 at the first key
@@ -560,9 +562,9 @@ extern "C" int ptl_attention_decode_kv(void* out, long out_stride, int out_f32, 
                                        float* part_ml, int n_seq, int Hq, int Hkv, int maps, int Dk,
                                        int Dv, int page_size, int window, int keep_first, int chunk,
                                        const float* sink, const float* gate, long gate_stride,
-                                       float scale, int num_splits, int dtype, hipStream_t stream) {
+                                       float softcap, float scale, int num_splits, int dtype, hipStream_t stream) {
   if (n_seq <= 0) return PTL_OK;
-  const AttnExtras ex{window, keep_first, chunk, sink, gate, gate_stride};
+  const AttnExtras ex{window, keep_first, chunk, sink, gate, gate_stride, softcap};
   if (Hq <= 0 || Hkv <= 0 || maps <= 0 || Hq % maps || (Hq / maps) % Hkv || Dk <= 0 || Dk % 16 ||
       Dk > 256 || Dv <= 0 || Dv % 16 || Dv > 256 || page_size <= 0 || num_splits < 1 ||
       num_splits > 1024 || (num_splits > 1 && (!part_acc || !part_ml)) || !extras_ok(ex))
@@ -599,11 +601,11 @@ extern "C" int ptl_attention_decode(void* out, long out_stride, const void* q, l
                                     const int32_t* block_table, int bt_stride, float* part_acc,
                                     float* part_ml, int n_seq, int Hq, int Hkv, int D, int page_size,
                                     int window, int keep_first, int chunk, const float* sink,
-                                    const float* gate, long gate_stride, float scale, int num_splits,
+                                    const float* gate, long gate_stride, float softcap, float scale, int num_splits,
                                     int dtype, hipStream_t stream) {
   return ptl_attention_decode_kv(out, out_stride, 0, q, q_stride, k_cache, v_cache, q_start, ctx_len,
                                  block_table, bt_stride, part_acc, part_ml, n_seq, Hq, Hkv, 1, D, D,
-                                 page_size, window, keep_first, chunk, sink, gate, gate_stride, scale,
+                                 page_size, window, keep_first, chunk, sink, gate, gate_stride, softcap, scale,
                                  num_splits, dtype, stream);
 }
 
@@ -638,8 +640,9 @@ __device__ __forceinline__ void wave_lds_fence() {
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 }
 
-// KEPT: a window that keeps the sequence's first keys (keep_first > 0).
-template <int NDT, int UNR, bool KEPT>
+// KEPT: a window that keeps the sequence's first keys (keep_first > 0). CAP: scores are capped; then
+// scale_log2 is softcap * log2 e and cap_in takes a raw score to tanh_exp2's argument.
+template <int NDT, int UNR, bool KEPT, bool CAP>
 __global__ void __launch_bounds__(256)
 attn_decode_mfma_kernel(bf16_t* __restrict__ out, long out_stride, const bf16_t* __restrict__ q,
                         long q_stride, const bf16_t* __restrict__ k_cache,
@@ -647,7 +650,7 @@ attn_decode_mfma_kernel(bf16_t* __restrict__ out, long out_stride, const bf16_t*
                         const int32_t* __restrict__ ctx_len, const int32_t* __restrict__ block_table,
                         int bt_stride, float* __restrict__ part_acc, float* __restrict__ part_ml,
                         int Hq, int Hkv, int page_size, int page_shift, AttnExtras ex, float scale_log2,
-                        int num_splits) {
+                        float cap_in, int num_splits) {
   constexpr int D = 32 * NDT;
   constexpr int NT = 2 * NDT;             // 16-wide tiles of the head dimension
   constexpr int TILE = 64 * UNR;          // keys per turn of the workgroup
@@ -767,7 +770,7 @@ attn_decode_mfma_kernel(bf16_t* __restrict__ out, long out_stride, const bf16_t*
     for (int u = 0; u < UNR; ++u)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        float sc = st[u][i] * scale_log2;
+        float sc = (CAP ? tanh_exp2(st[u][i] * cap_in) : st[u][i]) * scale_log2;
         sc = (kc + 16 * u + 4 * lg + i < k_end) ? sc : -INFINITY;
         st[u][i] = sc;
         tmax = fmaxf(tmax, sc);
@@ -873,16 +876,20 @@ static int launch_decode_mfma(void* out, long out_stride, const void* q, long q_
   const size_t lds_merge = (size_t)(4 * 16 * D + 4 * 16 * 2) * sizeof(float);
   const size_t lds_values = (size_t)4 * UNR * 16 * (D + 16) * sizeof(bf16_t);
   const size_t lds = lds_merge > lds_values ? lds_merge : lds_values;
-  if (ex.window > 0 && ex.keep_first > 0)
-    attn_decode_mfma_kernel<NDT, UNR, true><<<grid, 256, lds, stream>>>(
-        (bf16_t*)out, out_stride, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache,
-        (const bf16_t*)v_cache, q_start, ctx_len, block_table, bt_stride, part_acc, part_ml, Hq, Hkv,
-        page_size, page_shift, ex, scale * 1.4426950408889634f, num_splits);
-  else
-    attn_decode_mfma_kernel<NDT, UNR, false><<<grid, 256, lds, stream>>>(
-        (bf16_t*)out, out_stride, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache,
-        (const bf16_t*)v_cache, q_start, ctx_len, block_table, bt_stride, part_acc, part_ml, Hq, Hkv,
-        page_size, page_shift, ex, scale * 1.4426950408889634f, num_splits);
+  const bool kept = ex.window > 0 && ex.keep_first > 0, cap = ex.softcap > 0.f;
+  const float log2e = 1.4426950408889634f;
+  const float scale_log2 = (cap ? ex.softcap : scale) * log2e, cap_in = cap ? 2.0f * log2e * scale / ex.softcap : 0.f;
+#define GO(KEPT, CAP)                                                                                      \
+  attn_decode_mfma_kernel<NDT, UNR, KEPT, CAP><<<grid, 256, lds, stream>>>(                                \
+      (bf16_t*)out, out_stride, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, \
+      q_start, ctx_len, block_table, bt_stride, part_acc, part_ml, Hq, Hkv, page_size, page_shift, ex,      \
+      scale_log2, cap_in, num_splits)
+  if (kept) {
+    if (cap) GO(true, true); else GO(true, false);
+  } else {
+    if (cap) GO(false, true); else GO(false, false);
+  }
+#undef GO
   if (hipGetLastError() != hipSuccess) return PTL_ERR_LAUNCH;
   if (num_splits > 1) {
     dim3 mgrid(n_seq, Hq);
@@ -900,9 +907,9 @@ extern "C" int ptl_attention_decode_mfma(void* out, long out_stride, const void*
                                          float* part_ml, int n_seq, int Hq, int Hkv, int D,
                                          int page_size, int window, int keep_first, int chunk,
                                          const float* sink, const float* gate, long gate_stride,
-                                         float scale, int num_splits, int unroll, hipStream_t stream) {
+                                         float softcap, float scale, int num_splits, int unroll, hipStream_t stream) {
   if (n_seq <= 0) return PTL_OK;
-  const AttnExtras ex{window, keep_first, chunk, sink, gate, gate_stride};
+  const AttnExtras ex{window, keep_first, chunk, sink, gate, gate_stride, softcap};
   if (Hq <= 0 || Hkv <= 0 || Hq % Hkv || Hq / Hkv > 16 || D <= 0 || D % 32 || D > 128 ||
       page_size <= 0 || (page_size & (page_size - 1)) ||
       (long)Hkv * page_size * D * 2 >= (1L << 32) || q_stride % 8 || num_splits < 1 ||

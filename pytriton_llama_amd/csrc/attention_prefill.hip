@@ -67,8 +67,9 @@ template <> __device__ __forceinline__ void store4<float>(float* p, const float*
 
 // NDK, NDV: key and value sizes in units of 32. RT: 16-row query tiles per wave; the workgroup
 // takes 64 * RT query rows. KEPT: a window that keeps the sequence's first keys (keep_first > 0):
-// the key tiles then walk a list of two stretches of positions instead of one.
-template <int NDK, int NDV, int RT, typename TO, bool KEPT>
+// the key tiles then walk a list of two stretches of positions instead of one. CAP: scores are capped:
+// tanh_exp2(raw score * cap_in) takes the place of the raw score and scale_log2 is softcap * log2 e.
+template <int NDK, int NDV, int RT, typename TO, bool KEPT, bool CAP>
 __global__ void __launch_bounds__(256, (NDK + NDV) <= 4 ? 3 : 2)
 attn_prefill_mfma_kernel(TO* __restrict__ out, long out_stride, const bf16_t* __restrict__ q,
                          long q_stride, const bf16_t* __restrict__ k_cache,
@@ -76,7 +77,7 @@ attn_prefill_mfma_kernel(TO* __restrict__ out, long out_stride, const bf16_t* __
                          const int32_t* __restrict__ ctx_len, const int32_t* __restrict__ block_table,
                          int bt_stride, const int32_t* __restrict__ work_seq,
                          const int32_t* __restrict__ work_qoff, int n_work, int Hq, int Hkv, int maps,
-                         int page_size, int page_shift, AttnExtras ex, float scale_log2) {
+                         int page_size, int page_shift, AttnExtras ex, float scale_log2, float cap_in) {
   constexpr int DK = 32 * NDK, DV = 32 * NDV;
   constexpr int PBM = 64 * RT;
   constexpr int CPRK = DK / 8, CPRV = DV / 8;      // 16-byte chunks per row
@@ -300,6 +301,12 @@ attn_prefill_mfma_kernel(TO* __restrict__ out, long out_stride, const bf16_t* __
     Frag8 pb[RT][2];
 #pragma unroll
     for (int r = 0; r < RT; ++r) {
+      if (CAP) {
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) st[r][kt][i] = tanh_exp2(st[r][kt][i] * cap_in);
+      }
       if (MASKED) {
 #pragma unroll
         for (int kt = 0; kt < 4; ++kt)
@@ -424,16 +431,19 @@ static int launch_prefill_mfma(void* out, long out_stride, const void* q, long q
   int page_shift = -1;
   for (int sh = 0; sh < 31; ++sh)
     if ((1 << sh) == page_size) page_shift = sh;
-  if (ex.window > 0 && ex.keep_first > 0)
-    attn_prefill_mfma_kernel<NDK, NDV, RT, TO, true><<<grid, 256, 0, stream>>>(
-        (TO*)out, out_stride, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache,
-        (const bf16_t*)v_cache, q_start, ctx_len, block_table, bt_stride, work_seq, work_qoff,
-        n_work, Hq, Hkv, maps, page_size, page_shift, ex, scale * 1.4426950408889634f);
-  else
-    attn_prefill_mfma_kernel<NDK, NDV, RT, TO, false><<<grid, 256, 0, stream>>>(
-        (TO*)out, out_stride, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache,
-        (const bf16_t*)v_cache, q_start, ctx_len, block_table, bt_stride, work_seq, work_qoff,
-        n_work, Hq, Hkv, maps, page_size, page_shift, ex, scale * 1.4426950408889634f);
+  const bool kept = ex.window > 0 && ex.keep_first > 0, cap = ex.softcap > 0.f;
+  if (kept && cap) return PTL_ERR_ARG;
+  const float log2e = 1.4426950408889634f;
+  const float scale_log2 = (cap ? ex.softcap : scale) * log2e, cap_in = cap ? 2.0f * log2e * scale / ex.softcap : 0.f;
+#define GO(KEPT, CAP)                                                                                       \
+  attn_prefill_mfma_kernel<NDK, NDV, RT, TO, KEPT, CAP><<<grid, 256, 0, stream>>>(                          \
+      (TO*)out, out_stride, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache,     \
+      q_start, ctx_len, block_table, bt_stride, work_seq, work_qoff, n_work, Hq, Hkv, maps, page_size,      \
+      page_shift, ex, scale_log2, cap_in)
+  if (kept) GO(true, false);
+  else if (cap) GO(false, true);
+  else GO(false, false);
+#undef GO
   return ptl_launch_status();
 }
 
@@ -472,9 +482,9 @@ extern "C" int ptl_attention_prefill_mfma(void* out, long out_stride, const void
                                           int Hkv, int D,
                                           int page_size, int window, int keep_first, int chunk,
                                           const float* sink, const float* gate, long gate_stride,
-                                          float scale, hipStream_t stream) {
+                                          float softcap, float scale, hipStream_t stream) {
   if (n_work <= 0) return PTL_OK;
-  const AttnExtras ex{window, keep_first, chunk, sink, gate, gate_stride};
+  const AttnExtras ex{window, keep_first, chunk, sink, gate, gate_stride, softcap};
   if (Hq <= 0 || Hkv <= 0 || Hq % Hkv || D % 32 || D <= 0 || D > 128 || page_size <= 0 ||
       (page_size & (page_size - 1)) || (long)Hkv * page_size * D * 2 >= (1L << 32) ||
       Hq > 65535 || n_groups < 1 || n_groups > n_work || q_stride % 8 || out_stride % 4 ||
@@ -500,9 +510,9 @@ extern "C" int ptl_attention_prefill_mfma_kv(void* out, long out_stride, int out
                                              int n_work, int n_groups, int Hq, int Hkv, int maps, int Dk,
                                              int Dv, int page_size, int window, int keep_first, int chunk,
                                              const float* sink, const float* gate, long gate_stride,
-                                             float scale, hipStream_t stream) {
+                                             float softcap, float scale, hipStream_t stream) {
   if (n_work <= 0) return PTL_OK;
-  const AttnExtras ex{window, keep_first, chunk, sink, gate, gate_stride};
+  const AttnExtras ex{window, keep_first, chunk, sink, gate, gate_stride, softcap};
   if (Hq <= 0 || Hkv <= 0 || maps <= 0 || Hq % maps || (Hq / maps) % Hkv || Dk % 32 || Dk <= 0 ||
       Dk > 128 || Dv % 32 || Dv <= 0 || Dv > 128 || page_size <= 0 || (page_size & (page_size - 1)) ||
       (long)Hkv * maps * page_size * Dk * 2 >= (1L << 32) || (long)Hkv * page_size * Dv * 2 >= (1L << 32) ||

@@ -58,8 +58,12 @@ struct Plan {
   bool timed = false;                             // timed, or given up: not tried again
 };
 
-// (M, N, K, ldx, ldy, output type)
-using Key = std::tuple<int, int, int, long, long, int>;
+// (M, N, K, ldx, ldy, output type, products, and from one product to the next: of x, of W, of y)
+using Key = std::tuple<int, int, int, long, long, int, int, long, long, long>;
+
+// columns of y from the first product's first to the last one's last (the products of a batch leave their
+// results side by side in the rows of y)
+long columns(const Key& k) { return std::get<1>(k) + (std::get<6>(k) - 1) * std::get<9>(k); }
 
 struct State {
   hipblasLtHandle_t handle = nullptr;
@@ -141,7 +145,7 @@ __global__ void disagree_kernel(const T* got, const T* ref, int M, int N, long l
 // proposal's result, laid out as y). check: two words of device memory behind ref.
 bool agrees(State& s, const Plan& p, int i, const Key& key, void* y, const void* ref, unsigned* check,
             const void* x, const void* w, hipStream_t stream) {
-  const int M = std::get<0>(key), N = std::get<1>(key);
+  const int M = std::get<0>(key), N = (int)columns(key);
   const long ld = std::get<4>(key);
   const bool f32 = std::get<5>(key) == PTL_DTYPE_F32;
   if (!ok(run_algo(s, p, p.proposals[i].algo, y, x, w, stream))) return false;
@@ -215,7 +219,7 @@ void time_plan(State& s, Plan& p, const Key& key, void* y, const void* x, const 
   // caches here and cold in a step: a few per cent say nothing) and gives the same product
   const int M = std::get<0>(key);
   const long ld = std::get<4>(key);
-  const size_t bytes = (size_t)M * ld * (std::get<5>(key) == PTL_DTYPE_F32 ? 4 : 2);
+  const size_t bytes = ((size_t)(M - 1) * ld + columns(key)) * (std::get<5>(key) == PTL_DTYPE_F32 ? 4 : 2);
   char* ref = nullptr;
   for (;;) {
     int best_i = 0;
@@ -250,7 +254,8 @@ void time_plan(State& s, Plan& p, const Key& key, void* y, const void* x, const 
   }
 }
 
-int make_plan(State& s, Plan& p, int M, int N, int K, long ldx, long ldy, int out_dtype) {
+int make_plan(State& s, Plan& p, int M, int N, int K, long ldx, long ldy, int out_dtype, int batch, long sx, long sw,
+              long sy) {
   // Column-major view: y^T [N, M] = W [N, K] x^T [K, M]. W lies as a K x N column-major
   // matrix (leading dimension K) and is transposed; x as K x M (leading dimension ldx).
   const hipDataType out_type = out_dtype == PTL_DTYPE_F32 ? HIP_R_32F : HIP_R_16BF;
@@ -262,6 +267,16 @@ int make_plan(State& s, Plan& p, int M, int N, int K, long ldx, long ldy, int ou
       !ok(hipblasLtMatrixLayoutCreate(&p.b, HIP_R_16BF, K, M, ldx)) ||
       !ok(hipblasLtMatrixLayoutCreate(&p.c, out_type, N, M, ldy)))
     return PTL_ERR_LAUNCH;
+  if (batch > 1) {
+    const int32_t n = batch;
+    const int64_t step[3] = {sw, sx, sy};
+    const hipblasLtMatrixLayout_t layout[3] = {p.a, p.b, p.c};
+    for (int i = 0; i < 3; ++i)
+      if (!ok(hipblasLtMatrixLayoutSetAttribute(layout[i], HIPBLASLT_MATRIX_LAYOUT_BATCH_COUNT, &n, sizeof(n))) ||
+          !ok(hipblasLtMatrixLayoutSetAttribute(layout[i], HIPBLASLT_MATRIX_LAYOUT_STRIDED_BATCH_OFFSET, &step[i],
+                                                sizeof(step[i]))))
+        return PTL_ERR_LAUNCH;
+  }
   return propose(s, p) ? PTL_OK : PTL_ERR_ARG;
 }
 
@@ -269,11 +284,16 @@ int make_plan(State& s, Plan& p, int M, int N, int K, long ldx, long ldy, int ou
 
 // y [M, N] (row stride ldy; bfloat16 or float32) = x [M, K] (bfloat16, row stride ldx) W^T,
 // W [N, K] bfloat16 with dense rows. Rows of x and W 16-byte aligned.
+// batch > 1: that many such products, x_stride, w_stride and y_stride elements apart; their columns of y lie
+// side by side (y_stride >= N, all of them inside a row).
 // use_timed != 0: run the proposal that a timing of this shape kept, and time the shape now if
 // it has not been (unless the stream is being captured); 0: the library's first proposal.
 extern "C" int ptl_blaslt_gemm_bf16(void* y, const void* x, const void* w, int M, int N, int K,
-                                    long ldx, long ldy, int out_dtype, int use_timed, hipStream_t stream) {
+                                    long ldx, long ldy, int out_dtype, int batch, long x_stride, long w_stride,
+                                    long y_stride, int use_timed, hipStream_t stream) {
   if (M <= 0 || N <= 0) return PTL_OK;
+  if (batch < 1 || (batch > 1 && (y_stride < N || (batch - 1) * y_stride + N > ldy))) return PTL_ERR_ARG;
+  if (batch == 1) x_stride = w_stride = y_stride = 0;
   if (K <= 0 || ldx < K || ldy < N || (out_dtype != PTL_DTYPE_F32 && out_dtype != PTL_DTYPE_BF16))
     return PTL_ERR_ARG;
   static const bool never_timed = getenv("PTL_BLASLT_NO_TUNING") != nullptr;
@@ -294,7 +314,7 @@ extern "C" int ptl_blaslt_gemm_bf16(void* y, const void* x, const void* w, int M
     s.handle = handle;
     s.workspace = workspace;
   }
-  const Key key(M, N, K, ldx, ldy, out_dtype);
+  const Key key(M, N, K, ldx, ldy, out_dtype, batch, x_stride, w_stride, y_stride);
   auto it = s.plans.find(key);
   if (it == s.plans.end()) {
     if (s.plans.size() >= MAX_PLANS) {
@@ -307,7 +327,7 @@ extern "C" int ptl_blaslt_gemm_bf16(void* y, const void* x, const void* w, int M
       }
     }
     Plan p;
-    const int rc = make_plan(s, p, M, N, K, ldx, ldy, out_dtype);
+    const int rc = make_plan(s, p, M, N, K, ldx, ldy, out_dtype, batch, x_stride, w_stride, y_stride);
     if (rc != PTL_OK) {
       drop_plan(p);
       return rc;
@@ -331,6 +351,6 @@ extern "C" int ptl_blaslt_timed_shapes() {
 extern "C" int ptl_blaslt_timed_choice(int M, int N, int K, long ldx, long ldy, int out_dtype) {
   State& s = state();
   std::lock_guard<std::mutex> guard(s.lock);
-  auto it = s.plans.find(Key(M, N, K, ldx, ldy, out_dtype));
+  auto it = s.plans.find(Key(M, N, K, ldx, ldy, out_dtype, 1, 0, 0, 0));
   return it == s.plans.end() || !it->second.timed ? -1 : it->second.timed_choice;
 }

@@ -71,6 +71,22 @@ __device__ __forceinline__ float gelu_tanh(float z) {
 __device__ __forceinline__ float glu_act(int act, float g) {
   return act == GLU_GELU_TANH ? gelu_tanh(g) : g / (1.0f + expf(-g));
 }
+// The whole of a gated activation, act(gate, up). GLU_CLAMPED: g = min(gate, limit), u = up clamped to
+// [-limit, limit], g sigmoid(1.702 g) (u + 1); the others act(gate) * up.
+#define GLU_CLAMPED 2
+struct GluArgs {
+  int act;
+  float limit;
+};
+__device__ __forceinline__ float glu(const GluArgs& a, float g, float u) {
+  if (a.act == GLU_CLAMPED) {
+    g = fminf(g, a.limit);
+    u = fminf(fmaxf(u, -a.limit), a.limit);
+    return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
+  }
+  return glu_act(a.act, g) * u;
+}
+static inline bool glu_ok(int act) { return act == GLU_SILU || act == GLU_GELU_TANH || act == GLU_CLAMPED; }
 
 // block-wide sum for blockDim.x a multiple of 64, at most 1024; scratch holds 16 floats
 __device__ __forceinline__ float block_sum(float v, float* scratch) {

@@ -173,6 +173,14 @@ struct AddNormArgs {
   long ldr;
 };
 
+// Several products side by side (ptl_gemm_skinny_groups_bf16): the rows of W from g * cols on (the last
+// group: all that are left) multiply rows of x that lie g * x_stride elements further. cols == 0: one product.
+// cols is a multiple of 16: no tile has rows of two groups.
+struct GroupArgs {
+  int cols, last;
+  long x_stride;
+};
+
 // ROWS: weight rows a workgroup owns: 16 fill the MFMA tile; 8 (half the tile idle) give twice
 // the workgroups when N is so small that 16-row tiles would leave CUs without work.
 // ADD_NORM: the epilogue described at AddNormArgs (MT = 1, bfloat16 output).
@@ -180,11 +188,12 @@ struct AddNormArgs {
 template <int MT, int U, int ROWS, typename TY, bool ADD_NORM = false, int XR = 16, bool BLOCKED = false>
 __global__ void __launch_bounds__(1024)
 gemm_skinny_kernel(TY* __restrict__ y, const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
-                   int M, int N, int K, long ldx, long ldy, int k_per_wave, AddNormArgs an) {
+                   int M, int N, int K, long ldx, long ldy, int k_per_wave, AddNormArgs an, GroupArgs gr) {
   extern __shared__ float red[];                 // [waves][MT][64][4]
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, ln = lane & 15, lg = lane >> 4;
   const int nwaves = blockDim.x >> 6;
   const int n0 = blockIdx.x * ROWS;
+  if (!ADD_NORM && gr.cols) x += min(n0 / gr.cols, gr.last) * gr.x_stride;
   const bool wrow = ln < ROWS;
   const bf16_t* wp = gs_row_ptr<BLOCKED>(w, min(n0 + min(ln, ROWS - 1), N - 1), K, lg);
   static_assert(XR == 16 || MT == 1, "packed loads of x are for one tile of rows");
@@ -362,7 +371,7 @@ static int compute_units() {
 template <int MT, int U, int ROWS>
 static int launch_skinny_rows(void* y, const void* x, const void* w, int M, int N, int K, long ldx,
                               long ldy, int out_dtype, hipStream_t stream,
-                              const AddNormArgs* an = nullptr, bool blocked = false) {
+                              const AddNormArgs* an = nullptr, bool blocked = false, GroupArgs gr = {}) {
   if (blocked && K % 32) return PTL_ERR_ARG;
   const int blocks = (N + ROWS - 1) / ROWS;
   // enough waves to keep every SIMD of the chip busy a few times over (16 waves a compute
@@ -377,7 +386,7 @@ static int launch_skinny_rows(void* y, const void* x, const void* w, int M, int 
   const int xr = MT == 1 ? gs_rows_of(M) : 16;
 #define GO1(TY, AN, XR, BL, args)                                                                    \
   gemm_skinny_kernel<(XR == 16 ? MT : 1), U, ROWS, TY, AN, XR, BL><<<blocks, waves * 64, lds, stream>>>( \
-      (TY*)y, (const bf16_t*)x, (const bf16_t*)w, M, N, K, ldx, ldy, k_per_wave, args)
+      (TY*)y, (const bf16_t*)x, (const bf16_t*)w, M, N, K, ldx, ldy, k_per_wave, args, gr)
 #define GO(TY, AN, XR, args)                                                                         \
   if (blocked) GO1(TY, AN, XR, true, args); else GO1(TY, AN, XR, false, args)
 #define BY_ROWS(TY, AN, args)                                                                        \
@@ -408,12 +417,12 @@ static int skinny_rows(int N) { return (N + 15) / 16 <= few_tiles() ? 8 : 16; }
 template <int MT, int U>
 static int launch_skinny(void* y, const void* x, const void* w, int M, int N, int K, long ldx,
                          long ldy, int out_dtype, hipStream_t stream,
-                         const AddNormArgs* an = nullptr, bool blocked = false) {
+                         const AddNormArgs* an = nullptr, bool blocked = false, GroupArgs gr = {}) {
   // measured on MI355X at K = 2048 and 8192: N = 2048 (128 tiles of 16 rows) gains 10 to 20 %
   // from 8-row tiles, N = 3072 (192 tiles) loses
   if (skinny_rows(N) == 8)
-    return launch_skinny_rows<MT, U, 8>(y, x, w, M, N, K, ldx, ldy, out_dtype, stream, an, blocked);
-  return launch_skinny_rows<MT, U, 16>(y, x, w, M, N, K, ldx, ldy, out_dtype, stream, an, blocked);
+    return launch_skinny_rows<MT, U, 8>(y, x, w, M, N, K, ldx, ldy, out_dtype, stream, an, blocked, gr);
+  return launch_skinny_rows<MT, U, 16>(y, x, w, M, N, K, ldx, ldy, out_dtype, stream, an, blocked, gr);
 }
 
 // w_blocked != 0: ``w`` is the blocked copy of the matrix (see gs_row_ptr; rows padded to a
@@ -428,6 +437,23 @@ extern "C" int ptl_gemm_skinny_bf16(void* y, const void* x, const void* w, int w
   if (M <= 16) return launch_skinny<1, 8>(y, x, w, M, N, K, ldx, ldy, out_dtype, stream, nullptr, bl);
   if (M <= 32) return launch_skinny<2, 4>(y, x, w, M, N, K, ldx, ldy, out_dtype, stream, nullptr, bl);
   return launch_skinny<4, 2>(y, x, w, M, N, K, ldx, ldy, out_dtype, stream, nullptr, bl);
+}
+
+// Several products of M <= 64 rows in one launch: columns g * cols .. of y = x_g W_g^T with x_g = x + g *
+// x_stride, for the groups 0 .. last (see GroupArgs); W [N, K] holds the groups' rows one after the other.
+extern "C" int ptl_gemm_skinny_groups_bf16(void* y, const void* x, const void* w, int w_blocked, int M, int N, int K,
+                                           long ldx, long ldy, int cols, int last, long x_stride, int out_dtype,
+                                           hipStream_t stream) {
+  if (M <= 0 || N <= 0) return PTL_OK;
+  if (M > 64 || K <= 0 || K % 8 || ldx % 8 || ldx < K || ldy < N || cols <= 0 || cols % 16 || last < 0 ||
+      (long)last * cols >= N || x_stride % 8 || (out_dtype != PTL_DTYPE_F32 && out_dtype != PTL_DTYPE_BF16) ||
+      (w_blocked && K % 32))
+    return PTL_ERR_ARG;
+  const bool bl = w_blocked != 0;
+  const GroupArgs gr{cols, last, x_stride};
+  if (M <= 16) return launch_skinny<1, 8>(y, x, w, M, N, K, ldx, ldy, out_dtype, stream, nullptr, bl, gr);
+  if (M <= 32) return launch_skinny<2, 4>(y, x, w, M, N, K, ldx, ldy, out_dtype, stream, nullptr, bl, gr);
+  return launch_skinny<4, 2>(y, x, w, M, N, K, ldx, ldy, out_dtype, stream, nullptr, bl, gr);
 }
 
 // How many partial sums a row gets from ptl_gemm_skinny_add_norm_bf16 with N columns (on the
@@ -456,7 +482,7 @@ extern "C" int ptl_gemm_skinny_add_norm_bf16(void* y, const void* x, const void*
 // Decode-step products with their follow-up fused in, for at most 16 rows of x:
 //
 // ptl_gate_up_silu_bf16:  out[m, c] = act(x . Wg[c]) * (x . Wu[c])   (W = [Wg; Wu], [2I, K]; act SiLU or
-//     the tanh form of GELU)
+//     the tanh form of GELU; or the clamped form, see glu)
 // ptl_qkv_rope_store_bf16: q, k, v = x . Wqkv^T; q and k rotated by the angles
 //     positions[m] * inv_freq[j] on the pairs (j, j + D/2); q written out, the
 //     rotated k and v written into the cache pages at slots[m].
@@ -494,7 +520,7 @@ template <int MODE, int U, int ROWS, int XR, bool BLOCKED>
 __global__ void __launch_bounds__(1024)
 gemm_pair_kernel(bf16_t* __restrict__ y, const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
                  int M, int N_out, int K, long ldx, long ldy, int k_per_wave, int pair_offset,
-                 int tiles_per_group, int group_rows, RopeStoreArgs rs, RowScaleArgs sc, int act) {
+                 int tiles_per_group, int group_rows, RopeStoreArgs rs, RowScaleArgs sc, GluArgs act) {
   extern __shared__ float red[];                 // [waves][2][64][4]
   __shared__ float row_factor[16];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, ln = lane & 15, lg = lane >> 4;
@@ -613,7 +639,7 @@ gemm_pair_kernel(bf16_t* __restrict__ y, const bf16_t* __restrict__ x, const bf1
     for (int i = 0; i < 4; ++i) {
       // the gate and up products are rounded to bfloat16 as the unfused path stores them
       const float g = round_to<bf16_t>(acc1[i]), u = round_to<bf16_t>(acc2[i]);
-      o.e[i] = float_to_bf16(glu_act(act, g) * u);
+      o.e[i] = float_to_bf16(glu(act, g, u));
     }
     const int c0 = r1 + 4 * lg;
     if ((N_out & 3) == 0 && (ldy & 3) == 0 && (reinterpret_cast<uintptr_t>(y) & 7) == 0) {
@@ -667,9 +693,9 @@ static int pair_waves(int blocks, int K) {
 // w_blocked: as for ptl_gemm_skinny_bf16
 extern "C" int ptl_gate_up_silu_bf16(void* out, const void* x, const void* w, int w_blocked, int M, int I,
                                      int K, long ldx, const float* partials, int n_partials, float eps,
-                                     int act, hipStream_t stream) {
+                                     int act, float limit, hipStream_t stream) {
   if (M <= 0 || I <= 0) return PTL_OK;
-  if ((act != GLU_SILU && act != GLU_GELU_TANH) || M > 16 || I % 16 || K <= 0 || K % 8 || ldx % 8 || ldx < K || (partials && n_partials <= 0) ||
+  if (!glu_ok(act) || M > 16 || I % 16 || K <= 0 || K % 8 || ldx % 8 || ldx < K || (partials && n_partials <= 0) ||
       (w_blocked && K % 32))
     return PTL_ERR_ARG;
   const RowScaleArgs sc = {partials, n_partials, 1.0f / (float)K, eps};
@@ -680,7 +706,7 @@ extern "C" int ptl_gate_up_silu_bf16(void* out, const void* x, const void* w, in
   RopeStoreArgs none = {};
 #define GO1(XR, BL)                                                                                   \
   gemm_pair_kernel<PAIR_SILU, 8, 16, XR, BL><<<blocks, waves * 64, lds, stream>>>(                    \
-      (bf16_t*)out, (const bf16_t*)x, (const bf16_t*)w, M, I, K, ldx, I, k_per_wave, I, blocks, 0, none, sc, act)
+      (bf16_t*)out, (const bf16_t*)x, (const bf16_t*)w, M, I, K, ldx, I, k_per_wave, I, blocks, 0, none, sc, GluArgs{act, limit})
 #define GO(XR) if (w_blocked) GO1(XR, true); else GO1(XR, false)
   switch (gs_rows_of(M)) {
     case 4: GO(4); break;
@@ -716,7 +742,7 @@ extern "C" int ptl_qkv_rope_store_bf16(void* q_out, long ldq, const void* x, con
 #define GO1(ROWS, XR, BL)                                                                             \
   gemm_pair_kernel<PAIR_ROPE, 8, ROWS, XR, BL><<<blocks, waves * 64, lds, stream>>>(                  \
       (bf16_t*)q_out, (const bf16_t*)x, (const bf16_t*)w, M, Hq * D, K, ldx, ldq, k_per_wave, D / 2,  \
-      tiles, D, rs, sc, 0)
+      tiles, D, rs, sc, GluArgs{})
 #define GO(ROWS, XR) if (w_blocked) GO1(ROWS, XR, true); else GO1(ROWS, XR, false)
 #define BY_ROWS(ROWS)                                                                                 \
   switch (gs_rows_of(M)) {                                                                            \

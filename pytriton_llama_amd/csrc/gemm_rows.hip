@@ -6,7 +6,7 @@
 //   ptl_rows_sum_add_rmsnorm  sum of those partial sums + residual + RMSNorm (whole rows)
 //   ptl_rows_sum_rope_store   sum of the partial sums of a q | k | v projection, rotation of q
 //                             and k, k and v into the cache pages
-//   ptl_rows_gate_up_silu     act(x Wg^T) * (x Wu^T), act SiLU or the tanh form of GELU
+//   ptl_rows_gate_up_silu     act(x Wg^T) * (x Wu^T), act SiLU or the tanh form of GELU; or the clamped form
 // The reference runs these products through cuBLAS and the rest as kernels of their own
 // (lite_llama/models/llama.py:37-40,120, lite_llama/kernels/rope_emb.py, swiglu.py,
 // skip_rmsnorm.py).
@@ -80,7 +80,7 @@ template <int MT, int KC, int DEPTH, int WT, int MODE, typename TY>
 __global__ void __launch_bounds__((4 / WT + 1) * 64)
 gemm_rows_kernel(TY* __restrict__ y, const bf16_t* __restrict__ x, const bf16_t* __restrict__ wb,
                  int M, int N_out, int w_rows, int K, long ldx, long ldy, int k_per_split,
-                 int pair_offset, int act) {
+                 int pair_offset, GluArgs act) {
   constexpr int FRAGS = KC / 32;                 // weight fragments a wave and chunk
   constexpr int PIECES = KC / 8;                 // 16-byte pieces of a row of a chunk of x
   constexpr int XI = MT * 16 * PIECES / 64;      // load instructions that bring a chunk of x
@@ -285,7 +285,7 @@ gemm_rows_kernel(TY* __restrict__ y, const bf16_t* __restrict__ x, const bf16_t*
         for (int i = 0; i < 4; ++i) {
           // the gate and up products are rounded to bfloat16 as the unfused path stores them
           const float gt = round_to<bf16_t>(acc[j][t][i]), u = round_to<bf16_t>(up[i]);
-          o.e[i] = float_to_bf16(glu_act(act, gt) * u);
+          o.e[i] = float_to_bf16(glu(act, gt, u));
         }
         bf16_t* at = out + (size_t)m * ldy + c0;
         if ((ldy & 3) == 0 && (reinterpret_cast<uintptr_t>(out) & 7) == 0) {
@@ -320,7 +320,7 @@ int compute_units() {
 
 template <int MT, int KC, int DEPTH, int WT, int MODE, typename TY>
 int launch(void* y, const void* x, const void* wb, int M, int N_out, int w_rows, int K, long ldx, long ldy,
-           int blocks, int splits, int pair_offset, hipStream_t stream, int act = GLU_SILU) {
+           int blocks, int splits, int pair_offset, hipStream_t stream, GluArgs act = {GLU_SILU, 0.f}) {
   const size_t lds = (size_t)NB * MT * 16 * KC * sizeof(bf16_t);
   auto kernel = gemm_rows_kernel<MT, KC, DEPTH, WT, MODE, TY>;
   static bool raised = false;                  // (per instantiation)
@@ -396,11 +396,11 @@ extern "C" int ptl_rows_gemm_bf16(void* y, const void* x, const void* w_blocked,
 // out [M, I] = act(x Wg^T) * (x Wu^T) for W = [Wg; Wu] of shape [2 I, K] given as its blocked
 // copy; I % 32 == 0.
 extern "C" int ptl_rows_gate_up_silu(void* out, const void* x, const void* w_blocked, int M, int I, int K,
-                                     long ldx, int act, hipStream_t stream) {
+                                     long ldx, int act, float limit, hipStream_t stream) {
   if (I <= 0 || M == 0) return PTL_OK;
-  if (bad_common(M, K, ldx) || I % 32 || (act != GLU_SILU && act != GLU_GELU_TANH)) return PTL_ERR_ARG;
+  if (bad_common(M, K, ldx) || I % 32 || !glu_ok(act)) return PTL_ERR_ARG;
   const int blocks = I / 32;
-#define GO(MT, KC, DEPTH) launch<MT, KC, DEPTH, 1, MODE_SILU, bf16_t>(out, x, w_blocked, M, I, 2 * I, K, ldx, I, blocks, 1, I, stream, act)
+#define GO(MT, KC, DEPTH) launch<MT, KC, DEPTH, 1, MODE_SILU, bf16_t>(out, x, w_blocked, M, I, 2 * I, K, ldx, I, blocks, 1, I, stream, GluArgs{act, limit})
   switch (m_tiles(M)) {
     case 1: return GO(1, KC_1, DEPTH_1);
     case 2: return GO(2, KC_2, DEPTH_2);

@@ -2,30 +2,40 @@
 //
 //   S_t = diag(a_t) S_(t-1) + k_t v_t^T,     o_t = S_t^T q_t
 //
-// in two forms:
+// in three forms:
 //   MODE_SCALAR   one decay a head and token, a_t = exp(-exp(A_log) dt_t) with dt_t = softplus(raw +
 //                 bias); the value is dt_t v_t and skip v_t is added to the result: the state-space
 //                 duality of Mamba-2 (Dao, Gu: "Transformers are SSMs: Generalized Models and
 //                 Efficient Algorithms Through Structured State Space Duality") with S = state^T
 //   MODE_CHANNEL  a decay a key channel, a_t[d] in (0, 1]: gated linear attention (Yang, Wang, Shen,
 //                 Panda, Kim: "Gated Linear Attention Transformers with Hardware-Efficient Training")
+//   MODE_BONUS    the same decays, with a read-out in front of the update and a factor on the current
+//                 token's own product: o_t = (S_(t-1) + diag(u) k_t v_t^T)^T q_t, u [H, D]: the time
+//                 mixer of RWKV-6 (Peng et al.: "Eagle and Finch: RWKV with Matrix-Valued States and
+//                 Dynamic Recurrence")
 // Everything is float32. Query head h uses q/k head h / heads_per_qk. S lives in the request's state
 // slot as [H][Dv][DS] floats (a column of S after the other, DS = D rounded up to a multiple of 4).
 //
-// ptl_linear_decode_conv, ptl_linear_decode_lowrank: sequences of one token. A workgroup takes 16 to 64
+// ptl_linear_decode_conv, ptl_linear_decode_lowrank, ptl_linear_decode_bonus: sequences of one token. A workgroup takes 16 to 64
 //   columns of a head of a sequence, a column in 16 lanes (one row of a wave for the data-parallel lane moves); what is in front of the
 //   recurrence is done by the workgroup itself: the short causal convolution with SiLU (scalar form)
-//   or the low-rank decays (channel form). Bound by reading and writing S once.
+//   or the low-rank decays (channel and bonus forms). Bound by reading and writing S once.
 // ptl_linear_scan: portions. The rows of a sequence are walked in chunks of 32 tokens whose products
 //   run on the matrix cores in float32 (v_mfma_f32_16x16x4_f32):
 //     P[t, s] = sum_d q_t[d] k_s[d] a(s, t)[d]      s <= t, a(s, t) the decays of tokens s + 1 .. t
 //     O[t, :] = sum_s P[t, s] v_s + sum_d q_t[d] a(start, t)[d] S[d, :]
 //     S[d, :] = a(start, end)[d] S[d, :] + sum_s a(s, end)[d] k_s[d] v_s
+//   (bonus form: the read-outs of token t take the decays up to t - 1 only, and P[t, t] takes u)
 //   A workgroup of four waves takes 64 columns of a head; a wave keeps its 16 columns of S in the
 //   accumulators of the last product, which is also how the middle product wants them as an operand.
 //   Long sequences are cut into segments that are walked side by side: a local pass (what every
 //   segment makes of a zero state), a combine (the segments' start states) and the final pass.
-// ptl_lowrank_decay: a[t, c] = sigmoid(W2[c, :] . r_t + b[c])^(1 / tau) for all rows of a step.
+// ptl_lowrank_decay: the decays of all rows of a step, with z = W2[c, :] . f(r_t) + b[c]:
+//   DECAY_SIGMOID   a[t, c] = sigmoid(z)^(1 / tau), f the identity
+//   DECAY_EXP       a[t, c] = exp(-exp(z)), f = tanh
+// ptl_time_shift: the inputs of a time mixer, out[j, t, :] = x_t + (x_(t-1) - x_t) mu[j, :] for several
+//   mu at once; the row before a portion's first lies in the state slot (the scan and decode kernels
+//   that follow leave the portion's last row there: ShiftArgs).
 //
 // Decays between tokens are never formed as quotients or differences of large numbers: in the scalar
 // form the logarithms are summed in double, in the channel form products of decays are taken inside
@@ -35,6 +45,9 @@
 
 #define MODE_SCALAR 0
 #define MODE_CHANNEL 1
+#define MODE_BONUS 2
+#define DECAY_SIGMOID 0
+#define DECAY_EXP 1
 #define QC 32                // tokens of a chunk
 #define XLD 68               // row stride of the values in LDS
 #define PLD 36               // row stride of P in LDS
@@ -60,6 +73,25 @@ __device__ __forceinline__ float sigmoid_power(float z, float p) {
   return __builtin_amdgcn_exp2f(-p * l);
 }
 
+__device__ __forceinline__ float decay_in(int form, float r) { return form == DECAY_EXP ? tanhf(r) : r; }
+__device__ __forceinline__ float decay_of(int form, float z, float inv_tau) {
+  return form == DECAY_EXP ? expf(-expf(z)) : sigmoid_power(z, inv_tau);
+}
+
+// The last row of x that a sequence brings, kept as float32 [W] at ``off`` of its state slot (x null:
+// nothing is kept). Part ``part`` of ``parts`` of the row, 256 threads.
+struct ShiftArgs {
+  const void* x; long ldx; int dtype;
+  long off;
+  int W;
+};
+__device__ __forceinline__ void keep_row(const ShiftArgs& s, float* slot, size_t row, int part, int parts) {
+  const int per = (s.W + parts - 1) / parts;
+  for (int c = part * per + threadIdx.x; c < min(s.W, (part + 1) * per); c += 256)
+    slot[s.off + c] = s.dtype == PTL_DTYPE_F32 ? ((const float*)s.x)[row * s.ldx + c]
+                                               : bf16_to_float(((const bf16_t*)s.x)[row * s.ldx + c]);
+}
+
 struct LinArgs {
   float* out;                                     // [T, H, Dv]
   const float* q; long ldq;                       // q[t * ldq + g * D + d]
@@ -74,6 +106,8 @@ struct LinArgs {
   const int32_t* q_start; const int32_t* state_slots;
   int H, heads_per_qk, D, DS, Dv;
   int P, seg_len;                                 // segments a sequence at most, tokens of one
+  const float* bonus;                             // bonus: [H, D]
+  ShiftArgs shift;
 };
 
 // floats of one segment's work area: S, and its decays (one a head, or one a key channel)
@@ -85,9 +119,9 @@ __host__ __device__ static inline size_t work_floats(const LinArgs& A, int mode)
 template <int NDT, int MODE, bool FINAL>
 constexpr size_t chunk_lds_floats() {
   constexpr size_t rows = (size_t)QC * (16 * NDT + 4);
-  return rows * (1 + (FINAL ? 1 : 0) + (MODE == MODE_CHANNEL ? 1 : 0)) + (size_t)QC * XLD +
-         (FINAL ? (size_t)QC * PLD : 0) + (MODE == MODE_CHANNEL && FINAL ? (size_t)QC * 20 : 0) +
-         (MODE == MODE_CHANNEL ? 2 * 16 * NDT : 2 * 5 * QC);
+  return rows * (1 + (FINAL ? 1 : 0) + (MODE != MODE_SCALAR ? 1 : 0)) + (size_t)QC * XLD +
+         (FINAL ? (size_t)QC * PLD : 0) + (MODE != MODE_SCALAR && FINAL ? (size_t)QC * 20 : 0) +
+         (MODE != MODE_SCALAR ? 2 * 16 * NDT : 2 * 5 * QC) + (MODE == MODE_BONUS ? 16 * NDT : 0);
 }
 
 // workgroups a compute unit that the registers are shared out for (one where S takes many of them)
@@ -95,6 +129,8 @@ constexpr int chunk_workgroups(int ndt, bool final) { return ndt > 8 && final ? 
 
 template <int NDT, int MODE, bool FINAL>
 __global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chunk_kernel(LinArgs A, int vec) {
+  constexpr bool CHANNEL = MODE != MODE_SCALAR;      // a decay a key channel
+  constexpr bool BONUS = MODE == MODE_BONUS;
   constexpr int DP = 16 * NDT;              // key channels, padded
   constexpr int LD = DP + 4;                // row stride of q, k and the decays in LDS
   constexpr int NQ = DP / 4;                // float4 of a row
@@ -102,14 +138,15 @@ __global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chun
   float* Ks = lds;                                              // [QC][LD]
   float* Qs = Ks + QC * LD;                                     // FINAL: [QC][LD]
   float* As = Qs + (FINAL ? QC * LD : 0);                       // channel: [QC][LD]
-  float* Xs = As + (MODE == MODE_CHANNEL ? QC * LD : 0);        // [QC][XLD]
+  float* Xs = As + (CHANNEL ? QC * LD : 0);        // [QC][XLD]
   float* Ps = Xs + QC * XLD;                                    // FINAL: [QC][PLD]
   float* Pd = Ps + (FINAL ? QC * PLD : 0);                      // channel, FINAL: [QC][20], second halves of the
                                                                 // sums over d of the two diagonal tiles
-  float* tot = Pd + (MODE == MODE_CHANNEL && FINAL ? QC * 20 : 0);   // channel: [2][DP]
+  float* tot = Pd + (CHANNEL && FINAL ? QC * 20 : 0);   // channel: [2][DP]
   // scalar, twice (this chunk's and the next one's): [QC] each of the sums of the log decays from the
   // chunk's start, the step sizes, the decays from the chunk's start, the step sizes x decays to its end
   double* cums = reinterpret_cast<double*>(tot);
+  float* bon = tot + 2 * DP;                                    // bonus: [DP]
   float* dtss = reinterpret_cast<float*>(cums + 2 * QC);
   float* ess = dtss + 2 * QC;
   float* wss = ess + 2 * QC;
@@ -151,7 +188,7 @@ __global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chun
   // The rows of the next chunk are on their way from global memory into registers while the current
   // one is worked on from LDS: a thread holds NR float4 of k (and of q and the decays) and two of v.
   constexpr int NR = (QC * NQ + 255) / 256;
-  f32x4_t fk[NR], fq[FINAL ? NR : 1], fa[MODE == MODE_CHANNEL ? NR : 1], fv[2];
+  f32x4_t fk[NR], fq[FINAL ? NR : 1], fa[CHANNEL ? NR : 1], fv[2];
   float fdt = 0.f;                          // scalar: a token's raw step size
   auto fetch4 = [&](const float* p, int col, int most) {
     f32x4_t x = {0.f, 0.f, 0.f, 0.f};
@@ -173,7 +210,7 @@ __global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chun
       const bool in = r < steps && d < D;
       fk[n] = in ? fetch4(A.k + row * A.ldk + g * D, d, D) : zero;
       if (FINAL) fq[n] = in ? fetch4(A.q + row * A.ldq + g * D, d, D) : zero;
-      if (MODE == MODE_CHANNEL) fa[n] = in ? fetch4(A.decay + row * A.lda + h * D, d, D) : zero;
+      if (CHANNEL) fa[n] = in ? fetch4(A.decay + row * A.lda + h * D, d, D) : zero;
     }
 #pragma unroll
     for (int n = 0; n < 2; ++n) {
@@ -190,7 +227,7 @@ __global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chun
       *reinterpret_cast<f32x4_t*>(Ks + r * LD + d) = fk[n];
       if (FINAL) *reinterpret_cast<f32x4_t*>(Qs + r * LD + d) = fq[n] * A.qscale;
       // (rows past the end: zeros; their decay is taken as one where it matters, below)
-      if (MODE == MODE_CHANNEL) *reinterpret_cast<f32x4_t*>(As + r * LD + d) = fa[n];
+      if (CHANNEL) *reinterpret_cast<f32x4_t*>(As + r * LD + d) = fa[n];
     }
 #pragma unroll
     for (int n = 0; n < 2; ++n) {
@@ -222,6 +259,9 @@ __global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chun
     }
   };
 
+  if (BONUS) {
+    for (int d = tid; d < DP; d += 256) bon[d] = d < D ? A.bonus[(size_t)h * D + d] : 0.f;
+  }
   fetch(t_begin);
   fetch_dt(t_begin);
   if (scalar_wave) scalars(t_begin, 0);
@@ -240,9 +280,9 @@ __global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chun
       fetch_dt(t0 + 2 * QC);
     }
 
-    if (MODE == MODE_CHANNEL) {
+    if (CHANNEL) {
       // The two diagonal tiles: lane (t, lg) walks s from t down, w = q_t times the decays of
-      // s + 1 .. t; wave w takes tile w % 2 and half of the key channels, a lane every fourth float4.
+      // s + 1 .. t (bonus: of s + 1 .. t - 1 from s = t - 1 on, and q_t times u at s = t); wave w takes tile w % 2 and half of the key channels, a lane every fourth float4.
       if (FINAL) {
         const int base = 16 * (wave & 1), half = wave >> 1;
         float acc[16];
@@ -250,13 +290,15 @@ __global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chun
         for (int s = 0; s < 16; ++s) acc[s] = 0.f;
         for (int qd = half * (NQ / 2) + lg; qd < (half + 1) * (NQ / 2); qd += 4) {
           const f32x4_t qt = *reinterpret_cast<const f32x4_t*>(Qs + (base + ln) * LD + 4 * qd);
-          f32x4_t w = {0.f, 0.f, 0.f, 0.f};
+          f32x4_t w = {0.f, 0.f, 0.f, 0.f}, own = w;
+          if (BONUS) own = qt * *reinterpret_cast<const f32x4_t*>(bon + 4 * qd);
 #pragma unroll
           for (int s = 15; s >= 0; --s) {
             if (s < 15) w *= *reinterpret_cast<const f32x4_t*>(As + (base + s + 1) * LD + 4 * qd);
-            if (s == ln) w = qt;
+            if (s + (BONUS ? 1 : 0) == ln) w = qt;
+            const f32x4_t x = BONUS && s == ln ? own : w;
             const f32x4_t ks = *reinterpret_cast<const f32x4_t*>(Ks + (base + s) * LD + 4 * qd);
-            acc[s] += (w[0] * ks[0] + w[1] * ks[1]) + (w[2] * ks[2] + w[3] * ks[3]);
+            acc[s] += (x[0] * ks[0] + x[1] * ks[1]) + (x[2] * ks[2] + x[3] * ks[3]);
           }
         }
 #pragma unroll
@@ -273,7 +315,8 @@ __global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chun
         else *reinterpret_cast<f32x4_t*>(Pd + (base + ln) * 20 + 4 * lg) = mine;
         __syncthreads();
       }
-      // q_t times the decays from the start of its block of 16, k_s times those to the block's end
+      // q_t times the decays from the start of its block of 16 (bonus: without its own), k_s times those
+      // to the block's end
       for (int i = tid; i < 2 * DP; i += 256) {
         const int b = i / DP, d = i - b * DP;
         float* a = As + 16 * b * LD + d;
@@ -282,8 +325,9 @@ __global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chun
           float* q = Qs + 16 * b * LD + d;
 #pragma unroll
           for (int t = 0; t < 16; ++t) {
+            if (BONUS) q[t * LD] *= e;
             e *= 16 * b + t < steps ? a[t * LD] : 1.f;
-            q[t * LD] *= e;
+            if (!BONUS) q[t * LD] *= e;
           }
         }
         float f = 1.f;
@@ -327,7 +371,7 @@ __global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chun
         for (int dt = 0; dt < NDT; ++dt) {
           const f32x4_t q0 = *reinterpret_cast<const f32x4_t*>(Qs + ln * LD + 16 * dt + 4 * lg);
           f32x4_t q1 = *reinterpret_cast<const f32x4_t*>(Qs + (16 + ln) * LD + 16 * dt + 4 * lg);
-          if (MODE == MODE_CHANNEL) q1 *= *reinterpret_cast<const f32x4_t*>(tot + 16 * dt + 4 * lg);
+          if (CHANNEL) q1 *= *reinterpret_cast<const f32x4_t*>(tot + 16 * dt + 4 * lg);
 #pragma unroll
           for (int m = 0; m < 4; ++m) {
             O[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(q0[m], S[dt][m], O[0], 0, 0, 0);
@@ -346,7 +390,7 @@ __global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chun
 #pragma unroll
           for (int ts = 0; ts <= tt; ++ts) {
             f32x4_t pa = *reinterpret_cast<const f32x4_t*>(Ps + (16 * tt + ln) * PLD + 16 * ts + 4 * lg);
-            if (MODE == MODE_CHANNEL && ts == tt) pa += *reinterpret_cast<const f32x4_t*>(Pd + (16 * tt + ln) * 20 + 4 * lg);
+            if (CHANNEL && ts == tt) pa += *reinterpret_cast<const f32x4_t*>(Pd + (16 * tt + ln) * 20 + 4 * lg);
 #pragma unroll
             for (int m = 0; m < 4; ++m)
               O[tt] = __builtin_amdgcn_mfma_f32_16x16x4f32(pa[m], Xs[(16 * ts + 4 * lg + m) * XLD + 16 * wave + ln], O[tt], 0, 0, 0);
@@ -384,13 +428,13 @@ __global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chun
         }
         float f[NDT];                       // channel: the second block's decays on top of the first's
 #pragma unroll
-        for (int dt = 0; dt < NDT; ++dt) f[dt] = MODE == MODE_CHANNEL && ts == 0 ? tot[DP + 16 * dt + ln] : 1.f;
+        for (int dt = 0; dt < NDT; ++dt) f[dt] = CHANNEL && ts == 0 ? tot[DP + 16 * dt + ln] : 1.f;
 #pragma unroll
         for (int m = 0; m < 4; ++m) {
 #pragma unroll
           for (int dt = 0; dt < NDT; ++dt) {
             float ka = Ks[(16 * ts + 4 * lg + m) * LD + 16 * dt + ln];
-            if (MODE == MODE_CHANNEL && ts == 0) ka *= f[dt];
+            if (CHANNEL && ts == 0) ka *= f[dt];
             S[dt] = __builtin_amdgcn_mfma_f32_16x16x4f32(ka, x[m], S[dt], 0, 0, 0);
           }
         }
@@ -410,6 +454,9 @@ __global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chun
       if (live && d < DS) *reinterpret_cast<f32x4_t*>(column(to) + d) = S[dt];
     }
   }
+  // (the rows' inputs were made from the old kept row by a kernel in front of this one)
+  if (FINAL && seg == nseg - 1 && A.shift.x)
+    keep_row(A.shift, slot, (size_t)(row0 + qlen - 1), blockIdx.y * gridDim.x + blockIdx.x, gridDim.x * gridDim.y);
   if (!FINAL && blockIdx.x == 0) {
     float* decays = work_at(seg + 1) + (size_t)A.H * Dv * DS;
     if (MODE == MODE_SCALAR) {
@@ -480,21 +527,24 @@ static int launch_chunks(const LinArgs& A, int vec, int n_seqs, hipStream_t st) 
 
 template <int MODE>
 static int launch_scan(const LinArgs& A, int n_seqs, hipStream_t st) {
+  constexpr int LOCAL = MODE == MODE_SCALAR ? MODE_SCALAR : MODE_CHANNEL;      // (what does not read out)
   if (A.D <= 0 || A.D > 256 || A.Dv <= 0 || A.H <= 0 || A.H > 65535 || A.heads_per_qk <= 0 ||
       A.H % A.heads_per_qk || A.P < 1 || (long)n_seqs * A.P > 65535 || A.seg_len < 1 || (A.P > 1 && !A.work) ||
       A.slot_stride < (long)A.H * A.Dv * A.DS || A.slot_stride % 4 || ((uintptr_t)A.state & 15) ||
       ((uintptr_t)A.work & 15))
     return PTL_ERR_ARG;
   auto aligned = [](const float* p, long ld) { return ld % 4 == 0 && ((uintptr_t)p & 15) == 0; };
+  if (A.shift.x && (A.shift.W <= 0 || A.shift.off < (long)A.H * A.Dv * A.DS || A.shift.off + A.shift.W > A.slot_stride))
+    return PTL_ERR_ARG;
   const int vec = A.D % 4 == 0 && A.Dv % 4 == 0 && aligned(A.q, A.ldq) && aligned(A.k, A.ldk) && aligned(A.v, A.ldv) &&
                   (MODE == MODE_SCALAR || aligned(A.decay, A.lda));
   const int tiles = (A.D + 15) / 16;
 #define GO(N)                                                                                      \
   if (tiles <= N) {                                                                                \
     if (A.P > 1) {                                                                                 \
-      if (int e = launch_chunks<N, MODE, false>(A, vec, n_seqs, st)) return e;                     \
+      if (int e = launch_chunks<N, LOCAL, false>(A, vec, n_seqs, st)) return e;                    \
       const size_t quads = (size_t)A.H * A.Dv * (A.DS / 4);                                        \
-      linear_combine_kernel<MODE><<<dim3((unsigned)((quads + 255) / 256), n_seqs), 256, 0, st>>>(A); \
+      linear_combine_kernel<LOCAL><<<dim3((unsigned)((quads + 255) / 256), n_seqs), 256, 0, st>>>(A); \
       if (int e = ptl_launch_status()) return e;                                                   \
     }                                                                                              \
     return launch_chunks<N, MODE, true>(A, vec, n_seqs, st);                                       \
@@ -512,34 +562,40 @@ extern "C" long ptl_linear_work_floats(int mode, int n_seqs, int P, int H, int D
 }
 
 // Portions of n_seqs sequences. mode 0 (scalar): dt, A_log, dt_bias, skip; mode 1
-// (channel): decay. P: the most segments of seg_len rows that one of the sequences has.
+// (channel): decay; mode 2 (bonus): decay and bonus. P: the most segments of seg_len rows that one of the
+// sequences has. shift_x (or null): [T, ldx] of shift_dtype, whose row of every sequence's last token is
+// left in the sequence's slot (ShiftArgs).
 extern "C" int ptl_linear_scan(int mode, float* out, const float* q, long ldq, const float* k, long ldk,
                                const float* v, long ldv, float qscale, const float* dt, long ldt,
                                const float* A_log, const float* dt_bias, const float* skip, const float* decay,
-                               long lda, float* state, long slot_stride, float* work, int P, int seg_len,
-                               const int32_t* q_start, const int32_t* state_slots, int n_seqs, int H,
+                               long lda, const float* bonus, const void* shift_x, long shift_ldx, int shift_dtype,
+                               long shift_off, int shift_W, float* state, long slot_stride, float* work, int P,
+                               int seg_len, const int32_t* q_start, const int32_t* state_slots, int n_seqs, int H,
                                int G, int D, int Dv, hipStream_t st) {
   if (n_seqs <= 0) return PTL_OK;
   if (G <= 0 || H % G) return PTL_ERR_ARG;
   LinArgs A{out, q, ldq, k, ldk, v, ldv, qscale, dt, ldt, A_log, dt_bias, skip, decay, lda, state, slot_stride, work,
-            q_start, state_slots, H, H / G, D, (D + 3) / 4 * 4, Dv, P, seg_len};
+            q_start, state_slots, H, H / G, D, (D + 3) / 4 * 4, Dv, P, seg_len, bonus,
+            ShiftArgs{shift_x, shift_ldx, shift_dtype, shift_off, shift_W}};
   if (mode == MODE_SCALAR) {
     if (!dt || !A_log || !dt_bias || !skip) return PTL_ERR_ARG;
     return launch_scan<MODE_SCALAR>(A, n_seqs, st);
   }
-  if (mode != MODE_CHANNEL || !decay) return PTL_ERR_ARG;
+  if (!decay) return PTL_ERR_ARG;
+  if (mode == MODE_BONUS) return bonus ? launch_scan<MODE_BONUS>(A, n_seqs, st) : PTL_ERR_ARG;
+  if (mode != MODE_CHANNEL) return PTL_ERR_ARG;
   return launch_scan<MODE_CHANNEL>(A, n_seqs, st);
 }
 
 // ---- the low-rank decays of all rows ---------------------------------------------------------------
 // grid (blocks of 256 channels, blocks of DECAY_ROWS rows): a thread keeps its channel's row of W2 in
-// registers (up to 32 entries; a longer one is read again for every row), the rows of r go through LDS,
+// registers (up to 64 entries; a longer one is read again for every row), the rows of r go through LDS,
 // four entries a read
 #define DECAY_ROWS 8
 template <int RM>
 __global__ void __launch_bounds__(256)
 lowrank_decay_kernel(float* __restrict__ out, const float* __restrict__ r, long ldr, const float* __restrict__ w,
-                     const float* __restrict__ b, float inv_tau, int T, int C, int R, int RP) {
+                     const float* __restrict__ b, int form, float inv_tau, int T, int C, int R, int RP) {
   extern __shared__ __attribute__((aligned(16))) float rs[];       // [DECAY_ROWS][RP], zeros from R on
   const int t0 = blockIdx.y * DECAY_ROWS, rows = min(DECAY_ROWS, T - t0);
   const int c = blockIdx.x * 256 + threadIdx.x;
@@ -552,7 +608,7 @@ lowrank_decay_kernel(float* __restrict__ out, const float* __restrict__ r, long 
   const float bias = b[min(c, C - 1)];
   for (int i = threadIdx.x; i < rows * RP; i += 256) {
     const int t = i / RP, j = i - t * RP;
-    rs[i] = j < R ? r[(size_t)(t0 + t) * ldr + j] : 0.f;
+    rs[i] = j < R ? decay_in(form, r[(size_t)(t0 + t) * ldr + j]) : 0.f;
   }
   __syncthreads();
   if (c >= C) return;
@@ -562,7 +618,7 @@ lowrank_decay_kernel(float* __restrict__ out, const float* __restrict__ r, long 
     if (RM > 0) {
 #pragma unroll
       for (int j = 0; j < RM; j += 4) {
-        if (j >= RP) break;
+        if (j >= RP) continue;
         const f32x4_t x = *reinterpret_cast<const f32x4_t*>(rr + j);
 #pragma unroll
         for (int i = 0; i < 4; ++i) z = fmaf(wv[j + i], x[i], z);
@@ -570,20 +626,21 @@ lowrank_decay_kernel(float* __restrict__ out, const float* __restrict__ r, long 
     } else {
       for (int j = 0; j < R; ++j) z = fmaf(wr[j], rr[j], z);
     }
-    out[(size_t)(t0 + t) * C + c] = sigmoid_power(z, inv_tau);
+    out[(size_t)(t0 + t) * C + c] = decay_of(form, z, inv_tau);
   }
 }
 
 extern "C" int ptl_lowrank_decay(float* out, const float* r, long ldr, const float* w, const float* b,
-                                 float inv_tau, int T_, int C, int R, hipStream_t st) {
+                                 int form, float inv_tau, int T_, int C, int R, hipStream_t st) {
   if (T_ <= 0) return PTL_OK;
   const int RP = (R + 3) / 4 * 4;
   const size_t lds = (size_t)DECAY_ROWS * RP * sizeof(float);
-  if (C <= 0 || R <= 0 || lds > 48 * 1024 || (T_ + DECAY_ROWS - 1) / DECAY_ROWS > 65535) return PTL_ERR_ARG;
+  if (C <= 0 || R <= 0 || lds > 48 * 1024 || (form != DECAY_SIGMOID && form != DECAY_EXP) || (T_ + DECAY_ROWS - 1) / DECAY_ROWS > 65535) return PTL_ERR_ARG;
   const dim3 grid((C + 255) / 256, (T_ + DECAY_ROWS - 1) / DECAY_ROWS);
-  if (R <= 16) lowrank_decay_kernel<16><<<grid, 256, lds, st>>>(out, r, ldr, w, b, inv_tau, T_, C, R, RP);
-  else if (R <= 32) lowrank_decay_kernel<32><<<grid, 256, lds, st>>>(out, r, ldr, w, b, inv_tau, T_, C, R, RP);
-  else lowrank_decay_kernel<0><<<grid, 256, lds, st>>>(out, r, ldr, w, b, inv_tau, T_, C, R, RP);
+  if (R <= 16) lowrank_decay_kernel<16><<<grid, 256, lds, st>>>(out, r, ldr, w, b, form, inv_tau, T_, C, R, RP);
+  else if (R <= 32) lowrank_decay_kernel<32><<<grid, 256, lds, st>>>(out, r, ldr, w, b, form, inv_tau, T_, C, R, RP);
+  else if (R <= 64) lowrank_decay_kernel<64><<<grid, 256, lds, st>>>(out, r, ldr, w, b, form, inv_tau, T_, C, R, RP);
+  else lowrank_decay_kernel<0><<<grid, 256, lds, st>>>(out, r, ldr, w, b, form, inv_tau, T_, C, R, RP);
   return ptl_launch_status();
 }
 
@@ -601,15 +658,21 @@ struct DecodeArgs {
   // channel form
   int a_off;
   const float* w2; const float* b2; int R; float inv_tau;          // [H * D, R], [H * D]
+  int form;                                 // DECAY_SIGMOID, DECAY_EXP
   float* state; long slot_stride;
   const int32_t* q_start; const int32_t* state_slots;
   int H, heads_per_qk, D, DS, Dv;
+  const float* bonus;                       // bonus form: [H, D]
+  ShiftArgs shift;
 };
 
 // NB: blocks of 16 columns a workgroup takes (what is in front of the recurrence is then done less often)
 template <int J, int NB, int MODE>
 __global__ void __launch_bounds__(256) linear_decode_kernel(DecodeArgs A) {
-  __shared__ __attribute__((aligned(16))) float ks[64 * J], qs[64 * J], as[MODE == MODE_CHANNEL ? 64 * J : 4], xs[16 * NB];
+  constexpr bool CHANNEL = MODE != MODE_SCALAR, BONUS = MODE == MODE_BONUS;
+  __shared__ __attribute__((aligned(16))) float ks[64 * J], qs[64 * J], as[CHANNEL ? 64 * J : 4], xs[16 * NB];
+  __shared__ __attribute__((aligned(16))) float us[BONUS ? 64 * J : 4];
+  extern __shared__ float rs[];             // channel: [R], the decays' low-rank input
   const int tid = threadIdx.x, cg = tid >> 4, l = tid & 15;
   const int h = blockIdx.y, seq = blockIdx.z, g = h / A.heads_per_qk;
   const int row = A.q_start[seq];
@@ -649,6 +712,7 @@ __global__ void __launch_bounds__(256) linear_decode_kernel(DecodeArgs A) {
     } else if (i < 2 * DP) {
       const int d = i - DP;
       qs[d] = d < D ? value(A.q_off + g * D + d) * A.qscale : 0.f;
+      if (BONUS) us[d] = d < D ? A.bonus[h * D + d] : 0.f;
     } else {
       const int cc = c0 + i - 2 * DP;
       xs[i - 2 * DP] = cc < Dv ? value(A.v_off + h * Dv + cc) : 0.f;
@@ -659,17 +723,18 @@ __global__ void __launch_bounds__(256) linear_decode_kernel(DecodeArgs A) {
     step = softplus_f(p[A.dt_off + h] + A.dt_bias[h]);
     decay = expf(-expf(A.A_log[h]) * step);
   } else {
-    for (int d = tid; d < DP; d += 256) {
-      float a = 1.f;
-      if (d < D) {
-        const int ch = h * D + d;
-        const float* w = A.w2 + (size_t)ch * A.R;
-        const float* r = p + A.a_off;
-        float z = A.b2[ch];
-        for (int j = 0; j < A.R; ++j) z = fmaf(w[j], r[j], z);
-        a = sigmoid_power(z, A.inv_tau);
-      }
-      as[d] = a;
+    for (int j = tid; j < A.R; j += 256) rs[j] = decay_in(A.form, p[A.a_off + j]);
+    __syncthreads();
+    // 256 / (64 J) lanes a key channel share its row of W2
+    constexpr int LPC = J == 1 ? 4 : (J == 2 ? 2 : 1);
+    for (int i = tid; i < DP * LPC; i += 256) {
+      const int d = i / LPC, ch = h * D + min(d, D - 1);
+      const float* w = A.w2 + (size_t)ch * A.R;
+      float z = 0.f;
+      for (int j = i % LPC; j < A.R; j += LPC) z = fmaf(w[j], rs[j], z);
+#pragma unroll
+      for (int o = 1; o < LPC; o <<= 1) z += __shfl_xor(z, o, 64);
+      if (i % LPC == 0) as[d] = d < D ? decay_of(A.form, z + A.b2[ch], A.inv_tau) : 1.f;
     }
   }
   __syncthreads();
@@ -683,23 +748,28 @@ __global__ void __launch_bounds__(256) linear_decode_kernel(DecodeArgs A) {
     for (int j = 0; j < J; ++j) {
       const int d = 4 * (l + 16 * j);
       const f32x4_t k4 = *reinterpret_cast<const f32x4_t*>(ks + d), q4 = *reinterpret_cast<const f32x4_t*>(qs + d);
-      f32x4_t s = S[b][j];
-      if (MODE == MODE_CHANNEL) s *= *reinterpret_cast<const f32x4_t*>(as + d);
+      f32x4_t s = S[b][j], read;
+      if (BONUS) read = s + *reinterpret_cast<const f32x4_t*>(us + d) * k4 * v;
+      if (CHANNEL) s *= *reinterpret_cast<const f32x4_t*>(as + d);
       else s *= decay;
       s += k4 * v;
-      o += (s[0] * q4[0] + s[1] * q4[1]) + (s[2] * q4[2] + s[3] * q4[3]);
+      if (!BONUS) read = s;
+      o += (read[0] * q4[0] + read[1] * q4[1]) + (read[2] * q4[2] + read[3] * q4[3]);
       if (live && d < DS) __builtin_nontemporal_store(s, reinterpret_cast<f32x4_t*>(column(b) + d));
     }
     o = row16_sum(o);
     if (live && l == 0) A.out[((size_t)row * A.H + h) * Dv + c0 + 16 * b + cg] = fmaf(skip, x, o);
   }
+  if (A.shift.x) keep_row(A.shift, slot, (size_t)row, blockIdx.y * gridDim.x + blockIdx.x, gridDim.x * gridDim.y);
 }
 
 template <int MODE>
 static int launch_decode(const DecodeArgs& A, int n_seqs, hipStream_t st) {
   if (A.D <= 0 || A.D > 256 || A.Dv <= 0 || A.H <= 0 || A.H > 65535 || n_seqs > 65535 || A.heads_per_qk <= 0 ||
-      A.slot_stride < (long)A.H * A.Dv * A.DS || A.slot_stride % 4 || ((uintptr_t)A.state & 15))
+      A.slot_stride < (long)A.H * A.Dv * A.DS || A.slot_stride % 4 || ((uintptr_t)A.state & 15) || A.R > 8192 ||
+      (A.shift.x && (A.shift.W <= 0 || A.shift.off < (long)A.H * A.Dv * A.DS || A.shift.off + A.shift.W > A.slot_stride)))
     return PTL_ERR_ARG;
+  const size_t lds = MODE == MODE_SCALAR ? 0 : (size_t)A.R * sizeof(float);
   // as many columns a workgroup as leave about two workgroups a compute unit (of 256)
   const int blocks = (A.Dv + 15) / 16;
   const long all = (long)blocks * A.H * n_seqs;
@@ -707,8 +777,8 @@ static int launch_decode(const DecodeArgs& A, int n_seqs, hipStream_t st) {
   const dim3 grid((blocks + nb - 1) / nb, A.H, n_seqs);
 #define GO(J)                                                                       \
   {                                                                                 \
-    if (nb == 4) linear_decode_kernel<J, 4, MODE><<<grid, 256, 0, st>>>(A);         \
-    else if (nb == 2) linear_decode_kernel<J, 2, MODE><<<grid, 256, 0, st>>>(A);    \
+    if (nb == 4) linear_decode_kernel<J, 4, MODE><<<grid, 256, lds, st>>>(A);       \
+    else if (nb == 2) linear_decode_kernel<J, 2, MODE><<<grid, 256, lds, st>>>(A);  \
     else linear_decode_kernel<J, 1, MODE><<<grid, 256, 0, st>>>(A);                 \
     return ptl_launch_status();                                                     \
   }
@@ -741,6 +811,18 @@ extern "C" int ptl_linear_decode_conv(float* out, const float* p, long ldp, int 
   return launch_decode<MODE_SCALAR>(A, n_seqs, st);
 }
 
+static DecodeArgs lowrank_args(float* out, const float* p, long ldp, int q_off, int k_off, int v_off, int a_off,
+                               float qscale, const float* w2, const float* b2, int R, int form, float inv_tau,
+                               float* state, long slot_stride, const int32_t* q_start, const int32_t* state_slots,
+                               int H, int D, int Dv) {
+  DecodeArgs A{};
+  A.out = out; A.p = p; A.ldp = ldp; A.q_off = q_off; A.k_off = k_off; A.v_off = v_off; A.qscale = qscale;
+  A.a_off = a_off; A.w2 = w2; A.b2 = b2; A.R = R; A.form = form; A.inv_tau = inv_tau;
+  A.state = state; A.slot_stride = slot_stride; A.q_start = q_start; A.state_slots = state_slots;
+  A.H = H; A.heads_per_qk = 1; A.D = D; A.DS = (D + 3) / 4 * 4; A.Dv = Dv;
+  return A;
+}
+
 // The channel form: q, k (H heads of D), v (H of Dv) and the decays' low-rank input r [R] at columns of p;
 // w2 [H * D, R], b2 [H * D].
 extern "C" int ptl_linear_decode_lowrank(float* out, const float* p, long ldp, int q_off, int k_off, int v_off,
@@ -750,10 +832,118 @@ extern "C" int ptl_linear_decode_lowrank(float* out, const float* p, long ldp, i
                                          hipStream_t st) {
   if (n_seqs <= 0) return PTL_OK;
   if (R <= 0 || !w2 || !b2) return PTL_ERR_ARG;
-  DecodeArgs A{};
-  A.out = out; A.p = p; A.ldp = ldp; A.q_off = q_off; A.k_off = k_off; A.v_off = v_off; A.qscale = qscale;
-  A.a_off = a_off; A.w2 = w2; A.b2 = b2; A.R = R; A.inv_tau = inv_tau;
-  A.state = state; A.slot_stride = slot_stride; A.q_start = q_start; A.state_slots = state_slots;
-  A.H = H; A.heads_per_qk = 1; A.D = D; A.DS = (D + 3) / 4 * 4; A.Dv = Dv;
-  return launch_decode<MODE_CHANNEL>(A, n_seqs, st);
+  return launch_decode<MODE_CHANNEL>(lowrank_args(out, p, ldp, q_off, k_off, v_off, a_off, qscale, w2, b2, R,
+                                                  DECAY_SIGMOID, inv_tau, state, slot_stride, q_start, state_slots,
+                                                  H, D, Dv), n_seqs, st);
+}
+
+// The bonus form: as above with decays exp(-exp(w2 . tanh(r) + b2)), bonus [H, D]; the sequences' rows of
+// shift_x [T, ldx] are left in their slots (ShiftArgs).
+extern "C" int ptl_linear_decode_bonus(float* out, const float* p, long ldp, int q_off, int k_off, int v_off,
+                                       int a_off, const float* w2, const float* b2, int R, const float* bonus,
+                                       const void* shift_x, long shift_ldx, int shift_dtype, long shift_off,
+                                       int shift_W, float* state, long slot_stride, const int32_t* q_start,
+                                       const int32_t* state_slots, int n_seqs, int H, int D, int Dv, hipStream_t st) {
+  if (n_seqs <= 0) return PTL_OK;
+  if (R <= 0 || !w2 || !b2 || !bonus) return PTL_ERR_ARG;
+  DecodeArgs A = lowrank_args(out, p, ldp, q_off, k_off, v_off, a_off, 1.f, w2, b2, R, DECAY_EXP, 0.f, state,
+                              slot_stride, q_start, state_slots, H, D, Dv);
+  A.bonus = bonus;
+  A.shift = ShiftArgs{shift_x, shift_ldx, shift_dtype, shift_off, shift_W};
+  return launch_decode<MODE_BONUS>(A, n_seqs, st);
+}
+
+// ---- the inputs of a time mixer ----------------------------------------------------------------------
+// One workgroup a (row, block of 256 x VEC columns); a thread makes all n_mix results of its columns.
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256)
+time_shift_kernel(T* __restrict__ out, long mix_stride, const T* __restrict__ x, long ldx, const float* __restrict__ mu,
+                  int n_mix, const float* __restrict__ state, long slot_stride, long off,
+                  const int32_t* __restrict__ q_start, const int32_t* __restrict__ state_slots, int n_seqs, int W) {
+  const int t = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * VEC;
+  if (c >= W) return;
+  // the sequence of the row (the last one whose first row is not beyond t); a row behind all of them: none
+  int lo = 0, hi = n_seqs;
+  while (lo < hi) {
+    const int mid = (lo + hi + 1) >> 1;
+    if (q_start[mid] <= t) lo = mid; else hi = mid - 1;
+  }
+  float a[VEC], d[VEC];
+  auto read = [&](const T* p, float (&v)[VEC]) {
+    if (VEC == 1) {
+      v[0] = to_float<T>(p[0]);
+    } else if (sizeof(T) == 2) {
+      union { uint4 u; bf16_t e[8]; } r;
+      r.u = *reinterpret_cast<const uint4*>(p);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) v[j] = bf16_to_float(r.e[j]);
+    } else {
+#pragma unroll
+      for (int j = 0; j < VEC; j += 4) {
+        const float4 r = *reinterpret_cast<const float4*>(p + j);
+        v[j] = r.x; v[j + (VEC > 1)] = r.y; v[j + 2 * (VEC > 1)] = r.z; v[j + 3 * (VEC > 1)] = r.w;
+      }
+    }
+  };
+  read(x + (size_t)t * ldx + c, a);
+  if (lo < n_seqs && q_start[lo] < t) {
+    read(x + (size_t)(t - 1) * ldx + c, d);
+  } else {
+    const float* kept = lo < n_seqs ? state + (size_t)state_slots[lo] * slot_stride + off + c : nullptr;
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) d[j] = kept ? kept[j] : 0.f;
+  }
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) d[j] -= a[j];
+  for (int m = 0; m < n_mix; ++m) {
+    const float* f = mu + (size_t)m * W + c;
+    T* o = out + (size_t)m * mix_stride + (size_t)t * W + c;
+    if (VEC == 1) {
+      o[0] = from_float<T>(fmaf(d[0], f[0], a[0]));
+    } else {
+      float ff[VEC];
+#pragma unroll
+      for (int j = 0; j < VEC; j += 4) {
+        const float4 r = *reinterpret_cast<const float4*>(f + j);
+        ff[j] = r.x; ff[j + (VEC > 1)] = r.y; ff[j + 2 * (VEC > 1)] = r.z; ff[j + 3 * (VEC > 1)] = r.w;
+      }
+      if (sizeof(T) == 2) {
+        union { uint4 u; bf16_t e[8]; } r;
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) r.e[j] = float_to_bf16(fmaf(d[j], ff[j], a[j]));
+        *reinterpret_cast<uint4*>(o) = r.u;
+      } else {
+#pragma unroll
+        for (int j = 0; j < VEC; j += 4)
+          *reinterpret_cast<float4*>(o + j) =
+              make_float4(fmaf(d[j], ff[j], a[j]), fmaf(d[j + (VEC > 1)], ff[j + (VEC > 1)], a[j + (VEC > 1)]),
+                          fmaf(d[j + 2 * (VEC > 1)], ff[j + 2 * (VEC > 1)], a[j + 2 * (VEC > 1)]),
+                          fmaf(d[j + 3 * (VEC > 1)], ff[j + 3 * (VEC > 1)], a[j + 3 * (VEC > 1)]));
+      }
+    }
+  }
+}
+
+// out [n_mix, T, W] (mix_stride elements from one mix to the next, rows dense), x [T, ldx] of dtype, mu
+// float32 [n_mix, W]; the kept rows float32 [W] at off of the slots.
+extern "C" int ptl_time_shift(void* out, long mix_stride, const void* x, long ldx, const float* mu, int n_mix,
+                              const float* state, long slot_stride, long off, const int32_t* q_start,
+                              const int32_t* state_slots, int n_seqs, int T_, int W, int dtype, hipStream_t st) {
+  if (T_ <= 0 || n_mix <= 0) return PTL_OK;
+  if (W <= 0 || ldx < W || mix_stride < (long)T_ * W || off < 0 || off + W > slot_stride) return PTL_ERR_ARG;
+  const bool even = W % 8 == 0 && ldx % 8 == 0 && mix_stride % 8 == 0 &&
+                    (((uintptr_t)out | (uintptr_t)x | (uintptr_t)mu) & 15) == 0;
+  auto grid = [&](int vec) { return dim3(T_, (W + 256 * vec - 1) / (256 * vec)); };
+#define GO(T, VEC)                                                                                               \
+  time_shift_kernel<T, VEC><<<grid(VEC), 256, 0, st>>>((T*)out, mix_stride, (const T*)x, ldx, mu, n_mix, state,    \
+                                                       slot_stride, off, q_start, state_slots, n_seqs, W)
+  if (dtype == PTL_DTYPE_F32) {
+    if (even) GO(float, 4); else GO(float, 1);
+  } else if (dtype == PTL_DTYPE_BF16) {
+    if (even) GO(bf16_t, 8); else GO(bf16_t, 1);
+  } else {
+    return PTL_ERR_ARG;
+  }
+#undef GO
+  return ptl_launch_status();
 }

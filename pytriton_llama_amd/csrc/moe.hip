@@ -1,7 +1,7 @@
 // A routed feed-forward (mixture of experts) that never leaves the device, so that a step with
 // one can be recorded as a graph:
 //
-//   ptl_moe_topk      per token: scores = sigmoid(logits) or softmax(logits) in float32, the ``top``
+//   ptl_moe_topk      per token: logits (plus a per-expert bias, when one is given), scores = sigmoid(logits) or softmax(logits) in float32, the ``top``
 //                     largest (by score plus a per-expert correction, when one is given), their
 //                     experts and scores (the score without the correction is the weight, with or
 //                     without a renormalisation over the chosen ones, times a constant); with
@@ -57,8 +57,8 @@ __device__ __forceinline__ float unary_act(int kind, float u) {
 #define SCORE_SOFTMAX 1
 template <int TOPK_PER_LANE>
 __global__ void __launch_bounds__(256)
-moe_topk_kernel(const float* __restrict__ logits, int ld, int T_, int E, int top, int extra,
-                int renormalize, int score_fn, const float* __restrict__ bias, int real, float renorm_eps,
+moe_topk_kernel(const float* __restrict__ logits, int ld, const float* __restrict__ logit_bias, int T_, int E,
+                int top, int extra, int renormalize, int score_fn, const float* __restrict__ bias, int real, float renorm_eps,
                 float wscale, int n_groups, int keep_groups, int32_t* __restrict__ idx,
                 float* __restrict__ wgt, float* __restrict__ extra_out, float* __restrict__ ident_out) {
   __shared__ float choice[4][64 * TOPK_PER_LANE];      // a token's choice scores (groups only)
@@ -66,14 +66,15 @@ moe_topk_kernel(const float* __restrict__ logits, int ld, int T_, int E, int top
   const int lane = threadIdx.x & 63;
   if (t >= T_) return;
   const float* z = logits + (size_t)t * ld;
-  // v: what the choice goes by; sc: the score that becomes the weight. Sigmoid scores without a
-  // correction are chosen by their logits (the same order, and no ties where the sigmoid saturates).
+  // v: what the choice goes by; sc: the score that becomes the weight. Scores without a correction
+  // are chosen by their logits (the same order, and no ties where the sigmoid saturates or the
+  // softmax vanishes).
   float v[TOPK_PER_LANE], sc[TOPK_PER_LANE];
   float zmax = -INFINITY;
 #pragma unroll
   for (int i = 0; i < TOPK_PER_LANE; ++i) {
     const int e = lane + 64 * i;
-    v[i] = e < E ? z[e] : -INFINITY;
+    v[i] = e < E ? z[e] + (logit_bias ? logit_bias[e] : 0.f) : -INFINITY;
     zmax = fmaxf(zmax, v[i]);
   }
   if (score_fn == SCORE_SOFTMAX) {
@@ -91,7 +92,7 @@ moe_topk_kernel(const float* __restrict__ logits, int ld, int T_, int E, int top
 #pragma unroll
     for (int i = 0; i < TOPK_PER_LANE; ++i) sc[i] = sigmoidf_(v[i]);
   }
-  if (score_fn == SCORE_SOFTMAX || bias || n_groups > 1) {      // (a group's score sums scores)
+  if (bias || n_groups > 1) {      // (a group's score sums scores)
 #pragma unroll
     for (int i = 0; i < TOPK_PER_LANE; ++i) {
       const int e = lane + 64 * i;
@@ -196,13 +197,14 @@ moe_topk_kernel(const float* __restrict__ logits, int ld, int T_, int E, int top
   if (lane < extra) extra_out[(size_t)t * extra + lane] = sigmoidf_(z[E + lane]);
 }
 
-// logits [T, ld]: E router outputs a row, then ``extra`` columns. score_fn: 0 sigmoid, 1 softmax over
+// logits [T, ld]: E router outputs a row, then ``extra`` columns. logit_bias [E] or null: added to the
+// outputs before anything else. score_fn: 0 sigmoid, 1 softmax over
 // the E outputs. bias [E] or null: added to the scores for the choice only. real: the first ``real``
 // outputs are experts with matrices, the others return their input (idx -1; ident_out [T], which
 // must be given when real < E, receives the sum of their weights). Weights: the scores, divided by
 // their sum + renorm_eps when ``renormalize``, times wscale. n_groups > 1: the E outputs form that
 // many equal groups of neighbours (at most 64) of which the best keep_groups can be chosen from.
-extern "C" int ptl_moe_topk(const float* logits, int ld, int T_, int E, int top, int extra, int renormalize,
+extern "C" int ptl_moe_topk(const float* logits, int ld, const float* logit_bias, int T_, int E, int top, int extra, int renormalize,
                             int score_fn, const float* bias, int real, float renorm_eps, float wscale,
                             int n_groups, int keep_groups, int32_t* idx, float* wgt, float* extra_out,
                             float* ident_out, hipStream_t st) {
@@ -215,7 +217,7 @@ extern "C" int ptl_moe_topk(const float* logits, int ld, int T_, int E, int top,
       (score_fn != SCORE_SIGMOID && score_fn != SCORE_SOFTMAX))
     return PTL_ERR_ARG;
 #define GO(PER)                                                                                              \
-  moe_topk_kernel<PER><<<(T_ + 3) / 4, 256, 0, st>>>(logits, ld, T_, E, top, extra, renormalize, score_fn, bias, \
+  moe_topk_kernel<PER><<<(T_ + 3) / 4, 256, 0, st>>>(logits, ld, logit_bias, T_, E, top, extra, renormalize, score_fn, bias, \
                                                      real, renorm_eps, wscale, n_groups, keep_groups, idx, wgt,  \
                                                      extra_out, ident_out)
   if (E <= 64) GO(1);

@@ -11,6 +11,10 @@
 //   (k_cache [pages, Hk, page_size, Dk], v_cache [pages, Hv, page_size, Dv]). A layer that reads
 //   another's keys and values has none of its own: k_off < 0.
 //
+// ptl_conv_qkv_prepare: the same place of a mixer whose queries, keys and values pass a short causal
+//   convolution over time first and whose queries and keys are normed after the rotation. A wave
+//   takes one head of a run of neighbouring rows (where it stands, below).
+//
 // ptl_head_norm_gate: one wave a (token, head). From float32 results a [T, HA, Dv]:
 //   o = a[h * maps] - lam * a[h * maps + 1] (maps 2) or a[h] (maps 1); o / sqrt(mean(o^2) + eps)
 //   over the head's Dv values, times a weight (one for all heads, or one a head, or none), times a
@@ -165,6 +169,218 @@ extern "C" int ptl_qkv_prepare(void* q_out, const float* p, long ldp, int q_off,
   if (dtype == PTL_DTYPE_BF16) GO(bf16_t)
 #undef GO
   return PTL_ERR_ARG;
+}
+
+// ---- a short convolution, a rotation and then a norm ---------------------------------------------
+// u_t = p_t + bias (the columns of q, k and v: one row of channels q | k | v);
+// y_t = sum_j cw[:, j] u_(t - taps + 1 + j), inputs in front of the step's rows from the slot's kept
+//   ones [taps - 1, C] (bias included; zeros where a sequence starts);
+// q and k: the first rot_dims entries of a head turn by the row's position (pairs of neighbours, or
+//   entry i with entry i + rot_dims / 2), then, when ``norm``, the head is divided by its root mean square.
+// A wave takes one head for ``run`` rows one after the other, a lane NP pairs of its entries; with
+// TAPS > 0 the last TAPS - 1 inputs of a lane's entries stay in registers from row to row (TAPS = 0: any
+// number of taps, read again for every row). The first n_single sequences bring one row each: their
+// lanes also advance the kept inputs they have just read (those of longer portions are advanced
+// behind this kernel, when no wave reads them any more).
+#define PAIRS_NEIGHBOURS 0
+#define PAIRS_HALF 1
+
+struct ConvQkvArgs {
+  const float* p; long ldp; int off[3];
+  const float* bias;                        // [C] or null
+  const float* cw; int taps;                // [C, taps]; null with taps 1: no convolution
+  float* state; long slot_stride; long tail_off;
+  const int32_t* q_start; const int32_t* state_slots; int n_seqs, n_single;
+  const int32_t* positions; const int32_t* slots;
+  int rot_dims, layout; const float* inv_freq;
+  int norm; float eps;
+  int T, Hq, Hk, Hv, Dk, Dv, page_size, run;
+};
+
+template <int NP, int TAPS, typename TO>
+__global__ void __launch_bounds__(256)
+conv_qkv_prepare_kernel(TO* __restrict__ q_out, TO* __restrict__ k_cache, TO* __restrict__ v_cache, ConvQkvArgs A) {
+  const int lane = threadIdx.x & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int head = blockIdx.y * 4 + wave;
+  if (head >= A.Hq + A.Hk + A.Hv) return;
+  const int part = head < A.Hq ? 0 : (head < A.Hq + A.Hk ? 1 : 2);
+  const int h = head - (part == 0 ? 0 : (part == 1 ? A.Hq : A.Hq + A.Hk));
+  const int D = part == 2 ? A.Dv : A.Dk;
+  const int C = (A.Hq + A.Hk) * A.Dk + A.Hv * A.Dv;
+  const int c0 = (part == 0 ? 0 : (part == 1 ? A.Hq * A.Dk : (A.Hq + A.Hk) * A.Dk)) + h * D;      // channel of entry 0
+  const int col0 = A.off[part] + h * D;
+  const int rot = part == 2 ? 0 : A.rot_dims;
+  const int taps = TAPS > 0 ? TAPS : A.taps;
+  // the entries of this lane's pairs (-1: none)
+  int e[NP][2];
+#pragma unroll
+  for (int n = 0; n < NP; ++n) {
+    const int j = lane + 64 * n;
+    if (A.layout == PAIRS_HALF && 2 * j < rot) { e[n][0] = j; e[n][1] = j + rot / 2; }
+    else { e[n][0] = 2 * j; e[n][1] = 2 * j + 1; }
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+      if (e[n][i] >= D) e[n][i] = -1;
+  }
+  float w[NP][2][TAPS > 0 ? TAPS : 1], b[NP][2], f[NP];
+#pragma unroll
+  for (int n = 0; n < NP; ++n) {
+    f[n] = 2 * (lane + 64 * n) < rot ? A.inv_freq[lane + 64 * n] : 0.f;
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      b[n][i] = A.bias && e[n][i] >= 0 ? A.bias[c0 + e[n][i]] : 0.f;
+      if (TAPS > 0) {
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) w[n][i][j] = e[n][i] >= 0 ? (A.cw ? A.cw[(size_t)(c0 + e[n][i]) * TAPS + j] : 1.f) : 0.f;
+      }
+    }
+  }
+  auto input = [&](int row, int n, int i) {
+    return e[n][i] >= 0 ? A.p[(size_t)row * A.ldp + col0 + e[n][i]] + b[n][i] : 0.f;
+  };
+  const int t_begin = blockIdx.x * A.run, t_end = min(A.T, t_begin + A.run);
+  // the sequence of the first row: the last one whose first row is not beyond it
+  int seq = 0, hi = A.n_seqs;
+  while (seq < hi) {
+    const int mid = (seq + hi + 1) >> 1;
+    if (A.q_start[mid] <= t_begin) seq = mid; else hi = mid - 1;
+  }
+  bool fresh = true;                        // the window in registers is not of this sequence yet
+  float win[NP][2][TAPS > 1 ? TAPS - 1 : 1];
+  for (int t = t_begin; t < t_end; ++t) {
+    while (seq < A.n_seqs && A.q_start[seq + 1] <= t) { ++seq; fresh = true; }
+    if (seq >= A.n_seqs) return;            // rows that belong to no sequence
+    const int row0 = A.q_start[seq];
+    float* kept = taps > 1 ? A.state + (size_t)A.state_slots[seq] * A.slot_stride + A.tail_off : nullptr;
+    auto before = [&](int r, int n, int i) {                   // the input of row r of the sequence (r < 0: a kept one)
+      if (r >= 0) return input(row0 + r, n, i);
+      return e[n][i] >= 0 ? kept[(size_t)(taps - 1 + r) * C + c0 + e[n][i]] : 0.f;
+    };
+    const int r = t - row0;
+    float y[NP][2];
+#pragma unroll
+    for (int n = 0; n < NP; ++n)
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const float x = input(t, n, i);
+        if (TAPS > 0) {
+          if (fresh) {
+#pragma unroll
+            for (int j = 0; j < TAPS - 1; ++j) win[n][i][j] = before(r - (TAPS - 1) + j, n, i);
+          }
+          float s = 0.f;
+#pragma unroll
+          for (int j = 0; j < TAPS - 1; ++j) s = fmaf(w[n][i][j], win[n][i][j], s);
+          y[n][i] = fmaf(w[n][i][TAPS - 1], x, s);
+#pragma unroll
+          for (int j = 0; j < TAPS - 1; ++j) win[n][i][j] = j + 1 < TAPS - 1 ? win[n][i][j + 1] : x;
+          if (seq < A.n_single && e[n][i] >= 0) {
+#pragma unroll
+            for (int j = 0; j < TAPS - 1; ++j) kept[(size_t)j * C + c0 + e[n][i]] = win[n][i][j];
+          }
+        } else {
+          const float* wr = A.cw + (size_t)(c0 + max(e[n][i], 0)) * taps;
+          float s = 0.f;
+          for (int j = 0; j < taps - 1; ++j) s = fmaf(wr[j], before(r - (taps - 1) + j, n, i), s);
+          y[n][i] = fmaf(wr[taps - 1], x, s);
+          if (seq < A.n_single && e[n][i] >= 0) {
+            float* k = kept + c0 + e[n][i];
+            for (int j = 0; j < taps - 1; ++j) k[(size_t)j * C] = j + 1 < taps - 1 ? k[(size_t)(j + 1) * C] : x;
+          }
+        }
+      }
+    fresh = false;
+    float scale = 1.f;
+    if (part < 2) {
+      if (rot > 0) {
+        const float pos = (float)A.positions[t];
+#pragma unroll
+        for (int n = 0; n < NP; ++n) {
+          if (2 * (lane + 64 * n) >= rot) continue;
+          float sn, cs;
+          sincosf(pos * f[n], &sn, &cs);
+          const float u = y[n][0], v = y[n][1];
+          y[n][0] = u * cs - v * sn;
+          y[n][1] = v * cs + u * sn;
+        }
+      }
+      if (A.norm) {
+        float ss = 0.f;
+#pragma unroll
+        for (int n = 0; n < NP; ++n)
+#pragma unroll
+          for (int i = 0; i < 2; ++i)
+            if (e[n][i] >= 0) ss = fmaf(y[n][i], y[n][i], ss);
+        scale = 1.0f / sqrtf(wave_sum(ss) / (float)D + A.eps);
+      }
+    }
+    TO* dst = nullptr;
+    if (part == 0) {
+      dst = q_out + ((size_t)t * A.Hq + h) * D;
+    } else {
+      const int slot = A.slots ? A.slots[t] : -1;
+      if (slot < 0) continue;
+      const int page = slot / A.page_size, at = slot % A.page_size;
+      dst = part == 1 ? k_cache + (((size_t)page * A.Hk + h) * A.page_size + at) * D
+                      : v_cache + (((size_t)page * A.Hv + h) * A.page_size + at) * D;
+    }
+#pragma unroll
+    for (int n = 0; n < NP; ++n) {
+      if (sizeof(TO) == 2 && D % 2 == 0 && e[n][0] >= 0 && e[n][1] == e[n][0] + 1 && e[n][0] % 2 == 0) {
+        union { uint32_t u; bf16_t x[2]; } two;
+        two.x[0] = float_to_bf16(y[n][0] * scale);
+        two.x[1] = float_to_bf16(y[n][1] * scale);
+        *reinterpret_cast<uint32_t*>(dst + e[n][0]) = two.u;
+      } else {
+#pragma unroll
+        for (int i = 0; i < 2; ++i)
+          if (e[n][i] >= 0) dst[e[n][i]] = from_float<TO>(y[n][i] * scale);
+      }
+    }
+  }
+}
+
+// p float32 [T, ldp] with q (Hq heads of Dk), k (Hk of Dk) and v (Hv of Dv) at their columns; bias, cw: of the
+// channels q | k | v. q_out [T, Hq, Dk] and the caches of dtype; slots null: nothing is written to the caches.
+extern "C" int ptl_conv_qkv_prepare(void* q_out, const float* p, long ldp, int q_off, int k_off, int v_off,
+                                    const float* bias, const float* cw, int taps, float* state, long slot_stride,
+                                    long tail_off, const int32_t* q_start, const int32_t* state_slots, int n_seqs,
+                                    int n_single, const int32_t* positions, const int32_t* slots, int rot_dims,
+                                    int layout, const float* inv_freq, int norm, float eps, void* k_cache,
+                                    void* v_cache, int T_, int Hq, int Hk, int Hv, int Dk, int Dv, int page_size,
+                                    int dtype, hipStream_t st) {
+  if (T_ <= 0) return PTL_OK;
+  if (Hq <= 0 || Hk <= 0 || Hv <= 0 || Dk <= 0 || Dv <= 0 || Dk > 640 || Dv > 640 || page_size <= 0 || taps < 1 ||
+      (!cw && taps != 1) || rot_dims < 0 || rot_dims > Dk || (rot_dims & 1) || (rot_dims && !inv_freq) || n_seqs <= 0 ||
+      n_single < 0 || n_single > n_seqs || (layout != PAIRS_NEIGHBOURS && layout != PAIRS_HALF) || !positions ||
+      (slots && (!k_cache || !v_cache)) || (Hq + Hk + Hv + 3) / 4 > 65535 ||
+      (taps > 1 && (!state || tail_off < 0 ||
+                    tail_off + (long)(taps - 1) * ((Hq + Hk) * Dk + Hv * Dv) > slot_stride)))
+    return PTL_ERR_ARG;
+  ConvQkvArgs A{p, ldp, {q_off, k_off, v_off}, bias, cw, taps, state, slot_stride, tail_off, q_start, state_slots,
+                n_seqs, n_single, positions, slots, rot_dims, layout, inv_freq, norm, eps, T_, Hq, Hk, Hv, Dk, Dv,
+                page_size, 1};
+  // runs of rows that share their inputs, as long as the chip stays filled a few times over
+  const long waves = (long)T_ * (Hq + Hk + Hv);
+  A.run = waves >= 8 * 16384 ? 8 : (waves >= 4 * 16384 ? 4 : (waves >= 2 * 16384 ? 2 : 1));
+  const dim3 grid((T_ + A.run - 1) / A.run, (Hq + Hk + Hv + 3) / 4);
+  const bool wide = (Dk > Dv ? Dk : Dv) > 128;
+#define GO(NP, TAPS, TO)                                                                                           \
+  conv_qkv_prepare_kernel<NP, TAPS, TO><<<grid, 256, 0, st>>>((TO*)q_out, (TO*)k_cache, (TO*)v_cache, A)
+#define BY_TAPS(NP, TO)                                     \
+  if (taps == 4) GO(NP, 4, TO);                             \
+  else if (taps == 1) GO(NP, 1, TO);                        \
+  else GO(NP, 0, TO)
+#define BY_SIZE(TO)                                         \
+  if (wide) { BY_TAPS(5, TO); } else { BY_TAPS(1, TO); }
+  if (dtype == PTL_DTYPE_F32) { BY_SIZE(float) }
+  else if (dtype == PTL_DTYPE_BF16) { BY_SIZE(bf16_t) }
+  else return PTL_ERR_ARG;
+#undef BY_SIZE
+#undef BY_TAPS
+#undef GO
+  return ptl_launch_status();
 }
 
 #define ACT_NONE 0

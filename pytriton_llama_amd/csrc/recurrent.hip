@@ -853,27 +853,30 @@ extern "C" int ptl_conv_prepare(float* qn, float* kn, float* vv, const float* p,
 __global__ void __launch_bounds__(256)
 conv_tail_kernel(float* __restrict__ state, long slot_stride, long tail_off, const float* __restrict__ p,
                  long ldp, int x_off, const int32_t* __restrict__ q_start,
-                 const int32_t* __restrict__ state_slots, int C, int taps) {
+                 const int32_t* __restrict__ state_slots, const float* __restrict__ bias, int C, int taps) {
   const int seq = blockIdx.y;
   const int c = blockIdx.x * 256 + threadIdx.x;
   const int row0 = q_start[seq];
   const int qlen = q_start[seq + 1] - row0;
   if (qlen <= 0 || c >= C) return;
   float* tail = state + (size_t)state_slots[seq] * slot_stride + tail_off;
+  const float b = bias ? bias[c] : 0.f;
   // in order of rising i: an entry read from the old tail lies above the one being written
   for (int i = 0; i < taps - 1; ++i) {
     const int r = qlen - (taps - 1) + i;
-    tail[(size_t)i * C + c] = r >= 0 ? p[(size_t)(row0 + r) * ldp + x_off + c] : tail[(size_t)(i + qlen) * C + c];
+    tail[(size_t)i * C + c] = r >= 0 ? p[(size_t)(row0 + r) * ldp + x_off + c] + b : tail[(size_t)(i + qlen) * C + c];
   }
 }
 
+// bias [C] or null: added to the inputs of this step (the kept ones hold it already)
+
 extern "C" int ptl_conv_tail_update(float* state, long slot_stride, long tail_off, const float* p, long ldp,
                                     int x_off, const int32_t* q_start, const int32_t* state_slots,
-                                    int n_seqs, int C, int taps, hipStream_t st) {
+                                    int n_seqs, const float* bias, int C, int taps, hipStream_t st) {
   if (n_seqs <= 0 || taps <= 1) return PTL_OK;
   if (C <= 0 || n_seqs > 65535) return PTL_ERR_ARG;
   dim3 grid((C + 255) / 256, n_seqs);
   conv_tail_kernel<<<grid, 256, 0, st>>>(state, slot_stride, tail_off, p, ldp, x_off, q_start, state_slots,
-                                          C, taps);
+                                          bias, C, taps);
   return ptl_launch_status();
 }

@@ -12,6 +12,8 @@
 // ptl_stream_add_rmsnorm_sum: the same for a result that is a weighted sum of two and a bias.
 // ptl_stream_postnorm: stream = rmsnorm(alpha stream + y) * w, the norm behind the residual sum, with y a
 //   weighted sum of up to two results each of which may be RMS-normed first (where it stands, below).
+// ptl_stream_scaled_sum: stream += s1 (y1 + bias) + s2 y2 with a scale an entry, and the RMS norm in front
+//   of what reads the stream next: two sublayers side by side on one input (where it stands, below).
 // ptl_stream_rmsnorm: the RMS norm of rows of the stream, in the engine's type.
 // ptl_dyt: the norm alone, for rows that are no stream (the rows picked for the head).
 // ptl_embedding_scaled: stream[t] = table[ids[t]] * scale, in float32 (``copies`` times side by side in
@@ -343,6 +345,125 @@ extern "C" int ptl_stream_postnorm(float* stream, float alpha, const void* y1, f
   if (y_dtype == PTL_DTYPE_F32 && out_dtype == PTL_DTYPE_BF16) return launch_postnorm<float, bf16_t>(A, T_, st);
   if (y_dtype == PTL_DTYPE_BF16 && out_dtype == PTL_DTYPE_BF16) return launch_postnorm<bf16_t, bf16_t>(A, T_, st);
   if (y_dtype == PTL_DTYPE_BF16 && out_dtype == PTL_DTYPE_F32) return launch_postnorm<bf16_t, float>(A, T_, st);
+  return PTL_ERR_ARG;
+}
+
+// The residual sum of sublayers whose results are scaled entry by entry, and the norm that follows:
+//   stream += s1 * (y1 + bias) + s2 * y2;    out = stream * rsqrt(mean(stream^2) + eps) * w
+// (y1, y2, bias and both scales are optional: no y1 and no y2 leaves the stream as it is; w null: no
+// norm, no out). One workgroup a row; a thread keeps its VPT groups of VEC neighbouring entries in
+// registers from the one pass over memory to the last use.
+struct ScaledSumArgs {
+  float* stream;
+  const void* y1; const float* s1; const float* bias;
+  const void* y2; const float* s2;
+  const float* w; float eps;
+  void* out;
+  int H;
+};
+
+template <int VEC, typename T>
+__device__ __forceinline__ void read_vec(const T* p, float (&v)[VEC]) {
+  if (VEC == 1) {
+    v[0] = to_float<T>(p[0]);
+  } else if (sizeof(T) == 4) {
+    const float4 x = *reinterpret_cast<const float4*>(p);
+    v[0] = x.x; v[VEC > 1 ? 1 : 0] = x.y; v[VEC > 2 ? 2 : 0] = x.z; v[VEC > 3 ? 3 : 0] = x.w;
+  } else {
+    const uint2 x = *reinterpret_cast<const uint2*>(p);
+    v[0] = __uint_as_float(x.x << 16); v[VEC > 1 ? 1 : 0] = __uint_as_float(x.x & 0xffff0000u);
+    v[VEC > 2 ? 2 : 0] = __uint_as_float(x.y << 16); v[VEC > 3 ? 3 : 0] = __uint_as_float(x.y & 0xffff0000u);
+  }
+}
+
+template <int NT, int VPT, int VEC, typename T1, typename T2, typename TO>
+__global__ void __launch_bounds__(NT) stream_scaled_sum_kernel(ScaledSumArgs A) {
+  __shared__ float scratch[16];
+  const size_t row = (size_t)blockIdx.x * A.H;
+  float* stream = A.stream + row;
+  float u[VPT][VEC];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < VPT; ++k) {
+    const int i = (k * NT + threadIdx.x) * VEC;
+    if (i >= A.H) continue;
+    read_vec<VEC>((const float*)stream + i, u[k]);
+    if (A.y1) {
+      float y[VEC], f[VEC];
+      read_vec<VEC>((const T1*)A.y1 + row + i, y);
+      if (A.bias) {
+        read_vec<VEC>(A.bias + i, f);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) y[j] += f[j];
+      }
+      if (A.s1) read_vec<VEC>(A.s1 + i, f);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) u[k][j] = fmaf(A.s1 ? f[j] : 1.f, y[j], u[k][j]);
+    }
+    if (A.y2) {
+      float y[VEC], f[VEC];
+      read_vec<VEC>((const T2*)A.y2 + row + i, y);
+      if (A.s2) read_vec<VEC>(A.s2 + i, f);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) u[k][j] = fmaf(A.s2 ? f[j] : 1.f, y[j], u[k][j]);
+    }
+    if (A.y1 || A.y2) {
+      if (VEC == 1) stream[i] = u[k][0];
+      else *reinterpret_cast<float4*>(stream + i) = make_float4(u[k][0], u[k][VEC > 1 ? 1 : 0], u[k][VEC > 2 ? 2 : 0], u[k][VEC > 3 ? 3 : 0]);
+    }
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) ss = fmaf(u[k][j], u[k][j], ss);
+  }
+  if (!A.w) return;
+  const float r = 1.0f / sqrtf(block_sum(ss, scratch) / (float)A.H + A.eps);
+  TO* out = (TO*)A.out + row;
+#pragma unroll
+  for (int k = 0; k < VPT; ++k) {
+    const int i = (k * NT + threadIdx.x) * VEC;
+    if (i >= A.H) continue;
+    float w[VEC];
+    read_vec<VEC>(A.w + i, w);
+    TO e[VEC];
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) e[j] = from_float<TO>(u[k][j] * r * w[j]);
+    if (VEC == 1) out[i] = e[0];
+    else if (sizeof(TO) == 2) *reinterpret_cast<uint2*>(out + i) = *reinterpret_cast<const uint2*>(e);
+    else *reinterpret_cast<float4*>(out + i) = *reinterpret_cast<const float4*>(e);
+  }
+}
+
+template <typename T1, typename T2, typename TO>
+static int launch_scaled_sum(const ScaledSumArgs& A, int T_, hipStream_t st) {
+  auto odd = [](const void* p) { return ((uintptr_t)p & 15) != 0; };
+  const bool vec = A.H % 4 == 0 && !odd(A.stream) && !odd(A.y1) && !odd(A.s1) && !odd(A.bias) && !odd(A.y2) &&
+                   !odd(A.s2) && !odd(A.w) && !odd(A.out);
+  const int n = vec ? A.H / 4 : A.H;         // groups of entries of a row
+  // few rows: a row over 1,024 threads, so that a thread's loads are one or two deep
+  const bool few = T_ <= 512 && n > 256;
+#define GO(NT, VPT)                                                                      \
+  if (n <= NT * VPT) {                                                                   \
+    if (vec) stream_scaled_sum_kernel<NT, VPT, 4, T1, T2, TO><<<T_, NT, 0, st>>>(A);     \
+    else stream_scaled_sum_kernel<NT, VPT, 1, T1, T2, TO><<<T_, NT, 0, st>>>(A);         \
+    return ptl_launch_status();                                                          \
+  }
+  if (!few) { GO(256, 1) GO(256, 2) GO(256, 4) }
+  GO(1024, 1) GO(1024, 2) GO(1024, 4)
+  if (!vec) { GO(1024, 16) }
+#undef GO
+  return PTL_ERR_ARG;
+}
+
+// stream float32 [T, H], in place; y1 [T, H] float32 or null; y2 [T, H] of y2_dtype or null; s1, s2, bias, w
+// float32 [H] or null; out [T, H] of out_dtype (with w). H up to 16,384.
+extern "C" int ptl_stream_scaled_sum(float* stream, const float* y1, const float* s1, const float* bias,
+                                     const void* y2, int y2_dtype, const float* s2, const float* w, float eps,
+                                     void* out, int out_dtype, int T_, int H, hipStream_t st) {
+  if (T_ <= 0) return PTL_OK;
+  if (H <= 0 || !stream || (bias && !y1) || (w && !out) || (!y1 && !y2 && !w)) return PTL_ERR_ARG;
+  const ScaledSumArgs A{stream, y1, s1, bias, y2, s2, w, eps, out, H};
+  if (y2_dtype == PTL_DTYPE_F32 && out_dtype == PTL_DTYPE_F32) return launch_scaled_sum<float, float, float>(A, T_, st);
+  if (y2_dtype == PTL_DTYPE_F32 && out_dtype == PTL_DTYPE_BF16) return launch_scaled_sum<float, float, bf16_t>(A, T_, st);
+  if (y2_dtype == PTL_DTYPE_BF16 && out_dtype == PTL_DTYPE_BF16) return launch_scaled_sum<float, bf16_t, bf16_t>(A, T_, st);
   return PTL_ERR_ARG;
 }
 

@@ -5,3 +5,4 @@ from .virusun import build_virusun
 from .matusun import build_matusun
 from .senavik import build_senavik
 from .bimopel import build_bimopel
+from .fogapel import build_fogapel

@@ -144,6 +144,7 @@ def rmsnorm_cols(x: torch.Tensor, weight: torch.Tensor, eps: float) -> torch.Ten
 
 
 GLU_SILU, GLU_GELU_TANH = 0, 1        # activations of a gated feed-forward's gate
+GLU_CLAMPED = 2                       # gate and up clamped by a limit (gate_up_silu only)
 
 
 def silu_mul(gate_up: torch.Tensor, act: int = GLU_SILU) -> torch.Tensor:
@@ -230,6 +231,7 @@ def gemm_nt(x: torch.Tensor, w: torch.Tensor, out_dtype: Optional[torch.dtype] =
 
 
 SKINNY_MAX_ROWS = 64
+GROUPS_SKINNY_ROWS = 16    # rows up to which gemm_groups streams the weights itself
 BLOCKED_MAX_ROWS = 64      # rows of x up to which the kernels take the blocked copy of a weight
 
 
@@ -327,7 +329,45 @@ def gemm_library(x: torch.Tensor, w: torch.Tensor, out_dtype: Optional[torch.dty
     lib = library.load("blaslt")
     _check(lib.ptl_blaslt_gemm_bf16(_ptr(y), _ptr(x), _ptr(w), M, N, K, ctypes.c_long(ldx),
                                     ctypes.c_long(N), _F32 if out_dtype == torch.float32 else _BF16,
+                                    1, ctypes.c_long(0), ctypes.c_long(0), ctypes.c_long(0),
                                     1 if _timed_products else 0, _stream()), "gemm_library")
+    return y
+
+
+def gemm_groups(x: torch.Tensor, w: torch.Tensor, cols: int, blocked: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Several products side by side, float32 [M, N]: columns g * cols on (the last group: all that are left)
+    hold x[g] @ w[those rows].T. x [S, M, K] contiguous, w [N, K] with the groups' rows one after the other, cols a
+    multiple of 16. At most 64 rows of bfloat16 x: one launch of the weight-streaming kernel, which
+    takes ``blocked`` (blocked_weight(w)); more: the library, the groups of ``cols`` columns as one batch and the
+    last one by itself; float32: the vector-FMA kernel, group by group."""
+    _need_gpu(x, w)
+    S, M, K = x.shape
+    N = w.shape[0]
+    if (not x.is_contiguous() or not w.is_contiguous() or w.dim() != 2 or w.shape[1] != K or x.dtype != w.dtype
+            or cols <= 0 or cols % 16 or (S - 1) * cols >= N):
+        raise KernelError(f"gemm_groups: {S} groups of {cols} columns (a multiple of 16) do not fit w {tuple(w.shape)}")
+    y = torch.empty((M, N), dtype=torch.float32, device=x.device)
+    if M == 0:
+        return y
+    aligned = x.dtype == torch.bfloat16 and K % 8 == 0 and x.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0
+    if aligned and M <= GROUPS_SKINNY_ROWS:
+        wp, wb = _weight_arg(w, blocked, M, "gemm_groups")
+        _check(library.load("gemm").ptl_gemm_skinny_groups_bf16(
+            _ptr(y), _ptr(x), wp, wb, M, N, K, ctypes.c_long(K), ctypes.c_long(N), int(cols), S - 1,
+            ctypes.c_long(M * K), _F32, _stream()), "gemm_groups")
+        return y
+    if aligned and N % 4 == 0:
+        lib = library.load("blaslt")
+        for first, batch, n in ((0, S - 1, cols), (S - 1, 1, N - (S - 1) * cols)):
+            if batch:
+                _check(lib.ptl_blaslt_gemm_bf16(
+                    _ptr(y[:, first * cols:]), _ptr(x[first:]), _ptr(w[first * cols:]), M, n, K, ctypes.c_long(K),
+                    ctypes.c_long(N), _F32, batch, ctypes.c_long(M * K), ctypes.c_long(cols * K), ctypes.c_long(cols),
+                    1 if _timed_products else 0, _stream()), "gemm_groups")
+        return y
+    for g in range(S):
+        last = N if g == S - 1 else (g + 1) * cols
+        gemm_nt(x[g], w[g * cols:last], torch.float32, out=y[:, g * cols:last])
     return y
 
 
@@ -549,11 +589,12 @@ def gate_up_silu_fits(x: torch.Tensor, w: torch.Tensor, blocked: Optional[torch.
 
 
 def gate_up_silu(x: torch.Tensor, w: torch.Tensor, scale: Optional[RowScale] = None,
-                 blocked: Optional[torch.Tensor] = None, act: int = GLU_SILU) -> torch.Tensor:
+                 blocked: Optional[torch.Tensor] = None, act: int = GLU_SILU, limit: float = 0.0) -> torch.Tensor:
     """act(x Wg^T) * (x Wu^T) for w = [Wg; Wu] ([2I, K]) in one kernel (act as for silu_mul): for at most 16 rows
     of bfloat16 x the one of csrc/gemm.hip, from ROWS_MIN rows on, with the blocked copy of w,
     the one of csrc/gemm_rows.hip. ``scale``: the factor that the rows of x still lack (at most
-    16 rows); it is applied to both products."""
+    16 rows); it is applied to both products. ``act`` GLU_CLAMPED: with g = min(x Wg^T, limit) and u =
+    x Wu^T clamped to [-limit, limit], g sigmoid(1.702 g) (u + 1)."""
     rows = scale is None and _rows_x_ok(x, w, blocked) and w.shape[0] % 64 == 0
     if not (rows or (_fused_x_ok(x, w) and w.shape[0] % 32 == 0)):
         raise KernelError("gate_up_silu: needs bfloat16, K a multiple of 8, I a multiple of 16, aligned "
@@ -565,14 +606,14 @@ def gate_up_silu(x: torch.Tensor, w: torch.Tensor, scale: Optional[RowScale] = N
     if rows:
         _check(library.load("gemm_rows").ptl_rows_gate_up_silu(
             _ptr(out), _ptr(x), _rows_weight(w, blocked, "gate_up_silu"), M, I, K,
-            ctypes.c_long(x.stride(0)), int(act), _stream()), "gate_up_silu")
+            ctypes.c_long(x.stride(0)), int(act), ctypes.c_float(limit), _stream()), "gate_up_silu")
         return out
     lib = library.load("gemm")
     pp, count, eps = scale.args(M, K, "gate_up_silu") if scale is not None else _NO_SCALE
     wp, wb = _weight_arg(w, blocked, M, "gate_up_silu")
     _check(lib.ptl_gate_up_silu_bf16(_ptr(out), _ptr(x), wp, wb, M, I, K,
                                      ctypes.c_long(x.stride(0) if M > 1 else max(K, 8)),
-                                     pp, count, eps, int(act), _stream()),
+                                     pp, count, eps, int(act), ctypes.c_float(limit), _stream()),
            "gate_up_silu")
     return out
 
@@ -642,13 +683,16 @@ def qkv_rope_store(x: torch.Tensor, w: torch.Tensor, positions: torch.Tensor,
 
 
 def _mask_extras(what: str, T: int, Hq: int, window: int, keep_first: int, chunk: int,
-                 sink: Optional[torch.Tensor], gate: Optional[torch.Tensor]):
+                 sink: Optional[torch.Tensor], gate: Optional[torch.Tensor], softcap: float = 0.0):
     """The optional pieces every attention kernel takes, as kernel arguments: ``window`` (a query
     sees its own key and the window - 1 before it), ``keep_first`` (with a window: the keys at
     positions below it stay visible to every later query), ``chunk`` (a query sees the keys of its
     own chunk of so many positions), ``sink`` (float32 [Hq]: the softmax denominator of head h also
     holds exp(sink[h]), a term without key and value), ``gate`` (float32 [T, >= Hq], rows may be
-    strided: head h's result of row t is multiplied by sigmoid(gate[t, h]))."""
+    strided: head h's result of row t is multiplied by sigmoid(gate[t, h])), ``softcap`` (a scaled
+    score s becomes softcap * tanh(s / softcap); 0: it stays)."""
+    if softcap < 0:
+        raise KernelError(f"{what}: softcap is not negative")
     if keep_first < 0 or (keep_first and window <= 0):
         raise KernelError(f"{what}: keep_first goes with a window, and is not negative")
     if chunk < 0 or (chunk and window > 0):
@@ -662,7 +706,8 @@ def _mask_extras(what: str, T: int, Hq: int, window: int, keep_first: int, chunk
                 or gate.shape[0] != T or gate.shape[1] < Hq:
             raise KernelError(f"{what}: gate must be a float32 GPU matrix [{T}, >= {Hq}] with dense rows")
         stride = gate.stride(0)
-    return int(window), int(keep_first), int(chunk), _ptr(sink), _ptr(gate), ctypes.c_long(stride)
+    return (int(window), int(keep_first), int(chunk), _ptr(sink), _ptr(gate), ctypes.c_long(stride),
+            ctypes.c_float(softcap))
 
 
 def attention_generic(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
@@ -670,7 +715,7 @@ def attention_generic(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
                       block_table: torch.Tensor, work_seq: torch.Tensor, work_qoff: torch.Tensor,
                       scale: float, window: int = 0, keep_first: int = 0,
                       sink: Optional[torch.Tensor] = None, chunk: int = 0,
-                      gate: Optional[torch.Tensor] = None) -> None:
+                      gate: Optional[torch.Tensor] = None, softcap: float = 0.0) -> None:
     """Attention of a mixed batch over the paged cache (see csrc/attention.hip).
     q [T, Hq, D] (rows may be strided), out [T, Hq, D], caches
     [pages, Hkv, page_size, D], q_start [n+1], ctx_len [n], block_table [n, max_pages],
@@ -700,7 +745,7 @@ def attention_generic(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
     if block_table.dtype != torch.int32 or block_table.dim() != 2 or block_table.shape[0] < n \
             or block_table.stride(1) != 1:
         raise KernelError("attention: block_table must be int32 [n, max_pages]")
-    extras = _mask_extras("attention", T, Hq, window, keep_first, chunk, sink, gate)
+    extras = _mask_extras("attention", T, Hq, window, keep_first, chunk, sink, gate, softcap)
     lib = library.load("attention")
     _check(lib.ptl_attention_generic(
         _ptr(out), ctypes.c_long(out.stride(0)), _ptr(q), ctypes.c_long(q.stride(0)),
@@ -745,7 +790,7 @@ def attention_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
                      block_table: torch.Tensor, n_seq: int, scale: float, window: int = 0,
                      num_splits: int = 1, matrix_cores: bool = False, unroll: int = 0,
                      keep_first: int = 0, sink: Optional[torch.Tensor] = None, chunk: int = 0,
-                     gate: Optional[torch.Tensor] = None) -> None:
+                     gate: Optional[torch.Tensor] = None, softcap: float = 0.0) -> None:
     """Split-KV attention of the first ``n_seq`` sequences of the tables, each of
     which brings exactly one query token (see csrc/attention.hip). Head sizes in
     steps of 16 up to 256, float32 or bfloat16. ``matrix_cores``: the MFMA
@@ -760,7 +805,7 @@ def attention_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
         raise KernelError("attention_decode: tables are shorter than n_seq")
     if num_splits < 1:
         raise KernelError("attention_decode: num_splits must be >= 1")
-    extras = _mask_extras("attention_decode", T, Hq, window, keep_first, chunk, sink, gate)
+    extras = _mask_extras("attention_decode", T, Hq, window, keep_first, chunk, sink, gate, softcap)
     part_acc = part_ml = None
     if num_splits > 1:
         part_acc = torch.empty((n_seq, Hq, num_splits, D), dtype=torch.float32, device=q.device)
@@ -834,7 +879,7 @@ def attention_prefill_mfma(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Te
                            work_qoff: torch.Tensor, scale: float, window: int = 0,
                            block_rows: int = 64, groups: int = 0, keep_first: int = 0,
                            sink: Optional[torch.Tensor] = None, chunk: int = 0,
-                           gate: Optional[torch.Tensor] = None) -> None:
+                           gate: Optional[torch.Tensor] = None, softcap: float = 0.0) -> None:
     """bfloat16 attention of prompt portions on the matrix cores; the work list
     names query blocks of ``block_rows`` (64 or 128) rows, those with the most
     keys first. ``groups`` workgroups a head share the list (0: one for every
@@ -857,7 +902,9 @@ def attention_prefill_mfma(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Te
         raise KernelError("attention_prefill_mfma: query blocks are 64 or 128 rows")
     if q.stride(0) % 8 or out.stride(0) % 4 or q.data_ptr() % 16 or out.data_ptr() % 8:
         raise KernelError("attention_prefill_mfma: q rows must be 16-byte aligned, out rows 8-byte")
-    extras = _mask_extras("attention_prefill_mfma", T, Hq, window, keep_first, chunk, sink, gate)
+    if keep_first and softcap:
+        raise KernelError("attention_prefill_mfma: kept first keys with capped scores are not built")
+    extras = _mask_extras("attention_prefill_mfma", T, Hq, window, keep_first, chunk, sink, gate, softcap)
     lib = library.load("attention_prefill")
     n_work = int(work_seq.numel())
     _check(lib.ptl_attention_prefill_mfma(
@@ -1257,7 +1304,7 @@ def attention_generic_kv(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tens
                          q_start: torch.Tensor, ctx_len: torch.Tensor, block_table: torch.Tensor,
                          work_seq: torch.Tensor, work_qoff: torch.Tensor, scale: float, maps: int = 1,
                          window: int = 0, keep_first: int = 0, sink: Optional[torch.Tensor] = None,
-                         chunk: int = 0, gate: Optional[torch.Tensor] = None) -> None:
+                         chunk: int = 0, gate: Optional[torch.Tensor] = None, softcap: float = 0.0) -> None:
     """The vector-FMA attention kernel in its general form (csrc/attention.hip): q [T, Hq, Dk]
     with Hq = heads * maps (head after head, map after map), k_cache [pages, Hkv * maps, page_size,
     Dk], v_cache [pages, Hkv, page_size, Dv], out [T, Hq, Dv] in the caches' dtype or float32.
@@ -1289,7 +1336,7 @@ def attention_generic_kv(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tens
     if block_table.dtype != torch.int32 or block_table.dim() != 2 or block_table.shape[0] < n \
             or block_table.stride(1) != 1:
         raise KernelError("attention: block_table must be int32 [n, max_pages]")
-    extras = _mask_extras("attention", T, Hq, window, keep_first, chunk, sink, gate)
+    extras = _mask_extras("attention", T, Hq, window, keep_first, chunk, sink, gate, softcap)
     _check(library.load("attention").ptl_attention_generic_kv(
         _ptr(out), ctypes.c_long(out.stride(0)), int(out.dtype == torch.float32 and q.dtype != torch.float32),
         _ptr(q), ctypes.c_long(q.stride(0)), _ptr(k_cache), _ptr(v_cache), _ptr(q_start), _ptr(ctx_len),
@@ -1313,7 +1360,7 @@ def attention_prefill_mfma_kv(out: torch.Tensor, q: torch.Tensor, k_cache: torch
                               work_seq: torch.Tensor, work_qoff: torch.Tensor, scale: float, maps: int = 1,
                               groups: int = 1, window: int = 0, keep_first: int = 0,
                               sink: Optional[torch.Tensor] = None, chunk: int = 0,
-                              gate: Optional[torch.Tensor] = None) -> None:
+                              gate: Optional[torch.Tensor] = None, softcap: float = 0.0) -> None:
     """The matrix-core kernel for prompt portions in its general form (csrc/attention_prefill.hip):
     shapes as for attention_generic_kv, bfloat16 q and caches, out bfloat16 or float32; the work
     list names 64-row blocks, ``groups`` workgroups a head share it."""
@@ -1345,7 +1392,9 @@ def attention_prefill_mfma_kv(out: torch.Tensor, q: torch.Tensor, k_cache: torch
     n_work = int(work_seq.numel())
     if n_work == 0:
         return
-    extras = _mask_extras("attention_prefill_mfma_kv", T, Hq, window, keep_first, chunk, sink, gate)
+    if keep_first and softcap:
+        raise KernelError("attention_prefill_mfma_kv: kept first keys with capped scores are not built")
+    extras = _mask_extras("attention_prefill_mfma_kv", T, Hq, window, keep_first, chunk, sink, gate, softcap)
     _check(library.load("attention_prefill").ptl_attention_prefill_mfma_kv(
         _ptr(out), ctypes.c_long(out.stride(0)), int(out.dtype == torch.float32), _ptr(q),
         ctypes.c_long(q.stride(0)), _ptr(k_cache), _ptr(v_cache), _ptr(q_start), _ptr(ctx_len),
@@ -1363,7 +1412,7 @@ def attention_decode_kv(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tenso
                         q_start: torch.Tensor, ctx_len: torch.Tensor, block_table: torch.Tensor, n_seq: int,
                         scale: float, maps: int = 1, num_splits: int = 1, window: int = 0,
                         keep_first: int = 0, sink: Optional[torch.Tensor] = None, chunk: int = 0,
-                        gate: Optional[torch.Tensor] = None) -> None:
+                        gate: Optional[torch.Tensor] = None, softcap: float = 0.0) -> None:
     """Split-KV attention of the first ``n_seq`` sequences of the tables, each of which brings one
     query token, with keys and values of different sizes and ``maps`` score maps a head (shapes as
     for attention_generic_kv; sizes in steps of 16 up to 256)."""
@@ -1390,7 +1439,7 @@ def attention_decode_kv(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tenso
         raise KernelError("attention_decode_kv: block_table must be int32 [n, max_pages]")
     if n_seq > ctx_len.numel() or q_start.numel() < n_seq + 1 or block_table.shape[0] < n_seq or num_splits < 1:
         raise KernelError("attention_decode_kv: tables are shorter than n_seq, or no splits")
-    extras = _mask_extras("attention_decode_kv", T, Hq, window, keep_first, chunk, sink, gate)
+    extras = _mask_extras("attention_decode_kv", T, Hq, window, keep_first, chunk, sink, gate, softcap)
     part_acc = part_ml = None
     if num_splits > 1:
         part_acc = torch.empty((n_seq, Hq, num_splits, Dv), dtype=torch.float32, device=q.device)
@@ -1473,6 +1522,70 @@ def qkv_prepare(q_out: torch.Tensor, p: torch.Tensor, q_off: int, k_off: int, v_
         T, Hq, Hk, Hv, Dk, Dv, int(page_size), _dtype_code(q_out), _stream()), "qkv_prepare")
 
 
+ROT_PAIRS, ROT_HALF = 0, 1
+
+
+def conv_qkv_prepare(q_out: torch.Tensor, p: torch.Tensor, q_off: int, k_off: int, v_off: int,
+                     bias: Optional[torch.Tensor], conv_weight: Optional[torch.Tensor],
+                     state: Optional[torch.Tensor], tail_off: int, q_start: torch.Tensor,
+                     state_slots: torch.Tensor, n_single: int, positions: torch.Tensor, slots, rot_dims: int,
+                     layout: int, inv_freq, norm: bool, eps: float, k_cache, v_cache, Hq: int, Hk: int, Hv: int,
+                     Dk: int, Dv: int, page_size: int) -> None:
+    """Bias, short causal convolution over time, rotation, norm (without a weight, over every head of q
+    and k) and cache write for one step (csrc/prepare.hip). p float32 [T, columns] holds q (Hq heads of Dk),
+    k (Hk of Dk) and v (Hv of Dv); ``bias`` float32 [C] and ``conv_weight`` float32 [C, taps] (None: one
+    tap of one) of the channels q | k | v. The slots hold the last taps - 1 inputs [taps - 1, C], bias
+    included, at tail_off; those of the first ``n_single`` sequences, which bring one row each, are
+    advanced here, the others' by conv_tail_update behind this."""
+    _f32_rows(p, "conv_qkv_prepare: p")
+    T = p.shape[0]
+    nq, nk, nv = Hq * Dk, Hk * Dk, Hv * Dv
+    C = nq + nk + nv
+    for off, n in ((q_off, nq), (k_off, nk), (v_off, nv)):
+        if off < 0 or off + n > p.shape[1]:
+            raise KernelError("conv_qkv_prepare: the columns of q, k or v lie outside p")
+    if q_out.shape != (T, Hq, Dk) or not q_out.is_contiguous() or not q_out.is_cuda:
+        raise KernelError(f"conv_qkv_prepare: q_out must be a contiguous [{T}, {Hq}, {Dk}] GPU tensor")
+    _f32_vec(bias, C, "conv_qkv_prepare: bias")
+    taps = 1
+    if conv_weight is not None:
+        if conv_weight.dim() != 2 or conv_weight.shape[0] != C:
+            raise KernelError(f"conv_qkv_prepare: conv_weight must be [{C}, taps]")
+        taps = conv_weight.shape[1]
+        _f32_vec(conv_weight, C * taps, "conv_qkv_prepare: conv_weight")
+    _i32(q_start, "q_start")
+    _i32(state_slots, "state_slots")
+    _i32(positions, "positions")
+    n = state_slots.numel()
+    if q_start.numel() != n + 1 or not 0 <= n_single <= n or positions.numel() != T:
+        raise KernelError("conv_qkv_prepare: inconsistent sequence tables")
+    if taps > 1 and (state is None or state.dim() != 2 or state.dtype != torch.float32 or not state.is_contiguous()
+                     or not state.is_cuda or tail_off < 0 or tail_off + (taps - 1) * C > state.shape[1]):
+        raise KernelError("conv_qkv_prepare: the kept inputs lie outside the state")
+    if rot_dims:
+        if rot_dims % 2 or rot_dims > Dk:
+            raise KernelError(f"conv_qkv_prepare: {rot_dims} rotating entries of {Dk}")
+        _f32_vec(inv_freq, rot_dims // 2, "conv_qkv_prepare: frequencies")
+    if slots is not None:
+        _i32(slots, "slots")
+        _need_gpu(k_cache, v_cache, slots)
+        if (slots.numel() != T or k_cache.dim() != 4 or v_cache.dim() != 4
+                or k_cache.shape[1:] != (Hk, page_size, Dk) or v_cache.shape[1:] != (Hv, page_size, Dv)
+                or k_cache.shape[0] != v_cache.shape[0] or k_cache.dtype != q_out.dtype
+                or v_cache.dtype != q_out.dtype or not k_cache.is_contiguous() or not v_cache.is_contiguous()):
+            raise KernelError("conv_qkv_prepare: caches must be contiguous [pages, heads, page_size, size] of "
+                              "q_out's dtype, with one slot a row")
+    write = slots is not None
+    _check(library.load("prepare").ptl_conv_qkv_prepare(
+        _ptr(q_out), _ptr(p), ctypes.c_long(p.stride(0)), int(q_off), int(k_off), int(v_off), _ptr(bias),
+        _ptr(conv_weight), int(taps), _ptr(state) if taps > 1 else None,
+        ctypes.c_long(state.stride(0) if taps > 1 else 0), ctypes.c_long(tail_off), _ptr(q_start), _ptr(state_slots),
+        n, int(n_single), _ptr(positions), _ptr(slots), int(rot_dims), int(layout),
+        _ptr(inv_freq) if rot_dims else None, int(bool(norm)), ctypes.c_float(eps),
+        _ptr(k_cache) if write else None, _ptr(v_cache) if write else None, T, Hq, Hk, Hv, Dk, Dv, int(page_size),
+        _dtype_code(q_out), _stream()), "conv_qkv_prepare")
+
+
 def head_norm_gate(out: torch.Tensor, a: torch.Tensor, maps: int = 1, lam: float = 0.0, weight=None,
                    weight_per_head: bool = False, mult: float = 1.0, gate: Optional[torch.Tensor] = None,
                    gate_off: int = 0, act: int = GATE_NONE, eps: float = 0.0) -> None:
@@ -1549,6 +1662,36 @@ def stream_postnorm(stream: torch.Tensor, alpha: float, y1: torch.Tensor, a: flo
     return copy
 
 
+def stream_scaled_sum(stream: torch.Tensor, y1: Optional[torch.Tensor] = None, scale1: Optional[torch.Tensor] = None,
+                      bias: Optional[torch.Tensor] = None, y2: Optional[torch.Tensor] = None,
+                      scale2: Optional[torch.Tensor] = None, norm_weight: Optional[torch.Tensor] = None,
+                      eps: float = 0.0, out_dtype: Optional[torch.dtype] = None) -> Optional[torch.Tensor]:
+    """stream += scale1 * (y1 + bias) + scale2 * y2 in place, entry by entry (y1 float32; every piece is
+    optional, a scale that is None is one); with ``norm_weight`` returns rmsnorm(stream) * norm_weight in
+    ``out_dtype``."""
+    T, H = _check_stream(stream, "stream_scaled_sum")
+    if H > 16384:
+        raise KernelError(f"stream_scaled_sum: rows of up to 16384 entries, got {H}")
+    if y1 is None and y2 is None and norm_weight is None:
+        raise KernelError("stream_scaled_sum: nothing to do")
+    for y in (y1, y2):
+        if y is not None and (not y.is_cuda or y.shape != stream.shape or not y.is_contiguous()):
+            raise KernelError("stream_scaled_sum: the terms must be contiguous matrices of the stream's shape")
+    if (y1 is not None and y1.dtype != torch.float32) or (y1 is None and bias is not None):
+        raise KernelError("stream_scaled_sum: the first term is float32, and a bias goes with it")
+    out_dtype = out_dtype or torch.float32
+    if y2 is not None and y2.dtype == torch.bfloat16 and out_dtype == torch.float32:
+        y2 = y2.float()
+    for v, what in ((scale1, "scale1"), (bias, "bias"), (scale2, "scale2"), (norm_weight, "norm_weight")):
+        _f32_vec(v, H, f"stream_scaled_sum: {what}")
+    out = torch.empty((T, H), dtype=out_dtype, device=stream.device) if norm_weight is not None else None
+    _check(library.load("stream").ptl_stream_scaled_sum(
+        _ptr(stream), _ptr(y1), _ptr(scale1), _ptr(bias), _ptr(y2), _dtype_code(y2) if y2 is not None else _F32,
+        _ptr(scale2), _ptr(norm_weight), ctypes.c_float(eps), _ptr(out),
+        _F32 if out_dtype == torch.float32 else _BF16, T, H, _stream()), "stream_scaled_sum")
+    return out
+
+
 def stream_rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch.dtype) -> torch.Tensor:
     """rmsnorm(x) * weight for rows x of a float32 stream, in ``out_dtype``."""
     T, H = _check_stream(x, "stream_rmsnorm")
@@ -1616,9 +1759,11 @@ def conv_prepare(p: torch.Tensor, x_off: int, conv_weight: torch.Tensor, state: 
 
 
 def conv_tail_update(p: torch.Tensor, x_off: int, C: int, taps: int, state: torch.Tensor, tail_off: int,
-                     q_start: torch.Tensor, state_slots: torch.Tensor) -> None:
-    """The slots' last taps - 1 inputs after this step (after conv_prepare has read the old ones)."""
+                     q_start: torch.Tensor, state_slots: torch.Tensor, bias: Optional[torch.Tensor] = None) -> None:
+    """The slots' last taps - 1 inputs after this step (after conv_prepare has read the old ones).
+    ``bias`` float32 [C]: added to the step's inputs."""
     _f32_rows(p, "conv_tail_update: p")
+    _f32_vec(bias, C, "conv_tail_update: bias")
     _need_gpu(state, q_start, state_slots)
     if state.dim() != 2 or state.dtype != torch.float32 or not state.is_contiguous() \
             or tail_off + (taps - 1) * C > state.shape[1] or x_off + C > p.shape[1]:
@@ -1628,7 +1773,7 @@ def conv_tail_update(p: torch.Tensor, x_off: int, C: int, taps: int, state: torc
     _check(library.load("recurrent").ptl_conv_tail_update(
         _ptr(state), ctypes.c_long(state.stride(0)), ctypes.c_long(tail_off), _ptr(p),
         ctypes.c_long(p.stride(0)), int(x_off), _ptr(q_start), _ptr(state_slots), state_slots.numel(),
-        int(C), int(taps), _stream()), "conv_tail_update")
+        _ptr(bias), int(C), int(taps), _stream()), "conv_tail_update")
 
 
 # Segments of the delta rule (ptl_delta_scan_segments): 256 tokens, 512 from 2,048 rows on, used from
@@ -1754,7 +1899,7 @@ class Routing:
 def moe_route(logits: torch.Tensor, experts: int, top: int, extra: int = 0,
               renormalize: bool = False, score: int = SCORE_SIGMOID, correction: Optional[torch.Tensor] = None,
               identity: int = 0, renorm_eps: float = 0.0, weight_scale: float = 1.0,
-              groups: int = 1, keep_groups: int = 1) -> Routing:
+              groups: int = 1, keep_groups: int = 1, logit_bias: Optional[torch.Tensor] = None) -> Routing:
     """Route every row of float32 ``logits`` [T, experts + identity + extra] to ``top`` of its
     ``experts + identity`` router outputs and order the pairs by expert. Scores: the sigmoid of
     the logits, or their softmax over the router outputs; the choice goes by score +
@@ -1764,7 +1909,8 @@ def moe_route(logits: torch.Tensor, experts: int, top: int, extra: int = 0,
     products, and ``ident`` [T] holds the sum of their weights a token. ``groups`` > 1: the router
     outputs form that many equal groups of neighbours (at most 64); a group's score is the sum
     of its two largest choice scores (score + correction), and only outputs of the best
-    ``keep_groups`` groups can be chosen."""
+    ``keep_groups`` groups can be chosen. ``logit_bias`` [experts + identity]: added to the router's outputs
+    before anything else."""
     _need_gpu(logits)
     if logits.dim() != 2 or logits.dtype != torch.float32 or logits.stride(1) != 1 \
             or logits.shape[1] < experts + extra:
@@ -1777,6 +1923,7 @@ def moe_route(logits: torch.Tensor, experts: int, top: int, extra: int = 0,
                           "kernel takes")
     if correction is not None:
         _f32_vec(correction, outputs, "moe_route: correction")
+    _f32_vec(logit_bias, outputs, "moe_route: logit_bias")
     if groups < 1 or (groups > 1 and (groups > 64 or outputs % groups or not 1 <= keep_groups <= groups
                                       or keep_groups * (outputs // groups) < top)):
         raise KernelError(f"moe_route: {groups} groups of which {keep_groups} are kept do not fit "
@@ -1796,7 +1943,7 @@ def moe_route(logits: torch.Tensor, experts: int, top: int, extra: int = 0,
     r.wgt = torch.empty(A, dtype=torch.float32, device=dev)
     r.extra = torch.empty((T, extra), dtype=torch.float32, device=dev) if extra else None
     r.ident = torch.empty(T, dtype=torch.float32, device=dev) if identity else None
-    _check(lib.ptl_moe_topk(_ptr(logits), int(logits.stride(0)), T, outputs, top, extra, int(renormalize),
+    _check(lib.ptl_moe_topk(_ptr(logits), int(logits.stride(0)), _ptr(logit_bias), T, outputs, top, extra, int(renormalize),
                             int(score), _ptr(correction), experts, ctypes.c_float(renorm_eps),
                             ctypes.c_float(weight_scale), int(groups), int(keep_groups), _ptr(r.idx),
                             _ptr(r.wgt), _ptr(r.extra), _ptr(r.ident), _stream()), "moe_topk")
@@ -2037,17 +2184,32 @@ def _linear_columns(m, width, what):
         raise KernelError(f"{what}: float32 [T, >= {width}] with dense rows")
 
 
+def _kept_row(keep, T: int, state: torch.Tensor, matrices: int, what: str):
+    """The arguments (x, row stride, dtype, offset, width) of a row that is left in the state slots."""
+    if keep is None:
+        return None, ctypes.c_long(0), 0, ctypes.c_long(0), 0
+    x, off = keep
+    if not x.is_cuda or x.dim() != 2 or x.stride(1) != 1 or x.shape[0] != T or off < matrices \
+            or off + x.shape[1] > state.shape[1]:
+        raise KernelError(f"{what}: the kept row [T, W] lies outside the state slot, or inside the matrices")
+    return _ptr(x), ctypes.c_long(x.stride(0)), _dtype_code(x), ctypes.c_long(off), x.shape[1]
+
+
 def linear_scan(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, G: int, D: int,
                 state: torch.Tensor, q_start: torch.Tensor, state_slots: torch.Tensor, max_q_len: int,
                 qscale: float = 1.0, dt: Optional[torch.Tensor] = None, A_log: Optional[torch.Tensor] = None,
                 dt_bias: Optional[torch.Tensor] = None, skip: Optional[torch.Tensor] = None,
-                decay: Optional[torch.Tensor] = None, seg_len: int = 0) -> None:
+                decay: Optional[torch.Tensor] = None, seg_len: int = 0, bonus: Optional[torch.Tensor] = None,
+                keep=None) -> None:
     """S <- diag(a) S + k v^T, o = S^T (qscale q) over the rows of every sequence named by q_start and
     state_slots, from and to the state slots; out float32 [T, H, Dv] receives their rows. q, k:
     float32 matrices whose first G * D columns are the heads' (head h uses q/k head h / (H / G)); v:
     H * Dv columns. Either ``decay`` float32 [T, >= H * D] (a decay a key channel), or dt (raw step
     sizes, H columns), A_log, dt_bias, skip [H]: step = softplus(dt + dt_bias), a = exp(-exp(A_log)
-    step), the value is step * v and skip * v is added to the result. ``max_q_len``: the rows of the
+    step), the value is step * v and skip * v is added to the result. ``bonus`` float32 [H * D] (with
+    ``decay``): the read-out takes S from in front of the update, and the current token's own product times
+    the bonus, o = (S_old + diag(bonus) k v^T)^T q. ``keep`` = (x, off): every sequence's last row of x
+    [T, W] is left at ``off`` of its state slot. ``max_q_len``: the rows of the
     longest sequence (or a bound); ``seg_len``: rows of the segments that are walked side by side (0:
     chosen by linear_segment)."""
     if out.dim() != 3 or out.dtype != torch.float32 or not out.is_contiguous() or not out.is_cuda:
@@ -2073,6 +2235,11 @@ def linear_scan(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Te
         if G != H:
             raise KernelError("linear_scan: decays a key channel come with a q/k head a head")
         _linear_columns(decay, H * D, "linear_scan: decay")
+    if bonus is not None:
+        if scalar:
+            raise KernelError("linear_scan: a bonus goes with decays a key channel")
+        _f32_vec(bonus, H * D, "linear_scan: bonus")
+    kept = _kept_row(keep, T, state, linear_state_floats(H, D, Dv), "linear_scan")
     max_q_len = max(1, min(int(max_q_len), T))
     seg_len = int(seg_len) or linear_segment(n, max_q_len, H, Dv, compute_units(out.device))
     P = -(-max_q_len // seg_len)
@@ -2086,15 +2253,43 @@ def linear_scan(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Te
         else:
             work = torch.empty((floats,), dtype=torch.float32, device=out.device)
     _check(lib.ptl_linear_scan(
-        0 if scalar else 1, _ptr(out), _ptr(q), ctypes.c_long(q.stride(0)), _ptr(k), ctypes.c_long(k.stride(0)),
+        0 if scalar else (1 if bonus is None else 2), _ptr(out), _ptr(q), ctypes.c_long(q.stride(0)), _ptr(k), ctypes.c_long(k.stride(0)),
         _ptr(v), ctypes.c_long(v.stride(0)), ctypes.c_float(qscale), _ptr(dt),
         ctypes.c_long(dt.stride(0) if scalar else 0), _ptr(A_log), _ptr(dt_bias), _ptr(skip), _ptr(decay),
-        ctypes.c_long(0 if scalar else decay.stride(0)), _ptr(state), ctypes.c_long(state.stride(0)), _ptr(work),
+        ctypes.c_long(0 if scalar else decay.stride(0)), _ptr(bonus), *kept, _ptr(state), ctypes.c_long(state.stride(0)), _ptr(work),
         int(P), int(seg_len), _ptr(q_start), _ptr(state_slots), n, H, G, D, Dv, _stream()), "linear_scan")
 
 
-def lowrank_decay(r: torch.Tensor, w: torch.Tensor, bias: torch.Tensor, tau: float) -> torch.Tensor:
-    """sigmoid(w . r + bias)^(1 / tau): float32 [T, C] from r (float32, the first R columns of its
+def time_shift(x: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, off: int, q_start: torch.Tensor,
+               state_slots: torch.Tensor) -> torch.Tensor:
+    """out[j, t] = x[t] + (x' - x[t]) * mu[j], x' the row before in the sequence: [S, T, W] in x's dtype from
+    x [T, W] and mu float32 [S, W]. In front of a portion's first row stands the kept row, float32 [W] at
+    ``off`` of the sequence's state slot."""
+    _need_gpu(x, mu, state, q_start, state_slots)
+    if x.dim() != 2 or x.stride(1) != 1 or mu.dim() != 2 or mu.shape[1] != x.shape[1]:
+        raise KernelError("time_shift: x [T, W] with dense rows, mu [S, W]")
+    T, W = x.shape
+    S = mu.shape[0]
+    _f32_vec(mu, S * W, "time_shift: mu")
+    _i32(q_start, "q_start")
+    _i32(state_slots, "state_slots")
+    if state.dim() != 2 or state.dtype != torch.float32 or not state.is_contiguous() or off < 0 \
+            or off + W > state.shape[1] or q_start.numel() != state_slots.numel() + 1:
+        raise KernelError("time_shift: the kept rows lie outside the state, or inconsistent sequence tables")
+    out = torch.empty((S, T, W), dtype=x.dtype, device=x.device)
+    _check(library.load("linear_scan").ptl_time_shift(
+        _ptr(out), ctypes.c_long(T * W), _ptr(x), ctypes.c_long(x.stride(0) if T > 1 else W), _ptr(mu), S, _ptr(state),
+        ctypes.c_long(state.stride(0)), ctypes.c_long(off), _ptr(q_start), _ptr(state_slots), state_slots.numel(),
+        T, W, _dtype_code(x), _stream()), "time_shift")
+    return out
+
+
+DECAY_SIGMOID, DECAY_EXP = 0, 1
+
+
+def lowrank_decay(r: torch.Tensor, w: torch.Tensor, bias: torch.Tensor, tau: float = 1.0,
+                  form: int = DECAY_SIGMOID) -> torch.Tensor:
+    """sigmoid(w . r + bias)^(1 / tau), or with ``form`` DECAY_EXP exp(-exp(w . tanh(r) + bias)): float32 [T, C] from r (float32, the first R columns of its
     rows), w float32 [C, R], bias [C]."""
     C, R = w.shape
     _linear_columns(r, R, "lowrank_decay: r")
@@ -2105,8 +2300,8 @@ def lowrank_decay(r: torch.Tensor, w: torch.Tensor, bias: torch.Tensor, tau: flo
     T = r.shape[0]
     out = torch.empty((T, C), dtype=torch.float32, device=r.device)
     _check(library.load("linear_scan").ptl_lowrank_decay(
-        _ptr(out), _ptr(r), ctypes.c_long(r.stride(0)), _ptr(w), _ptr(bias), ctypes.c_float(1.0 / tau), T, C, R,
-        _stream()), "lowrank_decay")
+        _ptr(out), _ptr(r), ctypes.c_long(r.stride(0)), _ptr(w), _ptr(bias), int(form), ctypes.c_float(1.0 / tau),
+        T, C, R, _stream()), "lowrank_decay")
     return out
 
 
@@ -2143,29 +2338,51 @@ def linear_decode_conv(out: torch.Tensor, p: torch.Tensor, x_off: int, b_off: in
         H, G, D, Dv, _stream()), "linear_decode_conv")
 
 
+def _lowrank_columns(out, p, q_off, k_off, v_off, a_off, w, bias, state, q_start, state_slots, D, what):
+    _f32_rows(p, f"{what}: p")
+    T, H, Dv = out.shape
+    n = _linear_state(state, q_start, state_slots, H, D, Dv, 0, what)
+    if out.dtype != torch.float32 or not out.is_contiguous() or p.shape[0] != T:
+        raise KernelError(f"{what}: out must be contiguous float32 [T, H, Dv]")
+    C, R = w.shape
+    if C != H * D:
+        raise KernelError(f"{what}: w must have {H * D} rows")
+    for off, width in ((q_off, H * D), (k_off, H * D), (v_off, H * Dv), (a_off, R)):
+        if off < 0 or off + width > p.shape[1]:
+            raise KernelError(f"{what}: columns outside p")
+    _f32_vec(w, C * R, f"{what}: w")
+    _f32_vec(bias, C, f"{what}: bias")
+    return n, H, Dv, R
+
+
 def linear_decode_lowrank(out: torch.Tensor, p: torch.Tensor, q_off: int, k_off: int, v_off: int, a_off: int,
                           qscale: float, w: torch.Tensor, bias: torch.Tensor, tau: float, state: torch.Tensor,
                           q_start: torch.Tensor, state_slots: torch.Tensor, D: int) -> None:
     """One token of every sequence named by q_start and state_slots: the recurrence of linear_scan with
     a decay a key channel, sigmoid(w . r + bias)^(1 / tau), r the columns of p from a_off on."""
-    _f32_rows(p, "linear_decode_lowrank: p")
-    T, H, Dv = out.shape
-    n = _linear_state(state, q_start, state_slots, H, D, Dv, 0, "linear_decode_lowrank")
-    if out.dtype != torch.float32 or not out.is_contiguous() or p.shape[0] != T:
-        raise KernelError("linear_decode_lowrank: out must be contiguous float32 [T, H, Dv]")
-    C, R = w.shape
-    if C != H * D:
-        raise KernelError(f"linear_decode_lowrank: w must have {H * D} rows")
-    for off, width in ((q_off, H * D), (k_off, H * D), (v_off, H * Dv), (a_off, R)):
-        if off < 0 or off + width > p.shape[1]:
-            raise KernelError("linear_decode_lowrank: columns outside p")
-    _f32_vec(w, C * R, "linear_decode_lowrank: w")
-    _f32_vec(bias, C, "linear_decode_lowrank: bias")
+    n, H, Dv, R = _lowrank_columns(out, p, q_off, k_off, v_off, a_off, w, bias, state, q_start, state_slots, D,
+                                   "linear_decode_lowrank")
     _check(library.load("linear_scan").ptl_linear_decode_lowrank(
         _ptr(out), _ptr(p), ctypes.c_long(p.stride(0)), int(q_off), int(k_off), int(v_off), int(a_off),
         ctypes.c_float(qscale), _ptr(w), _ptr(bias), R, ctypes.c_float(1.0 / tau), _ptr(state),
         ctypes.c_long(state.stride(0)), _ptr(q_start), _ptr(state_slots), n, H, D, Dv, _stream()),
         "linear_decode_lowrank")
+
+
+def linear_decode_bonus(out: torch.Tensor, p: torch.Tensor, q_off: int, k_off: int, v_off: int, a_off: int,
+                        w: torch.Tensor, bias: torch.Tensor, bonus: torch.Tensor, state: torch.Tensor,
+                        q_start: torch.Tensor, state_slots: torch.Tensor, D: int, keep=None) -> None:
+    """One token of every sequence named by q_start and state_slots: the recurrence of linear_scan with a
+    ``bonus`` and the decays exp(-exp(w . tanh(r) + bias)), r the columns of p from a_off on; ``keep`` as
+    there."""
+    n, H, Dv, R = _lowrank_columns(out, p, q_off, k_off, v_off, a_off, w, bias, state, q_start, state_slots, D,
+                                   "linear_decode_bonus")
+    _f32_vec(bonus, H * D, "linear_decode_bonus: bonus")
+    kept = _kept_row(keep, out.shape[0], state, linear_state_floats(H, D, Dv), "linear_decode_bonus")
+    _check(library.load("linear_scan").ptl_linear_decode_bonus(
+        _ptr(out), _ptr(p), ctypes.c_long(p.stride(0)), int(q_off), int(k_off), int(v_off), int(a_off), _ptr(w),
+        _ptr(bias), R, _ptr(bonus), *kept, _ptr(state), ctypes.c_long(state.stride(0)), _ptr(q_start),
+        _ptr(state_slots), n, H, D, Dv, _stream()), "linear_decode_bonus")
 
 
 def gate_group_norm(y: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, groups: int, eps: float,

@@ -11,5 +11,5 @@ from .token_input import GatedTokenInput, TokenTable
 from .embedding import LinearHead, TokenEmbedding
 from .normed_attention import NormedAttention
 from .recurrent import GatedDeltaRule, MatrixMemory, ParallelMixers, SelectiveScan
-from .linear_recurrent import GatedLinearAttention, Mamba2
-from .block import HyperConnectionBlock, OutputNormBlock, PostNormBlock, PreNormBlock, SandwichBlock
+from .linear_recurrent import GatedLinearAttention, Mamba2, TimeMixer
+from .block import HyperConnectionBlock, OutputNormBlock, ParallelResidualBlock, PostNormBlock, PreNormBlock, SandwichBlock

@@ -417,3 +417,88 @@ class HyperConnectionBlock(Part):
         a = self._step(streams, y, 0, (c[0] if c is not None else None, self.norm2.weight, self.norm2.eps), dtype)
         y = self.feed_forward.forward(a)
         return streams, self._step(streams, y, 1, after, dtype)
+
+
+@register_part("block", "parallel_residual")
+class ParallelResidualBlock(Part):
+    """Two sublayers side by side on one normed input, on a residual stream kept in float32, their
+    results scaled entry by entry:
+
+        h = rmsnorm(x) w;    x <- x + s1 * mixer(h) + s2 * ffn(h)
+
+    The feed-forward with its scale is optional; ``scaled`` False: no scales in the checkpoint. The stream
+    is the block's ``h`` (float32 [T, hidden], updated in place). The sum, a bias that the mixer's result
+    still lacks (parts.base.PendingSum) and the norm in front of the block that runs next (``next_block``)
+    are one kernel; the normed rows travel where other blocks carry a residual. Sublayers read the
+    engine's dtype; the mixer may return float32 or it, and so may the feed-forward."""
+    takes_next_block = True
+
+    def __init__(self, hidden_size: int, mixer: Part, norm: Part, feed_forward: Part = None, scaled: bool = True,
+                 mixer_scale: str = "ls1", ffn_scale: str = "ls2"):
+        if not (hasattr(norm, "weight") and hasattr(norm, "eps")):
+            raise ValueError("the norm of this block is an RMS norm (a weight and an eps)")
+        self.hidden_size, self.scaled = int(hidden_size), bool(scaled)
+        self.mixer, self.norm1, self.feed_forward = mixer, norm, feed_forward
+        self.scale_names = (mixer_scale, ffn_scale)
+        self.scale1 = self.scale2 = None
+        libs = ("stream",)
+        for p in self._parts():
+            libs += tuple(p.kernel_libraries)
+        self.kernel_libraries = tuple(dict.fromkeys(libs))
+
+    def children(self):
+        roles = {"mixer": self.mixer, "norm1": self.norm1, "feed_forward": self.feed_forward,
+                 "scales": self if self.scaled else None}
+        return {k: p for k, p in roles.items() if p is not None}
+
+    def _parts(self):
+        return [p for p in (self.mixer, self.norm1, self.feed_forward) if p is not None]
+
+    def cache_spec(self):
+        return self.mixer.cache_spec() if hasattr(self.mixer, "cache_spec") else None
+
+    def work_lists(self):
+        lists = ()
+        for p in self._parts():
+            if hasattr(p, "work_lists"):
+                lists += tuple(p.work_lists())
+        return tuple(dict.fromkeys(lists))
+
+    def make_decode_copies(self) -> int:
+        return sum(p.make_decode_copies() for p in self._parts() if hasattr(p, "make_decode_copies"))
+
+    @property
+    def graph_capturable(self) -> bool:
+        return all(getattr(p, "graph_capturable", True) for p in self._parts())
+
+    # the block's own tensors: the scales of its sublayers' results
+    def param_sources(self):
+        if not self.scaled:
+            return []
+        names = self.scale_names if self.feed_forward is not None else self.scale_names[:1]
+        return [ParamSource(n, (self.hidden_size,), "vector", init=("normal", 1.0, 0.2)) for n in names]
+
+    def load(self, tensors, dtype, device) -> None:
+        a, b = self.scale_names
+        if a in tensors:
+            self.scale1 = place(tensors[a], "vector", dtype, device)
+        if b in tensors:
+            self.scale2 = place(tensors[b], "vector", dtype, device)
+
+    def forward(self, h, residual, ctx, cache, next_block=None):
+        if h.dtype != torch.float32 or h.shape[1] != self.hidden_size:
+            raise ops.KernelError("a parallel-residual block runs on a float32 residual stream")
+        stream, dtype = h, self.norm1.dtype
+        a = residual
+        if a is None:
+            a = ops.stream_scaled_sum(stream, norm_weight=self.norm1.weight, eps=self.norm1.eps, out_dtype=dtype)
+        y, bias = self.mixer.forward(a, ctx, cache), None
+        if isinstance(y, PendingSum) and len(y.terms) == 1 and y.terms[0][1] == 1.0 and y.norms is None \
+                and (y.bias is None or y.bias[1] == 1.0):
+            y, bias = y.terms[0][0], (y.bias[0] if y.bias is not None else None)
+        y = as_tensor(y)
+        z = as_tensor(self.feed_forward.forward(a)) if self.feed_forward is not None else None
+        norm = next_block.norm1 if isinstance(next_block, ParallelResidualBlock) else None
+        return stream, ops.stream_scaled_sum(stream, y if y.dtype == torch.float32 else y.float(), self.scale1, bias, z,
+                                             self.scale2, norm.weight if norm is not None else None,
+                                             norm.eps if norm is not None else 0.0, dtype)

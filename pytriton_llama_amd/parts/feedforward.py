@@ -71,7 +71,8 @@ class SwiGLU(Part):
 class GatedMLP(Part):
     """down(act(gate(x), up(x))) with the activation as a parameter: "silu" (silu(g) * u) or
     "clamped" (g' = min(g, limit), u' = clamp(u, -limit, limit), g' * sigmoid(1.702 g') * (u' + 1)).
-    No biases. gate and up are one [2I, hidden] matrix at run time."""
+    No biases. gate and up are one [2I, hidden] matrix at run time; the few rows of a decode step take the
+    product and the activation in one kernel."""
     kernel_libraries = ("moe",) + LINEAR_LIBRARIES
 
     def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "silu",
@@ -80,6 +81,7 @@ class GatedMLP(Part):
             raise ValueError(f"unknown gated activation {activation!r}")
         self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
         self.act = ops.ACT_CLAMPED if activation == "clamped" else ops.ACT_SILU
+        self.glu = ops.GLU_CLAMPED if activation == "clamped" else ops.GLU_SILU
         self.limit = float(limit)
         self.names = (gate_name, up_name, down_name)
         self.gate_up = self.down = self.gate_up_blocked = self.down_blocked = None
@@ -102,6 +104,9 @@ class GatedMLP(Part):
 
     def forward(self, x):
         x = as_tensor(x)
+        if ops.gate_up_silu_fits(x, self.gate_up, self.gate_up_blocked):
+            a = ops.gate_up_silu(x, self.gate_up, None, self.gate_up_blocked, self.glu, self.limit)
+            return linear(a, self.down, blocked=self.down_blocked)
         a = ops.gated_act(linear(x, self.gate_up, blocked=self.gate_up_blocked), self.act, self.limit)
         return linear(a, self.down, blocked=self.down_blocked)
 
@@ -148,7 +153,9 @@ class RoutedExperts(Part):
     "softmax", the softmax of z over all router outputs; the ``top`` outputs with the largest
     scores are taken (with ``correction_name``: the largest score + a per-output vector of the
     checkpoint; the weights stay the scores without it); their scores are the weights
-    (``renormalize``: divided by their sum + renorm_eps; then times route_scale).
+    (``renormalize``: divided by their sum + renorm_eps; then times route_scale). ``router_bias_name``: a
+    vector of the checkpoint, float32, added to z (with score "softmax", renormalize and no
+    correction the weights are the softmax over the chosen outputs' z alone).
     ``weight_on_input``: the weight multiplies what the expert reads, y = sum_k expert_k(s_k x),
     instead of what it returns. Experts are gated, down(act(gate(x), up(x))) with ``activation``
     "silu" or "clamped", or, with "relu2", down(relu(up(x))^2) without a gate. ``identity``: that
@@ -171,6 +178,7 @@ class RoutedExperts(Part):
                  renormalize: bool = False, shared: Optional[Part] = None, shared_gate: bool = True,
                  score: str = "sigmoid", correction_name: Optional[str] = None, identity: int = 0,
                  renorm_eps: float = 0.0, route_scale: float = 1.0, groups=None,
+                 router_bias_name: Optional[str] = None,
                  router_name: str = "router", expert_prefix: str = "e", shared_prefix: str = "shared.",
                  shared_gate_name: str = "shared.sg", gate_name: str = "gate", up_name: str = "up",
                  down_name: str = "down"):
@@ -196,13 +204,13 @@ class RoutedExperts(Part):
                 or self.keep_groups * (outputs // self.groups) < self.top or self.groups > 64:
             raise ValueError(f"{self.groups} groups of which {self.keep_groups} are kept do not fit {outputs} "
                              f"router outputs with {self.top} chosen (at most 64 equal groups)")
-        self.correction_name = correction_name
+        self.correction_name, self.router_bias_name = correction_name, router_bias_name
         self.shared = shared
         self.shared_gate = bool(shared_gate) and shared is not None
         self.router_name, self.expert_prefix = router_name, expert_prefix
         self.shared_prefix, self.shared_gate_name = shared_prefix, shared_gate_name
         self.names = (gate_name, up_name, down_name)
-        self.router = self.gate_up = self.down = self.correction = None
+        self.router = self.gate_up = self.down = self.correction = self.router_bias = None
         if shared is not None:
             self.kernel_libraries = tuple(dict.fromkeys(self.kernel_libraries + tuple(shared.kernel_libraries)))
 
@@ -213,6 +221,9 @@ class RoutedExperts(Part):
         if self.correction_name:
             out.append(ParamSource(self.correction_name, (self.num_experts + self.identity,), "vector",
                                    init=("normal", 0.0, 0.02)))
+        if self.router_bias_name:
+            out.append(ParamSource(self.router_bias_name, (self.num_experts + self.identity,), "vector",
+                                   init=("normal", 0.0, 0.2)))
         for e in range(self.num_experts):
             p = f"{self.expert_prefix}{e}."
             if self.gated:
@@ -233,6 +244,8 @@ class RoutedExperts(Part):
         self.router = place(torch.cat(router, dim=0), "matrix", dtype, device)
         if self.correction_name:
             self.correction = place(tensors[self.correction_name], "vector", dtype, device)
+        if self.router_bias_name:
+            self.router_bias = place(tensors[self.router_bias_name], "vector", dtype, device)
         names = [f"{self.expert_prefix}{e}." for e in range(self.num_experts)]
         first = (lambda p: torch.cat([tensors[p + g], tensors[p + u]], dim=0)) if self.gated \
             else (lambda p: tensors[p + u])
@@ -251,7 +264,7 @@ class RoutedExperts(Part):
         logits = linear(x, self.router, out_dtype=torch.float32)
         r = ops.moe_route(logits, self.num_experts, self.top, 1 if self.shared_gate else 0, self.renormalize,
                           self.score, self.correction, self.identity, self.renorm_eps, self.route_scale,
-                          self.groups, self.keep_groups)
+                          self.groups, self.keep_groups, self.router_bias)
         shared = self.shared.forward(x) if self.shared is not None else None
         return ops.moe_experts(x, r, self.gate_up, self.down, self.act, self.limit, self.weight_on_input,
                                shared, r.extra)

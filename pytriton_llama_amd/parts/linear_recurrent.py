@@ -1,6 +1,6 @@
 """Mixers whose memory is a matrix a head that decays and takes outer products
-(csrc/linear_scan.hip): Mamba-2 (one decay a head) and gated linear attention (a decay a key
-channel)."""
+(csrc/linear_scan.hip): Mamba-2 (one decay a head), gated linear attention (a decay a key
+channel) and the time mixer of RWKV (the same with a bonus on the current token)."""
 from __future__ import annotations
 
 from typing import List, Optional
@@ -14,7 +14,7 @@ from .normed_attention import pad_rows
 
 
 class _LinearStateMixer(Part):
-    """What the two mixers below share: one fused first projection whose result is taken in
+    """What the first two mixers below share: one fused first projection whose result is taken in
     float32, a float32 state slot, and an output projection with a float32 result. Sequences of one
     token (the leading ones of a step) take the decode kernel, the others the chunked one."""
     kernel_libraries = ("linear_scan", "prepare") + LINEAR_LIBRARIES
@@ -197,3 +197,87 @@ class GatedLinearAttention(_LinearStateMixer):
         out = torch.empty((y.shape[0], self.num_heads * self.vdim), dtype=dtype, device=y.device)
         ops.head_norm_gate(out, y, 1, 0.0, self.norm_weight, False, 1.0, p, self.g_off, ops.GATE_SILU, self.eps)
         return out
+
+
+@register_part("mixer", "time_mixer")
+class TimeMixer(Part):
+    """The time mixer of RWKV-6 (Peng et al.: "Eagle and Finch: RWKV with Matrix-Valued States and
+    Dynamic Recurrence"), without its data-dependent mixing: with x' the token's row before (zeros in front of
+    the first), each of r, k, v, g, w reads its own mix x + (x' - x) mu; r, k, v [heads, dim] are W_r, W_k,
+    W_v of theirs, the decay a key channel is a = exp(-exp(W_w2 tanh(W_w1 mix_w) + w0)), per head
+
+        o = (S + diag(u) k v^T)^T r;    S <- diag(a) S + k v^T
+
+    then each head's o divided by its root mean square, times a weight of all heads' size, times silu(W_g
+    mix_g), then W_o. S and the last row x live in the request's state slot in float32; W_w1's result is
+    taken in float32 and W_w2 held in float32. ``rank``: the rows of W_w1; None: the checkpoint says
+    (``rank_from``), and random weights are drawn with DEFAULT_RANK."""
+    kernel_libraries = ("linear_scan", "prepare") + LINEAR_LIBRARIES
+    DEFAULT_RANK = 16
+    MIXES = ("r", "k", "v", "g", "w")          # the order of the projections' rows (w: those of W_w1)
+
+    def __init__(self, hidden_size: int, num_heads: int, dim: int, eps: float, rank: Optional[int] = None,
+                 mu_prefix: str = "mu.", r_name: str = "r", k_name: str = "k", v_name: str = "v", g_name: str = "g",
+                 w1_name: str = "w1", w2_name: str = "w2", w0_name: str = "w0", u_name: str = "u",
+                 norm_name: str = "norm", o_name: str = "o"):
+        if dim > ops.LINEAR_MAX_KEYS:
+            raise ValueError(f"the recurrence kernels take key sizes up to {ops.LINEAR_MAX_KEYS}, got {dim}")
+        self.hidden_size, self.num_heads, self.dim, self.eps = int(hidden_size), int(num_heads), int(dim), float(eps)
+        self.rank = int(rank) if rank else self.DEFAULT_RANK
+        self.mu_prefix = mu_prefix
+        self.names = dict(r=r_name, k=k_name, v=v_name, g=g_name, w1=w1_name, w2=w2_name, w0=w0_name, u=u_name,
+                          norm=norm_name, o=o_name)
+        self.size = self.num_heads * self.dim
+        self.cols = -(-self.size // 16) * 16   # columns of a projection in their common result (padded)
+        self.x_off = ops.linear_state_floats(self.num_heads, self.dim, self.dim)       # the kept row in a slot
+        self.proj = self.o = self.proj_blocked = self.o_blocked = None
+        self.mu = self.w2 = self.w0 = self.bonus = self.norm_weight = None
+
+    def rank_from(self, prefix: str, shape_of) -> None:
+        """Take the rank from the shape of the checkpoint's W_w1 (``prefix``: of this mixer's tensors)."""
+        self.rank = int(shape_of(prefix + self.names["w1"])[0])
+
+    def cache_spec(self):
+        return StateSpec((-(-(self.x_off + self.hidden_size) // 4) * 4,), torch.float32)
+
+    def param_sources(self) -> List[ParamSource]:
+        n, W, C, R = self.names, self.hidden_size, self.size, self.rank
+        return [ParamSource(self.mu_prefix + m, (W,), "vector", init=("uniform", 0.0, 1.0)) for m in self.MIXES] + \
+               [ParamSource(n[x], (C, W)) for x in ("r", "k", "v", "g")] + \
+               [ParamSource(n["w1"], (R, W)), ParamSource(n["w2"], (C, R), "vector", init=("normal", 0.0, R ** -0.5)),
+                ParamSource(n["w0"], (C,), "vector", init=("uniform", -6.0, 0.5)),
+                ParamSource(n["u"], (self.num_heads, self.dim), "vector", init=("normal", 0.0, 0.5)),
+                ParamSource(n["norm"], (C,), "vector"), ParamSource(n["o"], (W, C))]
+
+    def load(self, tensors, dtype, device) -> None:
+        n = self.names
+        rows = [pad_rows(tensors[n[x]], 16) for x in ("r", "k", "v", "g", "w1")]
+        self.proj = place(torch.cat(rows, dim=0), "matrix", dtype, device)
+        self.o = place(tensors[n["o"]], "matrix", dtype, device)
+        self.mu = place(torch.stack([tensors[self.mu_prefix + m] for m in self.MIXES]), "vector", dtype, device)
+        for attr, key in (("w2", "w2"), ("w0", "w0"), ("bonus", "u"), ("norm_weight", "norm")):
+            setattr(self, attr, place(tensors[n[key]], "vector", dtype, device))
+
+    def make_decode_copies(self) -> int:
+        self.proj_blocked, self.o_blocked = decode_copy(self.proj), decode_copy(self.o)
+        return sum(t.numel() * t.element_size() for t in (self.proj_blocked, self.o_blocked)
+                   if t is not None)
+
+    def forward(self, x, ctx, cache):
+        x, state = as_tensor(x), cache.state
+        T, H, D, c = x.shape[0], self.num_heads, self.dim, self.cols
+        mixes = ops.time_shift(x, self.mu, state, self.x_off, ctx.q_start, ctx.state_slots)
+        p = ops.gemm_groups(mixes, self.proj, c, self.proj_blocked)
+        o = torch.empty((T, H, D), dtype=torch.float32, device=x.device)
+        keep = (x, self.x_off)              # (the recurrences' kernels leave the last rows in the slots)
+        n = ctx.num_decode_seqs
+        if n:
+            ops.linear_decode_bonus(o, p, 0, c, 2 * c, 4 * c, self.w2, self.w0, self.bonus, state, ctx.q_start[:n + 1],
+                                    ctx.state_slots[:n], D, keep)
+        if n < ctx.num_seqs:
+            decay = ops.lowrank_decay(p[:, 4 * c:], self.w2, self.w0, form=ops.DECAY_EXP)
+            ops.linear_scan(o, p, p[:, c:], p[:, 2 * c:], H, D, state, ctx.q_start[n:], ctx.state_slots[n:],
+                            max(ctx.q_lens[n:]), decay=decay, bonus=self.bonus, keep=keep)
+        out = torch.empty((T, H * D), dtype=x.dtype, device=x.device)
+        ops.head_norm_gate(out, o, 1, 0.0, self.norm_weight, True, 1.0, p, 3 * c, ops.GATE_SILU, self.eps)
+        return linear(out, self.o, out_dtype=torch.float32, blocked=self.o_blocked)

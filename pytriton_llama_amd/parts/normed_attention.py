@@ -9,7 +9,8 @@ import torch
 
 from .. import ops
 from .attention import ALL_16, PORTIONS_16, PORTIONS_64
-from .base import PagedSpec, PagedTensor, ParamSource, Part, PendingSum, as_tensor, place, register_part
+from .base import (PagedSpec, PagedTensor, ParamSource, Part, PendingSum, StateSpec, as_tensor, place,
+                   register_part)
 from .linear import LINEAR_LIBRARIES, decode_copy, linear
 from .rotary import banded_inv_freq, ramp_inv_freq
 
@@ -29,8 +30,10 @@ class NormedAttention(Part):
         v = W_v x + b_v [kv_heads, vdim]
         q, k <- RMS norm (``qk_norm`` "head": over the dim entries of every head and map, one weight
                 [dim] for all; "whole": over all of q and over all of k before they are split into
-                heads, weights of that size; None: no norm), then rotation of the first rot_dims
-                entries of every head (entry i with i + rot_dims / 2) by position * frequency
+                heads, weights of that size; None: no norm; "rotated": over every head behind the
+                rotation, without a weight), then rotation of the first rot_dims entries of every
+                head (entry i with i + rot_dims / 2; ``rot_layout`` "pairs", with qk_norm "rotated":
+                entry 2i with 2i + 1) by position * frequency
         a_m = softmax_j<=i (q_m(i) . k_m(j) * scale) v(j)         one result a map, same values
                 (``window``: over the keys with i - j < window only, the query's own and the
                 window - 1 before it; pages that every later query has left behind are given back.
@@ -40,8 +43,13 @@ class NormedAttention(Part):
                 without key and value that the scale does not touch; ``sink``: the same with one
                 fixed number for all heads. ``chunk``: over the keys of the query's own chunk, the
                 positions cut into chunks of so many from the sequence's start; pages of chunks that
-                are over are given back)
+                are over are given back. ``softcap``: a scaled score s becomes softcap * tanh(s / softcap)
+                first)
 
+    ``taps`` (with qk_norm "rotated"): behind their projections, biases included, q, k and v each pass a
+    causal convolution over time (``<name>.conv`` [channels, taps], the last tap is the current token's,
+    zeros in front of the sequence); the last taps - 1 projected values live in the request's state slot
+    in float32, and the mixer's cache layers are a pair (pages, state).
     maps = 1: out = W_o concat_h a + b_o.
     maps = 2 (differential attention: the second map is subtracted so that what both maps give
     to keys of no interest cancels): with lam = exp(lq1 . lk1) - exp(lq2 . lk2) + diff (one number
@@ -67,7 +75,8 @@ class NormedAttention(Part):
                  rot_dims: int = 0, rot_base: float = 10000.0, rot_scaling: Optional[dict] = None,
                  own_kv: bool = True, window: Optional[int] = None, keep_first: int = 0,
                  sink_name: Optional[str] = None, sink: Optional[float] = None, chunk: Optional[int] = None,
-                 head_gated: bool = False, o_bias: bool = True, q_name: str = "q", k_name: str = "k", v_name: str = "v",
+                 head_gated: bool = False, o_bias: bool = True, softcap: Optional[float] = None, taps: int = 0,
+                 rot_layout: str = "half", conv_suffix: str = ".conv", q_name: str = "q", k_name: str = "k", v_name: str = "v",
                  g_name: str = "g", o_name: str = "o", lambda_names=("lq1", "lk1", "lq2", "lk2")):
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} heads are not a multiple of {num_kv_heads} kv heads")
@@ -78,8 +87,21 @@ class NormedAttention(Part):
                              "are combined)")
         if head_gated and (maps != 1 or gated):
             raise ValueError("a gate a head is built for one map a head, and is the only gate")
-        if qk_norm not in (None, "head", "whole"):
-            raise ValueError(f"unknown query/key norm {qk_norm!r} (known: 'head', 'whole', None)")
+        if qk_norm not in (None, "head", "whole", "rotated"):
+            raise ValueError(f"unknown query/key norm {qk_norm!r} (known: 'head', 'whole', 'rotated', None)")
+        self.norm_rotated = qk_norm == "rotated"
+        if (taps or rot_layout != "half") and not self.norm_rotated:
+            raise ValueError("a convolution and pairs of neighbours are built for a norm behind the rotation")
+        if self.norm_rotated and (maps != 1 or not own_kv or rot_scaling):
+            raise ValueError("a norm behind the rotation is built for one map, keys and values of the layer's "
+                             "own and plain frequencies")
+        if rot_layout not in ("half", "pairs"):
+            raise ValueError(f"unknown layout of the rotating entries {rot_layout!r} (known: 'pairs', 'half')")
+        if taps < 0 or (softcap is not None and softcap <= 0):
+            raise ValueError("taps are not negative, and a softcap is positive")
+        self.taps, self.conv_suffix = int(taps), conv_suffix
+        self.rot_layout = ops.ROT_PAIRS if rot_layout == "pairs" else ops.ROT_HALF
+        self.softcap = float(softcap) if softcap else 0.0
         if rot_dims % 2 or not 0 <= rot_dims <= dim:
             raise ValueError(f"{rot_dims} rotating entries of {dim}: an even number, at most the head's size")
         if max(dim, vdim) > 640:
@@ -88,7 +110,8 @@ class NormedAttention(Part):
         self.dim, self.vdim, self.maps = int(dim), int(vdim), int(maps)
         self.scale = float(scale) if scale is not None else 1.0 / math.sqrt(dim)
         self.eps, self.diff = float(eps), float(diff)
-        self.norm_mode = {None: ops.NORM_NONE, "head": ops.NORM_HEAD, "whole": ops.NORM_WHOLE}[qk_norm]
+        self.norm_mode = {None: ops.NORM_NONE, "head": ops.NORM_HEAD, "whole": ops.NORM_WHOLE,
+                          "rotated": ops.NORM_NONE}[qk_norm]
         self.bias, self.gated, self.own_kv = bool(bias), bool(gated), bool(own_kv)
         self.head_gated, self.has_o_bias = bool(head_gated), bool(bias) and bool(o_bias)
         self.rot_dims = int(rot_dims)
@@ -130,12 +153,15 @@ class NormedAttention(Part):
         self.k_off = self.q_size if self.own_kv else -1
         self.v_off = self.q_size + self.k_size
         self.g_off = self.q_size + (self.k_size + self.v_size if self.own_kv else 0)
-        self.proj = self.o = self.proj_blocked = self.o_blocked = None
+        self.channels = self.q_size + self.k_size + self.v_size
+        self.proj = self.o = self.proj_blocked = self.o_blocked = self.conv_weight = self.qkv_bias = None
         self.q_bias = self.k_bias = self.v_bias = self.o_bias = None
         self.q_weight = self.k_weight = self.inv_freq = None
         self.lam = 0.0
         self.force_decode_splits = 0        # tests set it to try other splits
         libs = ("attention", "prepare", "stream") + LINEAR_LIBRARIES
+        if self.taps > 1:
+            libs += ("recurrent",)
         if self.dim % 32 == 0 and self.vdim % 32 == 0 and max(self.dim, self.vdim) <= 128:
             libs += ("attention_prefill",)          # the matrix-core kernel for prompt portions
         self.kernel_libraries = libs
@@ -177,7 +203,8 @@ class NormedAttention(Part):
         16-row blocks. ``gate``: float32 [T, >= heads], a factor sigmoid(gate) a row and head."""
         n_dec = ctx.num_decode_seqs if ops.attention_decode_kv_fits(self.dim, self.vdim) else 0
         window = self.window or 0
-        extras = dict(keep_first=self.keep_first, sink=self.sink, chunk=self.chunk or 0, gate=gate)
+        extras = dict(keep_first=self.keep_first, sink=self.sink, chunk=self.chunk or 0, gate=gate,
+                      softcap=self.softcap)
         # one map and keys as large as values: the matrix-core form of the split-KV kernel takes them
         mfma = (n_dec and self.maps == 1 and self.dim == self.vdim and q.stride(0) % 8 == 0
                 and ops.attention_decode_mfma_fits(q.dtype, self.num_heads, self.num_kv_heads, self.dim,
@@ -210,9 +237,12 @@ class NormedAttention(Part):
     def cache_spec(self):
         if not self.own_kv:
             return None
-        return PagedSpec((PagedTensor("k", (self.num_kv_heads * self.maps, self.dim), 1),
-                          PagedTensor("v", (self.num_kv_heads, self.vdim), 1)), self.window,
-                         self.keep_first, self.chunk)
+        pages = PagedSpec((PagedTensor("k", (self.num_kv_heads * self.maps, self.dim), 1),
+                           PagedTensor("v", (self.num_kv_heads, self.vdim), 1)), self.window,
+                          self.keep_first, self.chunk)
+        if self.taps <= 1:
+            return pages
+        return pages, StateSpec(((self.taps - 1) * self.channels,), torch.float32)
 
     def _norm_sizes(self):
         if self.norm_mode == ops.NORM_WHOLE:
@@ -231,6 +261,9 @@ class NormedAttention(Part):
             if self.bias:
                 out.append(ParamSource(n["k"] + ".b", (self.k_size,), "vector", init=small))
                 out.append(ParamSource(n["v"] + ".b", (self.v_size,), "vector", init=small))
+        if self.taps:
+            for x, size in (("q", self.q_size), ("k", self.k_size), ("v", self.v_size)):
+                out.append(ParamSource(n[x] + self.conv_suffix, (size, self.taps), "vector", init=("normal", 0.0, 0.5)))
         if self.norm_mode != ops.NORM_NONE:
             nq, nk = self._norm_sizes()
             out.append(ParamSource(n["q"] + ".norm", (nq,), "vector"))
@@ -269,6 +302,11 @@ class NormedAttention(Part):
             self.q_weight = place(tensors[n["q"] + ".norm"], "vector", dtype, device)
             if self.own_kv:
                 self.k_weight = place(tensors[n["k"] + ".norm"], "vector", dtype, device)
+        if self.taps:
+            self.conv_weight = place(torch.cat([tensors[n[x] + self.conv_suffix] for x in "qkv"], dim=0), "vector",
+                                     dtype, device)
+        if self.norm_rotated and self.bias:
+            self.qkv_bias = torch.cat([self.q_bias, self.k_bias, self.v_bias])
         if self.maps == 2:
             lq1, lk1, lq2, lk2 = (tensors[x].to(torch.float32).cpu() for x in self.lambda_names)
             self.lam = float(torch.exp((lq1 * lk1).sum()) - torch.exp((lq2 * lk2).sum())) + self.diff
@@ -284,20 +322,38 @@ class NormedAttention(Part):
         return sum(t.numel() * t.element_size() for t in (self.proj_blocked, self.o_blocked)
                    if t is not None)
 
+    def convolve(self, q, p, cache, tail, ctx, group) -> None:
+        """Bias, convolution, rotation, norm and cache write, and the slots' kept inputs."""
+        state = tail.state if tail is not None else None
+        n = ctx.num_decode_seqs
+        ops.conv_qkv_prepare(q, p, 0, self.k_off, self.v_off, self.qkv_bias, self.conv_weight, state, 0, ctx.q_start,
+                             ctx.state_slots, n, ctx.positions, group.slots if cache.writable else None, self.rot_dims,
+                             self.rot_layout, self.inv_freq, True, self.eps, cache.k, cache.v, self.num_heads,
+                             self.num_kv_heads, self.num_kv_heads, self.dim, self.vdim, cache.page_size)
+        if state is not None and n < ctx.num_seqs:
+            ops.conv_tail_update(p, 0, self.channels, self.taps, state, 0, ctx.q_start[n:], ctx.state_slots[n:],
+                                 self.qkv_bias)
+
     def heads_output(self, x, ctx, cache) -> torch.Tensor:
         """The concatenated heads [T, heads * vdim] in the engine's dtype: what the output
         projection reads."""
         x = as_tensor(x)
         T = x.shape[0]
         H, G, M, Dk, Dv = self.num_heads, self.num_kv_heads, self.maps, self.dim, self.vdim
+        tail = None
+        if self.taps > 1:
+            cache, tail = cache
         group = ctx.groups[cache.group]
         p = linear(x, self.proj, out_dtype=torch.float32, blocked=self.proj_blocked)
         q = torch.empty((T, H * M, Dk), dtype=x.dtype, device=x.device)
-        ops.qkv_prepare(q, p, 0, self.k_off, self.v_off, self.q_bias, self.k_bias, self.v_bias,
-                        self.norm_mode, self.q_weight, self.k_weight, self.eps, self.rot_dims,
-                        self.inv_freq, self.mag, ctx.positions,
-                        group.slots if (cache.writable and self.own_kv) else None, cache.k, cache.v,
-                        H * M, G * M, G, Dk, Dv, cache.page_size)
+        if self.norm_rotated:
+            self.convolve(q, p, cache, tail, ctx, group)
+        else:
+            ops.qkv_prepare(q, p, 0, self.k_off, self.v_off, self.q_bias, self.k_bias, self.v_bias,
+                            self.norm_mode, self.q_weight, self.k_weight, self.eps, self.rot_dims,
+                            self.inv_freq, self.mag, ctx.positions,
+                            group.slots if (cache.writable and self.own_kv) else None, cache.k, cache.v,
+                            H * M, G * M, G, Dk, Dv, cache.page_size)
         plain = M == 1
         a = torch.empty((T, H * M, Dv), dtype=x.dtype if plain else torch.float32, device=x.device)
         self.attend(a, q, cache, ctx, group, p[:, self.g_off:] if self.head_gated else None)
