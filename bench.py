@@ -381,6 +381,34 @@ BIMOPEL_SIZES = {
 }
 
 
+def fogapel_shape(width, layers, heads, kv_heads, dim, chunk, wkv_heads, wkv_dim, rank, dense_ff, experts, top,
+                  expert_ff, shared_ff, vocab):
+    """A Fogapel config.json of a real model's layer sizes: two time mixers and one attention layer in turn,
+    the first layer with a dense feed-forward, the others routed beside a shared expert."""
+    attn = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** 0.5 / 4, "conv": 4,
+            "softcap": 30.0, "mask": {"size": chunk}, "rot": {"base": 500000.0, "dims": dim}}
+    wkv = {"heads": wkv_heads, "dim": wkv_dim, "rank": rank}
+    moe = {"kind": "moe", "expert": {"ff": expert_ff}, "router": {"experts": experts, "top": top},
+           "shared": {"ff": shared_ff}}
+    out = [{"type": "attention" if i % 3 == 2 else "wkv", "mixer": attn if i % 3 == 2 else wkv,
+            "mlp": {"kind": "dense", "ff": dense_ff, "limit": 7.0} if i == 0 else moe} for i in range(layers)]
+    return {"architecture": "Fogapel", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+            "embedding": {"scale": 1.0}, "layers": out, "initializer_range": 0.02}
+
+
+# name -> (Fogapel sizes, the Llama shape of equal width, depth, heads and feed-forward width a token)
+FOGAPEL_SIZES = {
+    "2048": (dict(width=2048, layers=8, heads=16, kv_heads=4, dim=128, chunk=1024, wkv_heads=32, wkv_dim=64, rank=64,
+                  dense_ff=8192, experts=16, top=2, expert_ff=2048, shared_ff=4096, vocab=32000),
+             dict(num_hidden_layers=8, hidden_size=2048, num_attention_heads=16, num_key_value_heads=4,
+                  head_dim=128, intermediate_size=8192, vocab_size=32000, tie_word_embeddings=False)),
+    "4096": (dict(width=4096, layers=4, heads=32, kv_heads=8, dim=128, chunk=2048, wkv_heads=64, wkv_dim=64, rank=64,
+                  dense_ff=14336, experts=32, top=4, expert_ff=2048, shared_ff=6144, vocab=32000),
+             dict(num_hidden_layers=4, hidden_size=4096, num_attention_heads=32, num_key_value_heads=8,
+                  head_dim=128, intermediate_size=14336, vocab_size=32000, tie_word_embeddings=False)),
+}
+
+
 def engine_rates(cfg, dtype, S, batch, steps, warmup):
     """Prefill of one S-token prompt (one step) and decode steps of ``batch`` requests behind
     S-token prompts, through the whole engine, for any architecture."""
@@ -494,6 +522,15 @@ def bimopel_beside_llama(args):
                         others=(("virusun", VIRUSUN_SIZES, virusun_shape), ("matusun", MATUSUN_SIZES, matusun_shape)))
 
 
+def fogapel_beside_llama(args):
+    """Fogapel beside Llama and, with 'bimopel', 'senavik' or 'matusun' among --fogapel-models, beside the
+    designs whose layers are closest to its own (linear recurrences and attention inside chunks; routed
+    experts and a float32 stream)."""
+    return beside_llama(args, "fogapel", args.fogapel, args.fogapel_models, FOGAPEL_SIZES, fogapel_shape,
+                        others=(("bimopel", BIMOPEL_SIZES, bimopel_shape), ("senavik", SENAVIK_SIZES, senavik_shape),
+                                ("matusun", MATUSUN_SIZES, matusun_shape)))
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -547,6 +584,11 @@ def main():
     ap.add_argument("--bimopel-models", default="bimopel,llama",
                     help="with --bimopel: which models to run, of bimopel, llama, virusun and matusun (the designs "
                          "with the closest layers, at the same named size)")
+    ap.add_argument("--fogapel", default="", metavar="SIZES",
+                    help="the same for the Fogapel design (sizes of: 2048, 4096)")
+    ap.add_argument("--fogapel-models", default="fogapel,llama",
+                    help="with --fogapel: which models to run, of fogapel, llama, bimopel, senavik and matusun (the "
+                         "designs with the closest layers, at the same named size)")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py measures one GPU: this engine has no multi-GPU path, --gpus {args.gpus} is not run")
@@ -581,6 +623,8 @@ def main():
         return senavik_beside_llama(args)
     if args.bimopel:
         return bimopel_beside_llama(args)
+    if args.fogapel:
+        return fogapel_beside_llama(args)
     if args.mixed:
         return mixed_workload(args, cfg, short)
     if args.like_reference:

@@ -779,7 +779,7 @@ static int launch_decode(const DecodeArgs& A, int n_seqs, hipStream_t st) {
   {                                                                                 \
     if (nb == 4) linear_decode_kernel<J, 4, MODE><<<grid, 256, lds, st>>>(A);       \
     else if (nb == 2) linear_decode_kernel<J, 2, MODE><<<grid, 256, lds, st>>>(A);  \
-    else linear_decode_kernel<J, 1, MODE><<<grid, 256, 0, st>>>(A);                 \
+    else linear_decode_kernel<J, 1, MODE><<<grid, 256, lds, st>>>(A);                \
     return ptl_launch_status();                                                     \
   }
   switch ((A.DS + 63) / 64) {

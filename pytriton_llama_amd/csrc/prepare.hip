@@ -28,8 +28,8 @@
 //   sequences of one token it also advances the inputs that a short convolution keeps in the state
 //   slot (the recurrence in front of it has read the old ones).
 //
-// All arithmetic is float32: the angle is float(position) * frequency, sinf / cosf / expf are the
-// accurate ones.
+// All arithmetic is float32: the angle is float(position) * frequency (behind a convolution with the
+// product's rounding put back), sinf / cosf / expf are the accurate ones.
 #include "common.h"
 #include <math.h>
 
@@ -182,6 +182,17 @@ extern "C" int ptl_qkv_prepare(void* q_out, const float* p, long ldp, int q_off,
 // number of taps, read again for every row). The first n_single sequences bring one row each: their
 // lanes also advance the kept inputs they have just read (those of longer portions are advanced
 // behind this kernel, when no wave reads them any more).
+
+// Sine and cosine of pos * f, with what the product's rounding loses put back: at position 1,000 the
+// rounded angle of a fast entry is off by some 1e-5, and by another amount for a query than for its keys.
+__device__ __forceinline__ void turn_of(float pos, float f, float& sn, float& cs) {
+  const float a = pos * f, rest = fmaf(pos, f, -a);
+  float s, c;
+  sincosf(a, &s, &c);
+  sn = fmaf(rest, c, s);
+  cs = fmaf(-rest, s, c);
+}
+
 #define PAIRS_NEIGHBOURS 0
 #define PAIRS_HALF 1
 
@@ -299,7 +310,7 @@ conv_qkv_prepare_kernel(TO* __restrict__ q_out, TO* __restrict__ k_cache, TO* __
         for (int n = 0; n < NP; ++n) {
           if (2 * (lane + 64 * n) >= rot) continue;
           float sn, cs;
-          sincosf(pos * f[n], &sn, &cs);
+          turn_of(pos, f[n], sn, cs);
           const float u = y[n][0], v = y[n][1];
           y[n][0] = u * cs - v * sn;
           y[n][1] = v * cs + u * sn;
