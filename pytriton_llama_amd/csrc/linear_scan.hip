@@ -73,9 +73,16 @@ __device__ __forceinline__ float sigmoid_power(float z, float p) {
   return __builtin_amdgcn_exp2f(-p * l);
 }
 
-__device__ __forceinline__ float decay_in(int form, float r) { return form == DECAY_EXP ? tanhf(r) : r; }
+// The hardware's exponential in base 2 and reciprocal: tanh to a few 1e-7 (it enters a sum of R such terms),
+// e^z to a few 1e-7 of itself, which is what the decay's logarithm is known to.
+__device__ __forceinline__ float decay_in(int form, float r) {
+  return form == DECAY_EXP
+             ? fmaf(-2.0f, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(2.885390081777927f * r)), 1.0f)
+             : r;
+}
 __device__ __forceinline__ float decay_of(int form, float z, float inv_tau) {
-  return form == DECAY_EXP ? expf(-expf(z)) : sigmoid_power(z, inv_tau);
+  const float log2e = 1.4426950408889634f;
+  return form == DECAY_EXP ? __builtin_amdgcn_exp2f(-log2e * __builtin_amdgcn_exp2f(log2e * z)) : sigmoid_power(z, inv_tau);
 }
 
 // The last row of x that a sequence brings, kept as float32 [W] at ``off`` of its state slot (x null:
@@ -588,63 +595,111 @@ extern "C" int ptl_linear_scan(int mode, float* out, const float* q, long ldq, c
 }
 
 // ---- the low-rank decays of all rows ---------------------------------------------------------------
-// grid (blocks of 256 channels, blocks of DECAY_ROWS rows): a thread keeps its channel's row of W2 in
-// registers (up to 64 entries; a longer one is read again for every row), the rows of r go through LDS,
-// four entries a read
-#define DECAY_ROWS 8
-template <int RM>
+// grid (blocks of 64 channels, blocks of 64 rows), a wave 16 of the channels: z^T = W2 f(r)^T as
+// v_mfma_f32_16x16x4_f32. A lane holds its channel's entries 16 k + 4 lg .. + 3 of W2 as one float4 a
+// chunk of 16 (in the same order as those of r, which is all a sum needs), f(r) lies in LDS.
+template <int RC>
 __global__ void __launch_bounds__(256)
 lowrank_decay_kernel(float* __restrict__ out, const float* __restrict__ r, long ldr, const float* __restrict__ w,
-                     const float* __restrict__ b, int form, float inv_tau, int T, int C, int R, int RP) {
-  extern __shared__ __attribute__((aligned(16))) float rs[];       // [DECAY_ROWS][RP], zeros from R on
+                     const float* __restrict__ b, int form, float inv_tau, int T, int C, int R) {
+  constexpr int RP = 16 * RC, LD = RP + 4;
+  __shared__ __attribute__((aligned(16))) float rs[64 * LD];
+  const int tid = threadIdx.x, lane = tid & 63, ln = lane & 15, lg = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int t0 = blockIdx.y * 64, rows = min(64, T - t0), c0 = blockIdx.x * 64 + 16 * wave;
+  f32x4_t wf[RC];
+  const float* wr = w + (size_t)min(c0 + ln, C - 1) * R;
+#pragma unroll
+  for (int k = 0; k < RC; ++k)
+#pragma unroll
+    for (int m = 0; m < 4; ++m) wf[k][m] = 16 * k + 4 * lg + m < R ? wr[16 * k + 4 * lg + m] : 0.f;
+  for (int i = tid; i < 64 * RP; i += 256) {
+    const int t = i / RP, j = i - t * RP;
+    rs[t * LD + j] = t < rows && j < R ? decay_in(form, r[(size_t)(t0 + t) * ldr + j]) : 0.f;
+  }
+  f32x4_t bias;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) bias[i] = b[min(c0 + 4 * lg + i, C - 1)];
+  __syncthreads();
+  const bool four = C % 4 == 0 && ((uintptr_t)out & 15) == 0;
+  for (int tt = 0; tt < rows; tt += 16) {
+    f32x4_t z = bias;
+#pragma unroll
+    for (int k = 0; k < RC; ++k) {
+      const f32x4_t x = *reinterpret_cast<const f32x4_t*>(rs + (tt + ln) * LD + 16 * k + 4 * lg);
+#pragma unroll
+      for (int m = 0; m < 4; ++m) z = __builtin_amdgcn_mfma_f32_16x16x4f32(wf[k][m], x[m], z, 0, 0, 0);
+    }
+    // lane (ln, lg): channels c0 + 4 lg .. + 3 of row tt + ln
+    if (tt + ln >= rows) continue;
+    float* o = out + (size_t)(t0 + tt + ln) * C + c0 + 4 * lg;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) z[i] = decay_of(form, z[i], inv_tau);
+    if (four) {
+      if (c0 + 4 * lg < C) *reinterpret_cast<f32x4_t*>(o) = z;
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (c0 + 4 * lg + i < C) o[i] = z[i];
+    }
+  }
+}
+
+// ranks above 128: a thread a channel, its row of W2 read again for every row
+#define DECAY_ROWS 8
+__global__ void __launch_bounds__(256)
+lowrank_decay_wide_kernel(float* __restrict__ out, const float* __restrict__ r, long ldr, const float* __restrict__ w,
+                          const float* __restrict__ b, int form, float inv_tau, int T, int C, int R) {
+  extern __shared__ __attribute__((aligned(16))) float rw[];       // [DECAY_ROWS][R]
   const int t0 = blockIdx.y * DECAY_ROWS, rows = min(DECAY_ROWS, T - t0);
   const int c = blockIdx.x * 256 + threadIdx.x;
-  const float* wr = w + (size_t)min(c, C - 1) * R;
-  float wv[RM > 0 ? RM : 4];
-  if (RM > 0) {
-#pragma unroll
-    for (int j = 0; j < RM; ++j) wv[j] = j < R ? wr[j] : 0.f;
-  }
-  const float bias = b[min(c, C - 1)];
-  for (int i = threadIdx.x; i < rows * RP; i += 256) {
-    const int t = i / RP, j = i - t * RP;
-    rs[i] = j < R ? decay_in(form, r[(size_t)(t0 + t) * ldr + j]) : 0.f;
-  }
+  for (int i = threadIdx.x; i < rows * R; i += 256) rw[i] = decay_in(form, r[(size_t)(t0 + i / R) * ldr + i % R]);
   __syncthreads();
   if (c >= C) return;
-  for (int t = 0; t < rows; ++t) {
-    const float* rr = rs + t * RP;
-    float z = bias;
-    if (RM > 0) {
+  const float* wr = w + (size_t)c * R;
+  float z[DECAY_ROWS];
 #pragma unroll
-      for (int j = 0; j < RM; j += 4) {
-        if (j >= RP) continue;
-        const f32x4_t x = *reinterpret_cast<const f32x4_t*>(rr + j);
+  for (int t = 0; t < DECAY_ROWS; ++t) z[t] = b[c];
+  for (int j = 0; j < R; ++j) {
+    const float x = wr[j];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) z = fmaf(wv[j + i], x[i], z);
-      }
-    } else {
-      for (int j = 0; j < R; ++j) z = fmaf(wr[j], rr[j], z);
-    }
-    out[(size_t)(t0 + t) * C + c] = decay_of(form, z, inv_tau);
+    for (int t = 0; t < DECAY_ROWS; ++t) z[t] = fmaf(x, t < rows ? rw[t * R + j] : 0.f, z[t]);
   }
+#pragma unroll
+  for (int t = 0; t < DECAY_ROWS; ++t)
+    if (t < rows) out[(size_t)(t0 + t) * C + c] = decay_of(form, z[t], inv_tau);
 }
 
 extern "C" int ptl_lowrank_decay(float* out, const float* r, long ldr, const float* w, const float* b,
                                  int form, float inv_tau, int T_, int C, int R, hipStream_t st) {
   if (T_ <= 0) return PTL_OK;
-  const int RP = (R + 3) / 4 * 4;
-  const size_t lds = (size_t)DECAY_ROWS * RP * sizeof(float);
-  if (C <= 0 || R <= 0 || lds > 48 * 1024 || (form != DECAY_SIGMOID && form != DECAY_EXP) || (T_ + DECAY_ROWS - 1) / DECAY_ROWS > 65535) return PTL_ERR_ARG;
-  const dim3 grid((C + 255) / 256, (T_ + DECAY_ROWS - 1) / DECAY_ROWS);
-  if (R <= 16) lowrank_decay_kernel<16><<<grid, 256, lds, st>>>(out, r, ldr, w, b, form, inv_tau, T_, C, R, RP);
-  else if (R <= 32) lowrank_decay_kernel<32><<<grid, 256, lds, st>>>(out, r, ldr, w, b, form, inv_tau, T_, C, R, RP);
-  else if (R <= 64) lowrank_decay_kernel<64><<<grid, 256, lds, st>>>(out, r, ldr, w, b, form, inv_tau, T_, C, R, RP);
-  else lowrank_decay_kernel<0><<<grid, 256, lds, st>>>(out, r, ldr, w, b, form, inv_tau, T_, C, R, RP);
+  const size_t lds = (size_t)DECAY_ROWS * R * sizeof(float);
+  if (C <= 0 || R <= 0 || lds > 48 * 1024 || (form != DECAY_SIGMOID && form != DECAY_EXP) ||
+      (T_ + DECAY_ROWS - 1) / DECAY_ROWS > 65535)
+    return PTL_ERR_ARG;
+  const dim3 grid((C + 63) / 64, (T_ + 63) / 64);
+#define GO(RC) lowrank_decay_kernel<RC><<<grid, 256, 0, st>>>(out, r, ldr, w, b, form, inv_tau, T_, C, R)
+  if (R <= 16) GO(1);
+  else if (R <= 32) GO(2);
+  else if (R <= 64) GO(4);
+  else if (R <= 128) GO(8);
+  else
+    lowrank_decay_wide_kernel<<<dim3((C + 255) / 256, (T_ + DECAY_ROWS - 1) / DECAY_ROWS), 256, lds, st>>>(
+        out, r, ldr, w, b, form, inv_tau, T_, C, R);
+#undef GO
   return ptl_launch_status();
 }
 
 // ---- one token -------------------------------------------------------------------------------------
+// What follows the recurrence head by head: y = o / sqrt(mean(o^2) + eps) * w * silu(gate), [T, H * Dv] in
+// the engine's type (y null: the kernel leaves o). One workgroup has the whole head then.
+struct HeadArgs {
+  void* y; int dtype;
+  const float* w;                           // [H, Dv]
+  int gate_off;                             // column of p
+  float eps;
+};
+
 struct DecodeArgs {
   float* out;                               // [T, H, Dv]
   const float* p; long ldp;                 // the float32 projection
@@ -664,6 +719,7 @@ struct DecodeArgs {
   int H, heads_per_qk, D, DS, Dv;
   const float* bonus;                       // bonus form: [H, D]
   ShiftArgs shift;
+  HeadArgs head;
 };
 
 // NB: blocks of 16 columns a workgroup takes (what is in front of the recurrence is then done less often)
@@ -739,6 +795,7 @@ __global__ void __launch_bounds__(256) linear_decode_kernel(DecodeArgs A) {
   }
   __syncthreads();
   const float skip = MODE == MODE_SCALAR ? A.skip[h] : 0.f;
+  __shared__ float os[BONUS ? 16 * NB : 1];
 #pragma unroll
   for (int b = 0; b < NB; ++b) {
     const bool live = c0 + 16 * b + cg < Dv;
@@ -758,7 +815,24 @@ __global__ void __launch_bounds__(256) linear_decode_kernel(DecodeArgs A) {
       if (live && d < DS) __builtin_nontemporal_store(s, reinterpret_cast<f32x4_t*>(column(b) + d));
     }
     o = row16_sum(o);
-    if (live && l == 0) A.out[((size_t)row * A.H + h) * Dv + c0 + 16 * b + cg] = fmaf(skip, x, o);
+    if (BONUS && A.head.y) {
+      if (l == 0) os[16 * b + cg] = live ? o : 0.f;
+    } else if (live && l == 0) {
+      A.out[((size_t)row * A.H + h) * Dv + c0 + 16 * b + cg] = fmaf(skip, x, o);
+    }
+  }
+  if (BONUS && A.head.y) {
+    __syncthreads();
+    if (tid < 64) {                         // (Dv <= 16 NB <= 64: a lane a value)
+      const float o = tid < 16 * NB ? os[tid] : 0.f;
+      const float r = 1.0f / sqrtf(wave_sum(o * o) / (float)Dv + A.head.eps);
+      if (tid < Dv) {
+        const float y = o * r * A.head.w[h * Dv + tid] * silu_f(p[A.head.gate_off + h * Dv + tid]);
+        const size_t at = ((size_t)row * A.H + h) * Dv + tid;
+        if (A.head.dtype == PTL_DTYPE_F32) ((float*)A.head.y)[at] = y;
+        else ((bf16_t*)A.head.y)[at] = float_to_bf16(y);
+      }
+    }
   }
   if (A.shift.x) keep_row(A.shift, slot, (size_t)row, blockIdx.y * gridDim.x + blockIdx.x, gridDim.x * gridDim.y);
 }
@@ -773,7 +847,11 @@ static int launch_decode(const DecodeArgs& A, int n_seqs, hipStream_t st) {
   // as many columns a workgroup as leave about two workgroups a compute unit (of 256)
   const int blocks = (A.Dv + 15) / 16;
   const long all = (long)blocks * A.H * n_seqs;
-  const int nb = blocks >= 4 && all >= 4 * 512 ? 4 : (blocks >= 2 && all >= 2 * 512 ? 2 : 1);
+  int nb = blocks >= 4 && all >= 4 * 512 ? 4 : (blocks >= 2 && all >= 2 * 512 ? 2 : 1);
+  if (A.head.y) {                           // the heads are finished here: whole heads
+    if (blocks > 4) return PTL_ERR_ARG;
+    nb = blocks > 2 ? 4 : blocks;
+  }
   const dim3 grid((blocks + nb - 1) / nb, A.H, n_seqs);
 #define GO(J)                                                                       \
   {                                                                                 \
@@ -838,18 +916,21 @@ extern "C" int ptl_linear_decode_lowrank(float* out, const float* p, long ldp, i
 }
 
 // The bonus form: as above with decays exp(-exp(w2 . tanh(r) + b2)), bonus [H, D]; the sequences' rows of
-// shift_x [T, ldx] are left in their slots (ShiftArgs).
-extern "C" int ptl_linear_decode_bonus(float* out, const float* p, long ldp, int q_off, int k_off, int v_off,
+// shift_x [T, ldx] are left in their slots (ShiftArgs). y (or null; Dv up to 64): the heads are normed, weighted
+// and gated (HeadArgs) into y, and out is not written.
+extern "C" int ptl_linear_decode_bonus(float* out, void* y, int y_dtype, const float* head_w, int gate_off, float eps,
+                                       const float* p, long ldp, int q_off, int k_off, int v_off,
                                        int a_off, const float* w2, const float* b2, int R, const float* bonus,
                                        const void* shift_x, long shift_ldx, int shift_dtype, long shift_off,
                                        int shift_W, float* state, long slot_stride, const int32_t* q_start,
                                        const int32_t* state_slots, int n_seqs, int H, int D, int Dv, hipStream_t st) {
   if (n_seqs <= 0) return PTL_OK;
-  if (R <= 0 || !w2 || !b2 || !bonus) return PTL_ERR_ARG;
+  if (R <= 0 || !w2 || !b2 || !bonus || (y && (!head_w || gate_off < 0)) || (!y && !out)) return PTL_ERR_ARG;
   DecodeArgs A = lowrank_args(out, p, ldp, q_off, k_off, v_off, a_off, 1.f, w2, b2, R, DECAY_EXP, 0.f, state,
                               slot_stride, q_start, state_slots, H, D, Dv);
   A.bonus = bonus;
   A.shift = ShiftArgs{shift_x, shift_ldx, shift_dtype, shift_off, shift_W};
+  A.head = HeadArgs{y, y_dtype, head_w, gate_off, eps};
   return launch_decode<MODE_BONUS>(A, n_seqs, st);
 }
 

@@ -13,6 +13,7 @@
 //                     logit columns behind the experts' (a gate of a shared expert)
 //   ptl_moe_sort      the (token, choice) pairs ordered by expert: positions, the tiles of
 //                     MOE_TM rows that the products walk, all by one workgroup
+//   ptl_moe_route_few the two above in one kernel, for the few rows of a decode step
 //   ptl_moe_gate_up   per tile: rows gathered from x, the expert's gate and up matrices, and
 //                     the gated activation, written in sorted order. The routing weight scales
 //                     the expert's input (it is applied to both products, which are linear) or
@@ -55,17 +56,28 @@ __device__ __forceinline__ float unary_act(int kind, float u) {
 #define TOPK_MAX_PER_LANE 16
 #define SCORE_SIGMOID 0
 #define SCORE_SOFTMAX 1
+struct RouteArgs {
+  const float* logits; int ld;
+  const float* logit_bias;
+  int T, E, top, extra, renormalize, score_fn;
+  const float* bias;
+  int real;
+  float renorm_eps, wscale;
+  int n_groups, keep_groups;
+  int32_t* idx; float* wgt; float* extra_out; float* ident_out;
+};
+
+// One wave routes token t; cs: [64 * TOPK_PER_LANE] floats of LDS of the wave (groups only).
 template <int TOPK_PER_LANE>
-__global__ void __launch_bounds__(256)
-moe_topk_kernel(const float* __restrict__ logits, int ld, const float* __restrict__ logit_bias, int T_, int E,
-                int top, int extra, int renormalize, int score_fn, const float* __restrict__ bias, int real, float renorm_eps,
-                float wscale, int n_groups, int keep_groups, int32_t* __restrict__ idx,
-                float* __restrict__ wgt, float* __restrict__ extra_out, float* __restrict__ ident_out) {
-  __shared__ float choice[4][64 * TOPK_PER_LANE];      // a token's choice scores (groups only)
-  const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
+__device__ __forceinline__ void route_token(const RouteArgs& A, int t, float* cs) {
   const int lane = threadIdx.x & 63;
-  if (t >= T_) return;
-  const float* z = logits + (size_t)t * ld;
+  const int E = A.E, top = A.top, extra = A.extra, renormalize = A.renormalize, score_fn = A.score_fn, real = A.real;
+  const int n_groups = A.n_groups, keep_groups = A.keep_groups;
+  const float *logit_bias = A.logit_bias, *bias = A.bias;
+  const float renorm_eps = A.renorm_eps, wscale = A.wscale;
+  int32_t* idx = A.idx;
+  float *wgt = A.wgt, *extra_out = A.extra_out, *ident_out = A.ident_out;
+  const float* z = A.logits + (size_t)t * A.ld;
   // v: what the choice goes by; sc: the score that becomes the weight. Scores without a correction
   // are chosen by their logits (the same order, and no ties where the sigmoid saturates or the
   // softmax vanishes).
@@ -103,7 +115,6 @@ moe_topk_kernel(const float* __restrict__ logits, int ld, const float* __restric
     // Groups of E / n_groups neighbours; lane g scores group g by its two largest choice scores
     // (a group of one: by its only one); the best keep_groups groups stay (ties: the lower
     // group), the choice scores of all others become minus infinity.
-    float* cs = choice[threadIdx.x >> 6];
 #pragma unroll
     for (int i = 0; i < TOPK_PER_LANE; ++i)
       if (lane + 64 * i < E) cs[lane + 64 * i] = v[i];
@@ -197,6 +208,23 @@ moe_topk_kernel(const float* __restrict__ logits, int ld, const float* __restric
   if (lane < extra) extra_out[(size_t)t * extra + lane] = sigmoidf_(z[E + lane]);
 }
 
+template <int TOPK_PER_LANE>
+__global__ void __launch_bounds__(256) moe_topk_kernel(RouteArgs A) {
+  __shared__ float choice[4][64 * TOPK_PER_LANE];      // a token's choice scores (groups only)
+  const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (t < A.T) route_token<TOPK_PER_LANE>(A, t, choice[threadIdx.x >> 6]);
+}
+
+static bool route_ok(int ld, int E, int top, int extra, const float* extra_out, int real, const float* ident_out,
+                     int score_fn, int n_groups, int keep_groups) {
+  if (n_groups > 1 && (n_groups > 64 || E % n_groups || keep_groups < 1 || keep_groups > n_groups ||
+                       (long)keep_groups * (E / n_groups) < top))
+    return false;
+  return E > 0 && top > 0 && top <= E && E <= 64 * TOPK_MAX_PER_LANE && extra >= 0 && extra <= 64 && ld >= E + extra &&
+         (!extra || extra_out) && real >= 0 && real <= E && (real >= E || ident_out) &&
+         (score_fn == SCORE_SIGMOID || score_fn == SCORE_SOFTMAX);
+}
+
 // logits [T, ld]: E router outputs a row, then ``extra`` columns. logit_bias [E] or null: added to the
 // outputs before anything else. score_fn: 0 sigmoid, 1 softmax over
 // the E outputs. bias [E] or null: added to the scores for the choice only. real: the first ``real``
@@ -209,17 +237,11 @@ extern "C" int ptl_moe_topk(const float* logits, int ld, const float* logit_bias
                             int n_groups, int keep_groups, int32_t* idx, float* wgt, float* extra_out,
                             float* ident_out, hipStream_t st) {
   if (T_ <= 0) return PTL_OK;
-  if (n_groups > 1 && (n_groups > 64 || E % n_groups || keep_groups < 1 || keep_groups > n_groups ||
-                       (long)keep_groups * (E / n_groups) < top))
-    return PTL_ERR_ARG;
-  if (E <= 0 || top <= 0 || top > E || E > 64 * TOPK_MAX_PER_LANE || extra < 0 || extra > 64 || ld < E + extra ||
-      (extra && !extra_out) || real < 0 || real > E || (real < E && !ident_out) ||
-      (score_fn != SCORE_SIGMOID && score_fn != SCORE_SOFTMAX))
-    return PTL_ERR_ARG;
-#define GO(PER)                                                                                              \
-  moe_topk_kernel<PER><<<(T_ + 3) / 4, 256, 0, st>>>(logits, ld, logit_bias, T_, E, top, extra, renormalize, score_fn, bias, \
-                                                     real, renorm_eps, wscale, n_groups, keep_groups, idx, wgt,  \
-                                                     extra_out, ident_out)
+  if (!route_ok(ld, E, top, extra, extra_out, real, ident_out, score_fn, n_groups, keep_groups)) return PTL_ERR_ARG;
+  const RouteArgs A{logits, ld, logit_bias, T_, E, top, extra, renormalize, score_fn, bias, real, renorm_eps, wscale,
+                    n_groups, keep_groups, idx, wgt, extra_out, ident_out};
+#define GO(PER) \
+  moe_topk_kernel<PER><<<(T_ + 3) / 4, 256, 0, st>>>(A)
   if (E <= 64) GO(1);
   else if (E <= 256) GO(4);
   else GO(16);
@@ -231,11 +253,19 @@ extern "C" int ptl_moe_topk(const float* logits, int ld, const float* logit_bias
 // for a pair whose expert is outside 0..E-1 and takes no part in the products),
 // sorted[p] (the pair at position p), expert_end[e] (one past the last position of expert e),
 // and the tile list: tile_expert[i] (-1: no tile), tile_row0[i] for i < max_tiles.
-__global__ void __launch_bounds__(1024)
-moe_sort_kernel(const int32_t* __restrict__ idx, int A, int E, int32_t* __restrict__ pos_of,
-                int32_t* __restrict__ sorted, int32_t* __restrict__ expert_end,
-                int32_t* __restrict__ tile_expert, int32_t* __restrict__ tile_row0, int max_tiles) {
-  extern __shared__ int32_t sh[];        // count [E], start [E], n_tiles [1]
+struct SortArgs {
+  const int32_t* idx;
+  int A, E;
+  int32_t *pos_of, *sorted, *expert_end, *tile_expert, *tile_row0;
+  int max_tiles;
+};
+
+// sh: count [E], start [E], n_tiles [1]
+__device__ __forceinline__ void sort_pairs(const SortArgs& S, int32_t* sh) {
+  const int32_t* idx = S.idx;
+  const int A = S.A, E = S.E, max_tiles = S.max_tiles;
+  int32_t *pos_of = S.pos_of, *sorted = S.sorted, *expert_end = S.expert_end, *tile_expert = S.tile_expert,
+          *tile_row0 = S.tile_row0;
   int32_t* count = sh;
   int32_t* start = sh + E;
   int32_t* n_tiles = sh + 2 * E;
@@ -280,6 +310,22 @@ moe_sort_kernel(const int32_t* __restrict__ idx, int A, int E, int32_t* __restri
   }
 }
 
+__global__ void __launch_bounds__(1024) moe_sort_kernel(SortArgs S) {
+  extern __shared__ int32_t sh[];
+  sort_pairs(S, sh);
+}
+
+// The few rows of a decode step: both in one workgroup, a wave a token in turn.
+template <int TOPK_PER_LANE>
+__global__ void __launch_bounds__(1024) moe_route_few_kernel(RouteArgs A, SortArgs S) {
+  extern __shared__ int32_t sh[];
+  __shared__ float choice[16][64 * TOPK_PER_LANE];
+  const int wave = threadIdx.x >> 6;
+  for (int t = wave; t < A.T; t += 16) route_token<TOPK_PER_LANE>(A, t, choice[wave]);
+  __syncthreads();                       // (the choices, written to memory, are visible to the workgroup)
+  sort_pairs(S, sh);
+}
+
 extern "C" int ptl_moe_max_tiles(int A, int E) { return (A + MOE_TM - 1) / MOE_TM + (A < E ? A : E); }
 
 extern "C" int ptl_moe_sort(const int32_t* idx, int A, int E, int32_t* pos_of, int32_t* sorted,
@@ -287,8 +333,28 @@ extern "C" int ptl_moe_sort(const int32_t* idx, int A, int E, int32_t* pos_of, i
                             hipStream_t st) {
   if (A <= 0) return PTL_OK;
   if (E <= 0 || E > 8192 || max_tiles < ptl_moe_max_tiles(A, E)) return PTL_ERR_ARG;
-  moe_sort_kernel<<<1, 1024, (2 * E + 1) * sizeof(int32_t), st>>>(idx, A, E, pos_of, sorted, expert_end,
-                                                                  tile_expert, tile_row0, max_tiles);
+  moe_sort_kernel<<<1, 1024, (2 * E + 1) * sizeof(int32_t), st>>>(
+      SortArgs{idx, A, E, pos_of, sorted, expert_end, tile_expert, tile_row0, max_tiles});
+  return ptl_launch_status();
+}
+
+// ptl_moe_topk and ptl_moe_sort (of the first ``real`` outputs' pairs) in one kernel, for at most 64 rows and
+// 256 outputs.
+extern "C" int ptl_moe_route_few(const float* logits, int ld, const float* logit_bias, int T_, int E, int top,
+                                 int extra, int renormalize, int score_fn, const float* bias, int real,
+                                 float renorm_eps, float wscale, int n_groups, int keep_groups, int32_t* idx,
+                                 float* wgt, float* extra_out, float* ident_out, int32_t* pos_of, int32_t* sorted,
+                                 int32_t* expert_end, int32_t* tile_expert, int32_t* tile_row0, int max_tiles,
+                                 hipStream_t st) {
+  if (T_ <= 0) return PTL_OK;
+  if (T_ > 64 || E > 256 || real <= 0 || max_tiles < ptl_moe_max_tiles(T_ * top, real)) return PTL_ERR_ARG;
+  if (!route_ok(ld, E, top, extra, extra_out, real, ident_out, score_fn, n_groups, keep_groups)) return PTL_ERR_ARG;
+  const RouteArgs A{logits, ld, logit_bias, T_, E, top, extra, renormalize, score_fn, bias, real, renorm_eps, wscale,
+                    n_groups, keep_groups, idx, wgt, extra_out, ident_out};
+  const SortArgs S{idx, T_ * top, real, pos_of, sorted, expert_end, tile_expert, tile_row0, max_tiles};
+  const size_t lds = (2 * real + 1) * sizeof(int32_t);
+  if (E <= 64) moe_route_few_kernel<1><<<1, 1024, lds, st>>>(A, S);
+  else moe_route_few_kernel<4><<<1, 1024, lds, st>>>(A, S);
   return ptl_launch_status();
 }
 
@@ -399,10 +465,14 @@ moe_gemm_kernel(T* __restrict__ out, long ldo, const T* __restrict__ x, long ldx
 
 // Matrix-core forms for bfloat16 (K % 8 == 0, aligned rows).
 //
-// Few pairs (a decode step): fragments straight from memory, 64 result columns a workgroup. A
-// tile of at most 16 rows (nearly every tile of a decode step) is shared by the four waves
-// along K, 32 values in turn, so that four times as many loads of the expert's weights are under
-// way; their partial sums meet in LDS. Taller tiles: a wave owns 16 of the rows.
+// Few pairs (a decode step): fragments straight from memory, FEW_COLS result columns a workgroup. A
+// tile of at most 16 rows (nearly every tile of a decode step) is shared by the four waves, a quarter
+// of K each, so that four times as many loads of the expert's weights are under way; a wave asks for
+// the weights of its next turns (whole 128-byte lines of every row) before it multiplies those it has
+// (two sets of registers), and the waves' partial sums meet in LDS. Taller tiles: a wave owns 16 of
+// the rows. The columns of a workgroup are few so that the experts of a step, of which there may be no
+// more than one for every 25 compute units, are dealt out evenly.
+#define FEW_COLS 16
 template <int MODE>
 __global__ void __launch_bounds__(256)
 moe_gemm_mfma_kernel(bf16_t* __restrict__ out, long ldo, const bf16_t* __restrict__ x, long ldx,
@@ -412,8 +482,8 @@ moe_gemm_mfma_kernel(bf16_t* __restrict__ out, long ldo, const bf16_t* __restric
                      int act, float limit) {
   constexpr bool GATE_UP = MODE == MODE_GATE_UP;
   constexpr bool GATHER = MODE != MODE_DOWN;
-  constexpr int G = GATE_UP ? 2 : 1;
-  __shared__ float red[3][G * 4][4][64];
+  constexpr int G = GATE_UP ? 2 : 1, J = FEW_COLS / 16;
+  __shared__ float red[3][G * J][4][64];
   const int e = tile_expert[blockIdx.y];
   if (e < 0) return;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -423,7 +493,7 @@ moe_gemm_mfma_kernel(bf16_t* __restrict__ out, long ldo, const bf16_t* __restric
   const int row0 = tile_row0[blockIdx.y] + (split ? 0 : 16 * wave);
   const int rows = min(16, expert_end[e] - row0);
   if (rows <= 0) return;                 // (never in a split tile: its waves all stay)
-  const int n0 = blockIdx.x * 64;
+  const int n0 = blockIdx.x * FEW_COLS;
   const size_t wrows = GATE_UP ? 2 * (size_t)N : (size_t)N;
   w += (size_t)e * wrows * K;
   const int mr = min(ln, rows - 1);
@@ -435,40 +505,66 @@ moe_gemm_mfma_kernel(bf16_t* __restrict__ out, long ldo, const bf16_t* __restric
     if (wgt) f = wgt[a];
   }
   const bf16_t* arow = x + (size_t)src * ldx;
-  const bf16_t* brow[4];
+  const bf16_t* brow[J];
 #pragma unroll
-  for (int j = 0; j < 4; ++j) brow[j] = w + (size_t)min(n0 + 16 * j + ln, N - 1) * K;
-  f32x4_t acc[G][4];
+  for (int j = 0; j < J; ++j) brow[j] = w + (size_t)min(n0 + 16 * j + ln, N - 1) * K;
+  f32x4_t acc[G][J];
 #pragma unroll
   for (int g = 0; g < G; ++g)
 #pragma unroll
-    for (int j = 0; j < 4; ++j) acc[g][j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    for (int j = 0; j < J; ++j) acc[g][j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   const uint4 zero = make_uint4(0, 0, 0, 0);
   const size_t up = (size_t)N * K;
-  const int kstep = split ? 128 : 32;
-  for (int k0 = split ? 32 * wave : 0; k0 < K; k0 += kstep) {
+  struct Turn {
+    Frag8 a, b[G][J];
+  };
+  auto load = [&](Turn& f, int k0, int ke) {
     const int k = k0 + 8 * lg;
-    Frag8 a, b[G][4];
-    a.u = k < K ? *reinterpret_cast<const uint4*>(arow + k) : zero;
+    f.a.u = k < ke ? *reinterpret_cast<const uint4*>(arow + k) : zero;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      b[0][j].u = k < K ? load_once(brow[j] + k) : zero;
-      if (GATE_UP) b[G - 1][j].u = k < K ? load_once(brow[j] + up + k) : zero;
+    for (int j = 0; j < J; ++j) {
+      f.b[0][j].u = k < ke ? load_once(brow[j] + k) : zero;
+      if (GATE_UP) f.b[G - 1][j].u = k < ke ? load_once(brow[j] + up + k) : zero;
     }
+  };
+  auto multiply = [&](const Turn& f) {
 #pragma unroll
     for (int g = 0; g < G; ++g)
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        acc[g][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(b[g][j].v, a.v, acc[g][j], 0, 0, 0);
+      for (int j = 0; j < J; ++j)
+        acc[g][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f.b[g][j].v, f.a.v, acc[g][j], 0, 0, 0);
+  };
+  if (split) {
+    constexpr int U = 4;                 // turns a set of registers holds
+    const int per = ((K + 3) / 4 + 31) / 32 * 32, kb = wave * per, ke = min(K, kb + per);
+    Turn cur[U], nxt[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) load(cur[u], kb + 32 * u, ke);
+    for (int k0 = kb; k0 < ke; k0 += 64 * U) {
+#pragma unroll
+      for (int u = 0; u < U; ++u) load(nxt[u], k0 + 32 * (U + u), ke);
+#pragma unroll
+      for (int u = 0; u < U; ++u) multiply(cur[u]);
+#pragma unroll
+      for (int u = 0; u < U; ++u) load(cur[u], k0 + 32 * (2 * U + u), ke);
+#pragma unroll
+      for (int u = 0; u < U; ++u) multiply(nxt[u]);
+    }
+  } else {
+    for (int k0 = 0; k0 < K; k0 += 32) {
+      Turn f;
+      load(f, k0, K);
+      multiply(f);
+    }
   }
   if (split) {
     if (wave > 0) {
 #pragma unroll
       for (int g = 0; g < G; ++g)
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
+        for (int j = 0; j < J; ++j)
 #pragma unroll
-          for (int i = 0; i < 4; ++i) red[wave - 1][g * 4 + j][i][lane] = acc[g][j][i];
+          for (int i = 0; i < 4; ++i) red[wave - 1][g * J + j][i][lane] = acc[g][j][i];
     }
     __syncthreads();
     if (wave > 0) return;
@@ -477,13 +573,13 @@ moe_gemm_mfma_kernel(bf16_t* __restrict__ out, long ldo, const bf16_t* __restric
 #pragma unroll
       for (int g = 0; g < G; ++g)
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
+        for (int j = 0; j < J; ++j)
 #pragma unroll
-          for (int i = 0; i < 4; ++i) acc[g][j][i] += red[v][g * 4 + j][i][lane];
+          for (int i = 0; i < 4; ++i) acc[g][j][i] += red[v][g * J + j][i][lane];
   }
   if (ln < rows) {
 #pragma unroll
-    for (int j = 0; j < 4; ++j)
+    for (int j = 0; j < J; ++j)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int n = n0 + 16 * j + 4 * lg + i;
@@ -666,7 +762,7 @@ extern "C" int ptl_moe_gate_up(void* out, long ldo, const void* x, long ldx, con
                                hipStream_t st) {
   if (max_tiles <= 0) return PTL_OK;
   if (I <= 0 || K <= 0 || top <= 0 || max_tiles > 65535) return PTL_ERR_ARG;
-  dim3 grid((I + 63) / 64, max_tiles);
+  dim3 grid((I + 63) / 64, max_tiles), few((I + FEW_COLS - 1) / FEW_COLS, max_tiles);
   if (dtype == PTL_DTYPE_F32)
     moe_gemm_kernel<float, MODE_GATE_UP><<<grid, 256, 0, st>>>((float*)out, ldo, (const float*)x, ldx, (const float*)w,
                                                        tile_expert, tile_row0, expert_end, sorted, wgt, top, I,
@@ -678,7 +774,7 @@ extern "C" int ptl_moe_gate_up(void* out, long ldo, const void* x, long ldx, con
                                                       sorted, wgt, top, I, K, act, limit);
   }
   else if (dtype == PTL_DTYPE_BF16 && mfma_ok(x, ldx, w, K))
-    moe_gemm_mfma_kernel<MODE_GATE_UP><<<grid, 256, 0, st>>>((bf16_t*)out, ldo, (const bf16_t*)x, ldx,
+    moe_gemm_mfma_kernel<MODE_GATE_UP><<<few, 256, 0, st>>>((bf16_t*)out, ldo, (const bf16_t*)x, ldx,
                                                      (const bf16_t*)w, tile_expert, tile_row0, expert_end,
                                                      sorted, wgt, top, I, K, act, limit);
   else if (dtype == PTL_DTYPE_BF16)
@@ -698,7 +794,7 @@ extern "C" int ptl_moe_up(void* out, long ldo, const void* x, long ldx, const vo
                           int K, int act, int dtype, hipStream_t st) {
   if (max_tiles <= 0) return PTL_OK;
   if (I <= 0 || K <= 0 || top <= 0 || max_tiles > 65535 || act != 2) return PTL_ERR_ARG;
-  dim3 grid((I + 63) / 64, max_tiles);
+  dim3 grid((I + 63) / 64, max_tiles), few((I + FEW_COLS - 1) / FEW_COLS, max_tiles);
   if (dtype == PTL_DTYPE_F32)
     moe_gemm_kernel<float, MODE_UP><<<grid, 256, 0, st>>>((float*)out, ldo, (const float*)x, ldx,
                                                           (const float*)w, tile_expert, tile_row0, expert_end,
@@ -709,7 +805,7 @@ extern "C" int ptl_moe_up(void* out, long ldo, const void* x, long ldx, const vo
                                                          (const bf16_t*)w, tile_expert, tile_row0, expert_end,
                                                          sorted, wgt, top, I, K, act, 0.f);
   } else if (dtype == PTL_DTYPE_BF16 && mfma_ok(x, ldx, w, K))
-    moe_gemm_mfma_kernel<MODE_UP><<<grid, 256, 0, st>>>((bf16_t*)out, ldo, (const bf16_t*)x, ldx,
+    moe_gemm_mfma_kernel<MODE_UP><<<few, 256, 0, st>>>((bf16_t*)out, ldo, (const bf16_t*)x, ldx,
                                                         (const bf16_t*)w, tile_expert, tile_row0, expert_end,
                                                         sorted, wgt, top, I, K, act, 0.f);
   else if (dtype == PTL_DTYPE_BF16)
@@ -727,7 +823,7 @@ extern "C" int ptl_moe_down(void* out, long ldo, const void* x, long ldx, const 
                             int max_tiles, int pairs, int N, int K, int dtype, hipStream_t st) {
   if (max_tiles <= 0) return PTL_OK;
   if (N <= 0 || K <= 0 || max_tiles > 65535) return PTL_ERR_ARG;
-  dim3 grid((N + 63) / 64, max_tiles);
+  dim3 grid((N + 63) / 64, max_tiles), few((N + FEW_COLS - 1) / FEW_COLS, max_tiles);
   if (dtype == PTL_DTYPE_F32)
     moe_gemm_kernel<float, MODE_DOWN><<<grid, 256, 0, st>>>((float*)out, ldo, (const float*)x, ldx, (const float*)w,
                                                         tile_expert, tile_row0, expert_end, nullptr, nullptr, 1,
@@ -738,7 +834,7 @@ extern "C" int ptl_moe_down(void* out, long ldo, const void* x, long ldx, const 
                                                        (const bf16_t*)w, tile_expert, tile_row0, expert_end,
                                                        nullptr, nullptr, 1, N, K, 0, 0.f);
   } else if (dtype == PTL_DTYPE_BF16 && mfma_ok(x, ldx, w, K))
-    moe_gemm_mfma_kernel<MODE_DOWN><<<grid, 256, 0, st>>>((bf16_t*)out, ldo, (const bf16_t*)x, ldx,
+    moe_gemm_mfma_kernel<MODE_DOWN><<<few, 256, 0, st>>>((bf16_t*)out, ldo, (const bf16_t*)x, ldx,
                                                       (const bf16_t*)w, tile_expert, tile_row0, expert_end,
                                                       nullptr, nullptr, 1, N, K, 0, 0.f);
   else if (dtype == PTL_DTYPE_BF16)

@@ -177,7 +177,9 @@ extern "C" int ptl_qkv_prepare(void* q_out, const float* p, long ldp, int q_off,
 //   ones [taps - 1, C] (bias included; zeros where a sequence starts);
 // q and k: the first rot_dims entries of a head turn by the row's position (pairs of neighbours, or
 //   entry i with entry i + rot_dims / 2), then, when ``norm``, the head is divided by its root mean square.
-// A wave takes one head for ``run`` rows one after the other, a lane NP pairs of its entries; with
+// A wave takes one head for RUN rows one after the other, a lane NP pairs of its entries; the rows' inputs
+// are asked for before the first is worked on, and the four waves of a workgroup (four heads of the
+// same rows) share the rows' sines and cosines through LDS. With
 // TAPS > 0 the last TAPS - 1 inputs of a lane's entries stay in registers from row to row (TAPS = 0: any
 // number of taps, read again for every row). The first n_single sequences bring one row each: their
 // lanes also advance the kept inputs they have just read (those of longer portions are advanced
@@ -205,15 +207,29 @@ struct ConvQkvArgs {
   const int32_t* positions; const int32_t* slots;
   int rot_dims, layout; const float* inv_freq;
   int norm; float eps;
-  int T, Hq, Hk, Hv, Dk, Dv, page_size, run;
+  int T, Hq, Hk, Hv, Dk, Dv, page_size;
 };
 
-template <int NP, int TAPS, typename TO>
+template <int NP, int TAPS, int RUN, typename TO>
 __global__ void __launch_bounds__(256)
 conv_qkv_prepare_kernel(TO* __restrict__ q_out, TO* __restrict__ k_cache, TO* __restrict__ v_cache, ConvQkvArgs A) {
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int head = blockIdx.y * 4 + wave;
+  const int t_begin = blockIdx.x * RUN, t_end = min(A.T, t_begin + RUN);
+  __shared__ float2 turns[RUN][64 * NP];    // (sine, cosine) of every row and pair
+  if (A.rot_dims > 0 && (int)blockIdx.y * 4 < A.Hq + A.Hk) {
+    const int pairs = A.rot_dims / 2;
+    for (int i = threadIdx.x; i < RUN * pairs; i += 256) {
+      const int r = i / pairs, j = i - r * pairs;
+      if (t_begin + r < t_end) {
+        float2 v;
+        turn_of((float)A.positions[t_begin + r], A.inv_freq[j], v.x, v.y);
+        turns[r][j] = v;
+      }
+    }
+  }
+  __syncthreads();
   if (head >= A.Hq + A.Hk + A.Hv) return;
   const int part = head < A.Hq ? 0 : (head < A.Hq + A.Hk ? 1 : 2);
   const int h = head - (part == 0 ? 0 : (part == 1 ? A.Hq : A.Hq + A.Hk));
@@ -234,10 +250,28 @@ conv_qkv_prepare_kernel(TO* __restrict__ q_out, TO* __restrict__ k_cache, TO* __
     for (int i = 0; i < 2; ++i)
       if (e[n][i] >= D) e[n][i] = -1;
   }
-  float w[NP][2][TAPS > 0 ? TAPS : 1], b[NP][2], f[NP];
+  // two neighbouring entries at an even column, rows of an even length: one 8-byte load
+  const bool two = ((A.ldp | col0) & 1) == 0 && ((uintptr_t)A.p & 7) == 0 && !(A.layout == PAIRS_HALF && rot > 0) && D % 2 == 0;
+  float2 ahead[RUN][NP];                    // the rows' columns
+#pragma unroll
+  for (int r = 0; r < RUN; ++r)
+#pragma unroll
+    for (int n = 0; n < NP; ++n) {
+      float2 x = make_float2(0.f, 0.f);
+      const float* at = A.p + (size_t)(t_begin + r) * A.ldp + col0;
+      if (t_begin + r < t_end) {
+        if (two) {
+          if (e[n][0] >= 0) x = *reinterpret_cast<const float2*>(at + e[n][0]);
+        } else {
+          if (e[n][0] >= 0) x.x = at[e[n][0]];
+          if (e[n][1] >= 0) x.y = at[e[n][1]];
+        }
+      }
+      ahead[r][n] = x;
+    }
+  float w[NP][2][TAPS > 0 ? TAPS : 1], b[NP][2];
 #pragma unroll
   for (int n = 0; n < NP; ++n) {
-    f[n] = 2 * (lane + 64 * n) < rot ? A.inv_freq[lane + 64 * n] : 0.f;
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
       b[n][i] = A.bias && e[n][i] >= 0 ? A.bias[c0 + e[n][i]] : 0.f;
@@ -250,20 +284,30 @@ conv_qkv_prepare_kernel(TO* __restrict__ q_out, TO* __restrict__ k_cache, TO* __
   auto input = [&](int row, int n, int i) {
     return e[n][i] >= 0 ? A.p[(size_t)row * A.ldp + col0 + e[n][i]] + b[n][i] : 0.f;
   };
-  const int t_begin = blockIdx.x * A.run, t_end = min(A.T, t_begin + A.run);
   // the sequence of the first row: the last one whose first row is not beyond it
   int seq = 0, hi = A.n_seqs;
   while (seq < hi) {
     const int mid = (seq + hi + 1) >> 1;
     if (A.q_start[mid] <= t_begin) seq = mid; else hi = mid - 1;
   }
+  if (seq >= A.n_seqs) return;              // rows that belong to no sequence
+  const int my_slot = A.slots && lane < RUN && t_begin + lane < t_end ? A.slots[t_begin + lane] : -1;
   bool fresh = true;                        // the window in registers is not of this sequence yet
+  int row0 = 0, seq_end = A.q_start[seq + 1];
+  float* kept = nullptr;
   float win[NP][2][TAPS > 1 ? TAPS - 1 : 1];
-  for (int t = t_begin; t < t_end; ++t) {
-    while (seq < A.n_seqs && A.q_start[seq + 1] <= t) { ++seq; fresh = true; }
-    if (seq >= A.n_seqs) return;            // rows that belong to no sequence
-    const int row0 = A.q_start[seq];
-    float* kept = taps > 1 ? A.state + (size_t)A.state_slots[seq] * A.slot_stride + A.tail_off : nullptr;
+#pragma unroll
+  for (int q = 0; q < RUN; ++q) {
+    const int t = t_begin + q;
+    if (t >= t_end) return;
+    if (q == 0 || t >= seq_end) {           // (sequences without rows are skipped)
+      while (seq < A.n_seqs && A.q_start[seq + 1] <= t) ++seq;
+      if (seq >= A.n_seqs) return;
+      row0 = A.q_start[seq];
+      seq_end = A.q_start[seq + 1];
+      if (taps > 1) kept = A.state + (size_t)A.state_slots[seq] * A.slot_stride + A.tail_off;
+      fresh = true;
+    }
     auto before = [&](int r, int n, int i) {                   // the input of row r of the sequence (r < 0: a kept one)
       if (r >= 0) return input(row0 + r, n, i);
       return e[n][i] >= 0 ? kept[(size_t)(taps - 1 + r) * C + c0 + e[n][i]] : 0.f;
@@ -274,7 +318,7 @@ conv_qkv_prepare_kernel(TO* __restrict__ q_out, TO* __restrict__ k_cache, TO* __
     for (int n = 0; n < NP; ++n)
 #pragma unroll
       for (int i = 0; i < 2; ++i) {
-        const float x = input(t, n, i);
+        const float x = (i == 0 ? ahead[q][n].x : ahead[q][n].y) + b[n][i];
         if (TAPS > 0) {
           if (fresh) {
 #pragma unroll
@@ -305,12 +349,10 @@ conv_qkv_prepare_kernel(TO* __restrict__ q_out, TO* __restrict__ k_cache, TO* __
     float scale = 1.f;
     if (part < 2) {
       if (rot > 0) {
-        const float pos = (float)A.positions[t];
 #pragma unroll
         for (int n = 0; n < NP; ++n) {
           if (2 * (lane + 64 * n) >= rot) continue;
-          float sn, cs;
-          turn_of(pos, f[n], sn, cs);
+          const float sn = turns[q][lane + 64 * n].x, cs = turns[q][lane + 64 * n].y;
           const float u = y[n][0], v = y[n][1];
           y[n][0] = u * cs - v * sn;
           y[n][1] = v * cs + u * sn;
@@ -330,12 +372,12 @@ conv_qkv_prepare_kernel(TO* __restrict__ q_out, TO* __restrict__ k_cache, TO* __
     if (part == 0) {
       dst = q_out + ((size_t)t * A.Hq + h) * D;
     } else {
-      const int slot = A.slots ? A.slots[t] : -1;
-      if (slot < 0) continue;
-      const int page = slot / A.page_size, at = slot % A.page_size;
-      dst = part == 1 ? k_cache + (((size_t)page * A.Hk + h) * A.page_size + at) * D
+      const int slot = __builtin_amdgcn_readlane(my_slot, q);
+      const int page = max(slot, 0) / A.page_size, at = max(slot, 0) % A.page_size;
+      if (slot >= 0) dst = part == 1 ? k_cache + (((size_t)page * A.Hk + h) * A.page_size + at) * D
                       : v_cache + (((size_t)page * A.Hv + h) * A.page_size + at) * D;
     }
+    if (dst == nullptr) continue;
 #pragma unroll
     for (int n = 0; n < NP; ++n) {
       if (sizeof(TO) == 2 && D % 2 == 0 && e[n][0] >= 0 && e[n][1] == e[n][0] + 1 && e[n][0] % 2 == 0) {
@@ -371,20 +413,21 @@ extern "C" int ptl_conv_qkv_prepare(void* q_out, const float* p, long ldp, int q
     return PTL_ERR_ARG;
   ConvQkvArgs A{p, ldp, {q_off, k_off, v_off}, bias, cw, taps, state, slot_stride, tail_off, q_start, state_slots,
                 n_seqs, n_single, positions, slots, rot_dims, layout, inv_freq, norm, eps, T_, Hq, Hk, Hv, Dk, Dv,
-                page_size, 1};
-  // runs of rows that share their inputs, as long as the chip stays filled a few times over
-  const long waves = (long)T_ * (Hq + Hk + Hv);
-  A.run = waves >= 8 * 16384 ? 8 : (waves >= 4 * 16384 ? 4 : (waves >= 2 * 16384 ? 2 : 1));
-  const dim3 grid((T_ + A.run - 1) / A.run, (Hq + Hk + Hv + 3) / 4);
+                page_size};
+  // runs of rows that share their inputs where the chip stays filled
   const bool wide = (Dk > Dv ? Dk : Dv) > 128;
-#define GO(NP, TAPS, TO)                                                                                           \
-  conv_qkv_prepare_kernel<NP, TAPS, TO><<<grid, 256, 0, st>>>((TO*)q_out, (TO*)k_cache, (TO*)v_cache, A)
-#define BY_TAPS(NP, TO)                                     \
-  if (taps == 4) GO(NP, 4, TO);                             \
-  else if (taps == 1) GO(NP, 1, TO);                        \
-  else GO(NP, 0, TO)
-#define BY_SIZE(TO)                                         \
-  if (wide) { BY_TAPS(5, TO); } else { BY_TAPS(1, TO); }
+  const int run = !wide && (long)T_ * (Hq + Hk + Hv) >= 16384 ? 8 : 1;
+  const dim3 grid((T_ + run - 1) / run, (Hq + Hk + Hv + 3) / 4);
+#define GO(NP, TAPS, RUN, TO)                                                                                       \
+  conv_qkv_prepare_kernel<NP, TAPS, RUN, TO><<<grid, 256, 0, st>>>((TO*)q_out, (TO*)k_cache, (TO*)v_cache, A)
+#define BY_TAPS(NP, RUN, TO)                                     \
+  if (taps == 4) GO(NP, 4, RUN, TO);                             \
+  else if (taps == 1) GO(NP, 1, RUN, TO);                        \
+  else GO(NP, 0, RUN, TO)
+#define BY_SIZE(TO)                                                             \
+  if (wide) { BY_TAPS(5, 1, TO); }                                              \
+  else if (run == 8) { BY_TAPS(1, 8, TO); }                                     \
+  else { BY_TAPS(1, 1, TO); }
   if (dtype == PTL_DTYPE_F32) { BY_SIZE(float) }
   else if (dtype == PTL_DTYPE_BF16) { BY_SIZE(bf16_t) }
   else return PTL_ERR_ARG;
@@ -430,6 +473,68 @@ head_norm_gate_kernel(TO* __restrict__ out, long ldo, const float* __restrict__ 
   }
 }
 
+// One map, heads of up to 256 values that divide by 4: LPH lanes a head with a float4 each, 64 / LPH heads
+// (neighbours of one row after the other) a wave.
+template <int LPH, typename TO>
+__global__ void __launch_bounds__(256)
+head_norm_gate_vec_kernel(TO* __restrict__ out, long ldo, const float* __restrict__ a, const float* __restrict__ w,
+                          int w_stride, float mult, const float* __restrict__ gate, long ldg, int g_off, int act, float eps,
+                          long items, int H, int Dv) {
+  const long item = ((long)blockIdx.x * 256 + threadIdx.x) / LPH;
+  const int d = 4 * (threadIdx.x % LPH);
+  const bool in = item < items && d < Dv;
+  const long t = item / H;
+  const int h = (int)(item - t * H);
+  float4 o = make_float4(0.f, 0.f, 0.f, 0.f), g = o;
+  if (in) {
+    o = *reinterpret_cast<const float4*>(a + (size_t)item * Dv + d);
+    if (gate) g = *reinterpret_cast<const float4*>(gate + (size_t)t * ldg + g_off + (size_t)h * Dv + d);
+  }
+  float ss = fmaf(o.x, o.x, fmaf(o.y, o.y, fmaf(o.z, o.z, o.w * o.w)));
+#pragma unroll
+  for (int s = 1; s < LPH; s <<= 1) ss += __shfl_xor(ss, s, 64);
+  if (!in) return;
+  const float r = mult / sqrtf(ss / (float)Dv + eps);
+  float v[4] = {o.x * r, o.y * r, o.z * r, o.w * r};
+  const float z[4] = {g.x, g.y, g.z, g.w};
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    if (w) v[i] *= w[(size_t)h * w_stride + d + i];
+    if (gate) {
+      const float sg = 1.0f / (1.0f + expf(-z[i]));
+      v[i] *= act == ACT_SILU ? z[i] * sg : sg;
+    }
+  }
+  TO* dst = out + (size_t)t * ldo + (size_t)h * Dv + d;
+  if (sizeof(TO) == 2) {
+    union { uint2 u; bf16_t e[4]; } e;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) e.e[i] = float_to_bf16(v[i]);
+    *reinterpret_cast<uint2*>(dst) = e.u;
+  } else {
+    *reinterpret_cast<float4*>(dst) = make_float4(v[0], v[1], v[2], v[3]);
+  }
+}
+
+template <typename TO>
+static bool head_norm_gate_vec(void* out, long ldo, const float* a, const float* w, int w_stride, float mult,
+                               const float* gate, long ldg, int g_off, int act, float eps, long items, int H, int Dv,
+                               hipStream_t st) {
+  if (Dv % 4 || Dv > 256 || ldo % 4 || (((uintptr_t)a | (uintptr_t)out) & 15) ||
+      (gate && (ldg % 4 || g_off % 4 || ((uintptr_t)gate & 15))))
+    return false;
+  const int lanes = Dv / 4;
+#define GO(LPH)                                                                                                    \
+  if (lanes <= LPH) {                                                                                              \
+    head_norm_gate_vec_kernel<LPH, TO><<<(int)((items * LPH + 255) / 256), 256, 0, st>>>(                          \
+        (TO*)out, ldo, a, w, w_stride, mult, gate, ldg, g_off, act, eps, items, H, Dv);                            \
+    return true;                                                                                                   \
+  }
+  GO(4) GO(8) GO(16) GO(32) GO(64)
+#undef GO
+  return false;
+}
+
 // a float32 [T, H * maps, Dv] dense; out [T, ldo] (H * Dv columns used); gate float32 [T, ldg] read
 // at columns g_off .. g_off + H * Dv, or null; w float32 (w_stride 0: [Dv] for all heads, Dv: [H, Dv]),
 // or null.
@@ -441,7 +546,13 @@ extern "C" int ptl_head_norm_gate(void* out, long ldo, const float* a, int maps,
     return PTL_ERR_ARG;
   const long items = (long)T_ * H;
   const long blocks = (items + 3) / 4;
-  if (blocks > 0x7fffffff) return PTL_ERR_ARG;
+  if (items > 0x7fffffff / 16) return PTL_ERR_ARG;
+  if (maps == 1 && dtype == PTL_DTYPE_F32 &&
+      head_norm_gate_vec<float>(out, ldo, a, w, w_stride, mult, gate, ldg, g_off, act, eps, items, H, Dv, st))
+    return ptl_launch_status();
+  if (maps == 1 && dtype == PTL_DTYPE_BF16 &&
+      head_norm_gate_vec<bf16_t>(out, ldo, a, w, w_stride, mult, gate, ldg, g_off, act, eps, items, H, Dv, st))
+    return ptl_launch_status();
 #define GO(TO)                                                                                         \
   {                                                                                                    \
     head_norm_gate_kernel<TO><<<(int)blocks, 256, 0, st>>>((TO*)out, ldo, a, maps, lam, w, w_stride,   \

@@ -351,8 +351,21 @@ extern "C" int ptl_stream_postnorm(float* stream, float alpha, const void* y1, f
 // The residual sum of sublayers whose results are scaled entry by entry, and the norm that follows:
 //   stream += s1 * (y1 + bias) + s2 * y2;    out = stream * rsqrt(mean(stream^2) + eps) * w
 // (y1, y2, bias and both scales are optional: no y1 and no y2 leaves the stream as it is; w null: no
-// norm, no out). One workgroup a row; a thread keeps its VPT groups of VEC neighbouring entries in
+// norm, no out). y2 may also come as routed experts leave it: the rows of a token's choices times
+// their weights, and a shared expert's row (RoutedArgs). Behind the norm a time mixer's inputs can be made as
+// well, for rows that are sequences of one token (MixArgs): out_m = h + (h' - h) mu_m, h' the row kept in
+// the sequence's state slot. One workgroup a row; a thread keeps its VPT groups of VEC neighbouring entries in
 // registers from the one pass over memory to the last use.
+struct RoutedArgs {
+  const void* rows; long ldr;               // the experts' results, sorted by expert; null: none
+  const int32_t* pos_of; const float* wgt; int top;      // [T * top]; wgt null: ones
+  const void* shared;                       // [T, H] or null
+};
+struct MixArgs {
+  void* out; long mix_stride;               // [n, T, H]; null: none
+  const float* mu; int n;                   // [n, H]
+  const float* state; long slot_stride; long off; const int32_t* slots;
+};
 struct ScaledSumArgs {
   float* stream;
   const void* y1; const float* s1; const float* bias;
@@ -360,6 +373,8 @@ struct ScaledSumArgs {
   const float* w; float eps;
   void* out;
   int H;
+  RoutedArgs routed;
+  MixArgs mix;
 };
 
 template <int VEC, typename T>
@@ -381,13 +396,18 @@ __global__ void __launch_bounds__(NT) stream_scaled_sum_kernel(ScaledSumArgs A) 
   __shared__ float scratch[16];
   const size_t row = (size_t)blockIdx.x * A.H;
   float* stream = A.stream + row;
-  float u[VPT][VEC];
+  float u[VPT][VEC], d[VPT][VEC];          // d: the kept row, asked for long before it is needed
+  const float* kept = A.mix.out ? A.mix.state + (size_t)A.mix.slots[blockIdx.x] * A.mix.slot_stride + A.mix.off : nullptr;
   float ss = 0.f;
 #pragma unroll
   for (int k = 0; k < VPT; ++k) {
     const int i = (k * NT + threadIdx.x) * VEC;
     if (i >= A.H) continue;
     read_vec<VEC>((const float*)stream + i, u[k]);
+    if (kept) {
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) d[k][j] = kept[i + j];
+    }
     if (A.y1) {
       float y[VEC], f[VEC];
       read_vec<VEC>((const T1*)A.y1 + row + i, y);
@@ -400,14 +420,35 @@ __global__ void __launch_bounds__(NT) stream_scaled_sum_kernel(ScaledSumArgs A) 
 #pragma unroll
       for (int j = 0; j < VEC; ++j) u[k][j] = fmaf(A.s1 ? f[j] : 1.f, y[j], u[k][j]);
     }
-    if (A.y2) {
+    if (A.y2 || A.routed.rows) {
       float y[VEC], f[VEC];
-      read_vec<VEC>((const T2*)A.y2 + row + i, y);
+      if (A.routed.rows) {
+        const RoutedArgs& R = A.routed;
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) y[j] = 0.f;
+#pragma unroll 4
+        for (int c = 0; c < R.top; ++c) {
+          const size_t pair = (size_t)blockIdx.x * R.top + c;
+          const int p = R.pos_of[pair];
+          if (p < 0) continue;
+          const float g = R.wgt ? R.wgt[pair] : 1.f;
+          read_vec<VEC>((const T2*)R.rows + (size_t)p * R.ldr + i, f);
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) y[j] = fmaf(f[j], g, y[j]);
+        }
+        if (R.shared) {
+          read_vec<VEC>((const T2*)R.shared + row + i, f);
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) y[j] += f[j];
+        }
+      } else {
+        read_vec<VEC>((const T2*)A.y2 + row + i, y);
+      }
       if (A.s2) read_vec<VEC>(A.s2 + i, f);
 #pragma unroll
       for (int j = 0; j < VEC; ++j) u[k][j] = fmaf(A.s2 ? f[j] : 1.f, y[j], u[k][j]);
     }
-    if (A.y1 || A.y2) {
+    if (A.y1 || A.y2 || A.routed.rows) {
       if (VEC == 1) stream[i] = u[k][0];
       else *reinterpret_cast<float4*>(stream + i) = make_float4(u[k][0], u[k][VEC > 1 ? 1 : 0], u[k][VEC > 2 ? 2 : 0], u[k][VEC > 3 ? 3 : 0]);
     }
@@ -426,9 +467,35 @@ __global__ void __launch_bounds__(NT) stream_scaled_sum_kernel(ScaledSumArgs A) 
     TO e[VEC];
 #pragma unroll
     for (int j = 0; j < VEC; ++j) e[j] = from_float<TO>(u[k][j] * r * w[j]);
-    if (VEC == 1) out[i] = e[0];
-    else if (sizeof(TO) == 2) *reinterpret_cast<uint2*>(out + i) = *reinterpret_cast<const uint2*>(e);
-    else *reinterpret_cast<float4*>(out + i) = *reinterpret_cast<const float4*>(e);
+    auto put = [](TO* at, const TO (&v)[VEC]) {
+      if (VEC == 1) at[0] = v[0];
+      else if (sizeof(TO) == 2) *reinterpret_cast<uint2*>(at) = *reinterpret_cast<const uint2*>(v);
+      else *reinterpret_cast<float4*>(at) = *reinterpret_cast<const float4*>(v);
+    };
+    put(out + i, e);
+    if (A.mix.out) {
+      const MixArgs& M = A.mix;
+      float h[VEC];
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) {
+        h[j] = to_float<TO>(e[j]);
+        d[k][j] -= h[j];
+      }
+      constexpr int AT_ONCE = 5;            // the factors of so many mixes are asked for together
+      for (int m0 = 0; m0 < M.n; m0 += AT_ONCE) {
+        float f[AT_ONCE][VEC];
+#pragma unroll
+        for (int m = 0; m < AT_ONCE; ++m)
+          if (m0 + m < M.n) read_vec<VEC>(M.mu + (size_t)(m0 + m) * A.H + i, f[m]);
+#pragma unroll
+        for (int m = 0; m < AT_ONCE; ++m) {
+          if (m0 + m >= M.n) continue;
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) e[j] = from_float<TO>(fmaf(d[k][j], f[m][j], h[j]));
+          put((TO*)M.out + (size_t)(m0 + m) * M.mix_stride + row + i, e);
+        }
+      }
+    }
   }
 }
 
@@ -436,7 +503,8 @@ template <typename T1, typename T2, typename TO>
 static int launch_scaled_sum(const ScaledSumArgs& A, int T_, hipStream_t st) {
   auto odd = [](const void* p) { return ((uintptr_t)p & 15) != 0; };
   const bool vec = A.H % 4 == 0 && !odd(A.stream) && !odd(A.y1) && !odd(A.s1) && !odd(A.bias) && !odd(A.y2) &&
-                   !odd(A.s2) && !odd(A.w) && !odd(A.out);
+                   !odd(A.s2) && !odd(A.w) && !odd(A.out) && !odd(A.routed.rows) && !odd(A.routed.shared) &&
+                   A.routed.ldr % 4 == 0 && !odd(A.mix.out) && !odd(A.mix.mu) && A.mix.mix_stride % 4 == 0;
   const int n = vec ? A.H / 4 : A.H;         // groups of entries of a row
   // few rows: a row over 1,024 threads, so that a thread's loads are one or two deep
   const bool few = T_ <= 512 && n > 256;
@@ -453,14 +521,24 @@ static int launch_scaled_sum(const ScaledSumArgs& A, int T_, hipStream_t st) {
   return PTL_ERR_ARG;
 }
 
-// stream float32 [T, H], in place; y1 [T, H] float32 or null; y2 [T, H] of y2_dtype or null; s1, s2, bias, w
-// float32 [H] or null; out [T, H] of out_dtype (with w). H up to 16,384.
+// stream float32 [T, H], in place; y1 [T, H] float32 or null; y2 [T, H] of y2_dtype or null, or in its place rows
+// (ldr), pos_of, wgt, top and shared of y2_dtype (RoutedArgs); s1, s2, bias, w float32 [H] or null; out [T, H] of
+// out_dtype (with w); mix_out [n_mix, T, H] of out_dtype or null, with mu float32 [n_mix, H] and row t's kept
+// row at state + slots[t] * slot_stride + off (MixArgs). H up to 16,384.
 extern "C" int ptl_stream_scaled_sum(float* stream, const float* y1, const float* s1, const float* bias,
-                                     const void* y2, int y2_dtype, const float* s2, const float* w, float eps,
-                                     void* out, int out_dtype, int T_, int H, hipStream_t st) {
+                                     const void* y2, int y2_dtype, const float* s2, const void* rows, long ldr,
+                                     const int32_t* pos_of, const float* wgt, int top, const void* shared,
+                                     const float* w, float eps, void* out, int out_dtype, void* mix_out,
+                                     long mix_stride, const float* mu, int n_mix, const float* state,
+                                     long slot_stride, long off, const int32_t* slots, int T_, int H, hipStream_t st) {
   if (T_ <= 0) return PTL_OK;
-  if (H <= 0 || !stream || (bias && !y1) || (w && !out) || (!y1 && !y2 && !w)) return PTL_ERR_ARG;
-  const ScaledSumArgs A{stream, y1, s1, bias, y2, s2, w, eps, out, H};
+  if (H <= 0 || !stream || (bias && !y1) || (w && !out) || (!y1 && !y2 && !rows && !w) || (y2 && rows) ||
+      (rows && (!pos_of || top <= 0 || ldr < H)) || (shared && !rows) ||
+      (mix_out && (!w || !mu || n_mix <= 0 || !state || !slots || mix_stride < (long)T_ * H || off < 0 ||
+                   off + H > slot_stride)))
+    return PTL_ERR_ARG;
+  const ScaledSumArgs A{stream, y1, s1, bias, y2, s2, w, eps, out, H, RoutedArgs{rows, ldr, pos_of, wgt, top, shared},
+                        MixArgs{mix_out, mix_stride, mu, n_mix, state, slot_stride, off, slots}};
   if (y2_dtype == PTL_DTYPE_F32 && out_dtype == PTL_DTYPE_F32) return launch_scaled_sum<float, float, float>(A, T_, st);
   if (y2_dtype == PTL_DTYPE_F32 && out_dtype == PTL_DTYPE_BF16) return launch_scaled_sum<float, float, bf16_t>(A, T_, st);
   if (y2_dtype == PTL_DTYPE_BF16 && out_dtype == PTL_DTYPE_BF16) return launch_scaled_sum<float, bf16_t, bf16_t>(A, T_, st);

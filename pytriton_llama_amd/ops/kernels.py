@@ -1662,34 +1662,89 @@ def stream_postnorm(stream: torch.Tensor, alpha: float, y1: torch.Tensor, a: flo
     return copy
 
 
+class RoutedSum:
+    """What routed experts have computed but not added up: the rows of a step's (token, choice) pairs in the
+    experts' order, the routing that says where each token's rows lie and what they count, and a shared
+    expert's rows (or None)."""
+    __slots__ = ("rows", "routing", "weighted", "shared")
+
+    def __init__(self, rows, routing, weighted, shared):
+        self.rows, self.routing, self.weighted, self.shared = rows, routing, bool(weighted), shared
+
+    @property
+    def shape(self):
+        return (self.routing.idx.numel() // self.routing.top, self.rows.shape[1])
+
+    def tensor(self) -> torch.Tensor:
+        return moe_combine(self)
+
+
+class TimeMixes:
+    """The inputs of a time mixer that the norm in front of it is to make as well, for a step of single
+    tokens: mu float32 [n, H], and the row kept at ``off`` of every sequence's state slot."""
+    __slots__ = ("mu", "state", "off", "slots")
+
+    def __init__(self, mu, state, off, slots):
+        self.mu, self.state, self.off, self.slots = mu, state, int(off), slots
+
+
 def stream_scaled_sum(stream: torch.Tensor, y1: Optional[torch.Tensor] = None, scale1: Optional[torch.Tensor] = None,
-                      bias: Optional[torch.Tensor] = None, y2: Optional[torch.Tensor] = None,
-                      scale2: Optional[torch.Tensor] = None, norm_weight: Optional[torch.Tensor] = None,
-                      eps: float = 0.0, out_dtype: Optional[torch.dtype] = None) -> Optional[torch.Tensor]:
-    """stream += scale1 * (y1 + bias) + scale2 * y2 in place, entry by entry (y1 float32; every piece is
-    optional, a scale that is None is one); with ``norm_weight`` returns rmsnorm(stream) * norm_weight in
-    ``out_dtype``."""
+                      bias: Optional[torch.Tensor] = None, y2=None, scale2: Optional[torch.Tensor] = None,
+                      norm_weight: Optional[torch.Tensor] = None, eps: float = 0.0,
+                      out_dtype: Optional[torch.dtype] = None, mixes: Optional[TimeMixes] = None):
+    """stream += scale1 * (y1 + bias) + scale2 * y2 in place, entry by entry (y1 float32; y2 a matrix or a
+    RoutedSum; every piece is optional, a scale that is None is one); with ``norm_weight`` returns h =
+    rmsnorm(stream) * norm_weight in ``out_dtype``. ``mixes`` (every row is a sequence of one token): returns
+    (h, [n, T, H] of h + (h' - h) * mu, h' the sequence's kept row)."""
     T, H = _check_stream(stream, "stream_scaled_sum")
     if H > 16384:
         raise KernelError(f"stream_scaled_sum: rows of up to 16384 entries, got {H}")
     if y1 is None and y2 is None and norm_weight is None:
         raise KernelError("stream_scaled_sum: nothing to do")
+    out_dtype = out_dtype or torch.float32
+    routed = y2 if isinstance(y2, RoutedSum) else None
+    if routed is not None and routed.rows.dtype == torch.bfloat16 and out_dtype == torch.float32:
+        y2, routed = routed.tensor(), None
+    if routed is not None:
+        y2 = None
+        if routed.shape != (T, H) or routed.rows.stride(1) != 1:
+            raise KernelError("stream_scaled_sum: the routed rows do not fit the stream")
     for y in (y1, y2):
         if y is not None and (not y.is_cuda or y.shape != stream.shape or not y.is_contiguous()):
             raise KernelError("stream_scaled_sum: the terms must be contiguous matrices of the stream's shape")
     if (y1 is not None and y1.dtype != torch.float32) or (y1 is None and bias is not None):
         raise KernelError("stream_scaled_sum: the first term is float32, and a bias goes with it")
-    out_dtype = out_dtype or torch.float32
     if y2 is not None and y2.dtype == torch.bfloat16 and out_dtype == torch.float32:
         y2 = y2.float()
     for v, what in ((scale1, "scale1"), (bias, "bias"), (scale2, "scale2"), (norm_weight, "norm_weight")):
         _f32_vec(v, H, f"stream_scaled_sum: {what}")
     out = torch.empty((T, H), dtype=out_dtype, device=stream.device) if norm_weight is not None else None
+    code = _dtype_code(routed.rows if routed is not None else y2) if (routed is not None or y2 is not None) else _F32
+    if routed is not None:
+        r = routed.routing
+        more = (_ptr(routed.rows), ctypes.c_long(routed.rows.stride(0)), _ptr(r.pos_of),
+                _ptr(r.wgt) if routed.weighted else None, r.top, _ptr(routed.shared))
+    else:
+        more = (None, ctypes.c_long(0), None, None, 0, None)
+    mixed = None
+    if mixes is not None:
+        S = mixes.mu.shape[0]
+        _f32_vec(mixes.mu, S * H, "stream_scaled_sum: mu")
+        _i32(mixes.slots, "state_slots")
+        st = mixes.state
+        if norm_weight is None or mixes.slots.numel() != T or st.dim() != 2 or st.dtype != torch.float32 \
+                or not st.is_contiguous() or not st.is_cuda or mixes.off < 0 or mixes.off + H > st.shape[1]:
+            raise KernelError("stream_scaled_sum: mixes need a norm, a state slot a row and kept rows inside the slots")
+        mixed = torch.empty((S, T, H), dtype=out_dtype, device=stream.device)
+        mix = (_ptr(mixed), ctypes.c_long(T * H), _ptr(mixes.mu), S, _ptr(st), ctypes.c_long(st.stride(0)),
+               ctypes.c_long(mixes.off), _ptr(mixes.slots))
+    else:
+        mix = (None, ctypes.c_long(0), None, 0, None, ctypes.c_long(0), ctypes.c_long(0), None)
     _check(library.load("stream").ptl_stream_scaled_sum(
-        _ptr(stream), _ptr(y1), _ptr(scale1), _ptr(bias), _ptr(y2), _dtype_code(y2) if y2 is not None else _F32,
-        _ptr(scale2), _ptr(norm_weight), ctypes.c_float(eps), _ptr(out),
-        _F32 if out_dtype == torch.float32 else _BF16, T, H, _stream()), "stream_scaled_sum")
-    return out
+        _ptr(stream), _ptr(y1), _ptr(scale1), _ptr(bias), _ptr(y2), code, _ptr(scale2), *more, _ptr(norm_weight),
+        ctypes.c_float(eps), _ptr(out), _F32 if out_dtype == torch.float32 else _BF16, *mix, T, H, _stream()),
+        "stream_scaled_sum")
+    return out if mixes is None else (out, mixed)
 
 
 def stream_rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch.dtype) -> torch.Tensor:
@@ -1876,6 +1931,7 @@ def memory_scan(p: torch.Tensor, q_off: int, k_off: int, v_off: int, i_off: int,
 ACT_SILU, ACT_CLAMPED = 0, 1           # gated: act(gate) * up
 ACT_RELU2 = 2                          # no gate: relu(up)^2
 SCORE_SIGMOID, SCORE_SOFTMAX = 0, 1
+ROUTE_FEW_ROWS = 32                    # rows up to which choice and ordering are one kernel (one workgroup)
 
 
 def gated_act(gate_up: torch.Tensor, act: int, limit: float = 0.0) -> torch.Tensor:
@@ -1943,22 +1999,26 @@ def moe_route(logits: torch.Tensor, experts: int, top: int, extra: int = 0,
     r.wgt = torch.empty(A, dtype=torch.float32, device=dev)
     r.extra = torch.empty((T, extra), dtype=torch.float32, device=dev) if extra else None
     r.ident = torch.empty(T, dtype=torch.float32, device=dev) if identity else None
-    _check(lib.ptl_moe_topk(_ptr(logits), int(logits.stride(0)), _ptr(logit_bias), T, outputs, top, extra, int(renormalize),
-                            int(score), _ptr(correction), experts, ctypes.c_float(renorm_eps),
-                            ctypes.c_float(weight_scale), int(groups), int(keep_groups), _ptr(r.idx),
-                            _ptr(r.wgt), _ptr(r.extra), _ptr(r.ident), _stream()), "moe_topk")
-    _check(lib.ptl_moe_sort(_ptr(r.idx), A, experts, _ptr(r.pos_of), _ptr(r.sorted), _ptr(r.expert_end),
-                            _ptr(r.tile_expert), _ptr(r.tile_row0), r.max_tiles, _stream()), "moe_sort")
+    how = (_ptr(logits), int(logits.stride(0)), _ptr(logit_bias), T, outputs, top, extra, int(renormalize),
+           int(score), _ptr(correction), experts, ctypes.c_float(renorm_eps), ctypes.c_float(weight_scale),
+           int(groups), int(keep_groups), _ptr(r.idx), _ptr(r.wgt), _ptr(r.extra), _ptr(r.ident))
+    where = (_ptr(r.pos_of), _ptr(r.sorted), _ptr(r.expert_end), _ptr(r.tile_expert), _ptr(r.tile_row0), r.max_tiles)
+    if T <= ROUTE_FEW_ROWS and outputs <= 256:
+        _check(lib.ptl_moe_route_few(*how, *where, _stream()), "moe_route")
+        return r
+    _check(lib.ptl_moe_topk(*how, _stream()), "moe_topk")
+    _check(lib.ptl_moe_sort(_ptr(r.idx), A, experts, *where, _stream()), "moe_sort")
     return r
 
 
 def moe_experts(x: torch.Tensor, r: Routing, gate_up: torch.Tensor, down: torch.Tensor, act: int,
                 limit: float, weight_on_input: bool, shared: Optional[torch.Tensor] = None,
-                shared_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                shared_gate: Optional[torch.Tensor] = None, defer_sum: bool = False):
     """The routed experts on x [T, K]: gate_up [E, 2 I, K] (for an activation without a gate,
     ACT_RELU2: the up matrices [E, I, K]), down [E, N, I]; returns float32 [T, N] = sum over a
     row's choices of its experts' outputs (+ shared_gate[t] * shared[t], + r.ident[t] * x[t] for
-    the experts that return their input)."""
+    the experts that return their input). ``defer_sum`` (no gate, no such experts): a RoutedSum, the
+    sum being left to whoever reads the result."""
     _need_gpu(x, gate_up, down, shared, shared_gate)
     T, K = x.shape
     E, I2, _ = gate_up.shape
@@ -1994,12 +2054,25 @@ def moe_experts(x: torch.Tensor, r: Routing, gate_up: torch.Tensor, down: torch.
     _check(lib.ptl_moe_down(_ptr(rows), ctypes.c_long(N), _ptr(mid), ctypes.c_long(I), _ptr(down),
                             _ptr(r.tile_expert), _ptr(r.tile_row0), _ptr(r.expert_end), r.max_tiles, A, N, I,
                             code, _stream()), "moe_down")
-    y = torch.empty((T, N), dtype=torch.float32, device=x.device)
-    _check(lib.ptl_moe_combine(_ptr(y), _ptr(rows), ctypes.c_long(N), _ptr(r.pos_of),
-                               None if weight_on_input else _ptr(r.wgt), r.top, _ptr(shared), _ptr(shared_gate),
-                               int(shared_gate.stride(0)) if shared_gate is not None else 0,
-                               _ptr(x) if r.ident is not None else None, ctypes.c_long(x.stride(0)),
-                               _ptr(r.ident), T, N, code, _stream()), "moe_combine")
+    pending = RoutedSum(rows, r, not weight_on_input, shared)
+    if defer_sum:
+        if shared_gate is not None or r.ident is not None:
+            raise KernelError("moe_experts: a gate or experts that return their input need the sum made here")
+        return pending
+    return moe_combine(pending, shared_gate, x)
+
+
+def moe_combine(p: RoutedSum, shared_gate: Optional[torch.Tensor] = None, x: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """The sum that ``p`` stands for, float32 [T, N] (moe_experts: the gate of the shared expert, and x for
+    experts that return their input)."""
+    r, (T, N) = p.routing, p.shape
+    ident = r.ident is not None
+    y = torch.empty((T, N), dtype=torch.float32, device=p.rows.device)
+    _check(library.load("moe").ptl_moe_combine(
+        _ptr(y), _ptr(p.rows), ctypes.c_long(N), _ptr(r.pos_of), _ptr(r.wgt) if p.weighted else None, r.top,
+        _ptr(p.shared), _ptr(shared_gate), int(shared_gate.stride(0)) if shared_gate is not None else 0,
+        _ptr(x) if ident else None, ctypes.c_long(x.stride(0) if ident else 0), _ptr(r.ident), T, N,
+        _dtype_code(p.rows), _stream()), "moe_combine")
     return y
 
 
@@ -2369,18 +2442,31 @@ def linear_decode_lowrank(out: torch.Tensor, p: torch.Tensor, q_off: int, k_off:
         "linear_decode_lowrank")
 
 
+LINEAR_HEAD_FUSED = 64     # values a head up to which linear_decode_bonus can finish the heads itself
+
+
 def linear_decode_bonus(out: torch.Tensor, p: torch.Tensor, q_off: int, k_off: int, v_off: int, a_off: int,
                         w: torch.Tensor, bias: torch.Tensor, bonus: torch.Tensor, state: torch.Tensor,
-                        q_start: torch.Tensor, state_slots: torch.Tensor, D: int, keep=None) -> None:
+                        q_start: torch.Tensor, state_slots: torch.Tensor, D: int, keep=None, finish=None) -> None:
     """One token of every sequence named by q_start and state_slots: the recurrence of linear_scan with a
     ``bonus`` and the decays exp(-exp(w . tanh(r) + bias)), r the columns of p from a_off on; ``keep`` as
-    there."""
+    there. ``finish`` = (y [T, H * Dv], weight float32 [H * Dv], column of the gate in p, eps), for Dv up to
+    LINEAR_HEAD_FUSED: the heads' results divided by their root mean square, times the weight, times
+    silu(gate) into y; out then gives the sizes only."""
     n, H, Dv, R = _lowrank_columns(out, p, q_off, k_off, v_off, a_off, w, bias, state, q_start, state_slots, D,
                                    "linear_decode_bonus")
     _f32_vec(bonus, H * D, "linear_decode_bonus: bonus")
     kept = _kept_row(keep, out.shape[0], state, linear_state_floats(H, D, Dv), "linear_decode_bonus")
+    head = (None, 0, None, 0, ctypes.c_float(0.0))
+    if finish is not None:
+        y, weight, gate_off, eps = finish
+        _f32_vec(weight, H * Dv, "linear_decode_bonus: weight")
+        if y.shape != (out.shape[0], H * Dv) or not y.is_contiguous() or not y.is_cuda or Dv > LINEAR_HEAD_FUSED \
+                or gate_off < 0 or gate_off + H * Dv > p.shape[1]:
+            raise KernelError("linear_decode_bonus: finished heads of up to 64 values, a dense y, a gate inside p")
+        head = (_ptr(y), _dtype_code(y), _ptr(weight), int(gate_off), ctypes.c_float(eps))
     _check(library.load("linear_scan").ptl_linear_decode_bonus(
-        _ptr(out), _ptr(p), ctypes.c_long(p.stride(0)), int(q_off), int(k_off), int(v_off), int(a_off), _ptr(w),
+        _ptr(out), *head, _ptr(p), ctypes.c_long(p.stride(0)), int(q_off), int(k_off), int(v_off), int(a_off), _ptr(w),
         _ptr(bias), R, _ptr(bonus), *kept, _ptr(state), ctypes.c_long(state.stride(0)), _ptr(q_start),
         _ptr(state_slots), n, H, D, Dv, _stream()), "linear_decode_bonus")
 

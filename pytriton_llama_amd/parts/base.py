@@ -41,6 +41,8 @@ inside a kernel it launches anyway:
                               norm returns it when called with scale_ok=True; a mixer or
                               feed-forward whose class says ``takes_pending_scale`` applies the
                               factor to the results of its first product.
+    ops.RoutedSum             the rows of routed experts, not added up; a feed-forward whose class
+                              says ``can_defer_sum`` returns it when called with defer_sum=True.
     PendingSum(terms, bias)   a weighted sum of one or two results and a bias, not added up; a
                               block with a norm on its sublayers' outputs adds it up inside that
                               norm's kernel.
@@ -228,7 +230,8 @@ class PendingSum:
 
 def as_tensor(v):
     """``v`` finished, if it is one of the pending values."""
-    return v.tensor() if isinstance(v, (PendingProduct, PendingScale, PendingSum)) else v
+    from ..ops import RoutedSum
+    return v.tensor() if isinstance(v, (PendingProduct, PendingScale, PendingSum, RoutedSum)) else v
 
 
 def run_norm(norm, x, residual, consumer=None):

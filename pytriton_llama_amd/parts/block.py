@@ -427,10 +427,12 @@ class ParallelResidualBlock(Part):
         h = rmsnorm(x) w;    x <- x + s1 * mixer(h) + s2 * ffn(h)
 
     The feed-forward with its scale is optional; ``scaled`` False: no scales in the checkpoint. The stream
-    is the block's ``h`` (float32 [T, hidden], updated in place). The sum, a bias that the mixer's result
-    still lacks (parts.base.PendingSum) and the norm in front of the block that runs next (``next_block``)
-    are one kernel; the normed rows travel where other blocks carry a residual. Sublayers read the
-    engine's dtype; the mixer may return float32 or it, and so may the feed-forward."""
+    is the block's ``h`` (float32 [T, hidden], updated in place). The sum is not made by the block when one
+    of its kind runs next (``next_block``): it travels where other blocks carry a residual, and the next
+    block's first kernel adds it up (with a bias that the mixer's result still lacks, parts.base.PendingSum,
+    and the rows of routed experts, ops.RoutedSum), norms the new stream and, in front of a mixer that asks
+    for it (``mixes``), makes the mixer's inputs as well. Sublayers read the engine's dtype; the mixer may
+    return float32 or it, and so may the feed-forward."""
     takes_next_block = True
 
     def __init__(self, hidden_size: int, mixer: Part, norm: Part, feed_forward: Part = None, scaled: bool = True,
@@ -486,19 +488,33 @@ class ParallelResidualBlock(Part):
             self.scale2 = place(tensors[b], "vector", dtype, device)
 
     def forward(self, h, residual, ctx, cache, next_block=None):
+        """``residual``: what the block before has left to be added to the stream (y1, its scale, its bias,
+        y2, its scale), or None; returned the same way."""
         if h.dtype != torch.float32 or h.shape[1] != self.hidden_size:
             raise ops.KernelError("a parallel-residual block runs on a float32 residual stream")
         stream, dtype = h, self.norm1.dtype
-        a = residual
-        if a is None:
-            a = ops.stream_scaled_sum(stream, norm_weight=self.norm1.weight, eps=self.norm1.eps, out_dtype=dtype)
-        y, bias = self.mixer.forward(a, ctx, cache), None
+        left = residual if residual is not None else (None,) * 5
+        mixes = self.mixer.mixes(ctx, cache) if hasattr(self.mixer, "mixes") else None
+        a = ops.stream_scaled_sum(stream, *left, norm_weight=self.norm1.weight, eps=self.norm1.eps, out_dtype=dtype,
+                                  mixes=mixes)
+        if mixes is None:
+            y = self.mixer.forward(a, ctx, cache)
+        else:
+            a, mixed = a
+            y = self.mixer.forward(a, ctx, cache, mixed)
+        bias = None
         if isinstance(y, PendingSum) and len(y.terms) == 1 and y.terms[0][1] == 1.0 and y.norms is None \
                 and (y.bias is None or y.bias[1] == 1.0):
             y, bias = y.terms[0][0], (y.bias[0] if y.bias is not None else None)
         y = as_tensor(y)
-        z = as_tensor(self.feed_forward.forward(a)) if self.feed_forward is not None else None
-        norm = next_block.norm1 if isinstance(next_block, ParallelResidualBlock) else None
-        return stream, ops.stream_scaled_sum(stream, y if y.dtype == torch.float32 else y.float(), self.scale1, bias, z,
-                                             self.scale2, norm.weight if norm is not None else None,
-                                             norm.eps if norm is not None else 0.0, dtype)
+        z = None
+        if self.feed_forward is not None:
+            if getattr(self.feed_forward, "can_defer_sum", False):
+                z = self.feed_forward.forward(a, defer_sum=True)
+            else:
+                z = as_tensor(self.feed_forward.forward(a))
+        left = (y if y.dtype == torch.float32 else y.float(), self.scale1, bias, z, self.scale2)
+        if isinstance(next_block, ParallelResidualBlock):
+            return stream, left
+        ops.stream_scaled_sum(stream, *left, out_dtype=dtype)
+        return stream, None

@@ -259,7 +259,12 @@ class RoutedExperts(Part):
     def make_decode_copies(self) -> int:
         return self.shared.make_decode_copies() if self.shared is not None else 0
 
-    def forward(self, x):
+    @property
+    def can_defer_sum(self) -> bool:
+        return not self.shared_gate and not self.identity
+
+    def forward(self, x, defer_sum: bool = False):
+        """``defer_sum``: the sum over a token's experts is left to whoever reads it (ops.RoutedSum)."""
         x = as_tensor(x)
         logits = linear(x, self.router, out_dtype=torch.float32)
         r = ops.moe_route(logits, self.num_experts, self.top, 1 if self.shared_gate else 0, self.renormalize,
@@ -267,4 +272,4 @@ class RoutedExperts(Part):
                           self.groups, self.keep_groups, self.router_bias)
         shared = self.shared.forward(x) if self.shared is not None else None
         return ops.moe_experts(x, r, self.gate_up, self.down, self.act, self.limit, self.weight_on_input,
-                               shared, r.extra)
+                               shared, r.extra, defer_sum)

@@ -263,21 +263,34 @@ class TimeMixer(Part):
         return sum(t.numel() * t.element_size() for t in (self.proj_blocked, self.o_blocked)
                    if t is not None)
 
-    def forward(self, x, ctx, cache):
+    def mixes(self, ctx, cache):
+        """What the norm in front of this mixer needs to make its inputs as well (ops.TimeMixes), for a step
+        that brings single tokens only; None for any other step."""
+        if ctx.num_decode_seqs != ctx.num_seqs:
+            return None
+        return ops.TimeMixes(self.mu, cache.state, self.x_off, ctx.state_slots)
+
+    def forward(self, x, ctx, cache, mixed=None):
+        """``mixed``: the inputs [5, T, hidden], when the norm in front has made them (``mixes``)."""
         x, state = as_tensor(x), cache.state
         T, H, D, c = x.shape[0], self.num_heads, self.dim, self.cols
-        mixes = ops.time_shift(x, self.mu, state, self.x_off, ctx.q_start, ctx.state_slots)
-        p = ops.gemm_groups(mixes, self.proj, c, self.proj_blocked)
+        if mixed is None:
+            mixed = ops.time_shift(x, self.mu, state, self.x_off, ctx.q_start, ctx.state_slots)
+        p = ops.gemm_groups(mixed, self.proj, c, self.proj_blocked)
         o = torch.empty((T, H, D), dtype=torch.float32, device=x.device)
+        out = torch.empty((T, H * D), dtype=x.dtype, device=x.device)
         keep = (x, self.x_off)              # (the recurrences' kernels leave the last rows in the slots)
         n = ctx.num_decode_seqs
+        finish = None
+        if n == ctx.num_seqs and D <= ops.LINEAR_HEAD_FUSED:
+            finish = (out, self.norm_weight, 3 * c, self.eps)
         if n:
             ops.linear_decode_bonus(o, p, 0, c, 2 * c, 4 * c, self.w2, self.w0, self.bonus, state, ctx.q_start[:n + 1],
-                                    ctx.state_slots[:n], D, keep)
+                                    ctx.state_slots[:n], D, keep, finish)
         if n < ctx.num_seqs:
             decay = ops.lowrank_decay(p[:, 4 * c:], self.w2, self.w0, form=ops.DECAY_EXP)
             ops.linear_scan(o, p, p[:, c:], p[:, 2 * c:], H, D, state, ctx.q_start[n:], ctx.state_slots[n:],
                             max(ctx.q_lens[n:]), decay=decay, bonus=self.bonus, keep=keep)
-        out = torch.empty((T, H * D), dtype=x.dtype, device=x.device)
-        ops.head_norm_gate(out, o, 1, 0.0, self.norm_weight, True, 1.0, p, 3 * c, ops.GATE_SILU, self.eps)
+        if finish is None:
+            ops.head_norm_gate(out, o, 1, 0.0, self.norm_weight, True, 1.0, p, 3 * c, ops.GATE_SILU, self.eps)
         return linear(out, self.o, out_dtype=torch.float32, blocked=self.o_blocked)

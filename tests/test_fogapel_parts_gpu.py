@@ -168,6 +168,26 @@ def test_one_token_with_low_rank_decays_and_a_bonus(gpu_device, sizes, rank):
             close(y[i], want[s][step], 1e-5)
             assert torch.equal(state[slots[s], off:off + W].cpu().double(), x_all[s][step])
     assert bool((state[[2, 3, 5]] == 0).all())
+    if Dv > ops.LINEAR_HEAD_FUSED:
+        return
+    # the heads finished by the same kernel: norm, weight, gate
+    weight = rn(H * Dv)
+    state.zero_()
+    for step in range(max(lens)):
+        live = [s for s in range(3) if step < lens[s]]
+        gate = rn(len(live), H * Dv)
+        p = dev(torch.cat([torch.stack([p_all[s][step] for s in live]), gate], dim=1))
+        for dtype in DTYPES:
+            keep = state.clone()
+            y = torch.full((len(live), H * Dv), float("nan"), dtype=dtype, device="cuda")
+            ops.linear_decode_bonus(torch.empty(len(live), H, Dv, device="cuda"), p, 0, H * D, 2 * H * D,
+                                    2 * H * D + H * Dv, dev(w2), dev(w0), dev(u), keep,
+                                    i32(list(range(len(live) + 1))), i32([slots[s] for s in live]), D,
+                                    finish=(y, dev(weight), width, 1e-4))
+            for i, s in enumerate(live):
+                o = plain.rms(want[s][step], 1e-4).reshape(-1) * weight * plain.silu(gate[i])
+                close(y[i], o, 2e-5 if dtype == torch.float32 else 6e-3)
+        state = keep
 
 
 @pytest.mark.parametrize("T,C,R", [(1, 5, 1), (70, 33, 7), (300, 130, 64), (65, 64, 16), (17, 200, 65), (3, 70, 200)])
@@ -370,6 +390,29 @@ def test_scaled_sum_and_the_norm_that_follows(gpu_device, dtype, T, H):
         ops.stream_scaled_sum(dev(x), dev(y1)[:, :-1])
 
 
+@pytest.mark.parametrize("dtype", DTYPES, ids=["fp32", "bf16"])
+@pytest.mark.parametrize("T,H", [(1, 24), (7, 33), (9, 2048), (30, 1100)])
+def test_mixes_made_behind_the_norm(gpu_device, dtype, T, H):
+    """Rows that are sequences of one token: the norm's kernel makes the time mixer's inputs as well,
+    the same that time_shift makes from its result."""
+    from pytriton_llama_amd import ops
+    torch.manual_seed(H)
+    stream, y1 = torch.randn(T, H).cuda(), torch.randn(T, H).cuda()
+    w, mu = torch.randn(H).cuda(), torch.rand(5, H).cuda()
+    state = torch.randn(T + 2, H + 6).to(dtype).float().cuda()
+    slots = i32((torch.randperm(T + 2)[:T]).tolist())
+    again = stream.clone()
+    h, mixed = ops.stream_scaled_sum(stream, y1, norm_weight=w, eps=1e-5, out_dtype=dtype,
+                                     mixes=ops.TimeMixes(mu, state, 4, slots))
+    assert torch.equal(h, ops.stream_scaled_sum(again, y1, norm_weight=w, eps=1e-5, out_dtype=dtype))
+    assert torch.equal(stream, again)
+    assert torch.equal(mixed, ops.time_shift(h, mu, state, 4, i32(range(T + 1)), slots))
+    with pytest.raises(ops.KernelError):
+        ops.stream_scaled_sum(stream, y1, norm_weight=w, out_dtype=dtype, mixes=ops.TimeMixes(mu, state, 7, slots))
+    with pytest.raises(ops.KernelError):
+        ops.stream_scaled_sum(stream, y1, norm_weight=w, out_dtype=dtype, mixes=ops.TimeMixes(mu, state, 0, slots[:-1]))
+
+
 # ---- feed-forwards -----------------------------------------------------------------------------
 @pytest.mark.parametrize("M", [1, 5, 16, 24, 60, 130])
 @pytest.mark.parametrize("activation", ["clamped", "silu"])
@@ -424,6 +467,18 @@ def test_routed_experts(gpu_device, T, shared, dtype):
     want = plain.routed(x.double(), mlp, wd, "")
     got = part.forward(x.cuda()).cpu()
     close(got[clear], want[clear], 1e-5 if dtype == torch.float32 else 2e-2)
+    # the sum left to the kernel that adds it to the stream
+    from pytriton_llama_amd import ops
+    assert part.can_defer_sum
+    stream, scale, nw = torch.randn(T, W), torch.randn(W), torch.randn(W)
+    left = part.forward(x.cuda(), defer_sum=True)
+    assert isinstance(left, ops.RoutedSum) and left.shape == (T, W)
+    close(left.tensor()[clear.cuda()], want[clear], 1e-5 if dtype == torch.float32 else 2e-2)
+    held = stream.cuda()
+    out = ops.stream_scaled_sum(held, y2=left, scale2=scale.cuda(), norm_weight=nw.cuda(), eps=1e-5, out_dtype=dtype)
+    total = stream.double() + scale.double() * left.tensor().double().cpu()
+    close(held, total, 1e-6)
+    close(out, plain.rms(total, 1e-5) * nw.double(), 3e-6 if dtype == torch.float32 else 6e-3)
 
 
 # ---- attention with capped scores ----------------------------------------------------------------
