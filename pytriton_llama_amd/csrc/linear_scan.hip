@@ -289,7 +289,8 @@ __global__ void __launch_bounds__(256, chunk_workgroups(NDT, FINAL)) linear_chun
 
     if (CHANNEL) {
       // The two diagonal tiles: lane (t, lg) walks s from t down, w = q_t times the decays of
-      // s + 1 .. t (bonus: of s + 1 .. t - 1 from s = t - 1 on, and q_t times u at s = t); wave w takes tile w % 2 and half of the key channels, a lane every fourth float4.
+      // s + 1 .. t (bonus: of s + 1 .. t - 1 from s = t - 1 on, and q_t times u at s = t); wave w takes tile
+      // w % 2 and half of the key channels, a lane every fourth float4.
       if (FINAL) {
         const int base = 16 * (wave & 1), half = wave >> 1;
         float acc[16];

@@ -1,7 +1,8 @@
 // A routed feed-forward (mixture of experts) that never leaves the device, so that a step with
 // one can be recorded as a graph:
 //
-//   ptl_moe_topk      per token: logits (plus a per-expert bias, when one is given), scores = sigmoid(logits) or softmax(logits) in float32, the ``top``
+//   ptl_moe_topk      per token: logits (plus a per-expert bias, when one is given), scores =
+//                     sigmoid(logits) or softmax(logits) in float32, the ``top``
 //                     largest (by score plus a per-expert correction, when one is given), their
 //                     experts and scores (the score without the correction is the weight, with or
 //                     without a renormalisation over the chosen ones, times a constant); with
@@ -232,8 +233,8 @@ static bool route_ok(int ld, int E, int top, int extra, const float* extra_out, 
 // must be given when real < E, receives the sum of their weights). Weights: the scores, divided by
 // their sum + renorm_eps when ``renormalize``, times wscale. n_groups > 1: the E outputs form that
 // many equal groups of neighbours (at most 64) of which the best keep_groups can be chosen from.
-extern "C" int ptl_moe_topk(const float* logits, int ld, const float* logit_bias, int T_, int E, int top, int extra, int renormalize,
-                            int score_fn, const float* bias, int real, float renorm_eps, float wscale,
+extern "C" int ptl_moe_topk(const float* logits, int ld, const float* logit_bias, int T_, int E, int top, int extra,
+                            int renormalize, int score_fn, const float* bias, int real, float renorm_eps, float wscale,
                             int n_groups, int keep_groups, int32_t* idx, float* wgt, float* extra_out,
                             float* ident_out, hipStream_t st) {
   if (T_ <= 0) return PTL_OK;

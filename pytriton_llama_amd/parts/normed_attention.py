@@ -62,7 +62,8 @@ class NormedAttention(Part):
     The cache keeps the normed and rotated keys [kv_heads * maps, dim] and the values [kv_heads,
     vdim] of every token. ``own_kv`` False: the layer has no key and value tensors and reads the
     cache layer of another one (the run order hands it over, not writable); sizes and rotation
-    are the owner's. ``o_bias`` False: the output projection has no bias even with ``bias``. Scores, softmax, norms, angles and lam are float32; the projection's result is
+    are the owner's. ``o_bias`` False: the output projection has no bias even with ``bias``.
+    Scores, softmax, norms, angles and lam are float32; the projection's result is
     taken in float32 so that bias and norm see it unrounded. Tensor names are parameters; biases
     are the projection's name with ".b" added. ``rot_scaling``: None, or the numbers of a
     frequency scaling: factor, original, fast, slow (a ramp between the entries that turn fast and
@@ -76,8 +77,8 @@ class NormedAttention(Part):
                  own_kv: bool = True, window: Optional[int] = None, keep_first: int = 0,
                  sink_name: Optional[str] = None, sink: Optional[float] = None, chunk: Optional[int] = None,
                  head_gated: bool = False, o_bias: bool = True, softcap: Optional[float] = None, taps: int = 0,
-                 rot_layout: str = "half", conv_suffix: str = ".conv", q_name: str = "q", k_name: str = "k", v_name: str = "v",
-                 g_name: str = "g", o_name: str = "o", lambda_names=("lq1", "lk1", "lq2", "lk2")):
+                 rot_layout: str = "half", conv_suffix: str = ".conv", q_name: str = "q",
+                 k_name: str = "k", v_name: str = "v", g_name: str = "g", o_name: str = "o", lambda_names=("lq1", "lk1", "lq2", "lk2")):
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} heads are not a multiple of {num_kv_heads} kv heads")
         if maps not in (1, 2):
@@ -99,6 +100,8 @@ class NormedAttention(Part):
             raise ValueError(f"unknown layout of the rotating entries {rot_layout!r} (known: 'pairs', 'half')")
         if taps < 0 or (softcap is not None and softcap <= 0):
             raise ValueError("taps are not negative, and a softcap is positive")
+        if softcap and keep_first:
+            raise ValueError("capped scores with kept first tokens are not built")
         self.taps, self.conv_suffix = int(taps), conv_suffix
         self.rot_layout = ops.ROT_PAIRS if rot_layout == "pairs" else ops.ROT_HALF
         self.softcap = float(softcap) if softcap else 0.0

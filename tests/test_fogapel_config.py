@@ -156,7 +156,7 @@ def test_what_the_mixers_refuse():
     ok = dict(hidden_size=16, num_heads=2, num_kv_heads=1, dim=8, vdim=8)
     for bad in (dict(taps=3), dict(rot_layout="pairs"), dict(qk_norm="rotated", maps=2),
                 dict(qk_norm="rotated", own_kv=False), dict(qk_norm="rotated", rot_layout="thirds"),
-                dict(qk_norm="rotated", softcap=-1.0), dict(qk_norm="rotated", taps=-1), dict(qk_norm="last")):
+                dict(qk_norm="rotated", softcap=-1.0), dict(softcap=5.0, window=9, keep_first=2), dict(qk_norm="rotated", taps=-1), dict(qk_norm="last")):
         with pytest.raises(ValueError):
             NormedAttention(**ok, **bad)
     with pytest.raises(ValueError):
